@@ -15,29 +15,13 @@
 #include <string>
 #include <vector>
 
-namespace py = pybind11;
-#define P(x) reinterpret_cast<void*>(static_cast<uintptr_t>(x))
-#define CP(x) reinterpret_cast<const void*>(static_cast<uintptr_t>(x))
-#define FP(x) reinterpret_cast<float*>(static_cast<uintptr_t>(x))
-#define CFP(x) reinterpret_cast<const float*>(static_cast<uintptr_t>(x))
-#define IP(x) reinterpret_cast<int*>(static_cast<uintptr_t>(x))
-#define CIP(x) reinterpret_cast<const int*>(static_cast<uintptr_t>(x))
-#define ST(x) reinterpret_cast<hipStream_t>(static_cast<uintptr_t>(x))
-typedef uint64_t u64;
+#include "bindings_decoder.h"
 
 PYBIND11_MODULE(_dnn_hip, m) {
   m.doc() = "distributed_neural_networks_amd HIP/CDNA4 kernels (gfx950)";
   m.attr("arch") = "gfx950";
+  bind_decoder(m);
 
-  m.def("gemm_bf16", [](u64 A, int lda, u64 W, int ldw, u64 C, int ldc, u64 bias, u64 R, int ldr, int M, int N,
-                        int K, int act, int out_f32, u64 st, u64 wsh, u64 rowstat, u64 colsum, u64 ws,
-                        long long ws_bytes) {
-    return dnn_gemm_bf16(CP(A), lda, CP(W), ldw, P(C), ldc, CFP(bias), CP(R), ldr, M, N, K, act, out_f32, ST(st),
-                         CP(wsh), CFP(rowstat), CFP(colsum), P(ws), ws_bytes);
-  }, py::arg("A"), py::arg("lda"), py::arg("W"), py::arg("ldw"), py::arg("C"), py::arg("ldc"), py::arg("bias"),
-     py::arg("R"), py::arg("ldr"), py::arg("M"), py::arg("N"), py::arg("K"), py::arg("act"), py::arg("out_f32"),
-     py::arg("st"), py::arg("wsh") = 0, py::arg("rowstat") = 0, py::arg("colsum") = 0, py::arg("ws") = 0,
-     py::arg("ws_bytes") = 0);
   m.def("gemm_skinny", [](u64 A, int lda, u64 sa, u64 W, int ldw, u64 sw, u64 C, int ldc, u64 bias, u64 R, int ldr,
                           int M, int N, int K, int act, int out_f32, int fp8, u64 st) {
     return dnn_gemm_skinny(CP(A), lda, CFP(sa), CP(W), ldw, CFP(sw), P(C), ldc, CFP(bias), CP(R), ldr, M, N, K, act,
@@ -209,17 +193,6 @@ PYBIND11_MODULE(_dnn_hip, m) {
   }, py::arg("qkv"), py::arg("ldqkv"), py::arg("kc"), py::arg("vc"), py::arg("o"), py::arg("B"), py::arg("H"),
      py::arg("Hkv"), py::arg("hd"), py::arg("S"), py::arg("pos"), py::arg("cos"), py::arg("sin"), py::arg("scale"),
      py::arg("splits"), py::arg("ws"), py::arg("st"), py::arg("kv8") = 0);
-  m.def("sample_topk", [](u64 x, int ld, int M, int N, u64 out, float temperature, int topk, unsigned seed, u64 step,
-                          u64 st) {
-    return dnn_sample_topk(CP(x), ld, M, N, reinterpret_cast<int*>(out), temperature, topk, seed,
-                           reinterpret_cast<const int*>(step), ST(st));
-  });
-  m.def("argmax_rows", [](u64 x, int ld, int M, int N, u64 out, int f32in, u64 st, u64 out2, u64 pos_inc, u64 part,
-                          u64 hist, int hist_ld) {
-    return dnn_argmax_rows(CP(x), ld, M, N, IP(out), f32in, ST(st), IP(out2), IP(pos_inc),
-                           reinterpret_cast<void*>(static_cast<uintptr_t>(part)), IP(hist), hist_ld);
-  }, py::arg("x"), py::arg("ld"), py::arg("M"), py::arg("N"), py::arg("out"), py::arg("f32in"), py::arg("st"),
-     py::arg("out2") = 0, py::arg("pos_inc") = 0, py::arg("part") = 0, py::arg("hist") = 0, py::arg("hist_ld") = 0);
   m.def("quant_fp8_rows", [](u64 x, int ldx, u64 q, u64 scale, int M, int K, int kpad, u64 st, int split) {
     return dnn_quant_fp8_rows(CP(x), ldx, P(q), FP(scale), M, K, kpad, ST(st), split);
   }, py::arg("x"), py::arg("ldx"), py::arg("q"), py::arg("scale"), py::arg("M"), py::arg("K"), py::arg("kpad"),

@@ -270,9 +270,7 @@ long long dnn_comm_create(const void* id128, int nranks, int rank, int device, i
   std::memset(c->done_tok, 0, sizeof(c->done_tok));
   {
     DeviceGuard g(device);
-    int lo = 0, hi = 0;
-    hipDeviceGetStreamPriorityRange(&lo, &hi);  // hi = numerically smallest = most urgent
-    bool ok = hipStreamCreateWithPriority(&c->stream, hipStreamNonBlocking, hi) == hipSuccess;
+    bool ok = hipStreamCreateWithFlags(&c->stream, hipStreamNonBlocking) == hipSuccess;
     for (int i = 0; ok && i < Channel::RING; ++i)
       ok = hipEventCreateWithFlags(&c->in_ev[i], hipEventDisableTiming) == hipSuccess &&
            hipEventCreateWithFlags(&c->done_ev[i], hipEventDisableTiming) == hipSuccess;

@@ -71,6 +71,13 @@ __device__ __forceinline__ f32x2 gelu_erf2(f32x2 x) {
   return f32x2{x[0] >= 0.f ? x[0] - q[0] : q[0], x[1] >= 0.f ? x[1] - q[1] : q[1]};
 }
 
+// tanh-form GELU: 0.5 x (1 + tanh(u)) = x / (1 + exp(-2 u)), u = sqrt(2 / pi)
+// (x + 0.044715 x^3); one v_exp and one v_rcp (results feed bf16 stores).
+__device__ __forceinline__ float gelu_tanh(float x) {
+  const float u2 = x * fmaf(0.0713548162726f, x * x, 1.59576912160573f);  // 2 u
+  return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(u2 * -1.4426950408889634f));
+}
+
 __device__ __forceinline__ float silu(float x) { return x / (1.0f + __expf(-x)); }
 
 // DPP lane moves (VALU, no LDS round trip — __shfl_xor lowers to

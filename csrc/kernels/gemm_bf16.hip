@@ -138,10 +138,10 @@ __global__ __launch_bounds__(256, 2) void gemm_bf16_tn_kernel(
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int m = m0 + wm * 64 + i * 16 + (lane & 15);
-    if (ACT == ACT_SILU_MUL) {
+    if (is_glu(ACT)) {
 #pragma unroll
       for (int jp = 0; jp < 2; ++jp)
-        epi_silu_pair<OUT_F32>(acc[i][2 * jp], acc[i][2 * jp + 1], m, (n0 + wn * 64 + jp * 32) / 2, M, N / 2, Cv,
+        epi_glu_pair<ACT, OUT_F32>(acc[i][2 * jp], acc[i][2 * jp + 1], m, (n0 + wn * 64 + jp * 32) / 2, M, N / 2, Cv,
                                ldc, vec, lane);
     } else if (!OUT_F32 && pair) {
 #pragma unroll
@@ -525,7 +525,7 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
             acc[mq][nq][i][j] = acc[mq][nq][i][j] * rs[mq][i].x + rs[mq][i].y * cs[nq][j];
   }
   // the bias from the LDS copy, added here: the output calls get none to load
-  const bool badd = epv && bias != nullptr && ACT != ACT_SILU_MUL;  // uniform
+  const bool badd = epv && bias != nullptr && !is_glu(ACT);  // uniform
   if (badd) {
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq)
@@ -554,7 +554,7 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
   // first output is computed, so the tile pays one memory round trip for R
   // instead of one per output row group (-20..-25 % GEMM throughput otherwise,
   // profiles/archive/r2_gemm_epilogue_cost.jsonl).
-  if (res_pre && !OUT_F32 && ACT != ACT_SILU_MUL && pair && R != nullptr && n0 + TN - 1 < N && (gan & 4) == 0 &&
+  if (res_pre && !OUT_F32 && !is_glu(ACT) && pair && R != nullptr && n0 + TN - 1 < N && (gan & 4) == 0 &&
       (ldr & 7) == 0 && (reinterpret_cast<uintptr_t>(R) & 15) == 0) {
     // the residual tile by LDS-DMA into the dead operand buffers (res_tile_dma;
     // anatomy bit 4 = the per-lane gathers below)
@@ -575,7 +575,7 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
         }
     return;
   }
-  if (res_pre && !OUT_F32 && ACT != ACT_SILU_MUL && pair && R != nullptr && n0 + TN - 1 < N) {
+  if (res_pre && !OUT_F32 && !is_glu(ACT) && pair && R != nullptr && n0 + TN - 1 < N) {
     bf16x4 rr[2][NQ][4][2];
 #pragma unroll
     for (int mq = 0; mq < 2; ++mq)
@@ -604,8 +604,8 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
       for (int i = 0; i < 4; ++i) {
         const int m = m0 + mq * 128 + arow + i * 16 + (lane & 15);
         const int nb = n0 + nq * 128 + wc * 32;
-        if (ACT == ACT_SILU_MUL) {
-          epi_silu_pair<OUT_F32>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
+        if (is_glu(ACT)) {
+          epi_glu_pair<ACT, OUT_F32>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
         } else if (SCATTER) {
           // widened 16-B stores as in epi_pair_bf16, to the head-major / cache
           // destination of the lane's 8 columns (host: ACT_NONE, bf16 out, no
@@ -924,7 +924,7 @@ __global__ __launch_bounds__(512, 1) void gemm_fp8_256_kernel(
         }
     return;
   }
-  const bool badd = epv && bias != nullptr && ACT != ACT_SILU_MUL;  // uniform: bias added from the LDS copy
+  const bool badd = epv && bias != nullptr && !is_glu(ACT);  // uniform: bias added from the LDS copy
   const float* bias_e = badd ? nullptr : bias;
   // SCATTER: the cache positions of the lane's 8 rows, loaded before any store (qkv_row_pos)
   int spos[2][4] = {};
@@ -937,7 +937,7 @@ __global__ __launch_bounds__(512, 1) void gemm_fp8_256_kernel(
   const bool vec = epi_vec_ok(C, ldc, bias, R, ldr);
   const bool pair = vec && epi_pair_ok(C, ldc, bias, R, ldr);
   // residual rows of the whole tile in flight before the first output (as in the bf16 kernel)
-  const bool rpre = ACT != ACT_SILU_MUL && pair && R != nullptr && n0 + TN - 1 < N;
+  const bool rpre = !is_glu(ACT) && pair && R != nullptr && n0 + TN - 1 < N;
   // the residual tile by LDS-DMA into the dead operand buffers (res_tile_dma;
   // anatomy bit 4 = the per-lane gathers below)
   const bool rdma = rpre && (gan & 4) == 0 && (ldr & 7) == 0 && (reinterpret_cast<uintptr_t>(R) & 15) == 0;
@@ -986,8 +986,8 @@ __global__ __launch_bounds__(512, 1) void gemm_fp8_256_kernel(
         }
         if (SCATTER) {
           if (nb < N) epi_pair_scatter(v[0], v[1], m, nb + scat.c_off, M, bias_e, lane, scat, spos[mq][i]);
-        } else if (ACT == ACT_SILU_MUL) {
-          epi_silu_pair<false>(v[0], v[1], m, nb / 2, M, N / 2, C, ldc, vec, lane);
+        } else if (is_glu(ACT)) {
+          epi_glu_pair<ACT, false>(v[0], v[1], m, nb / 2, M, N / 2, C, ldc, vec, lane);
         } else if (rdma) {
           const int rl = m - m0, cl = nb - n0 + (lane >> 4) * 4;
           epi_pair_bf16<ACT, true>(v[0], v[1], m, nb, M, C, ldc, bias_e, R, ldr, lane, res_tile_read<TN>(smem, rl, cl),
@@ -1145,7 +1145,7 @@ static void launch_gemm(const void* A, int lda, const void* W, int ldw, void* C,
   // in a second launch — 1 + 1/2 rounds instead of 2 full ones, no workspace
   // and no reduction (the two launches write disjoint columns).
   const int ntm256 = (M + BG_M - 1) / BG_M;
-  const int Na = (big && ACT != ACT_SILU_MUL) ? tail_split_cols(M, N) : 0;
+  const int Na = (big && !is_glu(ACT)) ? tail_split_cols(M, N) : 0;
   if (Na > 0) {
     const int Nt = N - Na;
     const size_t cb = F32 ? sizeof(float) : sizeof(bf16_t);
@@ -1186,13 +1186,21 @@ extern "C" int dnn_gemm_bf16(const void* A, int lda, const void* W, int ldw, voi
     return (int)hipGetLastError();                                                                   \
   }
   DISPATCH(ACT_NONE)
+#ifndef DNN_DECODER_ONLY  // the other families' epilogues: not in the decoder subset (ops/build.py)
   DISPATCH(ACT_RELU)
   DISPATCH(ACT_GELU)
   DISPATCH(ACT_SILU_MUL)
+#endif
 #undef DISPATCH
+  if (act == ACT_GELU_TANH_MUL && !out_f32) {
+    launch_gemm<ACT_GELU_TANH_MUL, false>(A, lda, W, ldw, C, ldc, bias, R, ldr, M, N, K, st, Wsh, rs, colsum, ws,
+                                          ws_bytes);
+    return (int)hipGetLastError();
+  }
   return -2;
 }
 
+#ifndef DNN_DECODER_ONLY
 extern "C" int dnn_silu_mul_packed(const void* gu, int ld_in, void* out, int ld_out, int M, int F, hipStream_t st) {
   const int n = M * F;
   hipLaunchKernelGGL(silu_mul_packed_kernel, dim3((n + 255) / 256), dim3(256), 0, st, (const bf16_t*)gu, ld_in,
@@ -1275,10 +1283,10 @@ extern "C" int dnn_gemm_fp8_256(const void* A, const float* sa, const void* W, c
                                 const float* bias, const void* R, int ldr, int M, int N, int Kb, int act,
                                 hipStream_t st) {
   if (Kb % 128 != 0 || M <= 0 || N <= 0 || sa == nullptr || sw == nullptr) return -1;
-  if (act == ACT_SILU_MUL && N % 16 != 0) return -1;
+  if (is_glu(act) && N % 16 != 0) return -1;
   const int tiles = ((M + BG_M - 1) / BG_M) * ((N + BG_N - 1) / BG_N);
   // tail split (as launch_gemm's): GPT-2 XL O / c_proj (N = 1600) and c_fc (N = 6400) at M = 32768
-  const int Na = act != ACT_SILU_MUL ? tail_split_cols(M, N, true) : 0;
+  const int Na = !is_glu(act) ? tail_split_cols(M, N, true) : 0;
   const int ntm256 = (M + BG_M - 1) / BG_M, Nt = N - Na;
 #define F8L(a)                                                                                                    \
   if (act == a) {                                                                                                 \
@@ -1316,7 +1324,7 @@ extern "C" int dnn_gemm_fp8_mx(const void* A8, const void* sx, const void* W8, c
   if (qo != nullptr && (act != ACT_GELU || sxo == nullptr || kpo % 128 != 0 || kpo < N || ldq < kpo ||
                         (ldq & 7) != 0 || ((uintptr_t)qo & 7) != 0))
     return -1;
-  if (act == ACT_SILU_MUL && N % 16 != 0) return -1;
+  if (is_glu(act) && N % 16 != 0) return -1;
   const int tiles = ((M + BG_M - 1) / BG_M) * ((N + BG_N - 1) / BG_N);
   const uint32_t* sxw = reinterpret_cast<const uint32_t*>(sx);
   if (qo != nullptr) {
@@ -1353,3 +1361,4 @@ extern "C" int dnn_gemm_fp8_qkv_scatter_mx(const void* A8, const void* sx, const
                      N, Kb, sc, reinterpret_cast<const uint32_t*>(sx));
   return (int)hipGetLastError();
 }
+#endif  // DNN_DECODER_ONLY

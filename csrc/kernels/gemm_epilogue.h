@@ -7,7 +7,18 @@
 
 namespace dnn {
 
-enum Act { ACT_NONE = 0, ACT_RELU = 1, ACT_GELU = 2, ACT_SILU_MUL = 3 };
+enum Act { ACT_NONE = 0, ACT_RELU = 1, ACT_GELU = 2, ACT_SILU_MUL = 3, ACT_GELU_TANH_MUL = 4 };
+
+// Gated activations: the weight holds packed gate|up rows (ops/gemm.py
+// pack_gate_up) and the output act(gate) * up has half its columns.
+__host__ __device__ constexpr bool is_glu(int act) { return act == ACT_SILU_MUL || act == ACT_GELU_TANH_MUL; }
+
+// Activation of the gate half.
+template <int ACT>
+__device__ __forceinline__ float glu_gate(float g) {
+  if constexpr (ACT == ACT_GELU_TANH_MUL) return gelu_tanh(g);
+  return silu(g);
+}
 
 // Vector epilogue stores need 4-column-aligned rows and 16-B aligned bases.
 __device__ __forceinline__ bool epi_vec_ok(const void* C, int ldc, const float* bias, const bf16_t* R, int ldr) {
@@ -284,14 +295,14 @@ __device__ __forceinline__ bool epi_pair_ok(const void* C, int ldc, const float*
          ((uintptr_t)R & 7) == 0 && (R == nullptr || (ldr & 3) == 0);
 }
 
-// SwiGLU epilogue on a transposed accumulator tile of the packed gate|up
+// Gated (SwiGLU / tanh-GELU) epilogue on a transposed accumulator tile of the packed gate|up
 // weight (ops/gemm.py pack_gate_up: 8 gate rows, then the 8 matching up rows):
 // lanes 0-31 hold gate columns, lanes 32-63 the up columns of the same outputs,
 // so one xor-32 shuffle pairs them; lanes 0-31 write output columns
 // ncol0 + 4*(lane>>4) .. +3 of the [M, N/2] result.  Every lane must call this
 // (the shuffle), whatever its row.
-template <bool OUT_F32>
-__device__ __forceinline__ void epi_silu_t4(const f32x4& acc, int m, int ncol0, int M, int NO, void* __restrict__ Cv,
+template <int ACT, bool OUT_F32>
+__device__ __forceinline__ void epi_glu_t4(const f32x4& acc, int m, int ncol0, int M, int NO, void* __restrict__ Cv,
                                             int ldc, bool vec, int lane) {
   f32x4 other;
 #pragma unroll
@@ -300,7 +311,7 @@ __device__ __forceinline__ void epi_silu_t4(const f32x4& acc, int m, int ncol0, 
   const int ncol = ncol0 + (lane >> 4) * 4;
   f32x4 v;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) v[r] = silu(acc[r]) * other[r];
+  for (int r = 0; r < 4; ++r) v[r] = glu_gate<ACT>(acc[r]) * other[r];
   if (vec && ncol + 3 < NO) {
     if (OUT_F32) {
       *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(Cv) + (size_t)m * ldc + ncol) = v;
@@ -320,21 +331,24 @@ __device__ __forceinline__ void epi_silu_t4(const f32x4& acc, int m, int ncol0, 
     }
 }
 
-// SwiGLU epilogue of two adjacent 16-column tiles j, j+1 at full lane use: one
+// Gated epilogue of two adjacent 16-column tiles j, j+1 at full lane use: one
 // v_permlane32_swap per dword hands lanes 0-31 tile j's (gate, up) and lanes
-// 32-63 tile j+1's (epi_silu_t4 exchanged with ds_bpermute and left half the
+// 32-63 tile j+1's (epi_glu_t4 exchanged with ds_bpermute and left half the
 // lanes idle), and silu is x * rcp(1 + 2^(-x log2 e)) instead of an IEEE
 // divide.  Every lane writes output columns ncol0 + 4*(lane>>4) .. +3 of row m
 // (ncol0 = tile j's first output column).
-template <bool OUT_F32>
-__device__ __forceinline__ void epi_silu_pair(const f32x4& a0, const f32x4& a1, int m, int ncol0, int M, int NO,
+template <int ACT, bool OUT_F32>
+__device__ __forceinline__ void epi_glu_pair(const f32x4& a0, const f32x4& a1, int m, int ncol0, int M, int NO,
                                               void* __restrict__ Cv, int ldc, bool vec, int lane) {
   f32x4 v;
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const auto s = __builtin_amdgcn_permlane32_swap(__float_as_uint(a0[r]), __float_as_uint(a1[r]), false, false);
     const float g = __uint_as_float(s[0]), u = __uint_as_float(s[1]);
-    v[r] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * -1.4426950408889634f)) * u;
+    if constexpr (ACT == ACT_GELU_TANH_MUL)
+      v[r] = gelu_tanh(g) * u;
+    else
+      v[r] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * -1.4426950408889634f)) * u;
   }
   if (m >= M) return;
   const int ncol = ncol0 + (lane >> 4) * 4;

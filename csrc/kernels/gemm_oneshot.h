@@ -195,7 +195,7 @@ __global__ __launch_bounds__(256, 2) void gemm_oneshot_kernel(const uint8_t* __r
   // no memory round trip.  Uniform: vector-aligned operands, N % 4 == 0.
   constexpr int QPW = (NTW * MT + 3) / 4;  // epilogue tiles per wave
   // (14 VGPRs per tile: up to 2 tiles per wave; the 64 x 64 tiles spilled with 4)
-  constexpr bool PRE = QPW <= 2 && !SPLIT && ACT != ACT_SILU_MUL;
+  constexpr bool PRE = QPW <= 2 && !SPLIT && !is_glu(ACT);
   const bool pre = PRE && epi_pre && (N & 3) == 0 && epi_vec_ok(Cv, ldc, bias, R, ldr) &&
                    ((reinterpret_cast<uintptr_t>(sw) | reinterpret_cast<uintptr_t>(colsum)) & 15) == 0;
   // Unconditional, branch-free loads (absent operands read a valid dummy
@@ -519,8 +519,8 @@ __global__ __launch_bounds__(256, 2) void gemm_oneshot_kernel(const uint8_t* __r
       const bool vec = epi_vec_ok(Cv, ldc, bias, R, ldr);
       if constexpr (ABL & 8) {
         if (v[0] == 12345.f) reinterpret_cast<float*>(Cv)[0] = v[1];  // keep the sums live, store nothing
-      } else if constexpr (ACT == ACT_SILU_MUL) {
-        epi_silu_t4<false>(v, m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
+      } else if constexpr (is_glu(ACT)) {
+        epi_glu_t4<ACT, false>(v, m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
       } else if (pre && nb + 15 < N) {  // wave-uniform (epi_rowstat16 shuffles): the whole 16-column tile
         f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f};
         if (m < M) epi_t4_pre<ACT>(v, m, n, Cv, ldc, bias != nullptr, pre_b[k], R != nullptr, pre_r[k], &x);

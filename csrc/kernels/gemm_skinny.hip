@@ -173,7 +173,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_kernel(const uint8_t* __restr
   // and the epilogue pays no memory round trip after the barrier.  Uniform.
   // (14 VGPRs per column tile: only configs with room — the software-pipelined
   // and the wide ones spilled with it)
-  constexpr bool PRE = NT <= 2 && MT * NT * U <= 8 && !PIPE && !OUT_F32 && !FP8 && ACT != ACT_SILU_MUL;
+  constexpr bool PRE = NT <= 2 && MT * NT * U <= 8 && !PIPE && !OUT_F32 && !FP8 && !is_glu(ACT);
   constexpr int NP = PRE ? NT : 1;
   // (MT <= waves: wave t owns M tile t alone in the epilogue loop below, so its
   // prefetched operands are that tile's)
@@ -385,7 +385,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_kernel(const uint8_t* __restr
         }
       }
     }
-    if constexpr (ACT == ACT_SILU_MUL) {
+    if constexpr (is_glu(ACT)) {
 #pragma unroll
       for (int j = 0; j < NT; ++j) {
         if constexpr (FP8) {
@@ -393,7 +393,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_kernel(const uint8_t* __restr
 #pragma unroll
           for (int r = 0; r < 4; ++r) s[j][r] *= rs * (n + r < N ? sw[n + r] : 0.f);
         }
-        epi_silu_t4<OUT_F32>(s[j], m, (n0 + j * 16) / 2, M, N / 2, Cv, ldc, vec, lane);
+        epi_glu_t4<ACT, OUT_F32>(s[j], m, (n0 + j * 16) / 2, M, N / 2, Cv, ldc, vec, lane);
       }
     } else if (!OUT_F32 && !FP8 && (pre_t || rs_out != nullptr)) {  // uniform
 #pragma unroll
@@ -532,7 +532,7 @@ static int launch_stream_mt(const void* A, int lda_b, const void* Wsh, const flo
   hipLaunchKernelGGL((gemm_stream_kernel<MT, NT, W8, NORM, ACT, true>), grid, block, 0, st, (const uint8_t*)A, lda_b,
                      (const uint8_t*)Wsh, sw, C, ldc, bias, (const bf16_t*)R, ldr, M, N, nch, cps, colsum, eps, kelems,
                      (float*)ws, (unsigned*)nullptr);
-  const int NO = ACT == ACT_SILU_MUL ? N / 2 : N;
+  const int NO = is_glu(ACT) ? N / 2 : N;
   const long long threads = (long long)M * ((NO + 3) / 4);
   hipLaunchKernelGGL((gemm_stream_reduce<ACT, NORM, W8>), dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, st,
                      (const float*)ws, splitk, MP, ntiles * BN, (const uint8_t*)A, lda_b, sw, colsum, eps, kelems, C,
@@ -657,7 +657,7 @@ static int launch_os_cfg(const void* A, int lda_b, const void* Wsh, const float*
   if (splitk == 1) {
     // row statistics: partials of the output (not for the half-width SwiGLU
     // output); merged partials of the input when they fit OS_RS_SPT per thread
-    float2* rso = ACT != ACT_SILU_MUL ? g_rs_cur.out : nullptr;
+    float2* rso = !is_glu(ACT) ? g_rs_cur.out : nullptr;
     const float2* rsi = (NORM != 0 && (kelems + 15) / 16 <= OS_RS_SPT * (256 / MP)) ? g_rs_cur.in : nullptr;
     if constexpr (ABL == 0 && MT == 2 && STEPS == 1 && !W8 && NORM == 2 && ACT == ACT_GELU && NTW <= 2) {
       if (g_os_probe_abl != 0 && rsi == nullptr) {
@@ -684,7 +684,7 @@ static int launch_os_cfg(const void* A, int lda_b, const void* Wsh, const float*
   hipLaunchKernelGGL((gemm_oneshot_kernel<MT, NTW, W8, NORM, ACT, true, STEPS>), grid, block, smem, st,
                      (const uint8_t*)A, lda_b, (const uint8_t*)Wsh, sw, C, ldc, bias, (const bf16_t*)R, ldr, M, N, nch,
                      cps, colsum, eps, kelems, (float*)ws, ntiles, mgroups);
-  const int NO = ACT == ACT_SILU_MUL ? N / 2 : N;
+  const int NO = is_glu(ACT) ? N / 2 : N;
   const long long threads = (long long)M * ((NO + 3) / 4);
   hipLaunchKernelGGL((gemm_stream_reduce<ACT, NORM, W8>), dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, st,
                      (const float*)ws, splitk, mgroups * MP, ntiles * BN, (const uint8_t*)A, lda_b, sw, colsum, eps,
@@ -727,6 +727,7 @@ extern "C" int dnn_gemm_set_oneshot(int on, int mt, int ntw, int steps, int spli
   return 0;
 }
 
+#ifndef DNN_DECODER_ONLY  // probes: not in the decoder subset (ops/build.py)
 // Sweep / A-B entry (bench/oneshot_sweep.py): plain product (no epilogue), an
 // explicit config; returns -1 when the config does not apply to the shape.
 extern "C" int dnn_gemm_oneshot_sweep(const void* A, int lda, const void* Wsh, const float* sw, void* C, int ldc, int M,
@@ -790,6 +791,7 @@ extern "C" int dnn_gemm_oneshot_ablate(const void* A, int lda, const void* Wsh, 
 #undef ABLC
   return -2;
 }
+#endif
 
 template <int ACT, int NORM, bool W8>
 static bool stream_eligible(const void* A, int lda_b, const void* Wsh, int M, int N, int kbytes) {
@@ -840,7 +842,7 @@ static int launch_skinny_cfg(const void* A, int lda_b, const float* sa, const vo
   while (ks > 1 && kbytes / 64 < ks) ks >>= 1;
   size_t smem = (size_t)ks * NT * MT * 64 * sizeof(f32x4);
   if (NORM != NORM_NONE) smem += (size_t)ks * MT * 2 * 16 * sizeof(float);
-  float2* rso = (!F32 && !FP8 && ACT != ACT_SILU_MUL) ? g_rs_cur.out : nullptr;
+  float2* rso = (!F32 && !FP8 && !is_glu(ACT)) ? g_rs_cur.out : nullptr;
   hipLaunchKernelGGL((gemm_skinny_kernel<ACT, F32, MT, NT, FP8, U, PIPE, NORM, W8, MS>), dim3(groups), dim3(64 * ks), smem,
                      st, (const uint8_t*)A, lda_b, sa, (const uint8_t*)W, ldw_b, sw, C, ldc, bias, (const bf16_t*)R,
                      ldr, M, N, kbytes, colsum, eps, (const uint8_t*)Wsh, rso, g_rs_cur.out_ld, g_epi_pre);
@@ -977,9 +979,16 @@ extern "C" int dnn_gemm_skinny(const void* A, int lda, const float* sa, const vo
   const int eb = fp8 ? 1 : 2;
   const int kbytes = K * eb;
   if (M <= 0 || M > (fp8 ? 64 : SKINNY_MAX_M) || N <= 0 || kbytes % 64 != 0) return -1;
-  if (act == ACT_SILU_MUL && N % 16 != 0) return -1;  // packed gate|up groups of 8+8
+  if (is_glu(act) && N % 16 != 0) return -1;  // packed gate|up groups of 8+8
   if (fp8 && (sa == nullptr || sw == nullptr)) return -1;
   const int la = lda * eb, lw = ldw * eb;
+#ifdef DNN_DECODER_ONLY
+  if (act == ACT_NONE && !fp8)
+    return out_f32 ? launch_skinny<ACT_NONE, true, false>(A, la, sa, W, lw, sw, C, ldc, bias, R, ldr, M, N, kbytes, st,
+                                                          nullptr, 0.f, Wsh)
+                   : launch_skinny<ACT_NONE, false, false>(A, la, sa, W, lw, sw, C, ldc, bias, R, ldr, M, N, kbytes,
+                                                           st, nullptr, 0.f, Wsh, ws, ws_bytes);
+#else
 #define SKD(a)                                                                                              \
   if (act == a) {                                                                                           \
     if (fp8) {                                                                                              \
@@ -998,9 +1007,14 @@ extern "C" int dnn_gemm_skinny(const void* A, int lda, const float* sa, const vo
   SKD(ACT_GELU)
   SKD(ACT_SILU_MUL)
 #undef SKD
+#endif
+  if (act == ACT_GELU_TANH_MUL && !fp8 && !out_f32)
+    return launch_skinny<ACT_GELU_TANH_MUL, false, false>(A, la, sa, W, lw, sw, C, ldc, bias, R, ldr, M, N, kbytes, st,
+                                                          nullptr, 0.f, Wsh, ws, ws_bytes);
   return -2;
 }
 
+#ifndef DNN_DECODER_ONLY
 // Pre-norm fused skinny GEMM (bf16): y = act(rstd (A W'^T - mean colsum) + bias) (+ R),
 // norm = 1 RMSNorm, 2 LayerNorm (colsum required); W', bias', colsum from
 // ops/gemm.py fold_norm.  act: NONE / GELU / SILU_MUL.
@@ -1010,7 +1024,7 @@ extern "C" int dnn_gemm_skinny_norm(const void* A, int lda, const void* W, int l
                                     long long ws_bytes) {
   const int kbytes = K * 2;
   if (M <= 0 || M > SKINNY_MAX_M || N <= 0 || kbytes % 64 != 0) return -1;
-  if (act == ACT_SILU_MUL && N % 16 != 0) return -1;
+  if (is_glu(act) && N % 16 != 0) return -1;
   if (norm == NORM_LN && colsum == nullptr) return -1;
   const int la = lda * 2, lw = ldw * 2;
 #define SKN(a, nm)                                                                                                   \
@@ -1034,7 +1048,7 @@ extern "C" int dnn_gemm_skinny_w8(const void* A, int lda, const void* W, int ldw
                                   const float* colsum, float eps, hipStream_t st, const void* Wsh, void* ws,
                                   long long ws_bytes) {
   if (M <= 0 || M > SKINNY_MAX_M || N <= 0 || K % 64 != 0 || ldw < K || sw == nullptr) return -1;
-  if (act == ACT_SILU_MUL && N % 16 != 0) return -1;
+  if (is_glu(act) && N % 16 != 0) return -1;
   if (norm == NORM_LN && colsum == nullptr) return -1;
   const int la = lda * 2;
 #define SKW(a, nm)                                                                                                    \
@@ -1212,3 +1226,4 @@ extern "C" int dnn_gemm_head(const void* A, int lda, const void* Wsh, const floa
 }
 
 }  // namespace dnn
+#endif  // DNN_DECODER_ONLY

@@ -152,7 +152,7 @@ __device__ __forceinline__ void str_combine_item(const float* slab, int splitk, 
   float mean = 0.f, rstd = 1.f;
   if constexpr (NORM != 0)
     str_row_norm<NORM, SC1>(slab + (size_t)splitk * MP * Ns, splitk, MP, tile, m, A, lda_b, kelems, eps, mean, rstd);
-  if constexpr (ACT == ACT_SILU_MUL) {
+  if constexpr (is_glu(ACT)) {
     const int NO = N / 2;
     if (o >= NO) return;
     const int g = o >> 3, w = o & 7;
@@ -161,7 +161,7 @@ __device__ __forceinline__ void str_combine_item(const float* slab, int splitk, 
     bf16_t* C = reinterpret_cast<bf16_t*>(Cv) + (size_t)m * ldc + o;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      if (o + r < NO) C[r] = f2bf(silu(gt[r]) * up[r]);
+      if (o + r < NO) C[r] = f2bf(glu_gate<ACT>(gt[r]) * up[r]);
   } else {
     if (o >= N) return;
     const bool vec = epi_vec_ok(Cv, ldc, bias, R, ldr);
@@ -189,8 +189,8 @@ __device__ __forceinline__ void str_combine_tile(const float* slab, int splitk, 
                                                  float eps, int kelems, void* __restrict__ Cv, int ldc,
                                                  const float* __restrict__ bias, const bf16_t* __restrict__ R, int ldr,
                                                  int M, int N, int tid) {
-  const int per_row = (ACT == ACT_SILU_MUL ? BN / 2 : BN) / 4;
-  const int o0 = (ACT == ACT_SILU_MUL ? tile * BN / 2 : tile * BN);
+  const int per_row = (is_glu(ACT) ? BN / 2 : BN) / 4;
+  const int o0 = (is_glu(ACT) ? tile * BN / 2 : tile * BN);
   for (int i = tid; i < MP * per_row; i += 256) {
     const int m = i / per_row, o = o0 + (i - m * per_row) * 4;
     if (m < M)
@@ -504,8 +504,8 @@ __global__ __launch_bounds__(256, 1) void gemm_stream_kernel(const uint8_t* __re
         } else if constexpr (NORM == 1) {
           v *= rstd[t];
         }
-        if constexpr (ACT == ACT_SILU_MUL) {
-          epi_silu_t4<false>(v, m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
+        if constexpr (is_glu(ACT)) {
+          epi_glu_t4<ACT, false>(v, m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
         } else {
           epi_t4<ACT, false>(v, m, n, M, N, Cv, ldc, bias, R, ldr, vec);
         }
@@ -525,7 +525,7 @@ __global__ __launch_bounds__(256) void gemm_stream_reduce(const float* __restric
                                                           const float* __restrict__ bias,
                                                           const bf16_t* __restrict__ R, int ldr, int M, int N,
                                                           int epi_pre = 1) {
-  const int NO = ACT == ACT_SILU_MUL ? N / 2 : N;
+  const int NO = is_glu(ACT) ? N / 2 : N;
   const int per_row = (NO + 3) / 4;
   const int idx = blockIdx.x * 256 + threadIdx.x;
   const int m = idx / per_row, o = (idx - m * per_row) * 4;

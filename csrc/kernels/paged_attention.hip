@@ -1,0 +1,541 @@
+// Attention over a paged KV cache, for batches of unequal sequences (gfx950).
+//
+// Cache: 64-key pages, keys [page][G][64][DK], values [page][G][64][DV] (DK and
+// DV independent), addressed by a block table (slot, position / 64) -> page, so
+// a sequence's keys may lie anywhere in the pool.  A query at position i sees
+// key j when j <= i and (i - j < window or j < keep): a sliding window whose
+// first `keep` keys stay visible; window = INT_MAX is plain causal attention.
+// Only pages that hold a visible key are read.  The query heads of a KV head
+// (H / G, any number) are packed with the queries into the 32 columns of the
+// MFMA: column r of a sequence's chunk is (token r / R, head r % R), R = H / G.
+// An optional per-head output gate, sigmoid of a column of the projection row,
+// multiplies the head's output.
+//
+//   paged_write    new k / v rows -> pages
+//   paged_prefill  chunks of >= 2 tokens; a workgroup takes 128 packed rows
+//                  (4 waves x 32), pages staged through LDS
+//   paged_decode   one token per sequence: 32-key units dealt to the 4 waves of
+//                  a workgroup (and over `splits` workgroups), merged in LDS;
+//                  the token's own k / v are written to the cache on the way
+//   paged_attn_f32 fp32, one wave per (row, head): the exact mode
+//
+// Scores, softmax and accumulation are fp32; S^T = K Q^T keeps a query on one
+// lane pair, so row maxima and sums are in registers, and O^T += V^T P^T takes
+// P from the score registers and V^T by transposing LDS reads.
+#include "common.h"
+#include "residual_api.h"
+
+namespace dnn {
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+
+constexpr int PG = 64;  // keys per page
+constexpr float LOG2E = 1.4426950408889634f;
+
+__device__ __forceinline__ bool pa_sees(int i, int j, int window, int keep) {
+  return j <= i && (i - j < window || j < keep);
+}
+// page index of (slot, block), -1 outside the table or the pool
+__device__ __forceinline__ int pa_page(const PagedAttnArgs& a, int slot, int blk) {
+  if (blk < 0 || blk >= a.ldt) return -1;
+  const int p = a.table[(size_t)slot * a.ldt + blk];
+  return p < a.npages ? p : -1;
+}
+// Visible key units of `unit` keys for queries qlo..qhi: the first ke units
+// hold kept keys, wb..we the window.
+struct Units {
+  int ke, wb, total;
+  __device__ __forceinline__ int at(int i) const { return i < ke ? i : wb + i - ke; }
+};
+__device__ __forceinline__ Units pa_units(int qlo, int qhi, int window, int keep, int unit) {
+  const int we = qhi / unit + 1;
+  Units u;
+  u.ke = min((keep + unit - 1) / unit, we);
+  u.wb = max(qlo >= window ? (qlo - window + 1) / unit : 0, u.ke);
+  u.total = u.ke + max(we - u.wb, 0);
+  return u;
+}
+
+// ---------------------------------------------------------------- cache write
+template <typename T>
+__global__ __launch_bounds__(256) void paged_write_kernel(PagedAttnArgs a) {
+  constexpr int E = 16 / sizeof(T);
+  const int ck = a.G * a.DK / E, cv = a.G * a.DV / E;
+  const long i = blockIdx.x * 256L + threadIdx.x;
+  if (i >= (long)a.M * (ck + cv)) return;
+  const int m = (int)(i / (ck + cv));
+  int c = (int)(i % (ck + cv));
+  const int p = a.pos[m], page = pa_page(a, a.slots[m], p / PG);
+  if (page < 0) return;
+  const T* src = reinterpret_cast<const T*>(a.qkv) + (size_t)m * a.ldq + a.H * a.DK;
+  T* dst;
+  int d, g;
+  if (c < ck) {
+    g = c * E / a.DK;
+    d = c * E - g * a.DK;
+    src += c * E;
+    dst = reinterpret_cast<T*>(a.kp) + (((size_t)page * a.G + g) * PG + p % PG) * a.DK + d;
+  } else {
+    c -= ck;
+    g = c * E / a.DV;
+    d = c * E - g * a.DV;
+    src += a.G * a.DK + c * E;
+    dst = reinterpret_cast<T*>(a.vp) + (((size_t)page * a.G + g) * PG + p % PG) * a.DV + d;
+  }
+  *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(src);
+}
+
+// ---------------------------------------------------------------- MFMA pieces
+template <int D>
+__device__ __forceinline__ int pa_swz(int key, int chunk) {  // 16-B chunk of a K row in LDS
+  return D == 64 ? (chunk ^ ((key >> 1) & 7)) : (chunk ^ (key & 15));
+}
+template <int DV>
+struct PaV {
+  static constexpr int STRIDE = DV * 2 + 64;  // padded rows: conflict-free transposing reads
+};
+
+// Online softmax of 16 score registers per 32-key tile (NT tiles); returns the
+// rescale of what was accumulated so far.  sc: scale * log2(e).
+template <int NT>
+__device__ __forceinline__ float pa_softmax(f32x16 (&s)[NT], float sc, float& m_i, float& l_i) {
+  float mx = -INFINITY;
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int g = 0; g < 16; g += 2) mx = fmax_nan(mx, fmax_nan(s[t][g], s[t][g + 1]));
+  mx = fmax_nan(mx, __shfl_xor(mx, 32, 64));
+  const float m_new = fmax_nan(m_i, mx * sc);
+  const float m_use = m_new == -INFINITY ? 0.f : m_new;
+  const float alpha = __builtin_amdgcn_exp2f(m_i - m_use);
+  float rs = 0.f;
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int g = 0; g < 16; ++g) {
+      s[t][g] = __builtin_amdgcn_exp2f(fmaf(s[t][g], sc, -m_use));
+      rs += s[t][g];
+    }
+  rs += __shfl_xor(rs, 32, 64);
+  l_i = fmaf(l_i, alpha, rs);
+  m_i = m_new;
+  return alpha;
+}
+
+// O^T += V^T P^T for one 32-key tile staged at vbuf (row 0 = the tile's first key).
+template <int DV>
+__device__ __forceinline__ void pa_pv(const char* vbuf, const f32x16& p, f32x16 (&o)[DV / 32], int lane) {
+  const int h = lane >> 5;
+#pragma unroll
+  for (int s = 0; s < 2; ++s) {
+    bf16x8 pf;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) pf[j] = (short)f2bf(p[8 * s + j]);
+    const int krow = 16 * s + 4 * h + ((lane & 15) >> 2);
+    const int gsub = (lane >> 4) & 1;
+#pragma unroll
+    for (int dt = 0; dt < DV / 32; ++dt) {
+      const char* a0 = vbuf + krow * PaV<DV>::STRIDE + (dt * 32 + gsub * 16 + 4 * (lane & 3)) * 2;
+      const s16x4 v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(a0));
+      const s16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(a0 + 8 * PaV<DV>::STRIDE));
+      const bf16x8 vf = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+      o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pf, o[dt], 0, 0, 0);
+    }
+  }
+}
+
+__device__ __forceinline__ float pa_gate(const PagedAttnArgs& a, int row, int head) {
+  if (a.gate < 0) return 1.f;
+  const float z = bf2f(reinterpret_cast<const bf16_t*>(a.qkv)[(size_t)row * a.ldq + a.gate + head]);
+  return 1.0f / (1.0f + __expf(-z));
+}
+
+// ---------------------------------------------------------------- prefill
+// tiles: {first batch row of the chunk, its tokens, slot, first packed row}
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_prefill_kernel(PagedAttnArgs a,
+                                                                                      const int4* __restrict__ tiles) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  char* ks = smem;
+  char* vs = smem + PG * DK * 2;
+  constexpr int NKS = DK / 16, NDT = DV / 32, CK = DK / 8, CV = DV / 8;
+  constexpr int NIK = PG * CK / 256, NIV = PG * CV / 256;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int h = lane >> 5, r32 = lane & 31;
+  const int g = blockIdx.x, R = a.H / a.G;
+  const int4 t = tiles[blockIdx.y];
+  const int tok0 = t.x, n = t.y, slot = t.z, row0 = t.w;
+  const int p0 = a.pos[tok0];
+  const int last = n - 1;
+  const int wrow = row0 + wave * 32, row = wrow + r32;
+  const int tk = min(row / R, last), head = g * R + row % R;
+  const int q_abs = p0 + tk;
+  const int wq_min = p0 + min(wrow / R, last), wq_max = p0 + min((wrow + 31) / R, last);
+  const Units u = pa_units(p0 + min(row0 / R, last), p0 + min((row0 + 127) / R, last), a.window, a.keep, PG);
+
+  bf16x8 qf[NKS];
+  {
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.qkv) + (size_t)(tok0 + tk) * a.ldq + head * DK + 8 * h;
+#pragma unroll
+    for (int s = 0; s < NKS; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(qp + s * 16);
+  }
+  f32x16 o[NDT];
+#pragma unroll
+  for (int i = 0; i < NDT; ++i) o[i] = f32x16{};
+  float m_i = -INFINITY, l_i = 0.f;
+  const float sc = a.scale * LOG2E;
+
+  i32x4 pk[NIK], pv[NIV];
+  auto fetch = [&](int i) __attribute__((always_inline)) {
+    const int page = max(pa_page(a, slot, u.at(i)), 0);  // a missing page is never visible; stay in the pool
+    const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kp) + ((size_t)page * a.G + g) * PG * DK;
+    const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vp) + ((size_t)page * a.G + g) * PG * DV;
+#pragma unroll
+    for (int it = 0; it < NIK; ++it) pk[it] = *reinterpret_cast<const i32x4*>(kb + (it * 256 + tid) * 8);
+#pragma unroll
+    for (int it = 0; it < NIV; ++it) pv[it] = *reinterpret_cast<const i32x4*>(vb + (it * 256 + tid) * 8);
+  };
+  if (u.total > 0) fetch(0);
+  for (int i = 0; i < u.total; ++i) {
+    const int kb0 = u.at(i) * PG;
+    __syncthreads();
+#pragma unroll
+    for (int it = 0; it < NIK; ++it) {
+      const int e = it * 256 + tid, key = e / CK, c = e % CK;
+      *reinterpret_cast<i32x4*>(ks + key * DK * 2 + (pa_swz<DK>(key, c) << 4)) = pk[it];
+    }
+#pragma unroll
+    for (int it = 0; it < NIV; ++it) {
+      const int e = it * 256 + tid, key = e / CV, c = e % CV;
+      *reinterpret_cast<i32x4*>(vs + key * PaV<DV>::STRIDE + c * 16) = pv[it];
+    }
+    __syncthreads();
+    if (i + 1 < u.total) fetch(i + 1);
+    // any key of the page visible to the wave's queries wq_min..wq_max?
+    if (kb0 > wq_max || (wq_min - (kb0 + PG - 1) >= a.window && kb0 >= a.keep)) continue;
+    f32x16 s[2];
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) {
+      s[kt] = f32x16{};
+      const int key = kt * 32 + r32;
+#pragma unroll
+      for (int k = 0; k < NKS; ++k) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(ks + key * DK * 2 + (pa_swz<DK>(key, 2 * k + h) << 4));
+        s[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[k], s[kt], 0, 0, 0);
+      }
+    }
+    // every key visible to every query of the wave: no mask
+    if (kb0 + PG - 1 > wq_min || !(wq_max - kb0 < a.window || kb0 + PG <= a.keep)) {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+          if (!pa_sees(q_abs, kb0 + kt * 32 + (e & 3) + 8 * (e >> 2) + 4 * h, a.window, a.keep)) s[kt][e] = -INFINITY;
+    }
+    const float alpha = pa_softmax<2>(s, sc, m_i, l_i);
+    if (!__all(alpha == 1.f)) {
+#pragma unroll
+      for (int d = 0; d < NDT; ++d) o[d] *= alpha;
+    }
+    pa_pv<DV>(vs, s[0], o, lane);
+    pa_pv<DV>(vs + 32 * PaV<DV>::STRIDE, s[1], o, lane);
+  }
+  if (row >= n * R) return;
+  const float f = (l_i > 0.f ? 1.f / l_i : 0.f) * pa_gate(a, tok0 + tk, head);
+  bf16_t* op = reinterpret_cast<bf16_t*>(a.out) + (size_t)(tok0 + tk) * a.ldo + head * DV;
+#pragma unroll
+  for (int d = 0; d < NDT; ++d)
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      *reinterpret_cast<uint2*>(op + d * 32 + 8 * q + 4 * h) =
+          make_uint2(pack2bf(o[d][4 * q] * f, o[d][4 * q + 1] * f), pack2bf(o[d][4 * q + 2] * f, o[d][4 * q + 3] * f));
+}
+
+// ---------------------------------------------------------------- decode
+// grid (G * head tiles, sequences, splits); rows[e] = batch row of sequence e.
+// ws (splits > 1): [e][H][splits][DV + 2] = {max, sum, O} partials.
+constexpr int DU = 32;  // keys per unit
+
+template <int DV>
+__host__ __device__ constexpr int pa_dec_lds(int rt_rows) {
+  const int v = 4 * DU * (DV * 2 + 64), m = 4 * rt_rows * (DV + 2) * 4;
+  return v > m ? v : m;
+}
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_kernel(PagedAttnArgs a,
+                                                                                     const int* __restrict__ rows,
+                                                                                     float* __restrict__ ws) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr int NKS = DK / 16, NDT = DV / 32, CV = DV / 8;
+  constexpr int NIV = DU * CV / 64;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int h = lane >> 5, r32 = lane & 31;
+  const int R = a.H / a.G, nrt = (R + 31) / 32;
+  const int g = blockIdx.x / nrt, rt = blockIdx.x % nrt;
+  const int rr = min(R - rt * 32, 32);  // query heads of this workgroup
+  const int e = blockIdx.y, row = rows[e], ns = gridDim.z;
+  const int slot = a.slots[row], p = a.pos[row];
+  char* vs = smem + wave * DU * PaV<DV>::STRIDE;
+
+  const Units u = pa_units(p, p, a.window, a.keep, DU);
+  const int ub = (int)((long)u.total * blockIdx.z / ns), ue = (int)((long)u.total * (blockIdx.z + 1) / ns);
+
+  const bf16_t* rowp = reinterpret_cast<const bf16_t*>(a.qkv) + (size_t)row * a.ldq;
+  // the token's own key and value: the wave that reads their unit (the last of
+  // the list) stores them first
+  const int lastw = (u.total - 1 - ub) & 3;
+  if (ue == u.total && wave == lastw) {
+    const int page = pa_page(a, slot, p / PG);
+    if (page >= 0) {
+      bf16_t* kd = reinterpret_cast<bf16_t*>(a.kp) + (((size_t)page * a.G + g) * PG + p % PG) * DK;
+      bf16_t* vd = reinterpret_cast<bf16_t*>(a.vp) + (((size_t)page * a.G + g) * PG + p % PG) * DV;
+      if (lane < DK / 8)
+        *reinterpret_cast<uint4*>(kd + lane * 8) =
+            *reinterpret_cast<const uint4*>(rowp + a.H * DK + g * DK + lane * 8);
+      if (lane < DV / 8)
+        *reinterpret_cast<uint4*>(vd + lane * 8) =
+            *reinterpret_cast<const uint4*>(rowp + (a.H + a.G) * DK + g * DV + lane * 8);
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  }
+
+  bf16x8 qf[NKS];
+  {
+    const bf16_t* qp = rowp + (g * R + rt * 32 + min(r32, rr - 1)) * DK + 8 * h;
+#pragma unroll
+    for (int s = 0; s < NKS; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(qp + s * 16);
+  }
+  f32x16 o[NDT];
+#pragma unroll
+  for (int i = 0; i < NDT; ++i) o[i] = f32x16{};
+  float m_i = -INFINITY, l_i = 0.f;
+  const float sc = a.scale * LOG2E;
+
+  bf16x8 kf[NKS];
+  i32x4 pv[NIV];
+  auto load = [&](int i) __attribute__((always_inline)) {
+    const int unit = u.at(i);
+    const int page = max(pa_page(a, slot, unit / (PG / DU)), 0);
+    const size_t k0 = ((size_t)page * a.G + g) * PG + (unit % (PG / DU)) * DU;
+    const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kp) + (k0 + r32) * DK + 8 * h;
+    const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vp) + k0 * DV;
+#pragma unroll
+    for (int s = 0; s < NKS; ++s) kf[s] = *reinterpret_cast<const bf16x8*>(kb + s * 16);
+#pragma unroll
+    for (int it = 0; it < NIV; ++it) pv[it] = *reinterpret_cast<const i32x4*>(vb + (it * 64 + lane) * 8);
+  };
+  int i = ub + wave;
+  if (i < ue) load(i);
+  for (; i < ue; i += 4) {
+    const int kb0 = u.at(i) * DU;
+    f32x16 s[1];
+    s[0] = f32x16{};
+#pragma unroll
+    for (int k = 0; k < NKS; ++k) s[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[k], qf[k], s[0], 0, 0, 0);
+#pragma unroll
+    for (int it = 0; it < NIV; ++it) {
+      const int c = it * 64 + lane;
+      *reinterpret_cast<i32x4*>(vs + (c / CV) * PaV<DV>::STRIDE + (c % CV) * 16) = pv[it];
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    if (i + 4 < ue) load(i + 4);
+    if (kb0 + DU - 1 > p || !(p - kb0 < a.window || kb0 + DU <= a.keep)) {
+#pragma unroll
+      for (int q = 0; q < 16; ++q)
+        if (!pa_sees(p, kb0 + (q & 3) + 8 * (q >> 2) + 4 * h, a.window, a.keep)) s[0][q] = -INFINITY;
+    }
+    const float alpha = pa_softmax<1>(s, sc, m_i, l_i);
+    if (!__all(alpha == 1.f)) {
+#pragma unroll
+      for (int d = 0; d < NDT; ++d) o[d] *= alpha;
+    }
+    pa_pv<DV>(vs, s[0], o, lane);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  }
+
+  // merge the four waves: {m, l, O[DV]} of each query head
+  __syncthreads();
+  float* mg = reinterpret_cast<float*>(smem);
+  if (r32 < rr) {
+    float* d = mg + (wave * rr + r32) * (DV + 2);
+    if (h == 0) {
+      d[0] = m_i;
+      d[1] = l_i;
+    }
+#pragma unroll
+    for (int t = 0; t < NDT; ++t)
+#pragma unroll
+      for (int q = 0; q < 16; ++q) d[2 + t * 32 + (q & 3) + 8 * (q >> 2) + 4 * h] = o[t][q];
+  }
+  __syncthreads();
+  for (int x = tid; x < rr * DV; x += 256) {
+    const int r = x / DV, c = x % DV, head = g * R + rt * 32 + r;
+    float m = -INFINITY;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) m = fmaxf(m, mg[(w * rr + r) * (DV + 2)]);
+    float l = 0.f, v = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float* d = mg + (w * rr + r) * (DV + 2);
+      const float f = d[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(d[0] - m);
+      l = fmaf(d[1], f, l);
+      v = fmaf(d[2 + c], f, v);
+    }
+    if (ns == 1) {
+      reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * DV + c] =
+          f2bf((l > 0.f ? v / l : 0.f) * pa_gate(a, row, head));
+    } else {
+      float* d = ws + (((size_t)e * a.H + head) * ns + blockIdx.z) * (DV + 2);
+      if (c == 0) {
+        d[0] = m;
+        d[1] = l;
+      }
+      d[2 + c] = v;
+    }
+  }
+}
+
+__global__ __launch_bounds__(64) void paged_combine_kernel(PagedAttnArgs a, const int* __restrict__ rows, int ns,
+                                                           const float* __restrict__ ws) {
+  const int e = blockIdx.x / a.H, head = blockIdx.x % a.H, row = rows[e];
+  const float* d = ws + ((size_t)e * a.H + head) * ns * (a.DV + 2);
+  float m = -INFINITY;
+  for (int s = 0; s < ns; ++s) m = fmaxf(m, d[s * (a.DV + 2)]);
+  const float gate = pa_gate(a, row, head);
+  for (int c = threadIdx.x; c < a.DV; c += 64) {
+    float l = 0.f, v = 0.f;
+    for (int s = 0; s < ns; ++s) {
+      const float* q = d + s * (a.DV + 2);
+      const float f = q[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(q[0] - m);
+      l = fmaf(q[1], f, l);
+      v = fmaf(q[2 + c], f, v);
+    }
+    reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.DV + c] = f2bf((l > 0.f ? v / l : 0.f) * gate);
+  }
+}
+
+// ---------------------------------------------------------------- fp32
+__global__ __launch_bounds__(256) void paged_attn_f32_kernel(PagedAttnArgs a) {
+  __shared__ float qs[4][256], ps[4][PG];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int x = min((int)(blockIdx.x * 4 + wave), a.M * a.H - 1);  // surplus waves repeat the last row
+  const int row = x / a.H, head = x % a.H, g = head / (a.H / a.G);
+  const int slot = a.slots[row], p = a.pos[row];
+  const float* rowp = reinterpret_cast<const float*>(a.qkv) + (size_t)row * a.ldq;
+  for (int d = lane; d < a.DK; d += 64) qs[wave][d] = rowp[head * a.DK + d];
+  __syncthreads();
+  const Units u = pa_units(p, p, a.window, a.keep, PG);
+  float m = -INFINITY, l = 0.f, o[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < u.total; ++i) {
+    const int blk = u.at(i), page = pa_page(a, slot, blk);
+    if (page < 0) continue;
+    const int key = blk * PG + lane;
+    const float* kr = reinterpret_cast<const float*>(a.kp) + (((size_t)page * a.G + g) * PG + lane) * a.DK;
+    float s = -INFINITY;
+    if (pa_sees(p, key, a.window, a.keep)) {
+      s = 0.f;
+      for (int d = 0; d < a.DK; d += 4) {
+        const f32x4 k4 = *reinterpret_cast<const f32x4*>(kr + d);
+        s = fmaf(k4[0], qs[wave][d], s);
+        s = fmaf(k4[1], qs[wave][d + 1], s);
+        s = fmaf(k4[2], qs[wave][d + 2], s);
+        s = fmaf(k4[3], qs[wave][d + 3], s);
+      }
+      s *= a.scale;
+    }
+    const float m_new = fmaxf(m, wave_max(s));
+    if (m_new == -INFINITY) continue;
+    const float alpha = expf(m - m_new), pr = expf(s - m_new);
+    l = l * alpha + wave_sum(pr);
+    m = m_new;
+    ps[wave][lane] = pr;
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    const float* vb = reinterpret_cast<const float*>(a.vp) + ((size_t)page * a.G + g) * PG * a.DV;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int d = lane + 64 * c;
+      if (d >= a.DV) break;
+      float v = o[c] * alpha;
+      for (int j = 0; j < PG; ++j) v = fmaf(ps[wave][j], vb[(size_t)j * a.DV + d], v);
+      o[c] = v;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+  }
+  float f = l > 0.f ? 1.f / l : 0.f;
+  if (a.gate >= 0) f *= 1.0f / (1.0f + expf(-rowp[a.gate + head]));
+  float* op = reinterpret_cast<float*>(a.out) + (size_t)row * a.ldo + head * a.DV;
+#pragma unroll
+  for (int c = 0; c < 4; ++c)
+    if (lane + 64 * c < a.DV) op[lane + 64 * c] = o[c] * f;
+}
+
+}  // namespace dnn
+
+using namespace dnn;
+
+static bool pa_ok(const PagedAttnArgs& a, int elem) {
+  auto dim = [](int d) { return d == 64 || d == 128 || d == 256; };
+  const int vec = 16 / elem;
+  return a.M > 0 && a.G > 0 && a.H > 0 && a.H % a.G == 0 && dim(a.DK) && dim(a.DV) && a.ldq % vec == 0 &&
+         a.ldo % 4 == 0 && a.ldo >= a.H * a.DV && a.ldq >= (a.H + a.G) * a.DK + a.G * a.DV &&
+         (a.gate < 0 || a.gate + a.H <= a.ldq) && a.window > 0 && a.keep >= 0 && a.ldt > 0 && a.npages > 0 &&
+         a.table != nullptr && a.slots != nullptr && a.pos != nullptr;
+}
+
+extern "C" int dnn_paged_write(const PagedAttnArgs* a, int f32, hipStream_t st) {
+  if (!pa_ok(*a, f32 ? 4 : 2)) return -1;
+  const long n = (long)a->M * a->G * (a->DK + a->DV) / (f32 ? 4 : 8);
+  const dim3 grid((unsigned)((n + 255) / 256));
+  if (f32) hipLaunchKernelGGL(paged_write_kernel<float>, grid, dim3(256), 0, st, *a);
+  else hipLaunchKernelGGL(paged_write_kernel<bf16_t>, grid, dim3(256), 0, st, *a);
+  return (int)hipGetLastError();
+}
+
+#define PA_DISPATCH(F)                                                           \
+  {                                                                              \
+    if (a->DK == 64 && a->DV == 64) F(64, 64)                                    \
+    else if (a->DK == 64 && a->DV == 128) F(64, 128)                             \
+    else if (a->DK == 64 && a->DV == 256) F(64, 256)                             \
+    else if (a->DK == 128 && a->DV == 64) F(128, 64)                             \
+    else if (a->DK == 128 && a->DV == 128) F(128, 128)                           \
+    else if (a->DK == 128 && a->DV == 256) F(128, 256)                           \
+    else if (a->DK == 256 && a->DV == 64) F(256, 64)                             \
+    else if (a->DK == 256 && a->DV == 128) F(256, 128)                           \
+    else F(256, 256)                                                             \
+  }
+
+extern "C" int dnn_paged_prefill(const PagedAttnArgs* a, const int* tiles, int ntiles, hipStream_t st) {
+  if (!pa_ok(*a, 2) || ntiles <= 0 || ntiles > 65535 || !(a->scale > 0.f) || ((uintptr_t)tiles & 15) != 0) return -1;
+  const dim3 grid(a->G, ntiles);
+#define PF(K, V)                                                                                                     \
+  hipLaunchKernelGGL((paged_prefill_kernel<K, V>), grid, dim3(256), PG * (K * 2 + PaV<V>::STRIDE), st, *a, \
+                     (const int4*)tiles);
+  PA_DISPATCH(PF)
+#undef PF
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_paged_decode(const PagedAttnArgs* a, const int* rows, int nrows, int splits, float* ws,
+                                long long ws_elems, hipStream_t st) {
+  if (!pa_ok(*a, 2) || nrows <= 0 || nrows > 65535 || splits < 1 || splits > 256 || !(a->scale > 0.f)) return -1;
+  if (splits > 1 && (ws == nullptr || ws_elems < (long long)nrows * a->H * splits * (a->DV + 2))) return -1;
+  const int R = a->H / a->G, rr = R < 32 ? R : 32;
+  const dim3 grid(a->G * ((R + 31) / 32), nrows, splits);
+#define PD(K, V) \
+  hipLaunchKernelGGL((paged_decode_kernel<K, V>), grid, dim3(256), pa_dec_lds<V>(rr), st, *a, rows, ws);
+  PA_DISPATCH(PD)
+#undef PD
+  if (splits > 1)
+    hipLaunchKernelGGL(paged_combine_kernel, dim3((unsigned)(nrows * a->H)), dim3(64), 0, st, *a, rows, splits, ws);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_paged_attn_f32(const PagedAttnArgs* a, hipStream_t st) {
+  if (!pa_ok(*a, 4)) return -1;
+  hipLaunchKernelGGL(paged_attn_f32_kernel, dim3((unsigned)(((long)a->M * a->H + 3) / 4)), dim3(256), 0, st, *a);
+  return (int)hipGetLastError();
+}

@@ -9,6 +9,8 @@ Behavioural contract (reference ``node.py:222-290``, ``config.json:1-18``):
   ``num_parts >= 1`` is accepted as long as the ``part_index`` values are a
   permutation of ``0..num_parts-1`` — the only way a pipeline of more than two
   stages (GPT-2 4-stage, Llama-3 8-stage) can be described with this schema.
+* ``model`` names a registered model, or a folder whose ``config.json`` names its
+  architecture (``models/__init__.py``).
 * Additive optional fields (absent in the reference file, so it still loads):
   top level ``model``, ``dtype``, ``transport``, ``micro_batch_size``,
   ``num_microbatches``, ``seq_len``, ``decode_steps``, ``prompt_len``, ``temperature``, ``top_k``,
@@ -22,13 +24,14 @@ Nothing here touches torch, so it is cheap to import from the CLI and tests.
 from __future__ import annotations
 
 import json
+import os
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional, Tuple
 
 TRANSPORTS = ("grpc", "colocated", "rccl", "gloo", "gloo_gpu")
 DIST_TRANSPORTS = ("rccl", "gloo", "gloo_gpu")  # one rank per stage (and replica)
 MODELS = ("cifar10", "gpt2", "gpt2-medium", "gpt2-large", "gpt2-xl", "gpt2-tiny",
-          "llama3-8b", "llama3-tiny")
+          "llama3-8b", "llama3-tiny", "kozusun-tiny", "kozusun-1b", "kozusun-8b")
 
 
 class ConfigError(Exception):
@@ -180,8 +183,8 @@ def parse_pipeline(cfg: Dict[str, Any], path: str = "<config>") -> PipelineConfi
     if transport not in TRANSPORTS:
         raise ConfigError(f"ERROR: unknown transport '{transport}', expected one of {TRANSPORTS}")
     model = cfg.get("model", "cifar10")
-    if model not in MODELS:
-        raise ConfigError(f"ERROR: unknown model '{model}', expected one of {MODELS}")
+    if model not in MODELS and not os.path.isfile(os.path.join(str(model), "config.json")):
+        raise ConfigError(f"ERROR: unknown model '{model}', expected one of {MODELS} or a folder with a config.json")
     for key in ("micro_batch_size", "num_microbatches"):
         v = cfg.get(key, 1)
         if not isinstance(v, int) or v < 1:

@@ -8,6 +8,7 @@ build command; CPU-only processes never call into it.
 from __future__ import annotations
 
 import importlib
+import importlib.util
 import os
 
 import torch  # noqa: F401  (must precede the extension: shared HIP runtime)
@@ -23,7 +24,8 @@ def verify_stamp(path: str) -> dict:
     ``DNN_SKIP_STAMP=1`` skips the check (kernel development only)."""
     import hashlib
     import json
-    stamp_path = os.path.join(os.path.dirname(path), "_dnn_hip.build.json")
+    from .build import source_digest, sources, stamp_path as stamp_of
+    stamp_path = stamp_of(path)
     if os.environ.get("DNN_SKIP_STAMP"):
         return {}
     if not os.path.exists(stamp_path):
@@ -32,8 +34,7 @@ def verify_stamp(path: str) -> dict:
     stamp = json.load(open(stamp_path))
     if hashlib.sha256(open(path, "rb").read()).hexdigest() != stamp.get("library_sha256"):
         raise RuntimeError(f"{path} does not match its build stamp (library replaced after the build); rebuild")
-    from .build import source_digest
-    now = source_digest()
+    now = source_digest(sources("decoder" if os.path.basename(path).startswith("_dnn_decoder") else ""))
     stale = sorted(k for k in set(now) | set(stamp.get("sources", {})) if now.get(k) != stamp["sources"].get(k))
     if stale:
         raise RuntimeError(f"{path} was built from different sources ({', '.join(stale[:6])}); rebuild with "
@@ -59,20 +60,29 @@ def lib():
     if _lib is None and os.environ.get("DNN_HIP_LIB"):
         _lib = _load_override(os.environ["DNN_HIP_LIB"])
     if _lib is None:
-        try:
-            mod = importlib.import_module("distributed_neural_networks_amd._dnn_hip")
-        except ImportError as e:
-            raise RuntimeError(
-                "HIP kernel library _dnn_hip is not built; run "
-                "`python -m distributed_neural_networks_amd.ops.build` (hipcc, gfx950)") from e
-        verify_stamp(mod.__file__)
-        _lib = mod
+        errors = []
+        for name in ("_dnn_hip", "_dnn_decoder"):  # the full library, else the decoder subset (ops/build.py)
+            spec = importlib.util.find_spec("distributed_neural_networks_amd." + name)
+            if spec is None:
+                continue
+            try:
+                verify_stamp(spec.origin)
+            except RuntimeError as e:
+                errors.append(e)
+                continue
+            _lib = importlib.import_module("distributed_neural_networks_amd." + name)
+            return _lib
+        if errors:
+            raise errors[0]
+        raise RuntimeError("HIP kernel library _dnn_hip is not built; run "
+                           "`python -m distributed_neural_networks_amd.ops.build` (hipcc, gfx950)")
     return _lib
 
 
 def build_stamp() -> dict:
     import json
-    p = os.path.join(os.path.dirname(library_path()), "_dnn_hip.build.json")
+    from .build import stamp_path
+    p = stamp_path(library_path())
     return json.load(open(p)) if os.path.exists(p) else {}
 
 

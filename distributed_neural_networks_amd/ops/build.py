@@ -22,8 +22,6 @@ PKG = os.path.join(ROOT, "distributed_neural_networks_amd")
 BUILD = os.path.join(ROOT, "build", "hip")
 ARCH = os.environ.get("DNN_OFFLOAD_ARCH", "gfx950")
 EXT_SUFFIX = sysconfig.get_config_var("EXT_SUFFIX") or ".so"
-LIB_PATH = os.path.join(PKG, "_dnn_hip" + EXT_SUFFIX)
-
 TRANSFORMER_SRCS = ("norm_embed.hip", "attention.hip", "sampler.hip", "gemm_fp8.hip")
 # ReLU/max-pool epilogues: no NaN-canonicalising v_max before every fmaxf of an MFMA result
 # No SLP vectoriser where it packs scalar FP32 into cross-half v_pk_*_f32 (op_sel
@@ -31,14 +29,17 @@ TRANSFORMER_SRCS = ("norm_embed.hip", "attention.hip", "sampler.hip", "gemm_fp8.
 # workgroups per CU that read returned the pre-op value in lanes 48-63 (the
 # one-shot GEMM's row statistics, csrc/kernels/gemm_oneshot.h "The race of rounds
 # 5-6"; 100 -> 0 mismatches in 10000 calls, profiles/r6_oneshot_race_root_cause.md).
-# Explicit vector code keeps its packed ops.
 NO_SLP = ["-fno-slp-vectorize"]
+# No packed FP32 instructions anywhere (some v_pk_*_f32 forms returned wrong
+# lanes, see above): explicit float2 / ext_vector code is split per element too.
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 PER_FILE_FLAGS = {"cifar_fused.hip": ["-ffast-math"],
                   # fp32-accurate split path: keep IEEE rounding, only drop NaN canonicalisation in fmaxf
                   "cifar_x3.hip": ["-fno-honor-nans"],
                   # flash / decode softmax maxima over MFMA results: no v_max canonicalise
                   # per score (52 -> 17 v_max per GPT-2 flash block); -inf masking is kept
                   "attention.hip": ["-fno-honor-nans"] + NO_SLP,
+                  "paged_attention.hip": ["-fno-honor-nans"] + NO_SLP,
                   "gemm_skinny.hip": NO_SLP,
                   "gemm_bf16.hip": NO_SLP}
 
@@ -50,77 +51,124 @@ def _hipcc() -> str:
     raise RuntimeError("hipcc not found")
 
 
-def sources() -> List[str]:
+def sources(subset: str = "") -> List[str]:
+    names = SUBSETS[subset][1]
+    if names is not None:
+        return [os.path.join(CSRC, n) if n.endswith(".cpp") else os.path.join(CSRC, "kernels", n) for n in names]
     return (sorted(glob.glob(os.path.join(CSRC, "kernels", "*.hip"))) + sorted(glob.glob(os.path.join(CSRC, "comm", "*.cpp")))
             + [os.path.join(CSRC, "bindings.cpp")])
 
 
 def _flags(src: str) -> List[str]:
     f = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-I" + CSRC, "-Wno-unused-result",
-         "-Wno-unused-command-line-argument"]
+         "-Wno-unused-command-line-argument"] + NO_PACKED_FP32
     f += PER_FILE_FLAGS.get(os.path.basename(src), [])
     have_tf = all(os.path.exists(os.path.join(CSRC, "kernels", s)) for s in TRANSFORMER_SRCS)
     if have_tf:
         f.append("-DDNN_HAVE_TRANSFORMER")
-    if src.endswith("bindings.cpp"):
+    if os.path.basename(src).startswith("bindings"):
         import pybind11
         f += ["-x", "hip", "-I" + pybind11.get_include(), "-I" + sysconfig.get_paths()["include"]]
     return f
 
 
-def _headers_mtime() -> float:
-    hs = glob.glob(os.path.join(CSRC, "**", "*.h"), recursive=True)
-    return max([os.path.getmtime(h) for h in hs] + [0.0])
+def _includes(src: str, seen: set = None) -> set:
+    """``src`` and every in-tree header it includes, directly or not."""
+    import re
+    seen = set() if seen is None else seen
+    if src in seen:
+        return seen
+    seen.add(src)
+    with open(src) as f:
+        names = re.findall(r'^\s*#\s*include\s+"([^"]+)"', f.read(), re.M)
+    for n in names:
+        for d in (os.path.dirname(src), CSRC):
+            h = os.path.normpath(os.path.join(d, n))
+            if os.path.exists(h):
+                _includes(h, seen)
+                break
+    return seen
 
 
-def _obj(src: str) -> str:
+def _newest(src: str) -> float:
+    return max(os.path.getmtime(f) for f in _includes(src))
+
+
+def _obj(src: str, extra: List[str]) -> str:
     import hashlib
-    tag = hashlib.sha1(" ".join(_flags(src)).encode()).hexdigest()[:8]
+    tag = hashlib.sha1(" ".join(_flags(src) + extra).encode()).hexdigest()[:8]
     return os.path.join(BUILD, f"{os.path.basename(src)}.{tag}.o")
 
 
-def _compile(src: str, force: bool, hm: float) -> str:
-    obj = _obj(src)
-    if not force and os.path.exists(obj) and os.path.getmtime(obj) >= max(os.path.getmtime(src), hm):
+def _compile(src: str, force: bool, extra: List[str]) -> str:
+    obj = _obj(src, extra)
+    if not force and os.path.exists(obj) and os.path.getmtime(obj) >= _newest(src):
         return obj
-    cmd = [_hipcc()] + _flags(src) + ["-c", src, "-o", obj]
+    cmd = [_hipcc()] + _flags(src) + extra + ["-c", src, "-o", obj]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"hipcc failed for {src}:\n{' '.join(cmd)}\n{r.stdout}\n{r.stderr}")
     return obj
 
 
-def build(force: bool = False, jobs: int = 0, verbose: bool = True) -> str:
+# The full library, and the decoder subset: the kernels a paged decoder model
+# runs (runtime/decoder.py), compiled without the other families' entry points,
+# for a first use in a checkout that has no library yet (``ensure``).
+SUBSETS = {"": ("_dnn_hip", None, []),
+           "decoder": ("_dnn_decoder", ("gemm_bf16.hip", "gemm_skinny.hip", "sampler.hip", "gemm_f32.hip",
+                                        "residual_rows.hip", "paged_attention.hip", "bindings_decoder.cpp"),
+                       ["-DDNN_DECODER_ONLY"])}
+
+
+def lib_path(subset: str = "") -> str:
+    return os.path.join(PKG, SUBSETS[subset][0] + EXT_SUFFIX)
+
+
+def stamp_path(lib: str) -> str:
+    return lib[:-len(EXT_SUFFIX)] + ".build.json"
+
+
+def build(force: bool = False, jobs: int = 0, verbose: bool = True, subset: str = "") -> str:
     os.makedirs(BUILD, exist_ok=True)
-    srcs = sources()
-    hm = _headers_mtime()
+    srcs, lib, extra = sources(subset), lib_path(subset), SUBSETS[subset][2]
     jobs = jobs or min(len(srcs), int(os.environ.get("MAX_JOBS", "8")), os.cpu_count() or 4, 16)
     with cf.ThreadPoolExecutor(jobs) as ex:
-        objs = list(ex.map(lambda s: _compile(s, force, hm), srcs))
+        objs = list(ex.map(lambda s: _compile(s, force, extra), srcs))
     newest = max(os.path.getmtime(o) for o in objs)
-    if force or not os.path.exists(LIB_PATH) or os.path.getmtime(LIB_PATH) < newest:
-        cmd = [_hipcc(), "-shared", "-fPIC", f"--offload-arch={ARCH}"] + objs + ["-o", LIB_PATH]
+    if force or not os.path.exists(lib) or os.path.getmtime(lib) < newest:
+        part = lib + ".part"  # moved into place whole: another process may be loading it
+        cmd = [_hipcc(), "-shared", "-fPIC", f"--offload-arch={ARCH}"] + objs + ["-o", part]
         r = subprocess.run(cmd, capture_output=True, text=True)
         if r.returncode != 0:
             raise RuntimeError(f"link failed:\n{' '.join(cmd)}\n{r.stdout}\n{r.stderr}")
-    write_stamp(srcs)
+        os.replace(part, lib)
+    write_stamp(srcs, lib, extra)
     if verbose:
-        print(f"[build] {LIB_PATH} ({len(objs)} objects, arch {ARCH})")
-    return LIB_PATH
+        print(f"[build] {lib} ({len(objs)} objects, arch {ARCH})", file=sys.stderr)
+    return lib
 
 
-STAMP_PATH = os.path.join(PKG, "_dnn_hip.build.json")
+def ensure(subset: str) -> None:
+    """Compile ``subset`` unless a library that holds it is built from these sources."""
+    from ._lib import verify_stamp
+    for s in ("", subset):
+        try:
+            if os.path.exists(lib_path(s)):
+                verify_stamp(lib_path(s))
+                return
+        except RuntimeError:
+            pass
+    build(subset=subset)
 
 
 def source_digest(srcs: List[str] = None) -> dict:
     """sha256 of every source and header the library is built from."""
     import hashlib
-    srcs = srcs or sources()
-    files = sorted(set(srcs) | set(glob.glob(os.path.join(CSRC, "**", "*.h"), recursive=True)))
+    files = sorted(set().union(*(_includes(s) for s in (srcs or sources()))))
     return {os.path.relpath(f, ROOT): hashlib.sha256(open(f, "rb").read()).hexdigest() for f in files}
 
 
-def write_stamp(srcs: List[str]) -> None:
+def write_stamp(srcs: List[str], lib: str, extra: List[str]) -> None:
     """Build provenance next to the .so: source hashes, per-file flags, the
     compiler, the library's own hash (``_lib.verify_stamp`` checks them at
     load, so a stale or foreign binary fails loudly instead of running)."""
@@ -130,10 +178,10 @@ def write_stamp(srcs: List[str]) -> None:
     r = subprocess.run([_hipcc(), "--version"], capture_output=True, text=True)
     stamp = {"arch": ARCH, "built_at": time.strftime("%Y-%m-%dT%H:%M:%S"),
              "hipcc": (r.stdout or r.stderr).strip().splitlines()[:2],
-             "flags": {os.path.basename(s): _flags(s) for s in srcs},
+             "flags": {os.path.basename(s): _flags(s) + extra for s in srcs},
              "sources": source_digest(srcs),
-             "library_sha256": hashlib.sha256(open(LIB_PATH, "rb").read()).hexdigest()}
-    with open(STAMP_PATH, "w") as f:
+             "library_sha256": hashlib.sha256(open(lib, "rb").read()).hexdigest()}
+    with open(stamp_path(lib), "w") as f:
         json.dump(stamp, f, indent=1)
 
 
@@ -141,8 +189,9 @@ def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("-j", "--jobs", type=int, default=0)
     ap.add_argument("--force", action="store_true")
+    ap.add_argument("--subset", default="", choices=sorted(SUBSETS))
     a = ap.parse_args(argv)
-    build(a.force, a.jobs)
+    build(a.force, a.jobs, subset=a.subset)
     return 0
 
 

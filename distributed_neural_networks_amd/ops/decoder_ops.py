@@ -1,0 +1,224 @@
+"""Wrappers of the decoder kernels with an fp32 residual and a paged KV cache
+(``csrc/kernels/residual_rows.hip``, ``gemm_f32.hip``, ``paged_attention.hip``).
+
+Operands are bf16 (serving) or fp32 (exact mode: fp32 weights, activations,
+cache and MFMA); the residual stream is fp32 in both.  As in
+``transformer_ops``, every shape is validated on the host before a launch.
+"""
+from __future__ import annotations
+
+from typing import Optional
+
+import torch
+
+from . import gemm as G_
+from ._lib import check, lib, ptr, stream_ptr
+
+PAGE = 64                      # keys per cache page (paged_attention.hip PG)
+HEAD_DIMS = (64, 128, 256)     # head sizes the kernels are built for; others are zero-padded up
+TILE_ROWS = 128                # packed (token, head) rows of one prefill workgroup
+NO_WINDOW = (1 << 31) - 1
+WIDTH_MAX = 16384
+
+
+def pad_dim(d: int) -> int:
+    """Head size a ``d``-wide head is stored at."""
+    for p in HEAD_DIMS:
+        if d <= p:
+            return p
+    raise ValueError(f"head size {d} exceeds {HEAD_DIMS[-1]}")
+
+
+def pad64(n: int) -> int:
+    return -(-n // 64) * 64
+
+
+def _rows(t: Optional[torch.Tensor], M: int, N: int, name: str, dtypes) -> None:
+    if t is None:
+        return
+    if t.dim() != 2 or t.shape[0] < M or t.shape[1] < N or t.stride(1) != 1 or t.dtype not in dtypes:
+        raise ValueError(f"{name}: need >= ({M}, {N}) rows of {dtypes}, got {tuple(t.shape)} {t.dtype} "
+                         f"strides {t.stride()}")
+
+
+def _index(t: Optional[torch.Tensor], M: int, name: str) -> None:
+    if t is not None and (t.dtype != torch.int32 or t.numel() < M or not t.is_contiguous()):
+        raise ValueError(f"{name}: contiguous int32 with >= {M} entries expected")
+
+
+def _weight(t: Optional[torch.Tensor], N: int, name: str) -> None:
+    if t is not None and (t.dtype != torch.float32 or t.numel() < N or not t.is_contiguous()):
+        raise ValueError(f"{name}: contiguous fp32 with >= {N} entries expected")
+
+
+def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx: Optional[torch.Tensor] = None,
+                y: Optional[torch.Tensor] = None, yidx: Optional[torch.Tensor] = None, mult: float = 1.0,
+                y_norm: Optional[torch.Tensor] = None, x_out: Optional[torch.Tensor] = None,
+                copy: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
+                h: Optional[torch.Tensor] = None, eps: float = 1e-5) -> None:
+    """``x' = [x_in] + mult * y`` (``y`` RMS-normalised with weight ``y_norm``
+    first, if given), then any of ``x_out = x'`` (fp32), ``copy = x'`` and
+    ``h = RMSnorm(x') * norm``.  ``xidx`` / ``yidx`` gather the rows of ``x_in``
+    / ``y``.  Rows are zero-padded to a multiple of 4; means are over ``width``."""
+    f32, bf = torch.float32, torch.bfloat16
+    out = copy if copy is not None else h
+    od = out.dtype if out is not None else (y.dtype if y is not None else f32)
+    NP = next(t.shape[1] for t in (x_out, x_in, y) if t is not None)
+    _rows(x_in, 1 if xidx is not None else M, NP, "rows_update x_in", (f32,))
+    _rows(x_out, M, NP, "rows_update x_out", (f32,))
+    _rows(y, 1 if yidx is not None else M, NP, "rows_update y", (f32, bf))
+    _rows(copy, M, NP, "rows_update copy", (od,))
+    _rows(h, M, NP, "rows_update h", (od,))
+    _index(xidx, M, "rows_update xidx")
+    _index(yidx, M, "rows_update yidx")
+    _weight(y_norm, NP, "rows_update y_norm")
+    _weight(norm, NP, "rows_update norm")
+    if x_in is None and y is None or (norm is None) != (h is None) or width > NP or NP % 4 or NP > WIDTH_MAX:
+        raise ValueError(f"rows_update: unsupported call (width {width} of {NP})")
+    if x_in is not None and x_out is not None and x_in.stride(0) != x_out.stride(0):
+        raise ValueError("rows_update: x_in and x_out must share a row stride")
+    ldx = x_in.stride(0) if x_in is not None else (x_out.stride(0) if x_out is not None else 0)
+    y32 = y is None and od == f32 or y is not None and y.dtype == f32
+    check(lib().rows_update(ptr(x_in), ptr(xidx), 0 if x_in is None else x_in.shape[0], ptr(y), ptr(yidx),
+                            0 if y is None else y.shape[0], 0 if y is None else y.stride(0), float(mult), ptr(y_norm),
+                            ptr(x_out), ldx, ptr(copy), 0 if copy is None else copy.stride(0), ptr(norm), ptr(h),
+                            0 if h is None else h.stride(0), M, width, NP, float(eps), int(y32),
+                            int(od == f32), stream_ptr()), "rows_update")
+
+
+def token_gate(z: torch.Tensor, table: torch.Tensor, off: int, ids: torch.Tensor, out: torch.Tensor, M: int,
+               n: int) -> torch.Tensor:
+    """``out[m, c] = gelu_tanh(z[m, c]) * table[ids[m], off + c]`` for c < n; 0 in the padding columns."""
+    dt = (z.dtype,)
+    _rows(z, M, n, "token_gate z", (torch.float32, torch.bfloat16))
+    _rows(table, 1, off + n, "token_gate table", dt)
+    _rows(out, M, n, "token_gate out", dt)
+    _index(ids, M, "token_gate ids")
+    check(lib().token_gate(ptr(z), z.stride(0), ptr(table), table.stride(0), off, ptr(ids), table.shape[0], ptr(out),
+                           out.stride(0), M, n, out.shape[1], int(z.dtype == torch.float32), stream_ptr()),
+          "token_gate")
+    return out
+
+
+def linear_f32(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
+    """``x @ w.T + bias`` on the fp32 MFMA (K a multiple of 16)."""
+    M, K = x.shape
+    N = w.shape[0]
+    f = (torch.float32,)
+    _rows(x, M, K, "linear_f32 x", f)
+    _rows(w, N, K, "linear_f32 w", f)
+    _rows(out, M, N, "linear_f32 out", f)
+    _weight(bias, N, "linear_f32 bias")
+    check(lib().gemm_f32(ptr(x), x.stride(0), ptr(w), w.stride(0), ptr(out), out.stride(0), ptr(bias), M, N, K,
+                         stream_ptr()), "gemm_f32")
+    return out
+
+
+class Linear:
+    """A projection of the decoder layers: bf16 weights on the framework's MFMA
+    GEMMs (with the decode copy in fragment order, ``gemm.shuffle_weight``), or
+    fp32 weights on ``linear_f32``.  K (weight columns) is zero-padded to a
+    multiple of 64 by the caller."""
+
+    __slots__ = ("w", "bias", "ws", "act")
+
+    def __init__(self, w: torch.Tensor, bias: Optional[torch.Tensor], dtype: torch.dtype, device, glu: bool = False,
+                 decode_copy: bool = True):
+        self.w = w.to(device=device, dtype=dtype).contiguous()
+        self.bias = None if bias is None else bias.to(device=device, dtype=torch.float32).contiguous()
+        self.act = G_.ACT_GELU_TANH_MUL if glu else G_.ACT_NONE
+        self.ws = G_.shuffle_weight(self.w) if dtype == torch.bfloat16 and decode_copy else None
+
+    def __call__(self, x: torch.Tensor, out: torch.Tensor, gws: Optional[torch.Tensor] = None,
+                 scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """``scratch`` (fp32 gated projections): (M, weight rows) before the activation."""
+        if self.w.dtype == torch.bfloat16:
+            return G_.linear(x, self.w, self.bias, self.act, out=out, w_shuf=self.ws, ws=gws)
+        if self.act == G_.ACT_NONE:
+            return linear_f32(x, self.w, self.bias, out)
+        M, F = x.shape[0], self.w.shape[0] // 2
+        gu = linear_f32(x, self.w, self.bias, scratch[:M])
+        _rows(out, M, F, "gated linear out", (torch.float32,))
+        check(lib().glu_f32(ptr(gu), gu.stride(0), ptr(out), out.stride(0), M, F, stream_ptr()), "glu_f32")
+        return out
+
+
+def paged_args(qkv: torch.Tensor, kp: torch.Tensor, vp: torch.Tensor, table: torch.Tensor, slots: torch.Tensor,
+               pos: torch.Tensor, out: torch.Tensor, M: int, H: int, scale: float, window: Optional[int], keep: int,
+               gate: int = -1):
+    """Validated arguments of the paged-attention launches.
+
+    qkv rows ``[q H*DK | k G*DK | v G*DV | ...]``; ``kp`` (pages, G, 64, DK),
+    ``vp`` (pages, G, 64, DV); ``table`` (slots, pages per sequence) int32;
+    ``slots`` / ``pos`` per row; ``out`` rows ``[H*DV]``; ``gate``: first qkv
+    column of the per-head output gate (-1: none).  Every slot is the caller's:
+    ``0 <= slots[m] < table.shape[0]``."""
+    dt = qkv.dtype
+    if kp.dim() != 4 or vp.dim() != 4 or kp.shape[:3] != vp.shape[:3] or kp.shape[2] != PAGE:
+        raise ValueError(f"paged attention: pages {tuple(kp.shape)} / {tuple(vp.shape)}")
+    if kp.dtype != dt or vp.dtype != dt or out.dtype != dt or not (kp.is_contiguous() and vp.is_contiguous()):
+        raise ValueError("paged attention: the cache and output share the projection's dtype, pages contiguous")
+    P, G, _, DK = kp.shape
+    DV = vp.shape[3]
+    if DK not in HEAD_DIMS or DV not in HEAD_DIMS or H % G:
+        raise ValueError(f"paged attention: {H} heads over {G}, sizes {DK} / {DV}")
+    need = max((H + G) * DK + G * DV, gate + H if gate >= 0 else 0)
+    _rows(qkv, M, need, "paged attention qkv", (torch.float32, torch.bfloat16))
+    _rows(out, M, H * DV, "paged attention out", (dt,))
+    _index(slots, M, "paged attention slots")
+    _index(pos, M, "paged attention pos")
+    if table.dtype != torch.int32 or table.dim() != 2 or not table.is_contiguous():
+        raise ValueError("paged attention: block table must be contiguous int32 (slots, pages)")
+    if not scale > 0:
+        raise ValueError("paged attention: the score scale must be positive")
+    keep = min(int(keep), 1 << 30)
+    return lib().PagedAttnArgs(ptr(qkv), qkv.stride(0), ptr(kp), ptr(vp), ptr(table), table.shape[1], P, ptr(slots),
+                               ptr(pos), ptr(out), out.stride(0), M, H, G, DK, DV, gate,
+                               NO_WINDOW if window is None else int(window), keep, float(scale))
+
+
+def paged_write(args, f32: bool) -> None:
+    """Store the k / v columns of every row in its sequence's pages."""
+    check(lib().paged_write(args, int(f32), stream_ptr()), "paged_write")
+
+
+def paged_prefill(args, tiles: torch.Tensor) -> None:
+    """Attention of chunks of tokens already written to the cache.  ``tiles``
+    (n, 4) int32: {first row, tokens, slot, first packed row} (``chunk_tiles``)."""
+    if tiles.dtype != torch.int32 or tiles.dim() != 2 or tiles.shape[1] != 4 or not tiles.is_contiguous():
+        raise ValueError("paged_prefill: tiles must be contiguous int32 (n, 4)")
+    n = tiles.shape[0]
+    for i in range(0, n, 65535):
+        part = tiles[i:i + 65535]
+        check(lib().paged_prefill(args, ptr(part), part.shape[0], stream_ptr()), "paged_prefill")
+
+
+def chunk_tiles(row0: int, tokens: int, slot: int, group: int) -> list:
+    """Prefill workgroups of one chunk: ``tokens * group`` packed rows (group =
+    query heads per KV head), the last (longest) ones first."""
+    return [(row0, tokens, slot, r) for r in range(0, tokens * group, TILE_ROWS)][::-1]
+
+
+def paged_splits(n_seq: int, H: int, G: int, keys: int, window: Optional[int], keep: int) -> int:
+    """Workgroups per (sequence, KV head) of a decode launch: enough for two per
+    CU, with at least eight 32-key units each."""
+    if window is not None:
+        keys = min(keys, window + keep + 2 * PAGE)
+    units = -(-max(keys, 1) // 32)
+    wgs = n_seq * G * -(-(H // G) // 32)
+    return max(1, min(-(-512 // wgs), units // 8, 64))
+
+
+def paged_decode(args, rows: torch.Tensor, n: int, splits: int, ws: Optional[torch.Tensor]) -> None:
+    """One token of each of ``n`` sequences (``rows``: their batch rows); also
+    stores the tokens' k / v.  ``ws``: fp32, n * H * splits * (DV + 2) for splits > 1."""
+    _index(rows, n, "paged_decode rows")
+    if splits > 1 and (ws is None or ws.dtype != torch.float32 or not ws.is_contiguous()):
+        raise ValueError("paged_decode: splits > 1 needs an fp32 workspace")
+    check(lib().paged_decode(args, ptr(rows), n, splits, ptr(ws), 0 if ws is None else ws.numel(), stream_ptr()),
+          "paged_decode")
+
+
+def paged_attn_f32(args) -> None:
+    """fp32 attention of every row (cache already written)."""
+    check(lib().paged_attn_f32(args, stream_ptr()), "paged_attn_f32")

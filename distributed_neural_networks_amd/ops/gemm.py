@@ -12,7 +12,8 @@ import torch
 
 from ._lib import check, lib, ptr, stream_ptr
 
-ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU_MUL = 0, 1, 2, 3
+ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU_MUL, ACT_GELU_TANH_MUL = 0, 1, 2, 3, 4
+ACTS_GLU = (ACT_SILU_MUL, ACT_GELU_TANH_MUL)  # packed gate|up weight (pack_gate_up), half-width output
 SKINNY_MAX_M = 256
 
 
@@ -35,7 +36,8 @@ def set_skinny_max_m(m: int = 64) -> None:
     global SKINNY_ALWAYS_M
     check(lib().gemm_set_skinny_max_m(int(m)), "gemm_set_skinny_max_m")
     SKINNY_ALWAYS_M = int(m)
-_ACTS = {None: ACT_NONE, "none": ACT_NONE, "relu": ACT_RELU, "gelu": ACT_GELU, "silu_mul": ACT_SILU_MUL}
+_ACTS = {None: ACT_NONE, "none": ACT_NONE, "relu": ACT_RELU, "gelu": ACT_GELU, "silu_mul": ACT_SILU_MUL,
+         "gelu_tanh_mul": ACT_GELU_TANH_MUL}
 
 DECODE_WS_BYTES = 16 << 20
 _decode_ws = {}
@@ -145,7 +147,9 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
         raise TypeError("linear: bf16 operands required")
     if x2.stride(1) != 1 or w.stride(1) != 1:
         raise ValueError("linear: inner dims must be contiguous")
-    Nout = N // 2 if a == ACT_SILU_MUL else N
+    Nout = N // 2 if a in ACTS_GLU else N
+    if a in ACTS_GLU and N % 16:
+        raise ValueError(f"linear: packed gate|up rows {N} must be a multiple of 16")
     if out is None:
         out = torch.empty((M, Nout), dtype=out_dtype, device=x.device)
     o2 = out.reshape(-1, out.shape[-1]) if out.dim() != 2 else out

@@ -1,0 +1,414 @@
+"""Decoder stages with an fp32 residual over a paged KV cache (Kozusun).
+
+A stage runs a range of layer *runs* (``models/kozusun.py``; a looped layer
+counts once per pass and has a cache per pass, its weights are shared).  One
+forward pass serves both callers:
+
+* ``step_batch(StepBatch)`` — the engine's step (``runtime/engine.py``): tokens
+  of any number of sequences, portions of prompts beside single tokens;
+* ``step(x, pos, B, T, b0)`` — ``TransformerStage.step``'s contract for the
+  decode ring (``runtime/scheduler.py``): B sequences of T tokens on cache rows
+  [b0, b0 + B), each with its own fixed pages, so a decode step is one HIP
+  graph whose positions live on the device.
+
+Launches per layer run (bf16): q|k|v|gate projection; gate|up projection with
+the tanh-GELU product in its epilogue; attention (decode: cache write, attention
+and output gate in one launch; prefill: cache write, then flash attention) —
+both sublayers write one row ``[attention | feed-forward]``, so ONE projection
+with the two output matrices side by side gives their sum; residual update;
+token-input projections around ``token_gate``; residual update + the next run's
+norm in one pass.  The residual, norms, scores and softmax are fp32.
+
+``dtype="float32"`` runs the same sequence with fp32 weights, activations,
+cache and matrix products (``ops/decoder_ops.py``).
+
+Stage boundary: rows ``[residual | token id | padding]`` of fp32 (the token id
+as its bits): later stages need the tokens for their per-layer inputs, and the
+embedding output at a loop's entry.
+"""
+from __future__ import annotations
+
+from typing import Dict, List, Optional
+
+import torch
+
+from ..models import kozusun, model_info
+from ..ops import decoder_ops as D_
+from ..ops import transformer_ops as T_
+from ..ops.gemm import decode_workspace, pack_gate_up
+from .paging import PAGE, StepBatch, pages_for
+from .stages import StageCompute, StageOutput
+
+DTYPES = {None: torch.bfloat16, "bf16": torch.bfloat16, "bfloat16": torch.bfloat16, "fp32": torch.float32,
+          "float32": torch.float32}
+HOP_IDS = 4  # fp32 columns after the residual at a stage boundary: the token id's bits, padding
+
+
+def _pad(t: torch.Tensor, *shape: int) -> torch.Tensor:
+    """``t`` in the leading corner of a zero tensor of ``shape``."""
+    if tuple(t.shape) == shape:
+        return t
+    out = t.new_zeros(shape)
+    out[tuple(slice(0, n) for n in t.shape)] = t
+    return out
+
+
+def _pad_heads(w: torch.Tensor, heads: int, dim: int, to: int) -> torch.Tensor:
+    """Rows of ``heads`` groups of ``dim`` -> groups of ``to``, zeros between."""
+    w = w.view(heads, dim, *w.shape[1:])
+    return _pad(w, heads, to, *w.shape[2:]).reshape(heads * to, *w.shape[2:])
+
+
+class DecoderLayer:
+    """Packed weights of one layer."""
+
+    def __init__(self, cfg: kozusun.KozusunConfig, i: int, sd: Dict[str, torch.Tensor], dtype, device, wp: int):
+        L, m = cfg.layers[i], cfg.layers[i].mixer
+        self.mix, self.ff = m, L.ff
+        self.dk, self.dv = D_.pad_dim(m.dim), D_.pad_dim(m.vdim)
+        self.group = m.heads // m.kv_heads
+        ld = lambda n: sd[f"l{i}.{n}"].to(device=device, dtype=torch.float32)  # noqa: E731
+        lin = lambda w, b=None, glu=False: D_.Linear(w, b, dtype, device, glu)  # noqa: E731
+        self.norm1 = _pad(1 + ld("norm1"), wp)
+        self.norm1[cfg.n_embd:] = 0
+        heads = ((m.heads, m.dim, self.dk, "q"), (m.kv_heads, m.dim, self.dk, "k"), (m.kv_heads, m.vdim, self.dv, "v"))
+        w = [_pad_heads(_pad(ld(f"mix.{n}"), h * d, wp), h, d, p) for h, d, p, n in heads]
+        b = [_pad_heads(ld(f"mix.{n}.b"), h, d, p) for h, d, p, n in heads]
+        self.gate_col = sum(t.shape[0] for t in w)
+        n = self.gate_col + m.heads
+        self.n_qkv = -(-n // 16) * 16
+        self.w_qkv = lin(_pad(torch.cat(w + [_pad(ld("mix.g"), m.heads, wp)]), self.n_qkv, wp),
+                         _pad(torch.cat(b), self.n_qkv))
+        wo = ld("mix.o").view(cfg.n_embd, m.heads, m.vdim)
+        outs = [_pad(_pad(wo, cfg.n_embd, m.heads, self.dv).reshape(cfg.n_embd, -1), wp, m.heads * self.dv)]
+        self.n_att, self.n_ff = m.heads * self.dv, 0
+        self.w_up = None
+        if L.ff is not None:
+            self.n_ff = D_.pad64(L.ff)
+            self.w_up = lin(pack_gate_up(_pad(ld("mlp.gate"), self.n_ff, wp), _pad(ld("mlp.up"), self.n_ff, wp)),
+                            glu=True)
+            outs.append(_pad(ld("mlp.down"), wp, self.n_ff))
+        self.w_out = lin(torch.cat(outs, 1))
+        self.side_off = i * cfg.side_dim
+        if cfg.side_dim:
+            sp = D_.pad64(cfg.side_dim)
+            self.w_sgate = lin(_pad(ld("side.gate"), sp, wp))
+            self.w_sproj = lin(_pad(ld("side.proj"), wp, sp))
+            self.side_norm = _pad(ld("side.norm"), wp)
+
+
+class DecoderStage(StageCompute):
+    act_dtype = torch.float32  # stage-boundary rows
+
+    def __init__(self, model: str, sd: Dict[str, torch.Tensor], start: int, end: int, first: bool, last: bool,
+                 device, max_batch: int = 8, max_seq: int = 1024, max_tokens: Optional[int] = None,
+                 dtype: Optional[str] = None, temperature: float = 0.0, top_k: int = 0, seed: int = 0,
+                 num_pages: Optional[int] = None, cfg: Optional[kozusun.KozusunConfig] = None):
+        """``max_batch`` x ``max_seq``: the ring's cache rows (and the default
+        ``num_pages``).  ``num_pages``: the page pool of an engine.  ``max_tokens``:
+        rows of one step.  ``cfg`` overrides the registry's configuration."""
+        if dtype not in DTYPES:
+            raise ValueError(f"dtype {dtype!r}: this model runs in bf16 or float32")
+        self.model = model
+        self.cfg = c = cfg if cfg is not None else model_info(model).cfg
+        self.family = "kozusun"
+        self.start, self.end, self.first, self.last = start, end, first, last
+        self.device = dev = torch.device(device)
+        if dev.type != "cuda":
+            raise ValueError("DecoderStage runs on the GPU kernels only")
+        self.dtype = dt = DTYPES[dtype]
+        self.f32 = dt == torch.float32
+        self.temperature, self.top_k, self.seed = float(temperature), int(top_k), int(seed)
+        self.max_batch, self.max_seq = max_batch, max_seq
+        self.row_pages = pages_for(max_seq)
+        self.num_pages = num_pages or max_batch * self.row_pages
+        self.max_tokens = max(max_tokens or max_batch * max_seq, max_batch)
+        self.width, self.wp = c.n_embd, D_.pad64(c.n_embd)
+        self.V = c.vocab_size
+        self.Vpad = D_.pad64(self.V)
+        self.eps, self.mult = c.norm_eps, c.residual_mult
+        self.runs = c.runs[start:end + 1]
+        self.side = c.side_dim
+        self.enters = any(r.enters for r in self.runs)
+
+        def table(name, cols):  # gathered rows; columns padded so every row is aligned
+            t = sd[name].to(device=dev, dtype=dt)
+            return _pad(t, t.shape[0], cols).contiguous()
+        self.embed = table("embed", self.wp) if (first or self.enters) else None
+        if self.side:
+            self.side_embed = sd["side.embed"].to(device=dev, dtype=dt).contiguous()
+        if self.enters:
+            w = sd["loop.in"].to(device=dev, dtype=torch.float32)
+            w = torch.cat([_pad(w[:, :self.width], self.wp, self.wp), _pad(w[:, self.width:], self.wp, self.wp)], 1)
+            self.w_loop = D_.Linear(w, None, dt, dev)
+        layers = {i: DecoderLayer(c, i, sd, dt, dev, self.wp) for i in sorted({r.layer for r in self.runs})}
+        self.layers: List[DecoderLayer] = [layers[r.layer] for r in self.runs]
+        if last:
+            self.final_norm = _pad(1 + sd["final.norm"].to(device=dev, dtype=torch.float32), self.wp)
+            self.final_norm[self.width:] = 0
+            self.w_head = D_.Linear(_pad(sd["head"].to(device=dev, dtype=torch.float32), self.V, self.wp), None, dt, dev)
+        self.groups = sorted({L.group for L in self.layers})
+        self._alloc()
+        self._ring: Dict[tuple, dict] = {}
+        self._ring_table: Optional[torch.Tensor] = None
+        self._ring_ws: Optional[torch.Tensor] = None
+
+    def _alloc(self):
+        dev, dt, n = self.device, self.dtype, self.max_tokens
+        z = lambda cols, t=dt: torch.zeros((n, cols), dtype=t, device=dev)  # noqa: E731
+        self.x = z(self.wp, torch.float32)
+        self.cat = z(2 * self.wp)                     # [residual copy | embedding output]
+        self.h, self.y = z(self.wp), z(self.wp)
+        self.qkv = z(max(L.n_qkv for L in self.layers))
+        self.af = z(max(L.n_att + L.n_ff for L in self.layers))
+        ff = max(L.n_ff for L in self.layers)
+        self.gu = z(2 * ff) if self.f32 and ff else None
+        if self.side:
+            self.z, self.g = z(D_.pad64(self.side)), z(D_.pad64(self.side))
+        if self.enters:
+            self.y32 = self.y if self.f32 else z(self.wp, torch.float32)
+        if not self.first:
+            self.ids_in = torch.zeros((n,), dtype=torch.int32, device=dev)
+        P = self.num_pages
+        self.pages = [(torch.zeros((P, L.mix.kv_heads, PAGE, L.dk), dtype=dt, device=dev),
+                       torch.zeros((P, L.mix.kv_heads, PAGE, L.dv), dtype=dt, device=dev)) for L in self.layers]
+        if self.last:
+            self.hn = z(self.wp)
+            self.logits = torch.zeros((max(self.max_batch, 1), self.Vpad), dtype=dt, device=dev)
+            self.next_ids = torch.zeros((max(self.max_batch, 1),), dtype=torch.int32, device=dev)
+            self.amx_part = torch.empty((max(self.max_batch, 1) * 2 * T_.ARGMAX_PART_PER_ROW,), dtype=torch.int32,
+                                        device=dev)
+        self.ws: Optional[torch.Tensor] = None        # decode-attention partials (engine steps)
+
+    # ------------------------------------------------------------------ specs
+    @property
+    def d(self) -> int:
+        """Columns of a stage-boundary row."""
+        return self.wp + HOP_IDS
+
+    def in_spec(self, batch: int, T: int = 1):
+        return ((batch, T), torch.int32) if self.first else ((batch * T, self.d), torch.float32)
+
+    def out_spec(self, batch: int, T: int = 1):
+        return ((batch,), torch.int32) if self.last else ((batch * T, self.d), torch.float32)
+
+    @property
+    def fuses_step_tail(self) -> bool:
+        """Greedy last stage: the argmax launch writes the next input ids and advances the positions."""
+        return self.last and not self.temperature > 0
+
+    def reset(self):
+        for k, v in self.pages:
+            k.zero_()
+            v.zero_()
+
+    # ------------------------------------------------------------------ layers
+    def _prep(self, k: int, r0: int, M: int) -> dict:
+        """What the residual update before run ``k`` also produces."""
+        s = slice(r0, r0 + M)
+        if k == len(self.runs):
+            return {}
+        if self.runs[k].enters:
+            return {"copy": self.cat[s, :self.wp]}
+        return {"norm": self.layers[k].norm1, "h": self.h[s]}
+
+    def _splits(self, L: DecoderLayer, n: int, keys: int) -> int:
+        m = L.mix
+        return D_.paged_splits(n, m.heads, m.kv_heads, keys, m.window, m.keep_first)
+
+    def _ws_need(self, n: int, keys: int) -> int:
+        """fp32 partials the decode launches of ``n`` sequences need."""
+        return max((n * L.mix.heads * s * (L.dv + 2) for L in self.layers
+                    for s in [self._splits(L, n, keys)] if s > 1), default=0)
+
+    def _attention(self, k: int, b: StepBatch, qkv: torch.Tensor, out: torch.Tensor, ws) -> None:
+        L, (kp, vp), m = self.layers[k], self.pages[k], self.layers[k].mix
+        args = D_.paged_args(qkv, kp, vp, b.table, b.slots, b.pos, out, b.M, m.heads, m.scale, m.window, m.keep_first,
+                             L.gate_col)
+        if self.f32:
+            D_.paged_write(args, True)
+            D_.paged_attn_f32(args)
+            return
+        if b.chunks:
+            D_.paged_write(args, False)
+            D_.paged_prefill(args, b.tiles[L.group])
+        if b.n_dec:
+            D_.paged_decode(args, b.dec_rows, b.n_dec, self._splits(L, b.n_dec, b.max_len), ws)
+
+    def _layers(self, b: StepBatch, ids: torch.Tensor, r0: int, gws, ws) -> None:
+        """Residual rows [r0, r0 + M) through this stage's runs (``self.x`` holds
+        the incoming residual on a later stage)."""
+        M, wp, w, s = b.M, self.wp, self.width, slice(r0, r0 + b.M)
+        x, h, y, xc = self.x[s], self.h[s], self.y[s], self.cat[s, :self.wp]
+        up = lambda **kw: D_.rows_update(M, w, eps=self.eps, **kw)  # noqa: E731
+        if self.enters:  # the embedding output, kept for the loop's passes
+            up(y=self.embed, yidx=ids, mult=self.cfg.embed_scale, x_out=x if self.first else None,
+               copy=self.cat[s, wp:])
+            up(x_in=x, **self._prep(0, r0, M))
+        elif self.first:
+            up(y=self.embed, yidx=ids, mult=self.cfg.embed_scale, x_out=x, **self._prep(0, r0, M))
+        else:
+            up(x_in=x, **self._prep(0, r0, M))
+        for k, (run, L) in enumerate(zip(self.runs, self.layers)):
+            if run.enters:
+                up(y=self.w_loop(self.cat[s], self.y32[s], gws), x_out=x, norm=L.norm1, h=h)
+            qkv = self.qkv[s, :L.n_qkv]
+            af = self.af[s, :L.n_att + L.n_ff]
+            L.w_qkv(h, qkv, gws)
+            if L.w_up is not None:
+                L.w_up(h, af[:, L.n_att:], gws, None if self.gu is None else self.gu[:, :2 * L.n_ff])
+            self._attention(k, b, qkv, af[:, :L.n_att], ws)
+            L.w_out(af, y, gws)
+            nxt = self._prep(k + 1, r0, M)
+            if not self.side:
+                up(x_in=x, y=y, mult=self.mult, x_out=x, **nxt)
+                continue
+            up(x_in=x, y=y, mult=self.mult, x_out=x, copy=xc)
+            L.w_sgate(xc, self.z[s], gws)
+            D_.token_gate(self.z[s], self.side_embed, L.side_off, ids, self.g[s], M, self.side)
+            L.w_sproj(self.g[s], y, gws)
+            up(x_in=x, y=y, mult=self.mult, y_norm=L.side_norm, x_out=x, **nxt)
+
+    def _head(self, r0: int, M: int, rows: torch.Tensor, n: int, logits: torch.Tensor, gws=None) -> torch.Tensor:
+        """Logits of ``n`` rows (``rows``: their places among the M of the step)."""
+        hn = self.hn[r0:r0 + n]
+        D_.rows_update(n, self.width, x_in=self.x[r0:r0 + M], xidx=rows, norm=self.final_norm, h=hn, eps=self.eps)
+        self.w_head(hn, logits[:, :self.V], gws)
+        return logits
+
+    # ------------------------------------------------------------------ engine step
+    def step_batch(self, b: StepBatch, x: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+        """One step of an engine.  First stage: ``b.ids``; later ones: ``x``, the
+        previous stage's rows.  Returns boundary rows, or on the last stage the
+        logits of the wanted rows (n_want, V) (None when nothing is wanted)."""
+        if b.M > self.max_tokens:
+            raise ValueError(f"stage buffers hold {self.max_tokens} tokens, the step brings {b.M}")
+        if not self.f32 and b.n_dec:
+            need = self._ws_need(b.n_dec, b.max_len)
+            if need and (self.ws is None or self.ws.numel() < need):
+                self.ws = torch.empty((need,), dtype=torch.float32, device=self.device)
+        ids = self._enter(x, b.ids, 0, b.M)
+        gws = decode_workspace(self.device) if not self.f32 and b.M <= 64 else None
+        self._layers(b, ids, 0, gws, self.ws)
+        if not self.last:
+            return self._leave(ids, 0, b.M, None)
+        if not b.n_want:
+            return None
+        lg = torch.empty((b.n_want, self.Vpad), dtype=self.dtype, device=self.device)
+        return self._head(0, b.M, b.want, b.n_want, lg, gws if b.n_want <= 64 else None)[:, :self.V]
+
+    def sample(self, logits: torch.Tensor, pos: torch.Tensor) -> torch.Tensor:
+        """Next token of every logits row (int32), ``pos``: its position (sampling counter)."""
+        n = logits.shape[0]
+        out = torch.empty((n,), dtype=torch.int32, device=self.device)
+        if self.temperature > 0:
+            T_.sample_topk(logits if logits.dtype == torch.bfloat16 else logits.bfloat16(), out, self.V,
+                           self.temperature, self.top_k, self.seed, step=pos)
+        else:
+            T_.argmax_rows(logits, out, n=self.V)
+        return out
+
+    def _enter(self, x, ids, r0: int, M: int) -> torch.Tensor:
+        """Token ids of the step; a later stage takes the residual from ``x``."""
+        if self.first:
+            return ids
+        if x.dtype != torch.float32 or x.dim() != 2 or x.shape[0] < M or x.shape[1] != self.d:
+            raise ValueError(f"stage input {tuple(x.shape)} {x.dtype}: need ({M}, {self.d}) fp32 rows")
+        self.x[r0:r0 + M].copy_(x[:M, :self.wp])
+        ids_in = self.ids_in[r0:r0 + M]
+        ids_in.copy_(x[:M, self.wp:].view(torch.int32)[:, 0])
+        return ids_in
+
+    def _leave(self, ids, r0: int, M: int, out: Optional[torch.Tensor]) -> torch.Tensor:
+        if out is None:
+            out = torch.empty((M, self.d), dtype=torch.float32, device=self.device)
+        o = out.view(M, self.d)
+        o[:, :self.wp].copy_(self.x[r0:r0 + M])
+        o[:, self.wp:].view(torch.int32).copy_(ids.view(M, 1).expand(M, HOP_IDS))
+        return out
+
+    # ------------------------------------------------------------------ ring step
+    def _ring_batch(self, pos: torch.Tensor, B: int, T: int, b0: int) -> StepBatch:
+        """B sequences of T tokens on cache rows [b0, b0 + B), each with fixed pages."""
+        dev, W = self.device, self.row_pages
+        if self._ring_table is None:
+            if self.num_pages < self.max_batch * W:
+                raise ValueError(f"the page pool ({self.num_pages}) does not hold {self.max_batch} rows of {W} pages")
+            self._ring_table = torch.arange(self.max_batch * W, dtype=torch.int32, device=dev).view(self.max_batch, W)
+        c = self._ring.get((B, T, b0))
+        if c is None:
+            slots = torch.arange(b0, b0 + B, dtype=torch.int32, device=dev)
+            c = {"slots": slots.repeat_interleave(T).contiguous(),
+                 "last": torch.arange(T - 1, B * T, T, dtype=torch.int32, device=dev),
+                 "rows": torch.arange(B * T, dtype=torch.int32, device=dev), "chunks": [], "tiles": None}
+            if T > 1:
+                c["chunks"] = [(i * T, T, b0 + i) for i in range(B)]
+                c["tiles"] = {g: torch.tensor([t for ch in c["chunks"] for t in D_.chunk_tiles(*ch, g)],
+                                              dtype=torch.int32, device=dev) for g in self.groups}
+                c["steps"] = torch.arange(T, dtype=torch.int32, device=dev)
+            self._ring[(B, T, b0)] = c
+        p = pos if T == 1 else (pos.view(B, 1) + c["steps"]).view(-1).contiguous()
+        return StepBatch(M=B * T, pos=p, slots=c["slots"], table=self._ring_table,
+                         dec_rows=c["rows"] if T == 1 else None, n_dec=B if T == 1 else 0, chunks=c["chunks"],
+                         max_len=self.max_seq, tiles=c["tiles"])
+
+    def step(self, x: torch.Tensor, pos: torch.Tensor, B: int, T: int, b0: int = 0,
+             out: Optional[torch.Tensor] = None, last_only: bool = True, advance=None):
+        """``TransformerStage.step``'s contract (ids (B, T) on the first stage,
+        else boundary rows; ``pos`` (B,) device int32)."""
+        if advance is not None and not (self.fuses_step_tail and last_only):
+            raise ValueError("step(advance=...) needs a greedy last stage with last_only")
+        M, r0 = B * T, b0 if T == 1 else 0
+        if r0 + M > self.max_tokens or b0 + B > self.max_batch:
+            raise ValueError(f"step of {B} x {T} tokens at row {b0}: the stage holds {self.max_tokens} tokens, "
+                             f"{self.max_batch} sequences")
+        if self.first and (x.dtype != torch.int32 or tuple(x.shape) != (B, T)):
+            raise ValueError(f"first stage expects int32 ids ({B},{T}), got {x.dtype} {tuple(x.shape)}")
+        b = self._ring_batch(pos, B, T, b0)
+        ws = None
+        if T == 1 and not self.f32:
+            need = self._ws_need(B, self.max_seq)
+            if need:  # one slice per concurrent microbatch
+                per = -(-need // B)
+                if self._ring_ws is None or self._ring_ws.numel() < per * self.max_batch:
+                    self._ring_ws = torch.empty((per * self.max_batch,), dtype=torch.float32, device=self.device)
+                ws = self._ring_ws[per * b0:]
+        ids = self._enter(x, x.view(-1) if self.first else None, r0, M)
+        gws = decode_workspace(self.device, b0 // B) if T == 1 and not self.f32 else None
+        self._layers(b, ids, r0, gws, ws)
+        if not self.last:
+            return self._leave(ids, r0, M, out)
+        c = self._ring[(B, T, b0)]
+        if last_only:
+            n, rows, q0 = B, c["last"], r0 if T == 1 else b0
+            lg, nxt = self.logits[q0:q0 + n], self.next_ids[q0:q0 + n]
+        else:
+            n, rows = M, c["rows"]
+            lg = torch.empty((n, self.Vpad), dtype=self.dtype, device=self.device)
+            nxt = torch.empty((n,), dtype=torch.int32, device=self.device)
+        self._head(r0, M, rows, n, lg, gws)
+        if self.temperature > 0 and last_only:
+            T_.sample_topk(lg if not self.f32 else lg.bfloat16(), nxt, self.V, self.temperature, self.top_k, self.seed,
+                           step=pos)
+            if out is not None:
+                out.copy_(nxt)
+            return StageOutput(lg[:, :self.V], nxt)
+        dst = out if (last_only and out is not None) else nxt
+        also, adv, hist = (None, None, None) if advance is None else (tuple(advance) + (None,))[:3]
+        part = self.amx_part[q0 * 2 * T_.ARGMAX_PART_PER_ROW:] if last_only and not self.f32 else None
+        T_.argmax_rows(lg, dst, n=self.V, also=also, advance=adv, part=part, hist=hist)
+        return StageOutput(lg[:, :self.V], dst)
+
+    def forward(self, x: torch.Tensor, out: Optional[torch.Tensor] = None):
+        """Full-prefix forward of one request (``TransformerStage.forward``)."""
+        B, T = x.shape[0], x.shape[1]
+        if B > self.max_batch or T > self.max_seq:
+            raise ValueError(f"request (B={B}, T={T}) exceeds the stage cache ({self.max_batch}, {self.max_seq})")
+        if self.first:
+            h = x.to(device=self.device, dtype=torch.int32).contiguous()
+        else:
+            h = x.to(device=self.device, dtype=torch.float32).reshape(B * T, self.d).contiguous()
+        y = self.step(h, torch.zeros((B,), dtype=torch.int32, device=self.device), B, T, last_only=False)
+        if not self.last:
+            return y.view(B, T, self.d)
+        return StageOutput(y.probs.reshape(B, T, self.V), y.pred.view(B, T)[:, -1].contiguous())

@@ -1,0 +1,135 @@
+"""Paged KV cache bookkeeping: pages, block tables and the batch of one step.
+
+* ``PageTable`` — the allocator of a pool of ``PAGE``-key pages shared by every
+  layer of every stage: a sequence takes a slot (a row of the block table) when
+  it is admitted, pages as its length grows, and gives both back when it ends.
+  Freed pages and slots are used again first, so the pool only has to hold what
+  is live.
+* ``StepBatch`` — the device-side description of one engine step: tokens of any
+  number of sequences, prompt portions and single decoded tokens together.
+
+The page pools themselves belong to the stages (``runtime/decoder.py``); a page
+id addresses the same page in each of them.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import Dict, List, Optional, Sequence
+
+import numpy as np
+import torch
+
+from ..ops.decoder_ops import PAGE, chunk_tiles
+
+
+class OutOfPages(RuntimeError):
+    """The pool (or the slots) cannot hold what was asked for; nothing was taken."""
+
+
+def pages_for(tokens: int) -> int:
+    return -(-tokens // PAGE)
+
+
+class PageTable:
+    def __init__(self, num_pages: int, max_slots: int, pages_per_slot: Optional[int] = None):
+        if num_pages < 1 or max_slots < 1:
+            raise ValueError("PageTable: at least one page and one slot")
+        self.num_pages, self.max_slots = num_pages, max_slots
+        self.width = pages_per_slot or num_pages
+        self.table = np.full((max_slots, self.width), -1, dtype=np.int32)
+        self._free_pages = list(range(num_pages - 1, -1, -1))  # stacks: the last freed is used next
+        self._free_slots = list(range(max_slots - 1, -1, -1))
+        self._held: Dict[int, List[int]] = {}
+
+    @property
+    def free_pages(self) -> int:
+        return len(self._free_pages)
+
+    @property
+    def free_slots(self) -> int:
+        return len(self._free_slots)
+
+    def admit(self) -> int:
+        """A free slot (block-table row), without pages yet."""
+        if not self._free_slots:
+            raise OutOfPages(f"all {self.max_slots} sequence slots are in use")
+        slot = self._free_slots.pop()
+        self._held[slot] = []
+        return slot
+
+    def missing(self, slot: int, tokens: int) -> int:
+        """Pages the slot still needs to hold ``tokens`` positions."""
+        return max(0, pages_for(tokens) - len(self._held[slot]))
+
+    def reserve(self, slot: int, tokens: int) -> None:
+        """Pages for positions 0 .. tokens - 1 of the slot's sequence."""
+        held, need = self._held[slot], self.missing(slot, tokens)
+        if need > len(self._free_pages) or len(held) + need > self.width:
+            raise OutOfPages(f"{tokens} tokens need {need} more pages, {len(self._free_pages)} of {self.num_pages} free"
+                             f" (at most {self.width} per sequence)")
+        for _ in range(need):
+            p = self._free_pages.pop()
+            self.table[slot, len(held)] = p
+            held.append(p)
+
+    def release(self, slot: int) -> None:
+        held = self._held.pop(slot)
+        self._free_pages.extend(reversed(held))
+        self.table[slot, :] = -1
+        self._free_slots.append(slot)
+
+
+@dataclass
+class StepBatch:
+    """One step's rows on the device.  ``chunks``: (first row, tokens, slot) of
+    the sequences that bring two tokens or more; ``dec_rows``: rows of the
+    sequences that bring one; ``max_len``: the longest sequence after the step."""
+    M: int
+    pos: torch.Tensor
+    slots: torch.Tensor
+    table: torch.Tensor
+    dec_rows: Optional[torch.Tensor]
+    n_dec: int
+    chunks: Sequence[tuple]
+    max_len: int
+    ids: Optional[torch.Tensor] = None
+    want: Optional[torch.Tensor] = None
+    n_want: int = 0
+    tiles: Optional[Dict[int, torch.Tensor]] = None  # query heads per KV head -> prefill tiles
+
+
+def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[int], device) -> StepBatch:
+    """``entries``: (token ids, first position, slot, wanted places) per
+    sequence.  ``groups``: the query-heads-per-KV-head values of the model's
+    layers.  Everything travels in one host-to-device copy."""
+    ids, pos, slots, dec, want, chunks = [], [], [], [], [], []
+    for toks, p0, slot, places in entries:
+        n, row = len(toks), len(ids)
+        if n == 0:
+            raise ValueError("a step entry brings at least one token")
+        want += [row + w for w in places]
+        ids += toks
+        pos += range(p0, p0 + n)
+        slots += [slot] * n
+        if n == 1:
+            dec.append(row)
+        else:
+            chunks.append((row, n, slot))
+    parts = [("t%d" % g, np.array([t for c in chunks for t in chunk_tiles(*c, g)], dtype=np.int32).reshape(-1))
+             for g in sorted(set(groups))] if chunks else []
+    parts += [("ids", np.array(ids, dtype=np.int32)), ("pos", np.array(pos, dtype=np.int32)),
+              ("slots", np.array(slots, dtype=np.int32)), ("dec", np.array(dec, dtype=np.int32)),
+              ("want", np.array(want, dtype=np.int32)), ("table", table.reshape(-1))]
+    off, total = {}, 0
+    for name, a in parts:
+        off[name] = total
+        total += -(-a.size // 4) * 4  # 16-byte aligned starts
+    host = np.zeros(total, dtype=np.int32)
+    for name, a in parts:
+        host[off[name]:off[name] + a.size] = a
+    dev = torch.from_numpy(host).to(device)
+    v = {name: dev[off[name]:off[name] + a.size] for name, a in parts}
+    return StepBatch(M=len(ids), pos=v["pos"], slots=v["slots"], table=v["table"].view(table.shape),
+                     dec_rows=v["dec"] if dec else None, n_dec=len(dec), chunks=chunks,
+                     max_len=max(pos) + 1, ids=v["ids"], want=v["want"] if want else None, n_want=len(want),
+                     tiles={g: v["t%d" % g].view(-1, 4) for g in set(groups)} if chunks else None)

@@ -580,7 +580,14 @@ def _e4m3_amax(t: torch.Tensor) -> float:
 def build_device_stage(model: str, sd, start: int, end: int, first: bool, last: bool, device, dtype=None,
                        max_batch: int = 8, max_seq: int = 1024, max_tokens: Optional[int] = None,
                        temperature: float = 0.0, top_k: int = 0, seed: int = 0, kv_dtype: str = "bf16",
-                       kv_scale: str = "calibrated", fp8_prefill: str = "e4m3"):
+                       kv_scale: str = "calibrated", fp8_prefill: str = "e4m3", num_pages: Optional[int] = None):
+    """The GPU stage of a model family.  ``num_pages``: page pool of an engine (paged families)."""
+    if model_info(model).family == "kozusun":
+        from .decoder import DecoderStage
+        if kv_dtype != "bf16":
+            raise ValueError(f"model {model!r}: the paged cache follows the compute dtype, kv_cache_dtype {kv_dtype!r}")
+        return DecoderStage(model, sd, start, end, first, last, device, max_batch, max_seq, max_tokens, dtype,
+                            temperature, top_k, seed, num_pages=num_pages)
     fp8 = dtype in ("fp8", "float8_e4m3fn", "fp8_e4m3")
     info = model_info(model)
     max_seq = min(max_seq, getattr(info.cfg, "block_size", getattr(info.cfg, "max_seq", max_seq)))
@@ -589,14 +596,46 @@ def build_device_stage(model: str, sd, start: int, end: int, first: bool, last: 
 
 
 # ---------------------------------------------------------------------- smoke / golden check
+def decoder_smoke(dev) -> None:
+    """Kozusun-tiny, 2 stages: greedy tokens of the decode ring (fixed pages,
+    graphs) equal those of the engine (shared pool, prompts in portions) in the
+    exact mode, and the bf16 logits stay within 3e-2 of the exact ones."""
+    from .. import checkpoint as ckpt
+    from .engine import Engine, Entry
+    from .scheduler import DecodeRing, RingLinks
+    model = "kozusun-tiny"
+    n = model_info(model).num_layers
+    ranges = [(0, n // 2 - 1), (n // 2, n - 1)]
+    sds = [ckpt.random_stage_state_dict(model, a, b, i == 0, i == 1, 7, nontrivial=True)
+           for i, (a, b) in enumerate(ranges)]
+    prompt = torch.randint(0, model_info(model).cfg.vocab_size, (2, 70), generator=torch.Generator().manual_seed(3))
+    logits, toks = {}, {}
+    for dtype in ("float32", "bf16"):
+        def stages():
+            return [build_device_stage(model, sds[i], a, b, i == 0, i == 1, dev, dtype=dtype, max_batch=2, max_seq=96)
+                    for i, (a, b) in enumerate(ranges)]
+        toks[dtype] = DecodeRing(stages(), RingLinks(), 1, 1, 2).generate([prompt], 70, 6)
+        logits[dtype] = Engine(stages(), max_slots=2).step([Entry(i, p, [69]) for i, p in
+                                                           enumerate(prompt.tolist())]).float()
+    got = Engine([build_device_stage(model, sds[i], a, b, i == 0, i == 1, dev, dtype="float32", max_batch=2,
+                                     max_seq=96) for i, (a, b) in enumerate(ranges)],
+                 max_slots=2).generate(prompt.tolist(), 6, budget=33)
+    if got != toks["float32"].tolist():
+        raise AssertionError(f"smoke {model}: engine {got} vs ring {toks['float32'].tolist()}")
+    rel = ((logits["bf16"] - logits["float32"]).norm() / logits["float32"].norm()).item()
+    if not rel < 3e-2:
+        raise AssertionError(f"smoke {model}: bf16 logits rel err {rel:.3e}")
+
+
 def smoke(dev) -> None:
-    """GPT-2-tiny and Llama-tiny, 2 stages each on the decode ring, vs the fp32
-    torch golden: prefill logits within 2e-2 relative, the first generated
+    """Kozusun-tiny: decode ring vs engine (``decoder_smoke``); GPT-2-tiny and
+    Llama-tiny, 2 stages each on the decode ring, vs the fp32 torch golden: prefill logits within 2e-2 relative, the first generated
     token exact, and the greedy continuation equal to the golden's until the
     golden's top-2 logits come within bf16 resolution of each other."""
     from .. import checkpoint as ckpt
     from ..models import build_golden_stage
     from .scheduler import DecodeRing, RingLinks
+    decoder_smoke(dev)
     for model in ("gpt2-tiny", "llama3-tiny"):
         n = model_info(model).num_layers
         ranges = [(0, n // 2 - 1), (n // 2, n - 1)]
