@@ -50,7 +50,8 @@ def build_parser() -> argparse.ArgumentParser:
     p.add_argument("--input_image", help="Path to input image (only used by node with part_index 0)")
     # additive
     p.add_argument("--num_requests", type=int, default=1, help="requests stage 0 sends (default 1)")
-    p.add_argument("--prompt", default=None, help="GPT/Llama: comma-separated token ids (default: random)")
+    p.add_argument("--prompt", default=None, help="language models: comma-separated token ids (default: random); several prompts with ';' "
+                        "between them are batched continuously (transport colocated, paged models)")
     p.add_argument("--shutdown_pipeline", action="store_true",
                    help="stage 0 asks all peers to exit after its requests complete")
     p.add_argument("--serve_seconds", type=float, default=None, help="non-initiating nodes exit after this long")
@@ -97,7 +98,8 @@ def kv_needs(ctx: NodeContext, args) -> Tuple[int, int]:
     pipe = ctx.pipeline
     T = pipe.prompt_len or pipe.seq_len
     if getattr(args, "prompt", None):
-        T = len([v for v in args.prompt.split(",") if v.strip()])
+        from .runtime.generate import parse_prompts
+        T = max((len(p) for p in parse_prompts(args.prompt)), default=T)
     return pipe.micro_batch_size * pipe.num_microbatches, T + max(1, pipe.decode_steps or 1)
 
 
@@ -417,7 +419,9 @@ def run_colocated(ctx: NodeContext, args, device) -> int:
         st, full = build_stage(ctx, p, ranges, device, full, args)
         stages.append(st)
     if fam != "cifar":
-        from .runtime.generate import run_generate_colocated
+        from .runtime.generate import parse_prompts, run_generate_colocated, run_generate_engine
+        if len(parse_prompts(args.prompt)) > 1:
+            return run_generate_engine(ctx, args, stages, device)
         return run_generate_colocated(ctx, args, stages, device)
     mbs, M = pipe.micro_batch_size, pipe.num_microbatches
     cp = ColocatedPipeline(stages, mbs)

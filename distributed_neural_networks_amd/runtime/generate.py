@@ -1,4 +1,4 @@
-"""CLI generation drivers for the transformer families (GPT-2 / Llama-3).
+"""CLI generation drivers for the transformer families (GPT-2 / Llama-3 / Kozusun).
 
 The reference's GPT stages exist only as modules (``partitions/
 gpt_model_parts.py:6-50``) that recompute the whole prefix per call; nothing
@@ -9,6 +9,8 @@ greedily (or sampled) through the pipeline with the ``DecodeRing`` schedule
 
 * ``run_generate_colocated`` — every stage on one GPU (one ring group, each
   microbatch's decode step one HIP graph);
+* ``run_generate_engine`` — several prompts of unequal length (``--prompt
+  "1,2,3;4,5"``) through the paged engine's continuous batching;
 * ``run_generate_dist`` — one rank per stage over RCCL / gloo, tokens return to
   stage 0 over the back-edge.
 
@@ -29,6 +31,11 @@ from ..utils.log import log
 from .scheduler import DecodeRing, RingLinks
 
 
+def parse_prompts(prompt: Optional[str]) -> List[List[int]]:
+    """``--prompt``: comma-separated token ids, several prompts with ``;`` between them."""
+    return [ids for ids in ([int(v) for v in part.split(",") if v.strip()] for part in (prompt or "").split(";")) if ids]
+
+
 def make_prompts(pipe, prompt: Optional[str], replica: int = 0) -> torch.Tensor:
     """(micro_batch_size * num_microbatches, T) int64 prompt ids: ``--prompt``
     (comma-separated ids, replicated to every sequence) or seeded random ids
@@ -36,8 +43,10 @@ def make_prompts(pipe, prompt: Optional[str], replica: int = 0) -> torch.Tensor:
     info = model_info(pipe.model)
     n = pipe.micro_batch_size * pipe.num_microbatches
     if prompt:
-        ids = [int(v) for v in prompt.split(",") if v.strip()]
-        return torch.tensor([ids], dtype=torch.int64).repeat(n, 1)
+        several = parse_prompts(prompt)
+        if len(several) != 1:
+            raise ValueError("--prompt with several prompts: transport 'colocated' and a model with a paged cache only")
+        return torch.tensor(several, dtype=torch.int64).repeat(n, 1)
     g = torch.Generator().manual_seed(1234 + 7919 * replica)
     T = pipe.prompt_len or pipe.seq_len
     return torch.randint(0, info.cfg.vocab_size, (n, T), generator=g)
@@ -104,6 +113,28 @@ def run_generate_colocated(ctx, args, stages: List, device) -> int:
     prompts = [prompt[m * B:(m + 1) * B] for m in range(M)]
     pf, dec = _timed_generate(ring, prompts, T, steps, device, pipe.prefill_chunk)
     _report(ctx.node_id, ring.tokens(), pf, dec, n_seq, T, steps, M, 1)
+    return 0
+
+
+def run_generate_engine(ctx, args, stages: List, device) -> int:
+    """Several prompts of any lengths by continuous batching (``runtime/engine.py``):
+    ``micro_batch_size`` x ``num_microbatches`` sequences are live at a time, the
+    rest queue; ``prefill_chunk`` is the token budget of a step."""
+    from .engine import Engine
+    pipe = ctx.pipeline
+    prompts = parse_prompts(args.prompt)
+    steps = max(1, pipe.decode_steps or 1)
+    engine = Engine(stages, max_slots=pipe.micro_batch_size * pipe.num_microbatches)
+    t0 = time.perf_counter()
+    toks = engine.generate(prompts, steps, budget=pipe.prefill_chunk)
+    _sync(device)
+    dt = time.perf_counter() - t0
+    nid, first = ctx.node_id, [t[0] for t in toks]
+    log(f"[{nid}] ***** FINAL PREDICTION (Index): {first[0] if len(first) == 1 else first} *****")
+    log(f"[{nid}] generated tokens: {json.dumps(toks)}")
+    n = sum(len(p) for p in prompts) + len(prompts) * (steps - 1)
+    log("METRICS " + json.dumps({"node": nid, "sequences": len(prompts), "prompt_tokens": sum(map(len, prompts)),
+                                 "decode_steps": steps - 1, "tokens_per_s": round(n / dt, 1)}))
     return 0
 
 

@@ -9,6 +9,7 @@ capture serves every decode step.
 """
 from __future__ import annotations
 
+import gc
 from typing import Callable, Optional
 
 import torch
@@ -32,10 +33,20 @@ class GraphedStep:
             if reset is not None:
                 reset()
             s.synchronize()
+            # no garbage collection inside the capture: a graph of an earlier
+            # schedule that is collected there is destroyed while the stream
+            # captures, which the runtime answers with an abort
+            gc.collect()
+            collecting = gc.isenabled()
+            gc.disable()
             # thread-local capture: ProcessGroupNCCL's watchdog thread keeps
             # polling its events while a multi-GPU rank captures its decode step
-            with torch.cuda.graph(self.graph, stream=s, pool=pool, capture_error_mode="thread_local"):
-                self.result = fn()
+            try:
+                with torch.cuda.graph(self.graph, stream=s, pool=pool, capture_error_mode="thread_local"):
+                    self.result = fn()
+            finally:
+                if collecting:
+                    gc.enable()
         torch.cuda.current_stream(self.device).wait_stream(s)
 
     def __call__(self):

@@ -3,7 +3,9 @@
 Works on whole sequences (no cache, no batching, no fused weights) with
 ordinary torch CPU operations in ``dtype`` (float64 by default), straight from
 the config dictionary and the checkpoint tensors.  Shares no code with the
-package.
+package.  ``rnd`` rounds what a bf16 implementation may round (operands and
+results of the projections), so tests can ask how much error rounding alone
+makes.
 """
 from __future__ import annotations
 
@@ -11,6 +13,14 @@ import json
 import math
 
 import torch
+
+
+def exact(t):
+    return t
+
+
+def bf16(t):
+    return t.bfloat16().to(t.dtype)
 
 
 def rms_norm(x, eps):
@@ -56,12 +66,13 @@ def head_gate(h, wg):
     return torch.sigmoid(h @ wg.t())
 
 
-def attention_mixer(h, W, pre, m):
+def attention_mixer(h, W, pre, m, rnd=exact):
     H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     T = h.shape[0]
-    q = h @ W[pre + "q"].t() + W[pre + "q.b"]
-    k = h @ W[pre + "k"].t() + W[pre + "k.b"]
-    v = h @ W[pre + "v"].t() + W[pre + "v.b"]
+    h = rnd(h)
+    q = rnd(h @ W[pre + "q"].t() + W[pre + "q.b"])
+    k = rnd(h @ W[pre + "k"].t() + W[pre + "k.b"])
+    v = rnd(h @ W[pre + "v"].t() + W[pre + "v.b"])
     g = head_gate(h, W[pre + "g"])
     ok = visible(T, m.get("mask"))
     outs = []
@@ -69,34 +80,35 @@ def attention_mixer(h, W, pre, m):
         c = n // (H // G)
         s = attention_scores(q[:, n * dk:(n + 1) * dk], k[:, c * dk:(c + 1) * dk], m["scale"])
         outs.append(masked_softmax(s, ok) @ v[:, c * dv:(c + 1) * dv] * g[:, n:n + 1])
-    return torch.cat(outs, -1) @ W[pre + "o"].t()
+    return rnd(torch.cat(outs, -1)) @ W[pre + "o"].t()
 
 
-def gated_mlp(h, W, pre):
-    return (gelu_tanh(h @ W[pre + "gate"].t()) * (h @ W[pre + "up"].t())) @ W[pre + "down"].t()
+def gated_mlp(h, W, pre, rnd=exact):
+    h = rnd(h)
+    return rnd(gelu_tanh(h @ W[pre + "gate"].t()) * (h @ W[pre + "up"].t())) @ W[pre + "down"].t()
 
 
-def side_input(x, e, W, pre, eps):
+def side_input(x, e, W, pre, eps, rnd=exact):
     """Per-layer token input: e (T, side dim) this layer's part of the token's side embedding."""
-    g = gelu_tanh(x @ W[pre + "gate"].t()) * e
-    return rms_norm(g @ W[pre + "proj"].t(), eps) * W[pre + "norm"]
+    g = rnd(gelu_tanh(rnd(rnd(x) @ W[pre + "gate"].t())) * e)
+    return rms_norm(rnd(g @ W[pre + "proj"].t()), eps) * W[pre + "norm"]
 
 
-def loop_in(x, x0, w):
-    return torch.cat([x, x0], -1) @ w.t()
+def loop_in(x, x0, w, rnd=exact):
+    return rnd(torch.cat([x, x0], -1)) @ w.t()
 
 
-def layer(x, tokens, i, cfg, W):
+def layer(x, tokens, i, cfg, W, rnd=exact):
     L, eps, m = cfg["layers"][i], cfg["norm"]["eps"], cfg["residual_mult"]
     h = zero_centred_norm(x, W[f"l{i}.norm1"], eps)
-    y = attention_mixer(h, W, f"l{i}.mix.", L["mixer"])
+    y = attention_mixer(h, W, f"l{i}.mix.", L["mixer"], rnd)
     if L["mlp"] is not None:
-        y = y + gated_mlp(h, W, f"l{i}.mlp.")
-    x = x + m * y
+        y = y + gated_mlp(h, W, f"l{i}.mlp.", rnd)
+    x = x + m * rnd(y)
     if cfg.get("token_side"):
         d = cfg["token_side"]["dim"]
         e = W["side.embed"][tokens][:, i * d:(i + 1) * d]
-        x = x + m * side_input(x, e, W, f"l{i}.side.", eps)
+        x = x + m * side_input(x, e, W, f"l{i}.side.", eps, rnd)
     return x
 
 
@@ -112,16 +124,16 @@ def layer_runs(cfg):
     return runs + [(i, False) for i in range(lp["stop"], n)]
 
 
-def forward(tokens, cfg, W, trace=None):
+def forward(tokens, cfg, W, trace=None, rnd=exact):
     """tokens (T,) -> logits (T, vocab); ``trace``: list that receives the residual after every layer run."""
     x = x0 = embed(tokens, W["embed"], cfg["embedding"]["scale"])
     for i, starts in layer_runs(cfg):
         if starts:
-            x = loop_in(x, x0, W["loop.in"])
-        x = layer(x, tokens, i, cfg, W)
+            x = loop_in(x, x0, W["loop.in"], rnd)
+        x = layer(x, tokens, i, cfg, W, rnd)
         if trace is not None:
             trace.append(x)
-    return zero_centred_norm(x, W["final.norm"], cfg["norm"]["eps"]) @ W["head"].t()
+    return rnd(rnd(zero_centred_norm(x, W["final.norm"], cfg["norm"]["eps"])) @ W["head"].t())
 
 
 def tensor_shapes(cfg):
