@@ -37,7 +37,8 @@ Placements (the stage cut is the reference's at every N: conv | fc1+fc2+softmax,
 Scaling is weak: each stage-0 GPU sources ``--batch`` images per step.
 
 ``--model gpt2`` runs the GPT-2 4-stage token throughput bench instead
-(bench/gpt_bench.py).
+(bench/gpt_bench.py); ``--model kozusun`` times Kozusun layers beside Llama
+layers of the same size, prefill and decode (bench/decoder_bench.py).
 """
 from __future__ import annotations
 
@@ -784,6 +785,9 @@ def main():
         return rc
     if args.model != "cifar10":
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "bench"))
+        if args.model == "kozusun":
+            import decoder_bench
+            return decoder_bench.main(["--steps", str(args.steps)])
         import gpt_bench
         return gpt_bench.main(args)
     phases = {"startup_s": round(elapsed_s(), 2)}

@@ -1,0 +1,142 @@
+#!/usr/bin/env python3
+"""Kozusun layers beside Llama layers of the same size: prefill and decode.
+
+``bench.py --model kozusun`` runs it (one GPU).  For each size, ``--layers``
+layers of random weights of either model (no loop, no head; the residual enters
+from the embedding) run on the same box in turn, timed as HIP graphs for decode
+and eagerly for prefill; medians over alternating repeats.  Kozusun's extra work
+per layer (token input, output gate, fp32 residual) is part of its time.
+Prints one JSON line; ``--phase`` / ``--only`` restrict a profiler run.
+"""
+from __future__ import annotations
+
+import argparse
+import json
+import os
+import statistics
+import sys
+
+import torch
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+if ROOT not in sys.path:
+    sys.path.insert(0, ROOT)
+
+# name -> (Kozusun preset, Llama configuration of the same layer size)
+SIZES = {"8b": ("kozusun-8b", dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=4096, ffn_dim=14336)),
+         "1b": ("kozusun-1b", dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=2048, ffn_dim=5632))}
+
+
+def parse(argv=None):
+    ap = argparse.ArgumentParser()
+    ap.add_argument("--sizes", default="8b,1b")
+    ap.add_argument("--layers", type=int, default=4)
+    ap.add_argument("--batches", default="1,32,64", help="decode batch sizes")
+    ap.add_argument("--context", type=int, default=2048, help="tokens in the cache of a decode step, and of a prompt")
+    ap.add_argument("--prompts", type=int, default=4, help="prompts of a prefill")
+    ap.add_argument("--repeats", type=int, default=7)
+    ap.add_argument("--steps", type=int, default=20, help="decode steps of a repeat")
+    ap.add_argument("--phase", default="both", choices=["both", "prefill", "decode"])
+    ap.add_argument("--only", default="", choices=["", "kozusun", "llama"])
+    return ap.parse_args(argv)
+
+
+def build(size: str, layers: int, batch: int, seq: int, tokens: int, dev):
+    """{model: first-stage object with ``layers`` layers}"""
+    from dataclasses import replace
+    from distributed_neural_networks_amd import checkpoint as ckpt
+    from distributed_neural_networks_amd.models import kozusun, llama3
+    from distributed_neural_networks_amd.runtime.decoder import DecoderStage
+    from distributed_neural_networks_amd.runtime.transformer import TransformerStage
+    preset, lc = SIZES[size]
+    cfg = replace(kozusun.scaled(kozusun.KOZUSUN_CONFIGS[preset], layers), vocab_size=lc["vocab_size"])
+    sd = ckpt.random_kozusun_state(cfg, 0, layers - 1, True, False, 0, dev, True)
+    koz = DecoderStage(preset, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens,
+                       cfg=cfg)
+    del sd
+    name = "llama-layers-" + size
+    llama3.LLAMA_CONFIGS[name] = llama3.LlamaConfig(n_layer=layers, max_seq=seq, **lc)
+    sd = ckpt.random_stage_state_dict(name, 0, layers - 1, True, False, 0, device=dev)
+    lla = TransformerStage(name, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens)
+    return {"kozusun": koz, "llama": lla}
+
+
+def timed(fn, n: int) -> float:
+    """ms per call on the device, ``n`` calls between two events."""
+    a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    a.record()
+    for _ in range(n):
+        fn()
+    b.record()
+    b.synchronize()
+    return a.elapsed_time(b) / n
+
+
+def alternate(fns: dict, repeats: int, n: int) -> dict:
+    for f in fns.values():
+        f()
+    torch.cuda.synchronize()
+    t = {k: [] for k in fns}
+    for _ in range(repeats):
+        for k, f in fns.items():
+            t[k].append(timed(f, n))
+    return {k: statistics.median(v) for k, v in t.items()}
+
+
+def run(argv=None) -> dict:
+    a = parse(argv)
+    from distributed_neural_networks_amd.runtime.graph import GraphedStep
+    dev = torch.device("cuda", 0)
+    torch.cuda.set_device(dev)
+    rows = []
+    for size in a.sizes.split(","):
+        batches = [int(b) for b in a.batches.split(",")]
+        maxb = max(batches + [a.prompts])
+        seq, T = a.context + 64, a.context
+        stages = build(size, a.layers, maxb, seq, max(a.prompts * T, maxb), dev)
+        if a.only:
+            stages = {a.only: stages[a.only]}
+        g = torch.Generator().manual_seed(1)
+        ids = torch.randint(0, SIZES[size][1]["vocab_size"], (maxb, T), generator=g).to(device=dev, dtype=torch.int32)
+        zero = torch.zeros((maxb,), dtype=torch.int32, device=dev)
+        outs = {k: torch.empty(*s.out_spec(a.prompts, T)[:1], dtype=s.out_spec(a.prompts, T)[1], device=dev)
+                for k, s in stages.items()}
+        if a.phase != "decode":
+            B = a.prompts
+            ms = alternate({k: (lambda s=s, k=k: s.step(ids[:B], zero[:B], B, T, out=outs[k]))
+                            for k, s in stages.items()}, a.repeats, 2)
+            for k, v in ms.items():
+                rows.append({"size": size, "phase": "prefill", "model": k, "batch": B, "tokens": B * T,
+                             "us_per_layer": round(v * 1e3 / a.layers, 2),
+                             "tokens_per_s_layer": round(B * T / (v * 1e-3) * a.layers)})
+                print(json.dumps(rows[-1]), file=sys.stderr, flush=True)
+        for B in batches if a.phase != "prefill" else []:
+            pos = torch.full((B,), a.context, dtype=torch.int32, device=dev)
+            x = ids[:B, :1].contiguous()
+            graphs = {}
+            for k, s in stages.items():
+                out = torch.empty(*s.out_spec(B)[:1], dtype=s.out_spec(B)[1], device=dev)
+                graphs[k] = GraphedStep(lambda s=s, out=out: s.step(x, pos, B, 1, out=out), dev)
+            ms = alternate(graphs, a.repeats, a.steps)
+            for k, v in ms.items():
+                rows.append({"size": size, "phase": "decode", "model": k, "batch": B, "context": a.context,
+                             "us_per_layer": round(v * 1e3 / a.layers, 2),
+                             "tokens_per_s_layer": round(B / (v * 1e-3) * a.layers)})
+                print(json.dumps(rows[-1]), file=sys.stderr, flush=True)
+            del graphs
+        del stages, outs
+        torch.cuda.empty_cache()
+    big = [r for r in rows if r["model"] == "kozusun" and r["phase"] == "decode"] or \
+        [r for r in rows if r["model"] == "kozusun"]
+    return {"metric": "layer tokens/s, Kozusun decoder layers", "value": big[-1]["tokens_per_s_layer"] if big else None,
+            "unit": "tokens/s x layers", "n_gpus": 1, "higher_is_better": True, "vs_baseline": None, "dtype": "bf16",
+            "data": "synthetic (random weights)", "config": {"layers": a.layers, "context": a.context}, "rows": rows}
+
+
+def main(argv=None) -> int:
+    print(json.dumps(run(argv)), flush=True)
+    return 0
+
+
+if __name__ == "__main__":
+    sys.exit(main())

@@ -50,9 +50,14 @@ inline void bind_decoder(py::module_& m) {
     a.ldcopy = ldcopy, a.ldh = ldh, a.M = M, a.N = N, a.NP = NP, a.mult = mult, a.eps = eps;
     return dnn_rows_update(&a, y_f32, out_f32, ST(st));
   });
-  m.def("token_gate", [](u64 z, int ldz, u64 table, int ldt, int off, u64 tok, int V, u64 g, int ldg, int M, int n,
-                         int np, int f32, u64 st) {
-    return dnn_token_gate(CP(z), ldz, CP(table), ldt, off, CIP(tok), V, P(g), ldg, M, n, np, f32, ST(st));
+  m.def("token_gate", [](u64 x, int ldx, u64 w, int ldw, u64 wsh, int K, u64 table, int ldt, int off, u64 tok, int V,
+                         u64 g, int ldg, int M, int n, int np, u64 st) {
+    return dnn_token_gate(CP(x), ldx, CP(w), ldw, CP(wsh), K, CP(table), ldt, off, CIP(tok), V, P(g), ldg, M, n, np,
+                          ST(st));
+  });
+  m.def("token_gate_f32", [](u64 z, int ldz, u64 table, int ldt, int off, u64 tok, int V, u64 g, int ldg, int M, int n,
+                             int np, u64 st) {
+    return dnn_token_gate_f32(CFP(z), ldz, CFP(table), ldt, off, CIP(tok), V, FP(g), ldg, M, n, np, ST(st));
   });
   m.def("glu_f32", [](u64 gu, int ldi, u64 out, int ldo, int M, int F, u64 st) {
     return dnn_glu_f32(CFP(gu), ldi, FP(out), ldo, M, F, ST(st));

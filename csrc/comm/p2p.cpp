@@ -9,7 +9,7 @@
 //   * every pair channel is created eagerly and its collective init runs on a
 //     background thread (any creation order is deadlock-free; the id is
 //     published through the process group's TCP store by the lower rank);
-//   * an op posted on the channel's own high-priority stream is ordered after
+//   * an op posted on the channel's own stream is ordered after
 //     the work the caller's stream had queued when it was posted (the buffer
 //     is complete / free), and its completion is an event of a fixed ring that
 //     the caller's stream waits on device-side — the host never blocks on a

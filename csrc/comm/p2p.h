@@ -1,7 +1,7 @@
 // Native stage-to-stage data plane over RCCL (csrc/comm/p2p.cpp).
 //
 // A channel is one RCCL communicator (a peer pair, or a 1-rank loopback) with
-// its own high-priority HIP transfer stream and a ring of completion events.
+// its own HIP transfer stream and a ring of completion events.
 // Ops are posted either on the channel stream — ordered after the work the
 // caller's stream had queued at post time, completion returned as a token the
 // caller's stream can wait on without blocking the host — or directly on the

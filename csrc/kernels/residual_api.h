@@ -1,5 +1,6 @@
 // C ABI of the decoder kernels with an fp32 residual and a paged KV cache
-// (residual_rows.hip, gemm_f32.hip, paged_attention.hip).  As in api.h: every
+// (residual_rows.hip, token_gate.hip, gemm_f32.hip,
+// paged_attention.hip).  As in api.h: every
 // function enqueues on `st`; 0 = success, negative = rejected shape.
 #pragma once
 #include <hip/hip_runtime.h>
@@ -36,8 +37,11 @@ struct PagedAttnArgs {
 
 extern "C" {
 int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStream_t st);
-int dnn_token_gate(const void* z, int ldz, const void* table, int ldt, int off, const int* tok, int V, void* g, int ldg,
-                   int M, int n, int np, int f32, hipStream_t st);
+// g = gelu_tanh(x W^T) * table[tok]: bf16, wsh = W in fragment order; _f32: from z = x W^T
+int dnn_token_gate(const void* x, int ldx, const void* w, int ldw, const void* wsh, int K, const void* table, int ldt,
+                   int off, const int* tok, int V, void* g, int ldg, int M, int n, int np, hipStream_t st);
+int dnn_token_gate_f32(const float* z, int ldz, const float* table, int ldt, int off, const int* tok, int V, float* g,
+                       int ldg, int M, int n, int np, hipStream_t st);
 int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, hipStream_t st);
 int dnn_gemm_f32(const float* A, int lda, const float* W, int ldw, float* C, int ldc, const float* bias, int M, int N,
                  int K, hipStream_t st);

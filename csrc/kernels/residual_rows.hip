@@ -23,10 +23,6 @@ __device__ __forceinline__ void st4(float* p, const f32x4& v) { *reinterpret_cas
 __device__ __forceinline__ void st4(bf16_t* p, const f32x4& v) {
   *reinterpret_cast<uint2*>(p) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
 }
-__device__ __forceinline__ float to_f(float v) { return v; }
-__device__ __forceinline__ float to_f(bf16_t v) { return bf2f(v); }
-__device__ __forceinline__ void from_f(float* p, float v) { *p = v; }
-__device__ __forceinline__ void from_f(bf16_t* p, float v) { *p = f2bf(v); }
 
 // Sum over the TPR threads of a row (TPR = 64: the wave; 256: the workgroup).
 template <int TPR>
@@ -47,7 +43,9 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
   const int m = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
   if (m >= a.M) return;  // TPR 256: uniform over the workgroup
   const int xr = a.xidx != nullptr ? min(max(a.xidx[m], 0), a.xrows - 1) : m;
-  f32x4 x[NC], y[NC];
+  // few values per thread: the norm weights are issued with the row (one memory round trip)
+  constexpr bool PF = NC <= 4;
+  f32x4 x[NC], y[NC], yw[PF ? NC : 1], nw[PF ? NC : 1];
   const float* xp = a.x_in != nullptr ? a.x_in + (size_t)xr * a.ldx : nullptr;
   const YT* yp = nullptr;
   if (a.y != nullptr) {
@@ -62,6 +60,10 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
     if (c < a.NP) {
       if (xp != nullptr) x[i] = ld4(xp + c);
       if (yp != nullptr) y[i] = ld4(yp + c);
+      if constexpr (PF) {
+        if (a.y_w != nullptr) yw[i] = ld4(a.y_w + c);
+        if (a.n_w != nullptr) nw[i] = ld4(a.n_w + c);
+      }
     }
   }
   if (a.y_w != nullptr) {
@@ -74,7 +76,7 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
       const int c = (t + TPR * i) * 4;
-      if (c < a.NP) y[i] = y[i] * r * ld4(a.y_w + c);
+      if (c < a.NP) y[i] = y[i] * r * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c));
     }
   }
   float s = 0.f;
@@ -96,7 +98,7 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
     const int c = (t + TPR * i) * 4;
-    if (c < a.NP) st4(reinterpret_cast<OT*>(a.h) + (size_t)m * a.ldh + c, x[i] * r * ld4(a.n_w + c));
+    if (c < a.NP) st4(reinterpret_cast<OT*>(a.h) + (size_t)m * a.ldh + c, x[i] * r * (PF ? nw[PF ? i : 0] : ld4(a.n_w + c)));
   }
 }
 
@@ -122,26 +124,6 @@ static int rows_launch(const RowsArgs& a, hipStream_t st) {
   return -1;
 }
 
-// g[m, c] = gelu_tanh(z[m, c]) * table[token[m], off + c] for c < n, 0 up to np.
-template <typename T>
-__global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z, int ldz, const T* __restrict__ table,
-                                                         int ldt, int off, const int* __restrict__ tok, int V,
-                                                         T* __restrict__ g, int ldg, int M, int n, int np) {
-  const long i = blockIdx.x * 256L + threadIdx.x;
-  if (i >= (long)M * np) return;
-  const int m = (int)(i / np), c = (int)(i % np);
-  float v = 0.f;
-  if (c < n) {
-    const float x = to_f(z[(size_t)m * ldz + c]);
-    const float e = to_f(table[(size_t)min(max(tok[m], 0), V - 1) * ldt + off + c]);
-    if constexpr (sizeof(T) == 4)
-      v = 0.5f * x * (1.0f + tanhf(0.797884560802865f * (x + 0.044715f * x * x * x))) * e;
-    else
-      v = gelu_tanh(x) * e;
-  }
-  from_f(g + (size_t)m * ldg + c, v);
-}
-
 // fp32 gated activation of packed gate|up columns (8 gate, 8 up, ...): out = gelu_tanh(gate) * up.
 __global__ __launch_bounds__(256) void glu_f32_kernel(const float* __restrict__ gu, int ldi, float* __restrict__ out,
                                                       int ldo, int M, int F) {
@@ -163,19 +145,6 @@ extern "C" int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStr
   if ((a->xidx != nullptr && (a->xrows < 1 || a->x_out != nullptr)) || (a->yidx != nullptr && a->yrows < 1)) return -1;
   if (y_f32) return out_f32 ? rows_launch<float, float>(*a, st) : rows_launch<float, bf16_t>(*a, st);
   return out_f32 ? -1 : rows_launch<bf16_t, bf16_t>(*a, st);
-}
-
-extern "C" int dnn_token_gate(const void* z, int ldz, const void* table, int ldt, int off, const int* tok, int V,
-                              void* g, int ldg, int M, int n, int np, int f32, hipStream_t st) {
-  if (M <= 0 || n <= 0 || n > np || off < 0 || off + n > ldt || V < 1) return -1;
-  const dim3 grid((unsigned)(((long)M * np + 255) / 256));
-  if (f32)
-    hipLaunchKernelGGL(token_gate_kernel<float>, grid, dim3(256), 0, st, (const float*)z, ldz, (const float*)table, ldt,
-                       off, tok, V, (float*)g, ldg, M, n, np);
-  else
-    hipLaunchKernelGGL(token_gate_kernel<bf16_t>, grid, dim3(256), 0, st, (const bf16_t*)z, ldz, (const bf16_t*)table,
-                       ldt, off, tok, V, (bf16_t*)g, ldg, M, n, np);
-  return (int)hipGetLastError();
 }
 
 extern "C" int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, hipStream_t st) {

@@ -8,6 +8,7 @@
 #include <cstdio>
 
 #include "../kernels/api.h"
+#include "../kernels/residual_api.h"
 
 static int g_fail = 0;
 
@@ -33,6 +34,45 @@ int main() {
   float* f = reinterpret_cast<float*>(buf);
   int* ip = reinterpret_cast<int*>(buf);
   hipStream_t st = nullptr;
+  // decoder kernels
+  RowsArgs ra = {};
+  ra.x_in = f, ra.x_out = f, ra.ldx = ra.ldy = 64, ra.M = 1, ra.N = 64, ra.NP = 64;
+  RowsArgs rb = ra;
+  rb.M = 0;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows M=0");
+  rb = ra, rb.N = 65;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows N > NP");
+  rb = ra, rb.NP = 20000;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows too wide");
+  rb = ra, rb.xidx = ip, rb.xrows = 1;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows gathered in-place");
+  expect_reject(dnn_rows_update(&ra, 0, 1, st), "rows bf16 in, fp32 operand out");
+  expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 8, ip, 5, p, 64, 4, 24, 64, st), "token gate past the row");
+  expect_reject(dnn_token_gate(p, 64, p, 64, nullptr, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 64, st),
+                "token gate without the fragment copy");
+  expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 48, st), "token gate np%64");
+  expect_reject(dnn_gemm_f32(f, 24, f, 24, f, 8, nullptr, 4, 8, 24, st), "f32 gemm K%16");
+  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 12, st), "glu F%8");
+  PagedAttnArgs pa = {};
+  pa.qkv = pa.kp = pa.vp = pa.out = p, pa.table = pa.slots = pa.pos = ip;
+  pa.ldq = 256, pa.ldo = 64, pa.ldt = 1, pa.npages = 1, pa.M = 1, pa.H = pa.G = 1, pa.DK = pa.DV = 64;
+  pa.gate = 192, pa.window = 8, pa.keep = 0, pa.scale = 1.f;
+  auto bad = [&](auto edit, const char* what) {
+    PagedAttnArgs b = pa;
+    edit(b);
+    expect_reject(dnn_paged_decode(&b, ip, 1, 1, nullptr, 0, st), what);
+    expect_reject(dnn_paged_prefill(&b, ip, 1, st), what);
+  };
+  bad([](PagedAttnArgs& b) { b.DK = 96; }, "paged head size 96");
+  bad([](PagedAttnArgs& b) { b.G = 2; }, "paged heads % kv heads");
+  bad([](PagedAttnArgs& b) { b.ldq = 128; }, "paged qkv row too short");
+  bad([](PagedAttnArgs& b) { b.window = 0; }, "paged empty window");
+  bad([](PagedAttnArgs& b) { b.gate = 256; }, "paged gate past the row");
+  bad([](PagedAttnArgs& b) { b.scale = -1.f; }, "paged negative scale");
+  bad([](PagedAttnArgs& b) { b.table = nullptr; }, "paged without a block table");
+  expect_reject(dnn_paged_decode(&pa, ip, 1, 2, f, 4, st), "paged decode workspace too small");
+  expect_reject(dnn_paged_decode(&pa, ip, 0, 1, nullptr, 0, st), "paged decode of nothing");
+  expect_reject(dnn_paged_prefill(&pa, ip, 0, st), "paged prefill of nothing");
   // GEMMs
   expect_reject(dnn_gemm_bf16(p, 96, p, 96, p, 8, nullptr, nullptr, 0, 128, 128, 96, 0, 0, st), "gemm K%64");
   expect_reject(dnn_gemm_bf16(p, 64, p, 64, p, 8, nullptr, nullptr, 0, 0, 128, 64, 0, 0, st), "gemm M=0");

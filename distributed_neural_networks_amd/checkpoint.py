@@ -175,7 +175,7 @@ def random_stage_state_dict(model: str, start: int, end: int, first: bool, last:
                 if k.split(".")[0] in {n for u in range(start, end + 1) for n in cifar.UNIT_KEYS[u]}}
     dev = torch.device(device) if device is not None else torch.device("cpu")
     if info.family == "kozusun":
-        return _random_kozusun(info.cfg, start, end, first, last, seed, dev, nontrivial)
+        return random_kozusun_state(info.cfg, start, end, first, last, seed, dev, nontrivial)
     shapes = _stage_shapes(model, start, end, first, last)
     sd = {}
     for local, shape in shapes.items():
@@ -196,7 +196,7 @@ def random_stage_state_dict(model: str, start: int, end: int, first: bool, last:
     return sd
 
 
-def _random_kozusun(cfg, start, end, first, last, seed, dev, nontrivial) -> Dict[str, torch.Tensor]:
+def random_kozusun_state(cfg, start, end, first, last, seed, dev, nontrivial) -> Dict[str, torch.Tensor]:
     """Biases zero and norm weights one (stored around zero where the model adds
     the one), or noise around those with ``nontrivial``; projections of unit gain."""
     sd = {}

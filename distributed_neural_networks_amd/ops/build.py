@@ -116,7 +116,8 @@ def _compile(src: str, force: bool, extra: List[str]) -> str:
 # for a first use in a checkout that has no library yet (``ensure``).
 SUBSETS = {"": ("_dnn_hip", None, []),
            "decoder": ("_dnn_decoder", ("gemm_bf16.hip", "gemm_skinny.hip", "sampler.hip", "gemm_f32.hip",
-                                        "residual_rows.hip", "paged_attention.hip", "bindings_decoder.cpp"),
+                                        "residual_rows.hip", "token_gate.hip", "paged_attention.hip",
+                                        "bindings_decoder.cpp"),
                        ["-DDNN_DECODER_ONLY"])}
 
 

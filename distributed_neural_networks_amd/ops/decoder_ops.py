@@ -1,5 +1,6 @@
 """Wrappers of the decoder kernels with an fp32 residual and a paged KV cache
-(``csrc/kernels/residual_rows.hip``, ``gemm_f32.hip``, ``paged_attention.hip``).
+(``csrc/kernels/residual_rows.hip``, ``token_gate.hip``, ``gemm_f32.hip``,
+``paged_attention.hip``).
 
 Operands are bf16 (serving) or fp32 (exact mode: fp32 weights, activations,
 cache and MFMA); the residual stream is fp32 in both.  As in
@@ -86,20 +87,6 @@ def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx
                             int(od == f32), stream_ptr()), "rows_update")
 
 
-def token_gate(z: torch.Tensor, table: torch.Tensor, off: int, ids: torch.Tensor, out: torch.Tensor, M: int,
-               n: int) -> torch.Tensor:
-    """``out[m, c] = gelu_tanh(z[m, c]) * table[ids[m], off + c]`` for c < n; 0 in the padding columns."""
-    dt = (z.dtype,)
-    _rows(z, M, n, "token_gate z", (torch.float32, torch.bfloat16))
-    _rows(table, 1, off + n, "token_gate table", dt)
-    _rows(out, M, n, "token_gate out", dt)
-    _index(ids, M, "token_gate ids")
-    check(lib().token_gate(ptr(z), z.stride(0), ptr(table), table.stride(0), off, ptr(ids), table.shape[0], ptr(out),
-                           out.stride(0), M, n, out.shape[1], int(z.dtype == torch.float32), stream_ptr()),
-          "token_gate")
-    return out
-
-
 def linear_f32(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
     """``x @ w.T + bias`` on the fp32 MFMA (K a multiple of 16)."""
     M, K = x.shape
@@ -141,6 +128,32 @@ class Linear:
         _rows(out, M, F, "gated linear out", (torch.float32,))
         check(lib().glu_f32(ptr(gu), gu.stride(0), ptr(out), out.stride(0), M, F, stream_ptr()), "glu_f32")
         return out
+
+
+def token_gate(x: torch.Tensor, lin: Linear, table: torch.Tensor, off: int, ids: torch.Tensor, out: torch.Tensor,
+               n: int, scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[m, c] = gelu_tanh((x W^T)[m, c]) * table[ids[m], off + c]`` for c < n,
+    0 in the padding columns; ``lin``: W (rows padded to a multiple of 64).
+    ``scratch`` (fp32): (M, weight rows) for the projection."""
+    M, K = x.shape
+    dt, np_ = lin.w.dtype, lin.w.shape[0]
+    _rows(x, M, K, "token_gate x", (dt,))
+    _rows(table, 1, off + n, "token_gate table", (dt,))
+    _rows(out, M, np_, "token_gate out", (dt,))
+    _index(ids, M, "token_gate ids")
+    if lin.w.shape[1] != K or lin.bias is not None or np_ % 64 or not 0 < n <= np_:
+        raise ValueError(f"token_gate: x {tuple(x.shape)} vs w {tuple(lin.w.shape)}, {n} columns")
+    if dt == torch.float32:
+        z = linear_f32(x, lin.w, None, scratch[:M])
+        check(lib().token_gate_f32(ptr(z), z.stride(0), ptr(table), table.stride(0), off, ptr(ids), table.shape[0],
+                                   ptr(out), out.stride(0), M, n, np_, stream_ptr()), "token_gate_f32")
+        return out
+    if lin.ws is None or lin.ws.numel() != np_ * K * 2:
+        raise ValueError("token_gate: the weight needs its fragment-order copy")
+    check(lib().token_gate(ptr(x), x.stride(0), ptr(lin.w), lin.w.stride(0), ptr(lin.ws), K, ptr(table),
+                           table.stride(0), off, ptr(ids), table.shape[0], ptr(out), out.stride(0), M, n, np_,
+                           stream_ptr()), "token_gate")
+    return out
 
 
 def paged_args(qkv: torch.Tensor, kp: torch.Tensor, vp: torch.Tensor, table: torch.Tensor, slots: torch.Tensor,

@@ -5,7 +5,7 @@ The SURVEY §7.1 data plane: stage hops go straight to RCCL
 ProcessGroupNCCL's P2P.
 
 * ``Channel``: one RCCL communicator (a peer pair or a 1-rank loopback) with
-  its own high-priority transfer stream and a ring of completion events.  The
+  its own transfer stream and a ring of completion events.  The
   lower rank of a pair draws the RCCL unique id and publishes it in the
   process group's TCP store; the higher rank reads it, and both run the
   collective init, on a background thread, so opening a channel never blocks

@@ -16,8 +16,9 @@ the tanh-GELU product in its epilogue; attention (decode: cache write, attention
 and output gate in one launch; prefill: cache write, then flash attention) —
 both sublayers write one row ``[attention | feed-forward]``, so ONE projection
 with the two output matrices side by side gives their sum; residual update;
-token-input projections around ``token_gate``; residual update + the next run's
-norm in one pass.  The residual, norms, scores and softmax are fp32.
+token-input gate (projection, activation and product with the token's row in one
+launch) and its output projection; residual update + the next run's norm in one
+pass.  The residual, norms, scores and softmax are fp32.
 
 ``dtype="float32"`` runs the same sequence with fp32 weights, activations,
 cache and matrix products (``ops/decoder_ops.py``).
@@ -164,7 +165,8 @@ class DecoderStage(StageCompute):
         ff = max(L.n_ff for L in self.layers)
         self.gu = z(2 * ff) if self.f32 and ff else None
         if self.side:
-            self.z, self.g = z(D_.pad64(self.side)), z(D_.pad64(self.side))
+            self.g = z(D_.pad64(self.side))
+            self.z = z(D_.pad64(self.side)) if self.f32 else None
         if self.enters:
             self.y32 = self.y if self.f32 else z(self.wp, torch.float32)
         if not self.first:
@@ -264,8 +266,7 @@ class DecoderStage(StageCompute):
                 up(x_in=x, y=y, mult=self.mult, x_out=x, **nxt)
                 continue
             up(x_in=x, y=y, mult=self.mult, x_out=x, copy=xc)
-            L.w_sgate(xc, self.z[s], gws)
-            D_.token_gate(self.z[s], self.side_embed, L.side_off, ids, self.g[s], M, self.side)
+            D_.token_gate(xc, L.w_sgate, self.side_embed, L.side_off, ids, self.g[s], self.side, self.z)
             L.w_sproj(self.g[s], y, gws)
             up(x_in=x, y=y, mult=self.mult, y_norm=L.side_norm, x_out=x, **nxt)
 
