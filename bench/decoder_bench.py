@@ -50,7 +50,7 @@ def build(size: str, layers: int, batch: int, seq: int, tokens: int, dev):
     from distributed_neural_networks_amd.runtime.transformer import TransformerStage
     preset, lc = SIZES[size]
     cfg = replace(kozusun.scaled(kozusun.KOZUSUN_CONFIGS[preset], layers), vocab_size=lc["vocab_size"])
-    sd = ckpt.random_kozusun_state(cfg, 0, layers - 1, True, False, 0, dev, True)
+    sd = ckpt.random_decoder_state(kozusun, cfg, 0, layers - 1, True, False, 0, dev, True)
     koz = DecoderStage(preset, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens,
                        cfg=cfg)
     del sd

@@ -8,6 +8,7 @@
 #include <cstdint>
 
 #include "kernels/api.h"
+#include "kernels/mixer_api.h"
 #include "kernels/residual_api.h"
 
 namespace py = pybind11;
@@ -41,15 +42,65 @@ inline void bind_decoder(py::module_& m) {
                            reinterpret_cast<void*>(static_cast<uintptr_t>(part)), IP(hist), hist_ld);
   }, py::arg("x"), py::arg("ld"), py::arg("M"), py::arg("N"), py::arg("out"), py::arg("f32in"), py::arg("st"),
      py::arg("out2") = 0, py::arg("pos_inc") = 0, py::arg("part") = 0, py::arg("hist") = 0, py::arg("hist_ld") = 0);
-  m.def("rows_update", [](u64 x_in, u64 xidx, int xrows, u64 y, u64 yidx, int yrows, int ldy, float mult, u64 y_w,
-                          u64 x_out, int ldx, u64 copy, int ldcopy, u64 n_w, u64 h, int ldh, int M, int N, int NP,
-                          float eps, int y_f32, int out_f32, u64 st) {
-    RowsArgs a;
-    a.x_in = CFP(x_in), a.xidx = CIP(xidx), a.y = CP(y), a.yidx = CIP(yidx), a.y_w = CFP(y_w), a.x_out = FP(x_out);
-    a.copy = P(copy), a.n_w = CFP(n_w), a.h = P(h), a.xrows = xrows, a.yrows = yrows, a.ldx = ldx, a.ldy = ldy;
-    a.ldcopy = ldcopy, a.ldh = ldh, a.M = M, a.N = N, a.NP = NP, a.mult = mult, a.eps = eps;
+  // argument structs: pointers as addresses, every field by name
+#define PF(S, f) .def_property(#f, [](const S& a) { return (u64)(uintptr_t)a.f; }, [](S& a, u64 v) { a.f = reinterpret_cast<decltype(a.f)>(static_cast<uintptr_t>(v)); })
+#define VF(S, f) .def_readwrite(#f, &S::f)
+  py::class_<RowsArgs>(m, "RowsArgs")
+      .def(py::init([] { return RowsArgs{}; }))
+      PF(RowsArgs, x_in) PF(RowsArgs, xidx) PF(RowsArgs, y) PF(RowsArgs, yidx) PF(RowsArgs, y_w) PF(RowsArgs, x_out)
+      PF(RowsArgs, copy) PF(RowsArgs, n_w) PF(RowsArgs, h) PF(RowsArgs, x_add) PF(RowsArgs, y2) PF(RowsArgs, y2_w)
+      PF(RowsArgs, ys) PF(RowsArgs, ysi) PF(RowsArgs, ysw) PF(RowsArgs, n_b) PF(RowsArgs, pos) PF(RowsArgs, freq)
+      VF(RowsArgs, xrows) VF(RowsArgs, yrows) VF(RowsArgs, ldx) VF(RowsArgs, ldy) VF(RowsArgs, ldcopy) VF(RowsArgs, ldh)
+      VF(RowsArgs, M) VF(RowsArgs, N) VF(RowsArgs, NP) VF(RowsArgs, mult) VF(RowsArgs, eps) VF(RowsArgs, ldadd)
+      VF(RowsArgs, ldy2) VF(RowsArgs, ldys) VF(RowsArgs, ysrows) VF(RowsArgs, top) VF(RowsArgs, n_alpha);
+  m.def("rows_update", [](const RowsArgs& a, int y_f32, int out_f32, u64 st) {
     return dnn_rows_update(&a, y_f32, out_f32, ST(st));
   });
+  py::class_<QkNormArgs>(m, "QkNormArgs")
+      .def(py::init([] { return QkNormArgs{}; }))
+      PF(QkNormArgs, qkv) PF(QkNormArgs, kp) PF(QkNormArgs, kscale) PF(QkNormArgs, qw) PF(QkNormArgs, table)
+      PF(QkNormArgs, slots) PF(QkNormArgs, pos) VF(QkNormArgs, ldq) VF(QkNormArgs, ldt) VF(QkNormArgs, npages)
+      VF(QkNormArgs, M) VF(QkNormArgs, H) VF(QkNormArgs, G) VF(QkNormArgs, DK) VF(QkNormArgs, nq) VF(QkNormArgs, nk)
+      VF(QkNormArgs, t_every) VF(QkNormArgs, t_coef) VF(QkNormArgs, eps);
+  m.def("qk_norm", [](const QkNormArgs& a, int f32, u64 st) { return dnn_qk_norm(&a, f32, ST(st)); });
+  py::class_<ConvArgs>(m, "ConvArgs")
+      .def(py::init([] { return ConvArgs{}; }))
+      PF(ConvArgs, in) PF(ConvArgs, w) PF(ConvArgs, b) PF(ConvArgs, ring) PF(ConvArgs, out) PF(ConvArgs, start)
+      PF(ConvArgs, slots) PF(ConvArgs, pos) PF(ConvArgs, dt_bias) PF(ConvArgs, a_log) PF(ConvArgs, dt) PF(ConvArgs, la)
+      VF(ConvArgs, ldi) VF(ConvArgs, ldo) VF(ConvArgs, M) VF(ConvArgs, C) VF(ConvArgs, taps) VF(ConvArgs, dt_col)
+      VF(ConvArgs, H) VF(ConvArgs, nslots);
+  m.def("conv", [](const ConvArgs& a, int f32, u64 st) { return dnn_conv(&a, f32, ST(st)); });
+  m.def("conv_state", [](const ConvArgs& a, u64 ent, int nent, int f32, u64 st) {
+    return dnn_conv_state(&a, reinterpret_cast<const int4*>(CP(ent)), nent, f32, ST(st));
+  });
+  py::class_<ScanArgs>(m, "ScanArgs")
+      .def(py::init([] { return ScanArgs{}; }))
+      PF(ScanArgs, rows) PF(ScanArgs, dt) PF(ScanArgs, la) PF(ScanArgs, la_h) PF(ScanArgs, D) PF(ScanArgs, state)
+      PF(ScanArgs, y) PF(ScanArgs, ent) PF(ScanArgs, pos) VF(ScanArgs, ld) VF(ScanArgs, ldy) VF(ScanArgs, qcol)
+      VF(ScanArgs, kcol) VF(ScanArgs, vcol) VF(ScanArgs, qdiv) VF(ScanArgs, M) VF(ScanArgs, H) VF(ScanArgs, NP)
+      VF(ScanArgs, VP) VF(ScanArgs, vdim) VF(ScanArgs, nent) VF(ScanArgs, nslots) VF(ScanArgs, dt_c);
+  m.def("scan_steps", [](const ScanArgs& a, int f32, u64 st) { return dnn_scan_steps(&a, f32, ST(st)); });
+  m.def("scan_chunks", [](const ScanArgs& a, u64 st) { return dnn_scan_chunks(&a, ST(st)); });
+  py::class_<GatedNormArgs>(m, "GatedNormArgs")
+      .def(py::init([] { return GatedNormArgs{}; }))
+      PF(GatedNormArgs, y) PF(GatedNormArgs, z) PF(GatedNormArgs, w) PF(GatedNormArgs, out) VF(GatedNormArgs, ldy)
+      VF(GatedNormArgs, ldz) VF(GatedNormArgs, ldo) VF(GatedNormArgs, M) VF(GatedNormArgs, n) VF(GatedNormArgs, groups)
+      VF(GatedNormArgs, gate_first) VF(GatedNormArgs, eps);
+  m.def("gated_norm", [](const GatedNormArgs& a, int f32, u64 st) { return dnn_gated_norm(&a, f32, ST(st)); });
+  py::class_<RouteArgs>(m, "RouteArgs")
+      .def(py::init([] { return RouteArgs{}; }))
+      PF(RouteArgs, logits) PF(RouteArgs, idx) PF(RouteArgs, w) PF(RouteArgs, rank) PF(RouteArgs, counts)
+      PF(RouteArgs, order) PF(RouteArgs, place) PF(RouteArgs, offs) VF(RouteArgs, ldl) VF(RouteArgs, M) VF(RouteArgs, E)
+      VF(RouteArgs, groups) VF(RouteArgs, keep) VF(RouteArgs, top);
+  m.def("route", [](const RouteArgs& a, u64 st) { return dnn_route(&a, ST(st)); });
+  py::class_<GroupedArgs>(m, "GroupedArgs")
+      .def(py::init([] { return GroupedArgs{}; }))
+      PF(GroupedArgs, A) PF(GroupedArgs, W) PF(GroupedArgs, Wsh) PF(GroupedArgs, C) PF(GroupedArgs, offs)
+      PF(GroupedArgs, order) PF(GroupedArgs, counts) VF(GroupedArgs, lda) VF(GroupedArgs, ldc) VF(GroupedArgs, rows)
+      VF(GroupedArgs, arows) VF(GroupedArgs, div) VF(GroupedArgs, N) VF(GroupedArgs, K) VF(GroupedArgs, E)
+      VF(GroupedArgs, act);
+  m.def("grouped_gemm", [](const GroupedArgs& a, u64 st) { return dnn_grouped_gemm(&a, ST(st)); });
+  m.def("grouped_gemm_f32", [](const GroupedArgs& a, u64 st) { return dnn_grouped_gemm_f32(&a, ST(st)); });
   m.def("token_gate", [](u64 x, int ldx, u64 w, int ldw, u64 wsh, int K, u64 table, int ldt, int off, u64 tok, int V,
                          u64 g, int ldg, int M, int n, int np, u64 st) {
     return dnn_token_gate(CP(x), ldx, CP(w), ldw, CP(wsh), K, CP(table), ldt, off, CIP(tok), V, P(g), ldg, M, n, np,
@@ -59,8 +110,8 @@ inline void bind_decoder(py::module_& m) {
                              int np, u64 st) {
     return dnn_token_gate_f32(CFP(z), ldz, CFP(table), ldt, off, CIP(tok), V, FP(g), ldg, M, n, np, ST(st));
   });
-  m.def("glu_f32", [](u64 gu, int ldi, u64 out, int ldo, int M, int F, u64 st) {
-    return dnn_glu_f32(CFP(gu), ldi, FP(out), ldo, M, F, ST(st));
+  m.def("glu_f32", [](u64 gu, int ldi, u64 out, int ldo, int M, int F, int act, u64 st) {
+    return dnn_glu_f32(CFP(gu), ldi, FP(out), ldo, M, F, act, ST(st));
   });
   m.def("gemm_f32", [](u64 A, int lda, u64 W, int ldw, u64 C, int ldc, u64 bias, int M, int N, int K, u64 st) {
     return dnn_gemm_f32(CFP(A), lda, CFP(W), ldw, FP(C), ldc, CFP(bias), M, N, K, ST(st));
@@ -73,7 +124,9 @@ inline void bind_decoder(py::module_& m) {
         a.out = P(out), a.ldq = ldq, a.ldo = ldo, a.ldt = ldt, a.npages = npages, a.M = M, a.H = H, a.G = G;
         a.DK = DK, a.DV = DV, a.gate = gate, a.window = window, a.keep = keep, a.scale = scale;
         return a;
-      }));
+      }))
+      PF(PagedAttnArgs, kscale) PF(PagedAttnArgs, slopes) VF(PagedAttnArgs, gate_el) VF(PagedAttnArgs, shared)
+      VF(PagedAttnArgs, written);
   m.def("paged_write", [](const PagedAttnArgs& a, int f32, u64 st) { return dnn_paged_write(&a, f32, ST(st)); });
   m.def("paged_prefill", [](const PagedAttnArgs& a, u64 tiles, int ntiles, u64 st) {
     return dnn_paged_prefill(&a, CIP(tiles), ntiles, ST(st));

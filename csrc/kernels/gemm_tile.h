@@ -1,0 +1,556 @@
+// Tile pieces of the large bf16 GEMMs and the 256x256 / 256x128 kernel itself,
+// shared by the plain GEMMs (gemm_bf16.hip) and the products of rows grouped by
+// expert (moe.hip).
+#pragma once
+#include <type_traits>
+#include "common.h"
+#include "gemm_epilogue.h"
+#include "grouped_tile.h"
+
+namespace dnn {
+
+constexpr int GB_M = 128, GB_N = 128, GB_K = 64;
+constexpr int G_TILE_BYTES = GB_M * GB_K * 2;  // 16 KiB per operand tile
+
+__device__ __forceinline__ int swz_chunk(int row) { return (row >> 1) & 7; }
+
+// Stage one 128x64 bf16 tile (rows r0.., clamped to nrows-1) into LDS `dst`.
+__device__ __forceinline__ void stage_tile(const bf16_t* __restrict__ src, int ld, int r0, int nrows,
+                                           int k0, char* dst, int wave, int lane) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int piece = wave * 4 + i;            // 1 KiB = 8 rows per wave-instruction
+    const int rl = piece * 8 + (lane >> 3);    // row within the tile
+    const int cp = lane & 7;                   // destination 16B chunk (linear)
+    const int cs = cp ^ swz_chunk(rl);         // source chunk (inverse swizzle)
+    int r = r0 + rl;
+    r = r < nrows ? r : nrows - 1;
+    const bf16_t* g = src + (size_t)r * ld + k0 + cs * 8;
+    glds16(g, dst + piece * 1024);
+  }
+}
+
+__device__ __forceinline__ bf16x8 lds_frag(const char* tile, int row, int chunk) {
+  return *reinterpret_cast<const bf16x8*>(tile + row * 128 + ((chunk ^ swz_chunk(row)) << 4));
+}
+
+// Tile order: the XCD remap gives each XCD a contiguous run of logical ids;
+// inside it tiles go GROUP_M rows of M-tiles at a time, M fastest, so the ~32-64
+// tiles co-resident on one XCD share a few A and W panels in its L2.
+__device__ __forceinline__ void tile_coords(int logical, int ntm, int ntn, int& tm, int& tn) {
+  constexpr int GROUP_M = 8;
+  const int per_group = GROUP_M * ntn;
+  const int grp = logical / per_group;
+  const int first = grp * GROUP_M;
+  const int gm = min(ntm - first, GROUP_M);
+  const int r = logical - grp * per_group;
+  tm = first + r % gm;
+  tn = r / gm;
+}
+
+// ---------------------------------------------------------------------------
+// Large-tile GEMM: 256x256x64, 8 waves (2 M x 4 N), ~1 block per CU, the
+// 4-phase-per-K-tile schedule of the guide's 256^2 template (§5 "8-phase"):
+//
+//   LDS = [2 buffers][A0 A1 B0 B1] half-tiles of 128 rows x 64 k (16 KiB each),
+//   one __shared__ array (trap 4(a)).  Half-tile h of A holds the rows of every
+//   wave's output quadrant-row h, so a wave's 128x64 output is 2x2 quadrants of
+//   64x32 and each phase is one quadrant x K=64 = 16 MFMAs:
+//
+//     ph1: read B0 (4 ds_read_b128), A0 (8)  | stage A1[t+1] -> buf^1 | C00
+//     ph2: read B1 (4)                       | stage B0[t+1] -> buf^1 | C01
+//     ph3: read A1 (8)                       | stage A0[t+2] -> buf   | C11
+//     ph4: read B0 (4)                       | stage B1[t+2] -> buf   | C10
+//          + s_waitcnt vmcnt(4)  (retires everything of tile t+1)
+//
+//   Every restage lands >= 2 phases after the last read of that half-tile
+//   (WAR), every read is >= 1 phase after the vmcnt+barrier that retired its
+//   DMA (RAW).  Each phase = [ds_reads + 2 glds] s_barrier [lgkmcnt(0),
+//   setprio(1), 16 MFMA] s_barrier; waves of M-row 1 run one barrier behind
+//   M-row 0, so on every SIMD one wave issues LDS reads while its partner
+//   issues MFMAs.  glds stays in flight across barriers (raw s_barrier, counted
+//   vmcnt, never __syncthreads in the loop).  Loads past the last K-tile are
+//   clamped to it (harmless refills of dead buffers) so the vmcnt count is
+//   uniform.
+// ---------------------------------------------------------------------------
+constexpr int BG_M = 256, BG_N = 256, BG_K = 64;
+constexpr int BG_HALF = 128 * BG_K * 2;  // 16 KiB
+
+// Stage one 128x64 half-tile: 2 glds per thread, 8 rows per wave-instruction.
+__device__ __forceinline__ void stage_half(const bf16_t* __restrict__ src, int ld, int r0, int nrows, int k0,
+                                           char* dst, int wave, int lane) {
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int piece = i * 8 + wave;
+    const int rl = piece * 8 + (lane >> 3);
+    const int cs = (lane & 7) ^ swz_chunk(rl);
+    int r = r0 + rl;
+    r = r < nrows ? r : nrows - 1;
+    glds16(src + (size_t)r * ld + k0 + cs * 8, dst + piece * 1024);
+  }
+}
+
+// The same from a weight in fragment order (blocks of 16 rows x 32 columns): a
+// wave-instruction reads eight 128-B pieces, one per 8 columns of its 8 rows.
+__device__ __forceinline__ void stage_half_frag(const bf16_t* __restrict__ src, int K, int r0, int nrows, int k0,
+                                                char* dst, int wave, int lane) {
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int piece = i * 8 + wave;
+    const int rl = piece * 8 + (lane >> 3);
+    const int cs = (lane & 7) ^ swz_chunk(rl);
+    int r = r0 + rl;
+    r = r < nrows ? r : nrows - 1;
+    glds16(src + (size_t)(r >> 4) * 16 * K + ((size_t)(k0 >> 5) + (cs >> 2)) * 512 + (cs & 3) * 128 + (r & 15) * 8,
+           dst + piece * 1024);
+  }
+}
+
+// Epilogue operands of a 256^2 tile by LDS-DMA, into EPI_LDS bytes past the
+// operand buffers, issued before the first staging DMA (so the prologue's
+// counted wait retires them and no register carries them through the main
+// loop): wave 0 the bias of the tile's 256 columns, wave 1 the per-column
+// scale (fp8 channel scales / folded-norm column sums), waves 2-3 the row
+// statistics (float2) of its 256 rows, wave 4 the per-row fp8 activation
+// scales.  After the main loop every output group then reads them from LDS:
+// loaded there per group they cost one dependent memory round trip each (16
+// per tile), a load under a branch being waited for at the merge.  Addresses
+// past the matrix clamp to its last 16 B (host/kernel: N % 4 == 0, M even,
+// 16-B aligned vectors; those columns / rows are never stored).
+// Anatomy probe of the 256^2 kernels (bench/probes/gemm_anatomy.py; 0 in every
+// product launch): bit 1 skips the epilogue's stores (the accumulators stay
+// live through one sentinel compare), bit 2 skips the main loop (prologue DMAs,
+// their wait and the epilogue only), bit 8 runs the whole epilogue but
+// predicates its plain-path stores off, bit 4 reads the residual by per-lane
+// gathers instead of the LDS-DMA tile -- what a tile's fixed cost is made of
+// (profiles/r6_gemm_anatomy.jsonl: ~8-10 us of stores per tile at M = 32768;
+// row-staged, non-temporal or start-staggered stores were measured and
+// reverted, docs/ARCHITECTURE.md "Tried and reverted").
+static __device__ int g_gemm_anatomy = 0;
+
+constexpr int EPI_LDS = 5 * 1024;
+constexpr int EPI_B = 0, EPI_C = 1024, EPI_RS = 2048, EPI_SA = 4096;  // byte offsets
+
+__device__ __forceinline__ void epi_operands_dma(const float* bias, const float* col, const float2* rowstat,
+                                                 const float* sa, int n0, int N, int m0, int M, char* dst, int wave,
+                                                 int lane) {
+  if (wave == 0 && bias != nullptr) glds16(bias + min(n0 + 4 * lane, N - 4), dst + EPI_B);
+  if (wave == 1 && col != nullptr) glds16(col + min(n0 + 4 * lane, N - 4), dst + EPI_C);
+  if ((wave == 2 || wave == 3) && rowstat != nullptr)
+    glds16(rowstat + min(m0 + (wave - 2) * 128 + 2 * lane, M - 2), dst + EPI_RS + (wave - 2) * 1024);
+  if (wave == 4 && sa != nullptr) glds16(sa + min(m0 + 4 * lane, M - 4), dst + EPI_SA);
+}
+
+__device__ __forceinline__ void bg_barrier() {
+  __builtin_amdgcn_sched_barrier(0);
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_sched_barrier(0);
+}
+
+template <int MI, int NJ>
+__device__ __forceinline__ void bg_mfma(f32x4 (&acc)[MI][NJ], const bf16x8 (&a)[MI][2], const bf16x8 (&b)[NJ][2]) {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_setprio(1);
+#pragma unroll
+  for (int s = 0; s < 2; ++s)
+#pragma unroll
+    for (int i = 0; i < MI; ++i)
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[j][s], a[i][s], acc[i][j], 0, 0, 0);
+  __builtin_amdgcn_s_setprio(0);
+}
+
+template <int N>
+__device__ __forceinline__ void bg_read(bf16x8 (&f)[N][2], const char* half, int row0, int lane) {
+#pragma unroll
+  for (int i = 0; i < N; ++i)
+#pragma unroll
+    for (int s = 0; s < 2; ++s) f[i][s] = lds_frag(half, row0 + i * 16 + (lane & 15), s * 4 + (lane >> 4));
+}
+
+// QKV scatter epilogue (prefill c_attn, no RoPE): output column c of row
+// m = b*T + t lands head-major — q -> q[b][h][t][:], k / v -> the KV caches at
+// position pos[b] + t — instead of in a (M, (H+2Hkv) hd) qkv row, so the flash
+// prefill reads contiguous K/V from the cache and no longer copies them there
+// (bench/flash_copy_probe.py: 21 us of a 116 us GPT-2 attention layer).
+struct QkvScatter {
+  bf16_t* q;
+  bf16_t* k;
+  bf16_t* v;
+  const int* pos;
+  int T, H, Hkv, hd_shift, S;  // head dim = 1 << hd_shift
+  float invT;                  // 1 / T (row -> sequence without an integer division)
+  int c_off = 0;               // first qkv column of this launch (the tail-split launch covers the last 256)
+};
+
+// 8 consecutive output columns c..c+7 (one head) of row m -> destination.  The
+// store count is 32 per lane and tile, so the index math avoids integer
+// division: b = m / T from the fp32 reciprocal with a one-step correction
+// (exact for m < 2^24), head / dim by shifts (hd a power of two).
+__device__ __forceinline__ int qkv_batch(const QkvScatter& sc, int m) {
+  int b = (int)(((float)m + 0.5f) * sc.invT);
+  b -= b * sc.T > m ? 1 : 0;
+  b += (b + 1) * sc.T <= m ? 1 : 0;
+  return b;
+}
+// the cache position of row m (pos[b] + t), loaded for a lane's 8 rows before
+// the epilogue's first store: loaded per 32-column pair it waited, through the
+// in-order vmcnt, for every store issued before it
+__device__ __forceinline__ int qkv_row_pos(const QkvScatter& sc, int m) {
+  const int b = qkv_batch(sc, m);
+  return sc.pos[b] + (m - b * sc.T);
+}
+__device__ __forceinline__ bf16_t* qkv_dest(const QkvScatter& sc, int m, int c, int p) {
+  const int b = qkv_batch(sc, m);
+  const int t = m - b * sc.T;
+  const int hs = sc.hd_shift, hmask = (1 << hs) - 1;
+  const int qw = sc.H << hs, kw = sc.Hkv << hs;
+  if (c < qw) return sc.q + ((((size_t)b * sc.H + (c >> hs)) * sc.T + t) << hs) + (c & hmask);
+  if (p >= sc.S) return nullptr;  // past the cache capacity: dropped, as in qkv_split
+  const bool isk = c < qw + kw;
+  const int cc = isk ? c - qw : c - qw - kw;
+  return (isk ? sc.k : sc.v) + ((((size_t)b * sc.Hkv + (cc >> hs)) * sc.S + p) << hs) + (cc & hmask);
+}
+
+// One widened 16-B store per lane (as epi_pair_bf16) of a whole 32-column pair
+// to its head-major / cache destination (bias added first, no activation).
+__device__ __forceinline__ void epi_pair_scatter(f32x4 a0, f32x4 a1, int m, int nb, int M,
+                                                 const float* __restrict__ bias, int lane, const QkvScatter& sc,
+                                                 int p) {
+  const int q = lane >> 4;
+  if (bias != nullptr) {
+    a0 += *reinterpret_cast<const f32x4*>(bias + nb + q * 4);
+    a1 += *reinterpret_cast<const f32x4*>(bias + nb + 16 + q * 4);
+  }
+  const uint32_t x0 = pack2bf(a0[0], a0[1]), x1 = pack2bf(a0[2], a0[3]);
+  const uint32_t y0 = pack2bf(a1[0], a1[1]), y1 = pack2bf(a1[2], a1[3]);
+  const auto s0 = __builtin_amdgcn_permlane16_swap(x0, y0, false, false);
+  const auto s1 = __builtin_amdgcn_permlane16_swap(x1, y1, false, false);
+  if (m < M) {
+    bf16_t* d = qkv_dest(sc, m, nb + ((q & 1) << 4) + ((q >> 1) << 3), p);
+    if (d != nullptr) *reinterpret_cast<uint4*>(d) = make_uint4(s0[0], s1[0], s0[1], s1[1]);
+  }
+}
+
+// NQ = 2: 256x256 tiles (4 phases per K-tile, below).  NQ = 1: 256x128 tiles
+// for N where the 256^2 grid leaves its last round of 256 CUs half empty
+// (GPT-2's 768-wide projections at M = 32768: 384 tiles = 1.5 rounds; as
+// 256x128 768 tiles = 3 full rounds of half-size tiles).
+// Same waves (2 M x 4 N) and LDS images; a wave owns 2 x 1 quadrants of 64x32
+// and a K-tile is two phases:
+//     ph1: read B0 (4), A0 (8)  | stage A0, B0 [t+1] -> buf^1 | vmcnt(4) | C00
+//     ph2: read A1 (8)          | stage A1 [t+1]     -> buf^1 | vmcnt(2) | C10
+// (one tile ahead: every restage lands 2 phases after the last read of its
+// half-tile, every read 1 phase after the wait + barrier that retired it).
+// GRP: the rows are sorted by expert (grouped_tile.h): a tile belongs to one
+// expert's range of places, A rows are gathered, W holds every expert's weight
+// in fragment order (ops/gemm.py shuffle_weight) and C rows are places.
+template <int ACT, bool OUT_F32, bool SCATTER = false, int NQ = 2, bool GRP = false>
+__global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
+    const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__ W, int ldw, void* __restrict__ Cv,
+    int ldc, const float* __restrict__ bias, const bf16_t* __restrict__ R, int ldr, int M, int N, int K,
+    int res_pre, const float2* __restrict__ rowstat, const float* __restrict__ colsum, QkvScatter scat = {},
+    GroupedRows grp = {}) {
+  static_assert(NQ == 1 || NQ == 2, "256x256 or 256x128 tiles");
+  constexpr int TN = 128 * NQ;
+  __shared__ __attribute__((aligned(1024))) char smem[8 * BG_HALF + EPI_LDS];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int ntn = (N + TN - 1) / TN;
+  int tm, tn;
+  int ga[4] = {};  // GRP: the A rows this thread stages (2 of either half-tile)
+  if constexpr (GRP) {
+    const GroupTile t = group_tile(grp, BG_M, ntn, blockIdx.x, lane);
+    if (t.expert < 0) return;
+    tm = t.tm, tn = t.tn, M = t.rows;
+    W += (size_t)t.expert * N * K;
+    Cv = reinterpret_cast<bf16_t*>(Cv) + (size_t)t.first * ldc;
+#pragma unroll
+    for (int x = 0; x < 4; ++x)
+      ga[x] = grp.row(t.first + min(tm * BG_M + (x >> 1) * 128 + ((x & 1) * 8 + wave) * 8 + (lane >> 3), M - 1));
+  } else {
+    const int ntm = (M + BG_M - 1) / BG_M;
+    tile_coords(xcd_remap(blockIdx.x, ntm * ntn), ntm, ntn, tm, tn);
+  }
+  const int m0 = tm * BG_M, n0 = tn * TN;
+  const int wr = wave >> 2, wc = wave & 3;
+  const int nk = K / BG_K;
+  const int gan = GRP ? 0 : g_gemm_anatomy;
+  // epilogue operands in LDS (epi_operands_dma); uniform.  SCATTER: the bias
+  // is indexed by the global column (the tail launch's c_off).
+  char* epi = smem + 8 * BG_HALF;
+  const int boff = SCATTER ? scat.c_off : 0;
+  const bool epv = (N & 3) == 0 && (M & 1) == 0 && M >= 2 && N >= 4 &&
+                   ((reinterpret_cast<uintptr_t>(bias) | reinterpret_cast<uintptr_t>(colsum) |
+                     reinterpret_cast<uintptr_t>(rowstat)) & 15) == 0;
+  if (epv)
+    epi_operands_dma(bias != nullptr ? bias + boff : nullptr, colsum, rowstat, nullptr, n0, N, m0, M, epi, wave, lane);
+
+  f32x4 acc[2][NQ][4][2];
+#pragma unroll
+  for (int a = 0; a < 2; ++a)
+#pragma unroll
+    for (int b = 0; b < NQ; ++b)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[a][b][i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+  // half-tile h of buffer u: A0=0, A1=1, B0=2, B1=3
+  auto half = [&](int u, int h) { return smem + (u * 4 + h) * BG_HALF; };
+  auto stA = [&](int u, int h, int t) {
+    t = t < nk ? t : nk - 1;
+    if constexpr (GRP) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int piece = i * 8 + wave;
+        glds16(A + (size_t)(h == 0 ? ga[i] : ga[2 + i]) * lda + t * BG_K + ((lane & 7) ^ swz_chunk(piece * 8 + (lane >> 3))) * 8,
+               half(u, h) + piece * 1024);
+      }
+    } else {
+      stage_half(A, lda, m0 + h * 128, M, t * BG_K, half(u, h), wave, lane);
+    }
+  };
+  auto stB = [&](int u, int h, int t) {
+    t = t < nk ? t : nk - 1;
+    if constexpr (GRP) stage_half_frag(W, K, n0 + h * 128, N, t * BG_K, half(u, 2 + h), wave, lane);
+    else stage_half(W, ldw, n0 + h * 128, N, t * BG_K, half(u, 2 + h), wave, lane);
+  };
+
+  bf16x8 af[4][2], b0[2][2], b1[2][2];
+  const int arow = wr * 64, brow = wc * 32;
+  if constexpr (NQ == 1) {
+    // prologue: tile 0 complete
+    stA(0, 0, 0);
+    stB(0, 0, 0);
+    stA(0, 1, 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    bg_barrier();
+    if (wr == 1) bg_barrier();
+    auto ktile1 = [&](const int t, auto ucst) {
+      constexpr int u = decltype(ucst)::value;
+      // ph1
+      bg_read<2>(b0, half(u, 2), brow, lane);
+      __builtin_amdgcn_sched_barrier(0);
+      bg_read<4>(af, half(u, 0), arow, lane);
+      stA(u ^ 1, 0, t + 1);
+      stB(u ^ 1, 0, t + 1);
+      asm volatile("s_waitcnt vmcnt(4)" ::: "memory");  // A1 of tile t landed
+      bg_barrier();
+      bg_mfma<4, 2>(acc[0][0], af, b0);
+      bg_barrier();
+      // ph2
+      bg_read<4>(af, half(u, 1), arow, lane);
+      stA(u ^ 1, 1, t + 1);
+      asm volatile("s_waitcnt vmcnt(2)" ::: "memory");  // A0 / B0 of tile t+1 landed
+      bg_barrier();
+      bg_mfma<4, 2>(acc[1][0], af, b0);
+      bg_barrier();
+    };
+    int t = 0;
+    for (; t + 1 < nk; t += 2) {
+      ktile1(t, std::integral_constant<int, 0>{});
+      ktile1(t + 1, std::integral_constant<int, 1>{});
+    }
+    if (t < nk) ktile1(t, std::integral_constant<int, 0>{});
+  } else {
+  // prologue: tile 0 complete, A0/B1 of tile 1 in flight
+  stA(0, 0, 0);
+  stB(0, 1, 0);
+  stA(0, 1, 0);
+  stB(0, 0, 0);
+  stA(1, 0, 1);
+  stB(1, 1, 1);
+  asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+  bg_barrier();
+  if (wr == 1) bg_barrier();
+
+  // One K-tile; the loop runs two per iteration so the buffer index u is a
+  // compile-time constant and every LDS address an immediate offset.
+  auto ktile = [&](const int t, auto ucst) {
+    constexpr int u = decltype(ucst)::value;
+    // ph1
+    bg_read<2>(b0, half(u, 2), brow, lane);
+    __builtin_amdgcn_sched_barrier(0);
+    bg_read<4>(af, half(u, 0), arow, lane);
+    stA(u ^ 1, 1, t + 1);
+    bg_barrier();
+    bg_mfma<4, 2>(acc[0][0], af, b0);
+    bg_barrier();
+    // ph2
+    bg_read<2>(b1, half(u, 3), brow, lane);
+    stB(u ^ 1, 0, t + 1);
+    bg_barrier();
+    bg_mfma<4, 2>(acc[0][1], af, b1);
+    bg_barrier();
+    // ph3
+    bg_read<4>(af, half(u, 1), arow, lane);
+    stA(u, 0, t + 2);
+    bg_barrier();
+    bg_mfma<4, 2>(acc[1][1], af, b1);
+    bg_barrier();
+    // ph4
+    bg_read<2>(b0, half(u, 2), brow, lane);
+    stB(u, 1, t + 2);
+    asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+    bg_barrier();
+    bg_mfma<4, 2>(acc[1][0], af, b0);
+    bg_barrier();
+  };
+  int t = (gan & 2) ? nk : 0;
+  for (; t + 1 < nk; t += 2) {
+    ktile(t, std::integral_constant<int, 0>{});
+    ktile(t + 1, std::integral_constant<int, 1>{});
+  }
+  if (t < nk) ktile(t, std::integral_constant<int, 0>{});
+  }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  if (wr == 0) bg_barrier();
+  if (gan & 1) {  // anatomy probe: no stores
+    if (acc[0][0][0][0][0] == 1.2345e-30f) reinterpret_cast<bf16_t*>(Cv)[0] = 0;
+    return;
+  }
+
+  // Epilogue (transposed accumulators):
+  //   row m = m0 + mq*128 + wr*64 + i*16 + (lane&15), cols n..n+3 with
+  //   n = n0 + nq*128 + wc*32 + j*16 + (lane>>4)*4.
+  if (rowstat != nullptr) {  // folded pre-norm (prefill QKV / up projections)
+    // 8 row statistics and 4 column-sum vectors per lane (from the LDS copy)
+    float2 rs[2][4];
+    f32x4 cs[NQ][2];
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int rl = mq * 128 + arow + i * 16 + (lane & 15);
+        rs[mq][i] = epv ? reinterpret_cast<const float2*>(epi + EPI_RS)[rl] : rowstat[min(m0 + rl, M - 1)];
+      }
+#pragma unroll
+    for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const int n = n0 + nq * 128 + wc * 32 + j * 16 + (lane >> 4) * 4;
+        cs[nq][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (colsum != nullptr) {
+          if (epv) {
+            cs[nq][j] = *reinterpret_cast<const f32x4*>(epi + EPI_C + 4 * (n - n0));
+          } else if (n + 3 < N) {
+            cs[nq][j] = *reinterpret_cast<const f32x4*>(colsum + n);
+          } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) cs[nq][j][r] = n + r < N ? colsum[n + r] : 0.f;
+          }
+        }
+      }
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int j = 0; j < 2; ++j)
+            acc[mq][nq][i][j] = acc[mq][nq][i][j] * rs[mq][i].x + rs[mq][i].y * cs[nq][j];
+  }
+  // the bias from the LDS copy, added here: the output calls get none to load
+  const bool badd = epv && bias != nullptr && !is_glu(ACT);  // uniform
+  if (badd) {
+#pragma unroll
+    for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const f32x4 b4 = *reinterpret_cast<const f32x4*>(epi + EPI_B + 4 * (nq * 128 + wc * 32 + j * 16 + (lane >> 4) * 4));
+#pragma unroll
+        for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) acc[mq][nq][i][j] += b4;
+      }
+  }
+  const float* bias_e = badd ? nullptr : bias;
+  // SCATTER: the cache positions of the lane's 8 rows, loaded before any store (qkv_row_pos)
+  int spos[2][4] = {};
+  if constexpr (SCATTER) {
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) spos[mq][i] = qkv_row_pos(scat, min(m0 + mq * 128 + arow + i * 16 + (lane & 15), M - 1));
+  }
+  const bool vec = epi_vec_ok(Cv, ldc, bias, R, ldr);
+  const bool pair = vec && epi_pair_ok(Cv, ldc, bias, R, ldr);
+  // Residual epilogue: every residual load of the tile (32 x 8 B per lane, into
+  // the fragment registers the main loop no longer needs) is issued before the
+  // first output is computed, so the tile pays one memory round trip for R
+  // instead of one per output row group (-20..-25 % GEMM throughput otherwise,
+  // profiles/archive/r2_gemm_epilogue_cost.jsonl).
+  if (res_pre && !OUT_F32 && !is_glu(ACT) && pair && R != nullptr && n0 + TN - 1 < N && (gan & 4) == 0 &&
+      (ldr & 7) == 0 && (reinterpret_cast<uintptr_t>(R) & 15) == 0) {
+    // the residual tile by LDS-DMA into the dead operand buffers (res_tile_dma;
+    // anatomy bit 4 = the per-lane gathers below)
+    __syncthreads();  // every wave past its last operand read and DMA (vmcnt(0) above)
+    res_tile_dma<TN>(R, ldr, m0, n0, M, smem, wave, lane);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int rl = mq * 128 + arow + i * 16 + (lane & 15), cl = nq * 128 + wc * 32 + (lane >> 4) * 4;
+          epi_pair_bf16<ACT, true>(acc[mq][nq][i][0], acc[mq][nq][i][1], m0 + rl, n0 + nq * 128 + wc * 32, M,
+                                   reinterpret_cast<bf16_t*>(Cv), ldc, bias_e, R, ldr, lane,
+                                   res_tile_read<TN>(smem, rl, cl), res_tile_read<TN>(smem, rl, cl + 16));
+        }
+    return;
+  }
+  if (res_pre && !OUT_F32 && !is_glu(ACT) && pair && R != nullptr && n0 + TN - 1 < N) {
+    bf16x4 rr[2][NQ][4][2];
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          epi_pair_res_load(m0 + mq * 128 + arow + i * 16 + (lane & 15), n0 + nq * 128 + wc * 32, M, R, ldr, lane,
+                            rr[mq][nq][i][0], rr[mq][nq][i][1]);
+#pragma unroll
+    for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+      for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          epi_pair_bf16<ACT, true>(acc[mq][nq][i][0], acc[mq][nq][i][1], m0 + mq * 128 + arow + i * 16 + (lane & 15),
+                                   n0 + nq * 128 + wc * 32, M, reinterpret_cast<bf16_t*>(Cv), ldc, bias_e, R, ldr, lane,
+                                   rr[mq][nq][i][0], rr[mq][nq][i][1]);
+    return;
+  }
+#pragma unroll
+  for (int mq = 0; mq < 2; ++mq)
+#pragma unroll
+    for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int m = m0 + mq * 128 + arow + i * 16 + (lane & 15);
+        const int nb = n0 + nq * 128 + wc * 32;
+        if (is_glu(ACT)) {
+          epi_glu_pair<ACT, OUT_F32>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
+        } else if (SCATTER) {
+          // widened 16-B stores as in epi_pair_bf16, to the head-major / cache
+          // destination of the lane's 8 columns (host: ACT_NONE, bf16 out, no
+          // residual, N % 32 == 0, hd % 8 == 0 -> a 32-column pair is whole or
+          // past N, wave-uniformly)
+          if (nb < N)
+            epi_pair_scatter(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb + scat.c_off, M, bias_e, lane, scat,
+                             spos[mq][i]);
+        } else if (!OUT_F32 && pair && nb + 31 < N) {
+          epi_pair_bf16<ACT>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb, (gan & 8) ? 0 : M, reinterpret_cast<bf16_t*>(Cv), ldc,
+                             bias_e, R, ldr, lane);
+        } else {
+#pragma unroll
+          for (int j = 0; j < 2; ++j)
+            epi_t4<ACT, OUT_F32>(acc[mq][nq][i][j], m, nb + j * 16 + (lane >> 4) * 4, M, N, Cv, ldc, bias_e, R,
+                                 ldr, vec);
+        }
+      }
+}
+
+}  // namespace dnn

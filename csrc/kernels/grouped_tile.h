@@ -1,0 +1,65 @@
+// Tiles of rows that are sorted by expert: expert e owns the places
+// offs[e] .. offs[e + 1] - 1; a tile never crosses a border.
+#pragma once
+#include "common.h"
+
+namespace dnn {
+
+constexpr int EXPERTS_MAX = 256;
+
+struct GroupedRows {
+  const int* offs;   // [E + 1]
+  const int* order;  // source of a place: order[place] / div (nullptr: the place itself)
+  int* counts;       // zeroed by the first workgroup (nullptr: not)
+  int E, div, arows;
+  __device__ __forceinline__ int row(int place) const {
+    const int r = order != nullptr ? order[place] / div : place;
+    return min(max(r, 0), arows - 1);
+  }
+};
+
+struct GroupTile {
+  int expert, first, rows, tm, tn;  // first place and rows of the expert; expert < 0: past the last tile
+};
+
+// Tile `bid` of tiles of `bm` rows x ntn columns (m-tile major, neighbours on
+// one XCD).  Every lane of every wave calls it.
+__device__ __forceinline__ GroupTile group_tile(const GroupedRows& g, int bm, int ntn, int bid, int lane) {
+  if (g.counts != nullptr && bid == 0)
+    for (int e = threadIdx.x; e < g.E; e += blockDim.x) g.counts[e] = 0;
+  int first[4], rows[4], nt[4], sum = 0;  // lane l: experts 4 l .. 4 l + 3
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int e = min(lane * 4 + i, g.E);
+    first[i] = g.offs[e];
+    rows[i] = g.offs[min(e + 1, g.E)] - first[i];
+    nt[i] = (rows[i] + bm - 1) / bm;
+    sum += nt[i];
+  }
+  int incl = sum;
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const int u = __shfl_up(incl, o, 64);
+    if (lane >= o) incl += u;
+  }
+  const int total = __shfl(incl, 63, 64) * ntn;
+  GroupTile t{-1, 0, 0, 0, 0};
+  if (bid >= total) return t;
+  const int logical = xcd_remap(bid, total), mt = logical / ntn;
+  t.tn = logical - mt * ntn;
+  const int src = __ffsll((unsigned long long)__ballot(incl > mt)) - 1;  // the lane whose experts hold the tile
+  int base = incl - sum, e = lane * 4, f = first[0], r = rows[0];
+#pragma unroll
+  for (int i = 0; i < 3; ++i)
+    if (mt >= base + nt[i] && e == lane * 4 + i) base += nt[i], e = lane * 4 + i + 1, f = first[i + 1], r = rows[i + 1];
+  t.expert = __builtin_amdgcn_readfirstlane(__shfl(e, src, 64));
+  t.first = __builtin_amdgcn_readfirstlane(__shfl(f, src, 64));
+  t.rows = __builtin_amdgcn_readfirstlane(__shfl(r, src, 64));
+  t.tm = mt - __builtin_amdgcn_readfirstlane(__shfl(base, src, 64));
+  return t;
+}
+
+// Upper bound of the row tiles of `rows` places over E experts.
+inline int group_tiles_max(int rows, int bm, int E) { return rows / bm + (rows < E ? rows : E); }
+
+}  // namespace dnn

@@ -1,0 +1,93 @@
+// C ABI of the recurrent mixers (recurrence.hip) and the mixture of experts
+// (moe.hip).  Every function enqueues on `st`; 0 = success, negative = rejected shape.
+#pragma once
+#include <hip/hip_runtime.h>
+
+// Short causal convolution per channel over the rows of a step, with silu, and
+// the step sizes of a recurrence beside it.  `ring` keeps the last inputs of
+// every sequence: entry position % taps of [slot][taps][C].
+struct ConvArgs {
+  const void* in;      // rows, channels at column 0, stride ldi
+  const float* w;      // [taps][C], the current token's tap last
+  const float* b;      // [C]
+  void* ring;
+  void* out;           // rows [C], stride ldo
+  const int* start;    // per row: first row of its sequence's portion in this step
+  const int* slots;
+  const int* pos;
+  const float* dt_bias;  // [H]: dt = softplus(in[dt_col + h] + dt_bias[h])
+  const float* a_log;    // [H]: la = -exp(a_log[h]) * dt
+  float* dt;             // [M][H] (nullptr: no step sizes)
+  float* la;             // [M][H]
+  int ldi, ldo, M, C, taps, dt_col, H, nslots;
+};
+
+// Linear recurrence per head with a matrix state (fp32, [slot][H][VP][NP]):
+//   S <- exp(la) S + dt * k v^T,   y = S^T q + D v
+// la, dt per row and head, or la per head and dt one constant (la_h, dt_c).
+// Head h reads q / k of group h / qdiv.  A portion that begins at position 0
+// starts from a zero state.
+struct ScanArgs {
+  const void* rows;    // q, k, v columns of one row, stride ld
+  const float* dt;     // [M][H] or nullptr
+  const float* la;     // [M][H] or nullptr
+  const float* la_h;   // [H] (la == nullptr)
+  const float* D;      // [H] or nullptr
+  float* state;
+  void* y;             // rows [H * vdim], stride ldy
+  const int4* ent;     // sequences of the step: {first row, tokens, slot, -}
+  const int* pos;
+  int ld, ldy, qcol, kcol, vcol, qdiv, M, H, NP, VP, vdim, nent, nslots;
+  float dt_c;
+};
+
+// Gate and RMS norm of equal parts of a row:
+//   gate_first: out = norm(y * silu(z)) * w,   else: out = norm(y) * silu(z) [* w]
+struct GatedNormArgs {
+  const void* y;
+  const void* z;
+  const float* w;      // [n] or nullptr
+  void* out;
+  int ldy, ldz, ldo, M, n, groups, gate_first;
+  float eps;
+};
+
+// Router: softmax over E logits, the best `keep` of `groups` groups of
+// neighbours (by their largest score), the `top` best experts in them, weights
+// normalised over the chosen.  Sorted placement of every (row, choice):
+//   order[place] = row * top + choice,  place[row * top + choice],  offs[E + 1]
+struct RouteArgs {
+  const float* logits;
+  int* idx;       // [M * top] chosen expert
+  float* w;       // [M * top]
+  int* rank;      // [M * top] (scratch)
+  int* counts;    // [E], zero before and after
+  int* order;
+  int* place;
+  int* offs;
+  int ldl, M, E, groups, keep, top;
+};
+
+// Products of rows sorted by expert with that expert's weight:
+//   C[p] = act(A[row(p)] W_e^T),  e the expert whose range holds place p.
+struct GroupedArgs {
+  const void* A;       // row(p) = order[p] / div (order == nullptr: p)
+  const void* W;       // [E][N][K]
+  const void* Wsh;     // the same in fragment order (bf16, few rows per expert), or nullptr
+  void* C;             // [rows][N, or N / 2 for gated activations], stride ldc
+  const int* offs;     // [E + 1]
+  const int* order;
+  int* counts;         // zeroed on the way (nullptr: not)
+  int lda, ldc, rows, arows, div, N, K, E, act;
+};
+
+extern "C" {
+int dnn_conv(const ConvArgs* a, int f32, hipStream_t st);
+int dnn_conv_state(const ConvArgs* a, const int4* ent, int nent, int f32, hipStream_t st);
+int dnn_scan_steps(const ScanArgs* a, int f32, hipStream_t st);   // token by token
+int dnn_scan_chunks(const ScanArgs* a, hipStream_t st);           // bf16, 64-token chunks on the MFMA
+int dnn_gated_norm(const GatedNormArgs* a, int f32, hipStream_t st);
+int dnn_route(const RouteArgs* a, hipStream_t st);
+int dnn_grouped_gemm(const GroupedArgs* a, hipStream_t st);       // bf16
+int dnn_grouped_gemm_f32(const GroupedArgs* a, hipStream_t st);
+}

@@ -8,8 +8,11 @@
 // Only pages that hold a visible key are read.  The query heads of a KV head
 // (H / G, any number) are packed with the queries into the 32 columns of the
 // MFMA: column r of a sequence's chunk is (token r / R, head r % R), R = H / G.
-// An optional per-head output gate, sigmoid of a column of the projection row,
-// multiplies the head's output.
+// An optional output gate, sigmoid of a column of the projection row (one per
+// head, or one per head and value), multiplies the head's output.  Optional
+// score terms: a factor per cached key (a key norm that the cache does not
+// hold) and a per-head slope times the distance, taken off.  Values may be the
+// keys themselves (one pool; qk_norm.hip writes it).
 //
 //   paged_write    new k / v rows -> pages
 //   paged_prefill  chunks of >= 2 tokens; a workgroup takes 128 packed rows
@@ -60,7 +63,7 @@ __device__ __forceinline__ Units pa_units(int qlo, int qhi, int window, int keep
 template <typename T>
 __global__ __launch_bounds__(256) void paged_write_kernel(PagedAttnArgs a) {
   constexpr int E = 16 / sizeof(T);
-  const int ck = a.G * a.DK / E, cv = a.G * a.DV / E;
+  const int ck = a.G * a.DK / E, cv = a.shared ? 0 : a.G * a.DV / E;
   const long i = blockIdx.x * 256L + threadIdx.x;
   if (i >= (long)a.M * (ck + cv)) return;
   const int m = (int)(i / (ck + cv));
@@ -144,8 +147,26 @@ __device__ __forceinline__ void pa_pv(const char* vbuf, const f32x16& p, f32x16 
   }
 }
 
+// Terms of the score beyond the dot product, for 4 consecutive keys key0.. of
+// a page: s <- log2(e) * (s * kscale * scale - slope * (i - j)).
+__device__ __forceinline__ bool pa_has_terms(const PagedAttnArgs& a) { return a.kscale != nullptr || a.slopes != nullptr; }
+__device__ __forceinline__ f32x4 pa_kscale4(const PagedAttnArgs& a, int page, int key0) {
+  if (a.kscale == nullptr) return f32x4{1.f, 1.f, 1.f, 1.f};
+  return *reinterpret_cast<const f32x4*>(a.kscale + (size_t)page * PG + key0);
+}
+__device__ __forceinline__ float pa_slope(const PagedAttnArgs& a, int head) {
+  return a.slopes != nullptr ? a.slopes[head] * LOG2E : 0.f;
+}
+
+__device__ __forceinline__ float pa_sigmoid(const PagedAttnArgs& a, int row, int col) {
+  const float z = bf2f(reinterpret_cast<const bf16_t*>(a.qkv)[(size_t)row * a.ldq + a.gate + col]);
+  return 1.0f / (1.0f + __expf(-z));
+}
+__device__ __forceinline__ float pa_gate_el(const PagedAttnArgs& a, int row, int col) {
+  return a.gate >= 0 && a.gate_el ? pa_sigmoid(a, row, col) : 1.f;
+}
 __device__ __forceinline__ float pa_gate(const PagedAttnArgs& a, int row, int head) {
-  if (a.gate < 0) return 1.f;
+  if (a.gate < 0 || a.gate_el) return 1.f;
   const float z = bf2f(reinterpret_cast<const bf16_t*>(a.qkv)[(size_t)row * a.ldq + a.gate + head]);
   return 1.0f / (1.0f + __expf(-z));
 }
@@ -183,7 +204,9 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_prefill_k
 #pragma unroll
   for (int i = 0; i < NDT; ++i) o[i] = f32x16{};
   float m_i = -INFINITY, l_i = 0.f;
-  const float sc = a.scale * LOG2E;
+  const bool terms = pa_has_terms(a);
+  const float sc0 = a.scale * LOG2E, sc = terms ? 1.f : sc0;
+  const float slope = pa_slope(a, head);
 
   i32x4 pk[NIK], pv[NIV];
   auto fetch = [&](int i) __attribute__((always_inline)) {
@@ -224,6 +247,19 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_prefill_k
         s[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[k], s[kt], 0, 0, 0);
       }
     }
+    if (terms) {
+      const int page = max(pa_page(a, slot, u.at(i)), 0);
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const int k4 = kt * 32 + 8 * q + 4 * h;
+          const f32x4 f = pa_kscale4(a, page, k4) * sc0;
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            s[kt][4 * q + j] = fmaf(s[kt][4 * q + j], f[j], -slope * (float)(q_abs - (kb0 + k4 + j)));
+        }
+    }
     // every key visible to every query of the wave: no mask
     if (kb0 + PG - 1 > wq_min || !(wq_max - kb0 < a.window || kb0 + PG <= a.keep)) {
 #pragma unroll
@@ -246,9 +282,18 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_prefill_k
 #pragma unroll
   for (int d = 0; d < NDT; ++d)
 #pragma unroll
-    for (int q = 0; q < 4; ++q)
-      *reinterpret_cast<uint2*>(op + d * 32 + 8 * q + 4 * h) =
-          make_uint2(pack2bf(o[d][4 * q] * f, o[d][4 * q + 1] * f), pack2bf(o[d][4 * q + 2] * f, o[d][4 * q + 3] * f));
+    for (int q = 0; q < 4; ++q) {
+      float v[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = o[d][4 * q + j] * f;
+      if (a.gate >= 0 && a.gate_el) {
+        const bf16x4 z = *reinterpret_cast<const bf16x4*>(reinterpret_cast<const bf16_t*>(a.qkv) +
+                                                          (size_t)(tok0 + tk) * a.ldq + a.gate + head * DV + d * 32 + 8 * q + 4 * h);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] *= 1.0f / (1.0f + __expf(-bf2f_s(z[j])));
+      }
+      *reinterpret_cast<uint2*>(op + d * 32 + 8 * q + 4 * h) = make_uint2(pack2bf(v[0], v[1]), pack2bf(v[2], v[3]));
+    }
 }
 
 // ---------------------------------------------------------------- decode
@@ -285,7 +330,7 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
   // the token's own key and value: the wave that reads their unit (the last of
   // the list) stores them first
   const int lastw = (u.total - 1 - ub) & 3;
-  if (ue == u.total && wave == lastw) {
+  if (!a.written && ue == u.total && wave == lastw) {
     const int page = pa_page(a, slot, p / PG);
     if (page >= 0) {
       bf16_t* kd = reinterpret_cast<bf16_t*>(a.kp) + (((size_t)page * a.G + g) * PG + p % PG) * DK;
@@ -311,10 +356,13 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
 #pragma unroll
   for (int i = 0; i < NDT; ++i) o[i] = f32x16{};
   float m_i = -INFINITY, l_i = 0.f;
-  const float sc = a.scale * LOG2E;
+  const bool terms = pa_has_terms(a);
+  const float sc0 = a.scale * LOG2E, sc = terms ? 1.f : sc0;
+  const float slope = pa_slope(a, g * R + rt * 32 + min(r32, rr - 1));
 
   bf16x8 kf[NKS];
   i32x4 pv[NIV];
+  f32x4 ksc[4];
   auto load = [&](int i) __attribute__((always_inline)) {
     const int unit = u.at(i);
     const int page = max(pa_page(a, slot, unit / (PG / DU)), 0);
@@ -325,6 +373,10 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     for (int s = 0; s < NKS; ++s) kf[s] = *reinterpret_cast<const bf16x8*>(kb + s * 16);
 #pragma unroll
     for (int it = 0; it < NIV; ++it) pv[it] = *reinterpret_cast<const i32x4*>(vb + (it * 64 + lane) * 8);
+    if (terms) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) ksc[q] = pa_kscale4(a, page, (unit % (PG / DU)) * DU + 8 * q + 4 * h) * sc0;
+    }
   };
   int i = ub + wave;
   if (i < ue) load(i);
@@ -338,6 +390,13 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     for (int it = 0; it < NIV; ++it) {
       const int c = it * 64 + lane;
       *reinterpret_cast<i32x4*>(vs + (c / CV) * PaV<DV>::STRIDE + (c % CV) * 16) = pv[it];
+    }
+    if (terms) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          s[0][4 * q + j] = fmaf(s[0][4 * q + j], ksc[q][j], -slope * (float)(p - (kb0 + 8 * q + 4 * h + j)));
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     if (i + 4 < ue) load(i + 4);
@@ -385,7 +444,7 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     }
     if (ns == 1) {
       reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * DV + c] =
-          f2bf((l > 0.f ? v / l : 0.f) * pa_gate(a, row, head));
+          f2bf((l > 0.f ? v / l : 0.f) * pa_gate(a, row, head) * pa_gate_el(a, row, head * DV + c));
     } else {
       float* d = ws + (((size_t)e * a.H + head) * ns + blockIdx.z) * (DV + 2);
       if (c == 0) {
@@ -412,7 +471,7 @@ __global__ __launch_bounds__(64) void paged_combine_kernel(PagedAttnArgs a, cons
       l = fmaf(q[1], f, l);
       v = fmaf(q[2 + c], f, v);
     }
-    reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.DV + c] = f2bf((l > 0.f ? v / l : 0.f) * gate);
+    reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.DV + c] = f2bf((l > 0.f ? v / l : 0.f) * gate * pa_gate_el(a, row, head * a.DV + c));
   }
 }
 
@@ -444,6 +503,8 @@ __global__ __launch_bounds__(256) void paged_attn_f32_kernel(PagedAttnArgs a) {
         s = fmaf(k4[3], qs[wave][d + 3], s);
       }
       s *= a.scale;
+      if (a.kscale != nullptr) s *= a.kscale[(size_t)page * PG + lane];
+      if (a.slopes != nullptr) s -= a.slopes[head] * (float)(p - key);
     }
     const float m_new = fmaxf(m, wave_max(s));
     if (m_new == -INFINITY) continue;
@@ -466,11 +527,14 @@ __global__ __launch_bounds__(256) void paged_attn_f32_kernel(PagedAttnArgs a) {
     __builtin_amdgcn_wave_barrier();
   }
   float f = l > 0.f ? 1.f / l : 0.f;
-  if (a.gate >= 0) f *= 1.0f / (1.0f + expf(-rowp[a.gate + head]));
+  if (a.gate >= 0 && !a.gate_el) f *= 1.0f / (1.0f + expf(-rowp[a.gate + head]));
   float* op = reinterpret_cast<float*>(a.out) + (size_t)row * a.ldo + head * a.DV;
 #pragma unroll
-  for (int c = 0; c < 4; ++c)
-    if (lane + 64 * c < a.DV) op[lane + 64 * c] = o[c] * f;
+  for (int c = 0; c < 4; ++c) {
+    const int d = lane + 64 * c;
+    if (d >= a.DV) break;
+    op[d] = o[c] * f * (a.gate >= 0 && a.gate_el ? 1.0f / (1.0f + expf(-rowp[a.gate + head * a.DV + d])) : 1.f);
+  }
 }
 
 }  // namespace dnn
@@ -481,14 +545,15 @@ static bool pa_ok(const PagedAttnArgs& a, int elem) {
   auto dim = [](int d) { return d == 64 || d == 128 || d == 256; };
   const int vec = 16 / elem;
   return a.M > 0 && a.G > 0 && a.H > 0 && a.H % a.G == 0 && dim(a.DK) && dim(a.DV) && a.ldq % vec == 0 &&
-         a.ldo % 4 == 0 && a.ldo >= a.H * a.DV && a.ldq >= (a.H + a.G) * a.DK + a.G * a.DV &&
-         (a.gate < 0 || a.gate + a.H <= a.ldq) && a.window > 0 && a.keep >= 0 && a.ldt > 0 && a.npages > 0 &&
+         a.ldo % 4 == 0 && a.ldo >= a.H * a.DV && a.ldq >= (a.H + a.G) * a.DK + (a.shared ? 0 : a.G * a.DV) &&
+         (a.gate < 0 || a.gate + a.H * (a.gate_el ? a.DV : 1) <= a.ldq) && (!a.gate_el || a.gate % 4 == 0) &&
+         (!a.shared || (a.kp == a.vp && a.DK == a.DV && a.written)) && ((uintptr_t)a.kscale & 15) == 0 && a.window > 0 && a.keep >= 0 && a.ldt > 0 && a.npages > 0 &&
          a.table != nullptr && a.slots != nullptr && a.pos != nullptr;
 }
 
 extern "C" int dnn_paged_write(const PagedAttnArgs* a, int f32, hipStream_t st) {
   if (!pa_ok(*a, f32 ? 4 : 2)) return -1;
-  const long n = (long)a->M * a->G * (a->DK + a->DV) / (f32 ? 4 : 8);
+  const long n = (long)a->M * a->G * (a->DK + (a->shared ? 0 : a->DV)) / (f32 ? 4 : 8);
   const dim3 grid((unsigned)((n + 255) / 256));
   if (f32) hipLaunchKernelGGL(paged_write_kernel<float>, grid, dim3(256), 0, st, *a);
   else hipLaunchKernelGGL(paged_write_kernel<bf16_t>, grid, dim3(256), 0, st, *a);

@@ -1,0 +1,520 @@
+// Recurrent mixers over the rows of unequal sequences (gfx950): state-space
+// duality (Mamba-2) and retention are one recurrence with a matrix state,
+//   S_t = a_t S_{t-1} + dt_t k_t v_t^T,   y_t = S_t^T q_t + D v_t
+// whose decay is data-dependent in the one and a constant per head in the other.
+//
+//   conv        short causal convolution per channel + silu, and the step sizes
+//   conv_state  the last inputs of every sequence for its next step
+//   scan_chunks bf16, sequences of 2 tokens or more: 64-token chunks on the
+//               MFMA, the state in fp32 accumulators from chunk to chunk
+//   scan_steps  token by token in fp32: single decoded tokens, and the exact mode
+//   gated_norm  gate and RMS norm of equal parts of a row
+//
+// States are fp32 in pools by slot; a portion that begins at position 0 starts
+// from zero, so a slot needs no clearing between sequences.
+#include "common.h"
+#include "mixer_api.h"
+#include "vec16.h"
+
+namespace dnn {
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+constexpr float LOG2E = 1.4426950408889634f;
+
+// ---------------------------------------------------------------- convolution
+// grid M * ceil((C / E + H) / 256)
+template <typename T>
+__global__ __launch_bounds__(256) void conv_kernel(ConvArgs a) {
+  constexpr int E = Vec16<T>::N;
+  const int cv = a.C / E, gx = (cv + (a.dt != nullptr ? a.H : 0) + 255) / 256;
+  const int m = blockIdx.x / gx;
+  int i = (int)(blockIdx.x % gx) * 256 + threadIdx.x;
+  const T* row = reinterpret_cast<const T*>(a.in) + (size_t)m * a.ldi;
+  if (i >= cv) {
+    i -= cv;
+    if (a.dt == nullptr || i >= a.H) return;
+    const float z = to_f32(row[a.dt_col + i]) + a.dt_bias[i];
+    const float dt = z > 20.f ? z : log1pf(expf(z));
+    a.dt[(size_t)m * a.H + i] = dt;
+    a.la[(size_t)m * a.H + i] = fmaxf(-expf(a.a_log[i]) * dt, -88.f);  // exp(-88) is zero beside any state
+    return;
+  }
+  const int c = i * E, p = a.pos[m], s0 = a.start[m], slot = min(max(a.slots[m], 0), a.nslots - 1);
+  float acc[E], v[E];
+#pragma unroll
+  for (int j = 0; j < E; j += 4) {
+    const f32x4 b = *reinterpret_cast<const f32x4*>(a.b + c + j);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) acc[j + k] = b[k];
+  }
+  for (int t = 0; t < a.taps; ++t) {  // the input t positions back
+    if (p - t < 0) break;
+    const T* src = m - t >= s0 ? row - (size_t)t * a.ldi + c
+                               : reinterpret_cast<const T*>(a.ring) + ((size_t)slot * a.taps + (p - t) % a.taps) * a.C + c;
+    Vec16<T>::get(src, v);
+    const float* w = a.w + (size_t)(a.taps - 1 - t) * a.C + c;
+#pragma unroll
+    for (int j = 0; j < E; j += 4) {
+      const f32x4 w4 = *reinterpret_cast<const f32x4*>(w + j);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) acc[j + k] = fmaf(v[j + k], w4[k], acc[j + k]);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < E; ++j) acc[j] = silu(acc[j]);
+  Vec16<T>::put(reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + c, acc);
+}
+
+// grid (ceil(C / E / 256), sequences): the raw inputs of a portion's last tokens
+template <typename T>
+__global__ __launch_bounds__(256) void conv_state_kernel(ConvArgs a, const int4* __restrict__ ent) {
+  constexpr int E = Vec16<T>::N;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * E;
+  if (c >= a.C) return;
+  const int4 e = ent[blockIdx.y];
+  const int slot = min(max(e.z, 0), a.nslots - 1);
+  for (int t = max(e.y - a.taps, 0); t < e.y; ++t) {
+    const int m = e.x + t, p = a.pos[m];
+    *reinterpret_cast<uint4*>(reinterpret_cast<T*>(a.ring) + ((size_t)slot * a.taps + p % a.taps) * a.C + c) =
+        *reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(a.in) + (size_t)m * a.ldi + c);
+  }
+}
+
+// ---------------------------------------------------------------- token by token
+// grid (H, VP / 64, sequences); LPR lanes share a state row (one value column),
+// each holding float4s of it.
+template <typename T, int NP>
+__global__ __launch_bounds__(256) void scan_steps_kernel(ScanArgs a) {
+  constexpr int LPR = NP >= 64 ? 16 : NP / 4;  // lanes of a row
+  constexpr int NI = NP / (4 * LPR);           // float4s of a lane and row
+  constexpr int RPP = 256 / LPR, NR = 64 / RPP;
+  const int h = blockIdx.x, v0 = blockIdx.y * 64;
+  const int4 e = a.ent[blockIdx.z];
+  const int slot = min(max(e.z, 0), a.nslots - 1);
+  const int l = threadIdx.x % LPR, r0 = threadIdx.x / LPR;
+  float* st = a.state + (((size_t)slot * a.H + h) * a.VP + v0) * NP;
+  f32x4 S[NR][NI];
+  const bool fresh = a.pos[e.x] == 0;
+#pragma unroll
+  for (int r = 0; r < NR; ++r)
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      S[r][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (!fresh) S[r][i] = *reinterpret_cast<const f32x4*>(st + (size_t)(r0 + r * RPP) * NP + i * 4 * LPR + l * 4);
+    }
+  const float d = a.D != nullptr ? a.D[h] : 0.f;
+  for (int t = 0; t < e.y; ++t) {
+    const int m = e.x + t;
+    const T* row = reinterpret_cast<const T*>(a.rows) + (size_t)m * a.ld;
+    const float dt = a.dt != nullptr ? a.dt[(size_t)m * a.H + h] : a.dt_c;
+    const float la = a.la != nullptr ? a.la[(size_t)m * a.H + h] : a.la_h[h];
+    const float dec = expf(la);
+    const T* qp = row + a.qcol + (h / a.qdiv) * NP + l * 4;
+    const T* kp = row + a.kcol + (h / a.qdiv) * NP + l * 4;
+    f32x4 q[NI], k[NI];
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        q[i][j] = to_f32(qp[i * 4 * LPR + j]);
+        k[i][j] = to_f32(kp[i * 4 * LPR + j]) * dt;
+      }
+#pragma unroll
+    for (int r = 0; r < NR; ++r) {
+      const int v = v0 + r0 + r * RPP;
+      const float x = to_f32(row[a.vcol + h * a.VP + v]);
+      float y = 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          S[r][i][j] = fmaf(dec, S[r][i][j], k[i][j] * x);
+          y = fmaf(S[r][i][j], q[i][j], y);
+        }
+      y = group_sum<LPR>(y);
+      if (l == 0 && v < a.vdim) reinterpret_cast<T*>(a.y)[(size_t)m * a.ldy + h * a.vdim + v] = from_f32<T>(fmaf(d, x, y));
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < NR; ++r)
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+      *reinterpret_cast<f32x4*>(st + (size_t)(r0 + r * RPP) * NP + i * 4 * LPR + l * 4) = S[r][i];
+}
+
+// ---------------------------------------------------------------- chunks
+// Within a chunk, A_t the running sum of la:
+//   y_t = exp(A_t) S^T q_t + sum_{s <= t} (q_t . k_s) exp(A_t - A_s) dt_s v_s + D v_t
+//   S  <- exp(A_L) S + sum_s k_s (exp(A_L - A_s) dt_s v_s)^T
+// Everything that carries a decay, and the state as an operand, goes to the
+// MFMA as two bf16 terms (value and remainder), so the recurrence keeps about
+// 16 bits of mantissa; accumulators are fp32.  Wave w: tokens (w & 1) * 32..,
+// value columns (w >> 1) * 32.. of the output; the same value columns and half
+// of the state rows in the update.
+constexpr int SC_L = 64;            // tokens of a chunk
+constexpr int SC_VST = 64 * 2 + 64;  // bytes of a value row in LDS
+
+template <int NP>
+struct ScanLds {
+  static constexpr int KST = NP * 2 + 64, SST = NP * 2 + 16;
+  static constexpr int K = SC_L * KST, V = SC_L * SC_VST, S = 64 * SST;
+  static constexpr int TOTAL = K + V + 2 * S + 3 * SC_L * 4;
+};
+
+// 8 values of column (lane & 31) of a 64-row LDS tile at rows 16 s + 4 h + {0..3, 8..11}
+__device__ __forceinline__ bf16x8 sc_tr(const char* tile, int stride, int s, int col0, int lane) {
+  const char* p = tile + (16 * s + 4 * (lane >> 5) + ((lane & 15) >> 2)) * stride +
+                  (col0 + ((lane >> 4) & 1) * 16 + 4 * (lane & 3)) * 2;
+  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(p));
+  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(p + 8 * stride));
+  return bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+}
+__device__ __forceinline__ void sc_split(float v, short& hi, short& lo) {
+  const bf16_t h = f2bf(v);
+  hi = (short)h;
+  lo = (short)f2bf(v - bf2f(h));
+}
+
+template <int NP>
+__global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
+  using L = ScanLds<NP>;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  char* ks = smem;
+  char* vs = ks + L::K;
+  char* sh = vs + L::V;
+  char* sl = sh + L::S;
+  float* cum = reinterpret_cast<float*>(sl + L::S);
+  float* dts = cum + SC_L;
+  float* wst = dts + SC_L;
+  constexpr int NK = NP / 16, NT = NP / 32, NTW = NT > 1 ? NT / 2 : 1;
+  constexpr int CK = NP / 8, NIK = SC_L * CK / 256;  // 16-B pieces of a key row; per thread
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, hh = lane >> 5, r32 = lane & 31;
+  const int tt = wave & 1, vt = wave >> 1;
+  const int h = blockIdx.x, v0 = blockIdx.y * 64;
+  const int4 e = a.ent[blockIdx.z];
+  const int n = e.y, slot = min(max(e.z, 0), a.nslots - 1);
+  const bool mine = NT > 1 || tt == 0;  // this wave holds state rows
+  const int nt0 = NT > 1 ? tt * NTW : 0;
+  const bf16_t* base = reinterpret_cast<const bf16_t*>(a.rows) + (size_t)e.x * a.ld;
+  const int qc = a.qcol + (h / a.qdiv) * NP, kc = a.kcol + (h / a.qdiv) * NP, vc = a.vcol + h * a.VP + v0;
+  float* state = a.state + (((size_t)slot * a.H + h) * a.VP + v0 + vt * 32 + r32) * NP;
+  const float d = a.D != nullptr ? a.D[h] : 0.f;
+
+  f32x16 S[NTW];
+  const bool fresh = a.pos[e.x] == 0;
+#pragma unroll
+  for (int i = 0; i < NTW; ++i) {
+    S[i] = f32x16{};
+    if (!fresh && mine) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const f32x4 v = *reinterpret_cast<const f32x4*>(state + (nt0 + i) * 32 + 8 * q + 4 * hh);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) S[i][4 * q + j] = v[j];
+      }
+    }
+  }
+
+  i32x4 pk[NIK], pv[2];
+  float pla = 0.f, pdt = 0.f;
+  auto fetch = [&](int c0) __attribute__((always_inline)) {
+    const int len = min(SC_L, n - c0);
+#pragma unroll
+    for (int it = 0; it < NIK; ++it) {
+      const int x = it * 256 + tid, r = x / CK, c = x % CK;
+      pk[it] = i32x4{0, 0, 0, 0};
+      if (r < len) pk[it] = *reinterpret_cast<const i32x4*>(base + (size_t)(c0 + r) * a.ld + kc + c * 8);
+    }
+#pragma unroll
+    for (int it = 0; it < 2; ++it) {
+      const int x = it * 256 + tid, r = x >> 3, c = x & 7;
+      pv[it] = i32x4{0, 0, 0, 0};
+      if (r < len) pv[it] = *reinterpret_cast<const i32x4*>(base + (size_t)(c0 + r) * a.ld + vc + c * 8);
+    }
+    if (wave == 0) {
+      pla = pdt = 0.f;
+      if (lane < len) {
+        const size_t o = (size_t)(e.x + c0 + lane) * a.H + h;
+        pdt = a.dt != nullptr ? a.dt[o] : a.dt_c;
+        pla = a.la != nullptr ? a.la[o] : a.la_h[h];
+      }
+    }
+  };
+  fetch(0);
+  for (int c0 = 0; c0 < n; c0 += SC_L) {
+    const int len = min(SC_L, n - c0);
+    __syncthreads();  // the last chunk is read
+#pragma unroll
+    for (int it = 0; it < NIK; ++it) {
+      const int x = it * 256 + tid;
+      *reinterpret_cast<i32x4*>(ks + (x / CK) * L::KST + (x % CK) * 16) = pk[it];
+    }
+#pragma unroll
+    for (int it = 0; it < 2; ++it) {
+      const int x = it * 256 + tid;
+      *reinterpret_cast<i32x4*>(vs + (x >> 3) * SC_VST + (x & 7) * 16) = pv[it];
+    }
+    if (mine) {  // the state as an operand: rows of value columns, two terms
+#pragma unroll
+      for (int i = 0; i < NTW; ++i)
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          s16x4 hi, lo;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            short x, y;
+            sc_split(S[i][4 * q + j], x, y);
+            hi[j] = x;
+            lo[j] = y;
+          }
+          const int o = (vt * 32 + r32) * L::SST + ((nt0 + i) * 32 + 8 * q + 4 * hh) * 2;
+          *reinterpret_cast<s16x4*>(sh + o) = hi;
+          *reinterpret_cast<s16x4*>(sl + o) = lo;
+        }
+    }
+    if (wave == 0) {
+      float s = pla;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float u = __shfl_up(s, o, 64);
+        if (lane >= o) s += u;
+      }
+      cum[lane] = s;
+      dts[lane] = pdt;
+      const float end = __shfl(s, 63, 64);
+      wst[lane] = __expf(end - s) * pdt;
+    }
+    // this wave's queries as B operand: column = token
+    const int tok = tt * 32 + r32;
+    const bf16_t* qp = base + (size_t)min(c0 + tok, n - 1) * a.ld + qc + 8 * hh;
+    bf16x8 qf[NK];
+#pragma unroll
+    for (int k = 0; k < NK; ++k) qf[k] = *reinterpret_cast<const bf16x8*>(qp + k * 16);
+    __syncthreads();
+    if (c0 + SC_L < n) fetch(c0 + SC_L);
+
+    const float at = cum[tok];
+    f32x16 o = f32x16{};
+#pragma unroll
+    for (int k = 0; k < NK; ++k) {
+      const int off = (vt * 32 + r32) * L::SST + (k * 16 + 8 * hh) * 2;
+      o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(sh + off), qf[k], o, 0, 0, 0);
+      o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(sl + off), qf[k], o, 0, 0, 0);
+    }
+    o *= __expf(at);
+    for (int j = 0; j <= tt; ++j) {
+      f32x16 g = f32x16{};
+#pragma unroll
+      for (int k = 0; k < NK; ++k)
+        g = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
+            *reinterpret_cast<const bf16x8*>(ks + (j * 32 + r32) * L::KST + (k * 16 + 8 * hh) * 2), qf[k], g, 0, 0, 0);
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int s0 = j * 32 + 8 * q + 4 * hh;
+        const f32x4 cs = *reinterpret_cast<const f32x4*>(cum + s0), ds = *reinterpret_cast<const f32x4*>(dts + s0);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          g[4 * q + i] = s0 + i <= tok ? g[4 * q + i] * (__expf(at - cs[i]) * ds[i]) : 0.f;
+      }
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        bf16x8 hi, lo;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          short x, y;
+          sc_split(g[8 * s + i], x, y);
+          hi[i] = x;
+          lo[i] = y;
+        }
+        const bf16x8 vf = sc_tr(vs, SC_VST, 2 * j + s, vt * 32, lane);
+        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, hi, o, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, lo, o, 0, 0, 0);
+      }
+    }
+    if (tok < len) {
+      bf16_t* yp = reinterpret_cast<bf16_t*>(a.y) + (size_t)(e.x + c0 + tok) * a.ldy + h * a.vdim;
+      const bool vec = (a.vdim & 3) == 0 && (a.ldy & 3) == 0;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int vl = vt * 32 + 8 * q + 4 * hh, v = v0 + vl;
+        const s16x4 x = *reinterpret_cast<const s16x4*>(vs + tok * SC_VST + vl * 2);
+        float y[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y[i] = fmaf(d, bf2f_s(x[i]), o[4 * q + i]);
+        if (vec) {
+          if (v < a.vdim) *reinterpret_cast<uint2*>(yp + v) = make_uint2(pack2bf(y[0], y[1]), pack2bf(y[2], y[3]));
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (v + i < a.vdim) yp[v + i] = f2bf(y[i]);
+        }
+      }
+    }
+    if (mine) {
+      const float dec = __expf(cum[SC_L - 1]);
+#pragma unroll
+      for (int i = 0; i < NTW; ++i) S[i] *= dec;
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        const bf16x8 v = sc_tr(vs, SC_VST, s, vt * 32, lane);
+        const f32x4 w0 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh);
+        const f32x4 w1 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh + 8);
+        bf16x8 hi, lo;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          short x, y;
+          sc_split(bf2f_s(v[i]) * (i < 4 ? w0[i & 3] : w1[i & 3]), x, y);
+          hi[i] = x;
+          lo[i] = y;
+        }
+#pragma unroll
+        for (int i = 0; i < NTW; ++i) {
+          const bf16x8 kt = sc_tr(ks, L::KST, s, (nt0 + i) * 32, lane);
+          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, hi, S[i], 0, 0, 0);
+          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, lo, S[i], 0, 0, 0);
+        }
+      }
+    }
+  }
+  if (mine) {
+#pragma unroll
+    for (int i = 0; i < NTW; ++i)
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+        *reinterpret_cast<f32x4*>(state + (nt0 + i) * 32 + 8 * q + 4 * hh) =
+            f32x4{S[i][4 * q], S[i][4 * q + 1], S[i][4 * q + 2], S[i][4 * q + 3]};
+  }
+}
+
+// ---------------------------------------------------------------- gate and norm
+// TPR threads per part; E values a piece (16 bytes, or one value where parts are not aligned)
+template <typename T, int TPR, int E>
+__global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs a) {
+  __shared__ float red[4];
+  const int t = threadIdx.x % TPR;
+  const long x = blockIdx.x * (256L / TPR) + threadIdx.x / TPR;
+  if (x >= (long)a.M * a.groups) return;  // TPR 256: uniform over the workgroup
+  const int m = (int)(x / a.groups), g = (int)(x % a.groups), n = a.n / a.groups;
+  const T* y = reinterpret_cast<const T*>(a.y) + (size_t)m * a.ldy + g * n;
+  const T* z = reinterpret_cast<const T*>(a.z) + (size_t)m * a.ldz + g * n;
+  T* out = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + g * n;
+  float s = 0.f;
+  auto get = [&](const T* p, float (&v)[E]) __attribute__((always_inline)) {
+    if constexpr (E == 1) v[0] = to_f32(*p);
+    else Vec16<T>::get(p, v);
+  };
+  for (int c = t * E; c < n; c += TPR * E) {
+    float u[E], v[E];
+    get(y + c, u);
+    if (a.gate_first) get(z + c, v);
+#pragma unroll
+    for (int j = 0; j < E; ++j) {
+      if (a.gate_first) u[j] *= silu(v[j]);
+      s = fmaf(u[j], u[j], s);
+    }
+  }
+  s = wave_sum(s);
+  if constexpr (TPR == 256) {
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+    __syncthreads();
+    s = red[0] + red[1] + red[2] + red[3];
+  }
+  const float r = 1.0f / sqrtf(s / (float)n + a.eps);
+  for (int c = t * E; c < n; c += TPR * E) {
+    float u[E], v[E];
+    get(y + c, u);
+    get(z + c, v);
+#pragma unroll
+    for (int j = 0; j < E; ++j) {
+      u[j] *= silu(v[j]) * r;
+      if (a.w != nullptr) u[j] *= a.w[g * n + c + j];
+    }
+    if constexpr (E == 1) out[c] = from_f32<T>(u[0]);
+    else Vec16<T>::put(out + c, u);
+  }
+}
+
+}  // namespace dnn
+
+using namespace dnn;
+
+extern "C" int dnn_conv(const ConvArgs* a, int f32, hipStream_t st) {
+  const int e = f32 ? 4 : 8;
+  if (a->M <= 0 || a->C <= 0 || a->C % e != 0 || a->taps < 1 || a->ldi % e != 0 || a->ldo % e != 0 || a->ldi < a->C ||
+      a->ldo < a->C || a->nslots < 1)
+    return -1;
+  if (a->dt != nullptr && (a->H <= 0 || a->la == nullptr || a->dt_col < 0 || a->dt_col + a->H > a->ldi)) return -1;
+  const long n = (long)a->M * ((a->C / e + (a->dt != nullptr ? a->H : 0) + 255) / 256);
+  if (n > 0x7fffffff) return -1;
+  if (f32) hipLaunchKernelGGL(conv_kernel<float>, dim3((unsigned)n), dim3(256), 0, st, *a);
+  else hipLaunchKernelGGL(conv_kernel<bf16_t>, dim3((unsigned)n), dim3(256), 0, st, *a);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_conv_state(const ConvArgs* a, const int4* ent, int nent, int f32, hipStream_t st) {
+  const int e = f32 ? 4 : 8;
+  if (nent <= 0 || nent > 65535 || a->C % e != 0 || a->ldi % e != 0 || a->taps < 1 || ((uintptr_t)ent & 15) != 0) return -1;
+  const dim3 grid((unsigned)((a->C / e + 255) / 256), nent);
+  if (f32) hipLaunchKernelGGL(conv_state_kernel<float>, grid, dim3(256), 0, st, *a, ent);
+  else hipLaunchKernelGGL(conv_state_kernel<bf16_t>, grid, dim3(256), 0, st, *a, ent);
+  return (int)hipGetLastError();
+}
+
+static bool scan_ok(const ScanArgs& a) {
+  return a.M > 0 && a.H > 0 && a.VP % 64 == 0 && a.vdim > 0 && a.vdim <= a.VP && a.nent > 0 && a.nent <= 65535 &&
+         a.nslots > 0 && a.qdiv > 0 && a.ldy >= a.H * a.vdim && ((uintptr_t)a.ent & 15) == 0 &&
+         (a.la != nullptr || a.la_h != nullptr) && a.vcol + a.H * a.VP <= a.ld &&
+         a.qcol + ((a.H - 1) / a.qdiv + 1) * a.NP <= a.ld && a.kcol + ((a.H - 1) / a.qdiv + 1) * a.NP <= a.ld &&
+         (a.NP == 32 || a.NP == 64 || a.NP == 128 || a.NP == 256) && a.state != nullptr && a.pos != nullptr;
+}
+
+#define SCAN_NP(F)                                 \
+  switch (a->NP) {                                 \
+    case 32: F(32) break;                          \
+    case 64: F(64) break;                          \
+    case 128: F(128) break;                        \
+    default: F(256) break;                         \
+  }
+
+extern "C" int dnn_scan_steps(const ScanArgs* a, int f32, hipStream_t st) {
+  if (!scan_ok(*a)) return -1;
+  const dim3 grid(a->H, a->VP / 64, a->nent);
+#define SS(N)                                                                                       \
+  {                                                                                                 \
+    if (f32) hipLaunchKernelGGL((scan_steps_kernel<float, N>), grid, dim3(256), 0, st, *a);         \
+    else hipLaunchKernelGGL((scan_steps_kernel<bf16_t, N>), grid, dim3(256), 0, st, *a);            \
+  }
+  SCAN_NP(SS)
+#undef SS
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_scan_chunks(const ScanArgs* a, hipStream_t st) {
+  if (!scan_ok(*a) || (a->ld | a->qcol | a->kcol | a->vcol) % 8 != 0) return -1;
+  const dim3 grid(a->H, a->VP / 64, a->nent);
+#define SK(N) hipLaunchKernelGGL((scan_chunks_kernel<N>), grid, dim3(256), ScanLds<N>::TOTAL, st, *a);
+  SCAN_NP(SK)
+#undef SK
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_gated_norm(const GatedNormArgs* a, int f32, hipStream_t st) {
+  if (a->M <= 0 || a->n <= 0 || a->groups <= 0 || a->n % a->groups != 0 || a->ldy < a->n || a->ldz < a->n || a->ldo < a->n)
+    return -1;
+  const int n = a->n / a->groups, e = f32 ? 4 : 8;
+  const bool vec = n % e == 0 && (a->ldy | a->ldz | a->ldo) % e == 0 &&
+                   (((uintptr_t)a->y | (uintptr_t)a->z | (uintptr_t)a->out) & 15) == 0;
+  const long parts = (long)a->M * a->groups;
+#define GN(T, E)                                                                                                         \
+  {                                                                                                                      \
+    if (n > 1024) hipLaunchKernelGGL((gated_norm_kernel<T, 256, E>), dim3((unsigned)parts), dim3(256), 0, st, *a);       \
+    else hipLaunchKernelGGL((gated_norm_kernel<T, 64, E>), dim3((unsigned)((parts + 3) / 4)), dim3(256), 0, st, *a);     \
+  }
+  if (f32) {
+    if (vec) GN(float, 4) else GN(float, 1)
+  } else {
+    if (vec) GN(bf16_t, 8) else GN(bf16_t, 1)
+  }
+#undef GN
+  return (int)hipGetLastError();
+}

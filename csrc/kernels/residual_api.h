@@ -13,10 +13,22 @@ struct RowsArgs {
   const float* y_w;    // RMS-norm weight of y (nullptr: y as it is)
   float* x_out;        // updated residual (may be x_in)
   void* copy;          // optional copy of x' as a GEMM operand
-  const float* n_w;    // RMS-norm weight of h (nullptr: no h)
+  const float* n_w;    // norm weight of h (nullptr: no h)
   void* h;
   int xrows, yrows, ldx, ldy, ldcopy, ldh, M, N, NP;
   float mult, eps;
+  // optional parts (zero: absent)
+  const float* x_add = nullptr;     // fp32 rows joined to x as they are (stride ldadd)
+  const void* y2 = nullptr;         // second sublayer output, RMS-normed with y2_w, joined like y
+  const float* y2_w = nullptr;
+  const void* ys = nullptr;         // weighted rows joined to y: sum over t < top of ysw[m * top + t] * ys[ysi[m * top + t]]
+  const int* ysi = nullptr;
+  const float* ysw = nullptr;
+  const float* n_b = nullptr;       // with it the norm is tanh(n_alpha x') * n_w + n_b (no mean, no variance)
+  const int* pos = nullptr;         // with freq: a sinusoidal position vector joins x (columns < N), entry 2i
+  const double* freq = nullptr;     //   sin, 2i + 1 cos of 2 pi * pos * freq[i] (freq in turns)
+  int ldadd = 0, ldy2 = 0, ldys = 0, ysrows = 0, top = 0;
+  float n_alpha = 0.f;
 };
 
 // One sequence's key range, masks and scales of a paged attention launch.
@@ -30,9 +42,32 @@ struct PagedAttnArgs {
   void* out;           // [row][H*DV], row stride ldo
   int ldq, ldo, ldt, npages, M;
   int H, G, DK, DV;
-  int gate;            // first column of the per-head output gate logits in qkv, -1: none
+  int gate;            // first column of the output gate logits in qkv, -1: none
   int window, keep;    // key j seen by query i: j <= i and (i - j < window or j < keep)
   float scale;
+  // optional parts (zero: absent)
+  const float* kscale = nullptr;  // [page][64]: factor of every key's scores (fp32, all heads)
+  const float* slopes = nullptr;  // [H]: slope_h * (i - j) is taken off the scaled score
+  int gate_el = 0;                // the gate has a column per head and value (H*DV) instead of one per head
+  int shared = 0;                 // values are the keys: vp == kp, rows [q H*DK | k G*DK | ...]
+  int written = 0;                // the cache already holds the rows' keys and values (paged_decode does not store them)
+};
+
+// Query / key norm over whole projections, and the cache write of shared
+// keys = values:  q <- q * rsqrt(mean(q^2) + eps) * qw * temp(pos) in place,
+// page keys <- k as projected, kscale <- rsqrt(mean(k^2) + eps); qw holds the
+// product of both norm weights.  temp = 1 + t_coef * ln(floor((pos + 1) / t_every) + 1).
+struct QkNormArgs {
+  void* qkv;
+  void* kp;
+  float* kscale;
+  const float* qw;  // [H*DK]
+  const int* table;
+  const int* slots;
+  const int* pos;
+  int ldq, ldt, npages, M, H, G, DK, nq, nk;  // nq, nk: true widths of the projections
+  int t_every;                                 // 0: no temperature
+  float t_coef, eps;
 };
 
 extern "C" {
@@ -42,7 +77,8 @@ int dnn_token_gate(const void* x, int ldx, const void* w, int ldw, const void* w
                    int off, const int* tok, int V, void* g, int ldg, int M, int n, int np, hipStream_t st);
 int dnn_token_gate_f32(const float* z, int ldz, const float* table, int ldt, int off, const int* tok, int V, float* g,
                        int ldg, int M, int n, int np, hipStream_t st);
-int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, hipStream_t st);
+int dnn_qk_norm(const QkNormArgs* a, int f32, hipStream_t st);
+int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act, hipStream_t st);
 int dnn_gemm_f32(const float* A, int lda, const float* W, int ldw, float* C, int ldc, const float* bias, int M, int N,
                  int K, hipStream_t st);
 int dnn_paged_write(const PagedAttnArgs* a, int f32, hipStream_t st);

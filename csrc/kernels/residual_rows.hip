@@ -1,15 +1,19 @@
 // Row kernels of decoder layers with an fp32 residual stream.
 //
-// rows_update: one pass over a row that joins a sublayer's output into the
+// rows_update: one pass over a row that joins sublayer outputs into the
 // residual and prepares the next projection's input,
-//   x' = [x +] mult * y * [rsqrt(mean(y^2) + eps) * yw]      (fp32)
+//   z  = y * [rsqrt(mean(y^2) + eps) * yw] [+ the same of y2] [+ sum_t w_t ys_t]
+//   x' = [x] [+ x_add] [+ position vector] + mult * z        (fp32)
 //   copy = T(x')              the residual as a GEMM operand
-//   h    = T(x' * rsqrt(mean(x'^2) + eps) * nw)               RMS norm
+//   h    = T(x' * rsqrt(mean(x'^2) + eps) * nw)               RMS norm, or
+//        = T(tanh(alpha x') * nw + nb)                        dynamic tanh
 // each part optional.  y rows may be gathered (the embedding: y = table,
-// yidx = tokens, mult = the embedding scale), x rows too (the head's rows).
+// yidx = tokens, mult = the embedding scale), x rows too (the head's rows);
+// ys are the rows of a mixture of experts, w_t their router weights.
 // Rows are NP wide (padded, zeros past N); means are over the true width N.
 // bf16 y / T in serving, fp32 in the exact mode.
 #include "common.h"
+#include "gemm_epilogue.h"
 #include "residual_api.h"
 
 namespace dnn {
@@ -36,37 +40,85 @@ __device__ __forceinline__ float row_sum(float v, float* red) {
   return red[0] + red[1] + red[2] + red[3];
 }
 
+// Two sums at once over the TPR threads of a row.
+template <int TPR>
+__device__ __forceinline__ void row_sum2(float& u, float& v, float* red) {
+  u = wave_sum(u);
+  v = wave_sum(v);
+  if constexpr (TPR == 64) return;
+  const int wave = threadIdx.x >> 6;
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[wave] = u, red[4 + wave] = v;
+  __syncthreads();
+  u = red[0] + red[1] + red[2] + red[3];
+  v = red[4] + red[5] + red[6] + red[7];
+}
+
+// Entry c of the sinusoidal position vector: the angle in turns, reduced in
+// fp64 before it becomes fp32.
+__device__ __forceinline__ float pos_entry(int p, const double* freq, int c) {
+  double t = (double)p * freq[c >> 1];
+  t -= floor(t);
+  const float a = 6.283185307179586f * (float)t;
+  return (c & 1) != 0 ? cosf(a) : sinf(a);
+}
+
 template <typename YT, typename OT, int TPR, int NC>
 __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
-  __shared__ float red[4];
+  __shared__ float red[8];
   const int t = threadIdx.x % TPR;
   const int m = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
   if (m >= a.M) return;  // TPR 256: uniform over the workgroup
   const int xr = a.xidx != nullptr ? min(max(a.xidx[m], 0), a.xrows - 1) : m;
-  // few values per thread: the norm weights are issued with the row (one memory round trip)
+  // few values per thread: the norm weights and y2 are issued with the row (one memory round trip)
   constexpr bool PF = NC <= 4;
-  f32x4 x[NC], y[NC], yw[PF ? NC : 1], nw[PF ? NC : 1];
+  f32x4 x[NC], y[NC], yw[PF ? NC : 1], nw[PF ? NC : 1], y2[PF ? NC : 1];
   const float* xp = a.x_in != nullptr ? a.x_in + (size_t)xr * a.ldx : nullptr;
   const YT* yp = nullptr;
   if (a.y != nullptr) {
     const int yr = a.yidx != nullptr ? min(max(a.yidx[m], 0), a.yrows - 1) : m;
     yp = reinterpret_cast<const YT*>(a.y) + (size_t)yr * a.ldy;
   }
+  const YT* y2p = a.y2 != nullptr ? reinterpret_cast<const YT*>(a.y2) + (size_t)m * a.ldy2 : nullptr;
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
     const int c = (t + TPR * i) * 4;
     x[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if constexpr (PF) y2[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c < a.NP) {
       if (xp != nullptr) x[i] = ld4(xp + c);
       if (yp != nullptr) y[i] = ld4(yp + c);
       if constexpr (PF) {
         if (a.y_w != nullptr) yw[i] = ld4(a.y_w + c);
         if (a.n_w != nullptr) nw[i] = ld4(a.n_w + c);
+        if (y2p != nullptr) y2[i] = ld4(y2p + c);
       }
     }
   }
-  if (a.y_w != nullptr) {
+  if (y2p != nullptr) {  // both outputs normalised
+    float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (t + TPR * i) * 4;
+      f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+      if constexpr (PF) v = y2[i];
+      else if (c < a.NP) v = ld4(y2p + c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        s1 = fmaf(y[i][j], y[i][j], s1);
+        s2 = fmaf(v[j], v[j], s2);
+      }
+    }
+    row_sum2<TPR>(s1, s2, red);
+    const float r1 = 1.0f / sqrtf(s1 / (float)a.N + a.eps), r2 = 1.0f / sqrtf(s2 / (float)a.N + a.eps);
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (t + TPR * i) * 4;
+      if (c < a.NP)
+        y[i] = y[i] * r1 * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c)) + (PF ? y2[PF ? i : 0] : ld4(y2p + c)) * r2 * ld4(a.y2_w + c);
+    }
+  } else if (a.y_w != nullptr) {
     float s = 0.f;
 #pragma unroll
     for (int i = 0; i < NC; ++i)
@@ -78,6 +130,37 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
       const int c = (t + TPR * i) * 4;
       if (c < a.NP) y[i] = y[i] * r * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c));
     }
+  }
+  if (a.ys != nullptr) {
+    const int* si = a.ysi + (size_t)m * a.top;
+    const float* sw = a.ysw + (size_t)m * a.top;
+#pragma unroll 4
+    for (int k = 0; k < a.top; ++k) {
+      const YT* p = reinterpret_cast<const YT*>(a.ys) + (size_t)min(max(si[k], 0), a.ysrows - 1) * a.ldys;
+      const float w = sw[k];
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const int c = (t + TPR * i) * 4;
+        if (c < a.NP) y[i] = y[i] + w * ld4(p + c);
+      }
+    }
+  }
+  if (a.x_add != nullptr) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (t + TPR * i) * 4;
+      if (c < a.NP) x[i] = x[i] + ld4(a.x_add + (size_t)m * a.ldadd + c);
+    }
+  }
+  if (a.freq != nullptr) {
+    const int p = a.pos[m];
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int c = (t + TPR * i) * 4 + j;
+        if (c < a.N) x[i][j] += pos_entry(p, a.freq, c);
+      }
   }
   float s = 0.f;
 #pragma unroll
@@ -94,6 +177,19 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
     }
   }
   if (a.n_w == nullptr) return;
+  if (a.n_b != nullptr) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (t + TPR * i) * 4;
+      if (c >= a.NP) continue;
+      const f32x4 w = PF ? nw[PF ? i : 0] : ld4(a.n_w + c), b = ld4(a.n_b + c);
+      f32x4 v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = fmaf(tanhf(a.n_alpha * x[i][j]), w[j], b[j]);
+      st4(reinterpret_cast<OT*>(a.h) + (size_t)m * a.ldh + c, v);
+    }
+    return;
+  }
   const float r = 1.0f / sqrtf(row_sum<TPR>(s, red) / (float)a.N + a.eps);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
@@ -124,15 +220,17 @@ static int rows_launch(const RowsArgs& a, hipStream_t st) {
   return -1;
 }
 
-// fp32 gated activation of packed gate|up columns (8 gate, 8 up, ...): out = gelu_tanh(gate) * up.
+// fp32 gated activation of packed gate|up columns (8 gate, 8 up, ...): out = act(gate) * up.
 __global__ __launch_bounds__(256) void glu_f32_kernel(const float* __restrict__ gu, int ldi, float* __restrict__ out,
-                                                      int ldo, int M, int F) {
+                                                      int ldo, int M, int F, int act) {
   const long i = blockIdx.x * 256L + threadIdx.x;
   if (i >= (long)M * F) return;
   const int m = (int)(i / F), c = (int)(i % F);
   const float* p = gu + (size_t)m * ldi + (c >> 3) * 16 + (c & 7);
   const float x = p[0];
-  out[(size_t)m * ldo + c] = 0.5f * x * (1.0f + tanhf(0.797884560802865f * (x + 0.044715f * x * x * x))) * p[8];
+  const float g = act == ACT_SILU_MUL ? x / (1.0f + expf(-x))
+                                      : 0.5f * x * (1.0f + tanhf(0.797884560802865f * (x + 0.044715f * x * x * x)));
+  out[(size_t)m * ldo + c] = g * p[8];
 }
 
 }  // namespace dnn
@@ -142,14 +240,19 @@ using namespace dnn;
 extern "C" int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStream_t st) {
   if (a->M <= 0 || a->N <= 0 || a->N > a->NP || a->NP % 4 != 0 || (a->ldx | a->ldy | a->ldcopy | a->ldh) % 4 != 0)
     return -1;
+  if ((a->ldadd | a->ldy2 | a->ldys) % 4 != 0 || (a->y2 != nullptr && (a->y2_w == nullptr || a->y_w == nullptr)) ||
+      (a->ys != nullptr && (a->ysi == nullptr || a->ysw == nullptr || a->top < 1 || a->ysrows < 1)) ||
+      (a->freq != nullptr && a->pos == nullptr))
+    return -1;
   if ((a->xidx != nullptr && (a->xrows < 1 || a->x_out != nullptr)) || (a->yidx != nullptr && a->yrows < 1)) return -1;
   if (y_f32) return out_f32 ? rows_launch<float, float>(*a, st) : rows_launch<float, bf16_t>(*a, st);
   return out_f32 ? -1 : rows_launch<bf16_t, bf16_t>(*a, st);
 }
 
-extern "C" int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, hipStream_t st) {
-  if (M <= 0 || F <= 0 || F % 8 != 0 || ldi < 2 * F || ldo < F) return -1;
+extern "C" int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act,
+                           hipStream_t st) {
+  if (M <= 0 || F <= 0 || F % 8 != 0 || ldi < 2 * F || ldo < F || !is_glu(act)) return -1;
   hipLaunchKernelGGL(glu_f32_kernel, dim3((unsigned)(((long)M * F + 255) / 256)), dim3(256), 0, st, gu, ldi, out, ldo,
-                     M, F);
+                     M, F, act);
   return (int)hipGetLastError();
 }

@@ -26,7 +26,7 @@ from typing import Dict, Iterable, List, Optional, Tuple
 
 import torch
 
-from .models import cifar, gpt2, kozusun, llama3, model_info
+from .models import DECODERS, cifar, gpt2, llama3, model_info
 
 
 class CheckpointError(Exception):
@@ -125,8 +125,8 @@ def stage_state_dict(model: str, full_sd, start: int, end: int, first: bool,
     elif info.family == "gpt2":
         full_sd = _gpt2_normalise(full_sd)
         want = gpt2.stage_key_map(info.cfg, start, end, first, last)
-    elif info.family == "kozusun":
-        want = kozusun.stage_key_map(info.cfg, start, end, first, last)
+    elif info.family in DECODERS:
+        want = DECODERS[info.family].stage_key_map(info.cfg, start, end, first, last)
     else:
         want = llama3.stage_key_map(info.cfg, start, end, first, last)
         if last and "lm_head.weight" not in full_sd and "model.embed_tokens.weight" in full_sd:
@@ -136,8 +136,8 @@ def stage_state_dict(model: str, full_sd, start: int, end: int, first: bool,
         raise CheckpointError(f"missing keys for stage layers [{start},{end}]: {missing[:8]}"
                               + (f" (+{len(missing) - 8} more)" if len(missing) > 8 else ""))
     sd = {local: full_sd[full] for local, full in want.items()}
-    if info.family == "kozusun":  # every size comes from the config: the tensors must agree with it
-        shapes = kozusun.stage_shapes(info.cfg, start, end, first, last)
+    if info.family in DECODERS:  # every size comes from the config: the tensors must agree with it
+        shapes = DECODERS[info.family].stage_shapes(info.cfg, start, end, first, last)
         bad = [f"{k} {tuple(v.shape)} (config: {shapes[k]})" for k, v in sd.items() if tuple(v.shape) != shapes[k]]
         if bad:
             raise CheckpointError(f"tensors that do not fit the config: {bad[:8]}")
@@ -152,8 +152,8 @@ def unexpected_keys(model: str, full_sd, start: int, end: int, first: bool, last
     elif info.family == "gpt2":
         full_sd = _gpt2_normalise(full_sd)
         mine = set(gpt2.stage_key_map(info.cfg, start, end, first, last).values())
-    elif info.family == "kozusun":
-        mine = set(kozusun.stage_key_map(info.cfg, start, end, first, last).values())
+    elif info.family in DECODERS:
+        mine = set(DECODERS[info.family].stage_key_map(info.cfg, start, end, first, last).values())
     else:
         mine = set(llama3.stage_key_map(info.cfg, start, end, first, last).values())
     return [k for k in full_sd.keys() if k not in mine]
@@ -174,8 +174,8 @@ def random_stage_state_dict(model: str, start: int, end: int, first: bool, last:
         return {k: v for k, v in cifar.random_state_dict(seed).items()
                 if k.split(".")[0] in {n for u in range(start, end + 1) for n in cifar.UNIT_KEYS[u]}}
     dev = torch.device(device) if device is not None else torch.device("cpu")
-    if info.family == "kozusun":
-        return random_kozusun_state(info.cfg, start, end, first, last, seed, dev, nontrivial)
+    if info.family in DECODERS:
+        return random_decoder_state(DECODERS[info.family], info.cfg, start, end, first, last, seed, dev, nontrivial)
     shapes = _stage_shapes(model, start, end, first, last)
     sd = {}
     for local, shape in shapes.items():
@@ -196,22 +196,12 @@ def random_stage_state_dict(model: str, start: int, end: int, first: bool, last:
     return sd
 
 
-def random_kozusun_state(cfg, start, end, first, last, seed, dev, nontrivial) -> Dict[str, torch.Tensor]:
-    """Biases zero and norm weights one (stored around zero where the model adds
-    the one), or noise around those with ``nontrivial``; projections of unit gain."""
+def random_decoder_state(family, cfg, start, end, first, last, seed, dev, nontrivial) -> Dict[str, torch.Tensor]:
+    """Random weights of a paged decoder's stage (``family``: its description module)."""
     sd = {}
-    for k, shape in kozusun.stage_shapes(cfg, start, end, first, last).items():
+    for k, shape in family.stage_shapes(cfg, start, end, first, last).items():
         g = torch.Generator(device=dev).manual_seed(_key_seed(seed, k))
-        t = torch.randn(shape, generator=g, device=dev)
-        if len(shape) == 1:
-            noise = 0.1 * t if nontrivial else torch.zeros_like(t)
-            sd[k] = 1 + noise if k.endswith("side.norm") else noise
-        elif k == "embed":
-            sd[k] = t / cfg.embed_scale
-        elif k == "side.embed":
-            sd[k] = t
-        else:
-            sd[k] = t * shape[1] ** -0.5
+        sd[k] = family.random_tensor(cfg, k, torch.randn(shape, generator=g, device=dev), nontrivial)
     return sd
 
 
@@ -252,8 +242,8 @@ def make_full_checkpoint(model: str, path: str, seed: int = 0) -> None:
         st = random_stage_state_dict(model, 0, n - 1, True, True, seed)
         if info.family == "gpt2":
             km = gpt2.stage_key_map(info.cfg, 0, n - 1, True, True)
-        elif info.family == "kozusun":
-            km = kozusun.stage_key_map(info.cfg, 0, n - 1, True, True)
+        elif info.family in DECODERS:
+            km = DECODERS[info.family].stage_key_map(info.cfg, 0, n - 1, True, True)
         else:
             km = llama3.stage_key_map(info.cfg, 0, n - 1, True, True)
         sd = {km[k]: v for k, v in st.items()}

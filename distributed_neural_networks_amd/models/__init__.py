@@ -11,16 +11,22 @@ import os
 from dataclasses import dataclass
 from typing import List, Tuple
 
-from . import cifar, gpt2, kozusun, llama3
+from . import cifar, funepel, gpt2, kozusun, llama3
+from .decoder_config import CONFIG_FILE
 
 # "architecture" of a model folder's config.json -> (family, config loader)
-ARCHITECTURES = {kozusun.ARCHITECTURE: ("kozusun", kozusun.load_config)}
+ARCHITECTURES = {kozusun.ARCHITECTURE: ("kozusun", kozusun.load_config),
+                 funepel.ARCHITECTURE: ("funepel", funepel.load_config)}
+# families of the paged decoder stage (runtime/decoder.py): descriptions with
+# stage_shapes / stage_key_map / random_tensor / run_flops over layer runs
+DECODERS = {"kozusun": kozusun, "funepel": funepel}
+_DECODER_PRESETS = {"kozusun": kozusun.KOZUSUN_CONFIGS, "funepel": funepel.FUNEPEL_CONFIGS}
 
 
 @dataclass(frozen=True)
 class ModelInfo:
     name: str
-    family: str           # "cifar" | "gpt2" | "llama3" | "kozusun"
+    family: str           # "cifar" | "gpt2" | "llama3" | a key of DECODERS
     num_layers: int       # layer units that can be split across stages
     cfg: object = None
 
@@ -34,9 +40,9 @@ def model_info(name: str) -> ModelInfo:
     if name in llama3.LLAMA_CONFIGS:
         c = llama3.LLAMA_CONFIGS[name]
         return ModelInfo(name, "llama3", c.n_layer, c)
-    if name in kozusun.KOZUSUN_CONFIGS:
-        c = kozusun.KOZUSUN_CONFIGS[name]
-        return ModelInfo(name, "kozusun", c.n_layer, c)
+    for family, presets in _DECODER_PRESETS.items():
+        if name in presets:
+            return ModelInfo(name, family, presets[name].n_layer, presets[name])
     if is_model_folder(name):
         return _folder_info(os.path.abspath(name))
     raise KeyError(f"unknown model {name!r}")
@@ -44,12 +50,12 @@ def model_info(name: str) -> ModelInfo:
 
 def is_model_folder(name: str) -> bool:
     """A folder with a config.json (a model by path instead of by name)."""
-    return os.path.isfile(os.path.join(name, kozusun.CONFIG_FILE))
+    return os.path.isfile(os.path.join(name, CONFIG_FILE))
 
 
 @functools.lru_cache(maxsize=None)
 def _folder_info(path: str) -> ModelInfo:
-    with open(os.path.join(path, kozusun.CONFIG_FILE)) as f:
+    with open(os.path.join(path, CONFIG_FILE)) as f:
         arch = json.load(f).get("architecture")
     if arch not in ARCHITECTURES:
         raise KeyError(f"{path}: unknown architecture {arch!r}, expected one of {sorted(ARCHITECTURES)}")
@@ -69,8 +75,8 @@ def default_ranges(name: str, num_stages: int) -> List[Tuple[int, int]]:
         head = (2 * c.n_embd * c.vocab_size) / (24 * c.n_embd * c.n_embd)
         return balanced_ranges(info.num_layers, num_stages, 0.0, min(head, 2.0))
     c = info.cfg
-    if info.family == "kozusun":
-        head = 2 * c.n_embd * c.vocab_size / kozusun.run_flops(c, 0, 0)
+    if info.family in DECODERS:
+        head = 2 * c.n_embd * c.vocab_size / DECODERS[info.family].run_flops(c, 0, 0)
         return balanced_ranges(info.num_layers, num_stages, 0.0, min(head, 2.0))
     head = (2 * c.n_embd * c.vocab_size) / (2 * (2 * c.n_embd * c.n_embd * 2 + 3 * c.n_embd * c.ffn_dim))
     return balanced_ranges(info.num_layers, num_stages, 0.0, min(head, 2.0))
@@ -82,6 +88,6 @@ def build_golden_stage(name: str, start: int, end: int, first: bool, last: bool)
         return cifar.CifarStage(start, end)
     if info.family == "gpt2":
         return gpt2.GPTStage(info.cfg, start, end, first, last)
-    if info.family == "kozusun":
+    if info.family in DECODERS:
         raise ValueError(f"model {name!r} runs on the GPU kernels only (runtime/decoder.py); it has no torch stage")
     return llama3.LlamaStage(info.cfg, start, end, first, last)

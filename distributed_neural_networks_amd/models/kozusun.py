@@ -29,17 +29,13 @@ This module holds the description only; ``runtime/decoder.py`` runs it.
 """
 from __future__ import annotations
 
-import json
-import os
 from dataclasses import dataclass, replace
 from typing import Dict, List, Optional, Tuple
 
+from .decoder_config import (ModelConfigError, LayerRun, get_loop, get_number as _get, get_size as _size, layer_runs,
+                             load_json)
+
 ARCHITECTURE = "Kozusun"
-CONFIG_FILE = "config.json"
-
-
-class ModelConfigError(ValueError):
-    """config.json does not describe a model of this design."""
 
 
 @dataclass(frozen=True)
@@ -60,13 +56,6 @@ class LayerConfig:
 
 
 @dataclass(frozen=True)
-class LayerRun:
-    """One execution of a layer; ``enters``: a loop pass starts here."""
-    layer: int
-    enters: bool
-
-
-@dataclass(frozen=True)
 class KozusunConfig:
     vocab_size: int
     n_embd: int
@@ -84,26 +73,7 @@ class KozusunConfig:
 
     @property
     def runs(self) -> List[LayerRun]:
-        n = len(self.layers)
-        if self.loop is None:
-            return [LayerRun(i, False) for i in range(n)]
-        a, b, times = self.loop
-        body = [LayerRun(i, i == a) for i in range(a, b)]
-        return ([LayerRun(i, False) for i in range(a)] + body * times + [LayerRun(i, False) for i in range(b, n)])
-
-
-def _get(d, key, where, kinds=(int, float)):
-    v = d.get(key) if isinstance(d, dict) else None
-    if not isinstance(v, kinds) or isinstance(v, bool):
-        raise ModelConfigError(f"{where}: '{key}' is missing or not a number, got {v!r}")
-    return v
-
-
-def _size(d, key, where, low=1):
-    v = _get(d, key, where, (int,))
-    if v < low:
-        raise ModelConfigError(f"{where}: '{key}' must be >= {low}, got {v}")
-    return v
+        return layer_runs(len(self.layers), self.loop, first_pass_enters=True)
 
 
 def _attention(d, where) -> AttentionConfig:
@@ -137,26 +107,15 @@ def parse_config(d: Dict) -> KozusunConfig:
     if not isinstance(raw, list) or not raw:
         raise ModelConfigError("'layers' must be a list with at least one layer")
     layers = tuple(_layer(x, i) for i, x in enumerate(raw))
-    loop = None
-    if d.get("loop"):
-        a, b, t = (_size(d["loop"], k, "loop", low) for k, low in (("start", 0), ("stop", 1), ("times", 1)))
-        if not a < b <= len(layers):
-            raise ModelConfigError(f"loop: layers {a} .. {b - 1} of {len(layers)}")
-        loop = (a, b, t)
     return KozusunConfig(vocab_size=_size(d, "vocab", "config"), n_embd=_size(d, "width", "config"), layers=layers,
                          embed_scale=float(_get(d.get("embedding"), "scale", "embedding")),
                          norm_eps=float(_get(d.get("norm"), "eps", "norm")),
-                         residual_mult=float(_get(d, "residual_mult", "config")), loop=loop,
+                         residual_mult=float(_get(d, "residual_mult", "config")), loop=get_loop(d, len(layers)),
                          side_dim=_size(d["token_side"], "dim", "token_side") if d.get("token_side") else 0)
 
 
 def load_config(folder: str) -> KozusunConfig:
-    path = os.path.join(folder, CONFIG_FILE)
-    try:
-        with open(path) as f:
-            return parse_config(json.load(f))
-    except json.JSONDecodeError as e:
-        raise ModelConfigError(f"{path}: {e}") from e
+    return load_json(folder, parse_config)
 
 
 def make_config(vocab: int, width: int, n_layers: int, heads: int, kv_heads: int, dim: int, ff: Optional[int],
@@ -218,6 +177,18 @@ def stage_shapes(cfg: KozusunConfig, start: int, end: int, first: bool, last: bo
 
 def stage_key_map(cfg: KozusunConfig, start: int, end: int, first: bool, last: bool) -> Dict[str, str]:
     return {k: k for k in stage_shapes(cfg, start, end, first, last)}
+
+
+def random_tensor(cfg: KozusunConfig, name: str, noise, nontrivial: bool):
+    """A random weight from unit ``noise`` of its shape: projections of unit
+    gain, biases zero and norm weights one (stored around zero where the model
+    adds the one), or noise around those with ``nontrivial``."""
+    if noise.dim() == 1:
+        extra = 0.1 * noise if nontrivial else 0 * noise
+        return 1 + extra if name.endswith("side.norm") else extra
+    if name == "embed":
+        return noise / cfg.embed_scale
+    return noise if name == "side.embed" else noise * noise.shape[1] ** -0.5
 
 
 def run_flops(cfg: KozusunConfig, layer: int, ctx: int) -> float:

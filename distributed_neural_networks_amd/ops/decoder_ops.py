@@ -54,37 +54,74 @@ def _weight(t: Optional[torch.Tensor], N: int, name: str) -> None:
 
 def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx: Optional[torch.Tensor] = None,
                 y: Optional[torch.Tensor] = None, yidx: Optional[torch.Tensor] = None, mult: float = 1.0,
-                y_norm: Optional[torch.Tensor] = None, x_out: Optional[torch.Tensor] = None,
+                y_norm: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None,
+                y2_norm: Optional[torch.Tensor] = None, ys: Optional[torch.Tensor] = None,
+                ysi: Optional[torch.Tensor] = None, ysw: Optional[torch.Tensor] = None, top: int = 0,
+                x_add: Optional[torch.Tensor] = None, pos: Optional[torch.Tensor] = None,
+                freq: Optional[torch.Tensor] = None, x_out: Optional[torch.Tensor] = None,
                 copy: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
-                h: Optional[torch.Tensor] = None, eps: float = 1e-5) -> None:
-    """``x' = [x_in] + mult * y`` (``y`` RMS-normalised with weight ``y_norm``
-    first, if given), then any of ``x_out = x'`` (fp32), ``copy = x'`` and
-    ``h = RMSnorm(x') * norm``.  ``xidx`` / ``yidx`` gather the rows of ``x_in``
-    / ``y``.  Rows are zero-padded to a multiple of 4; means are over ``width``."""
+                norm_b: Optional[torch.Tensor] = None, alpha: float = 0.0, h: Optional[torch.Tensor] = None,
+                eps: float = 1e-5) -> None:
+    """``x' = [x_in] [+ x_add] [+ positions] + mult * z`` with ``z = y`` (RMS-
+    normalised with weight ``y_norm`` first, if given) ``[+ y2`` normalised with
+    ``y2_norm] [+ sum_t ysw[m, t] ys[ysi[m, t]]]``, then any of ``x_out = x'``
+    (fp32), ``copy = x'`` and ``h = RMSnorm(x') * norm``, or with ``norm_b`` the
+    dynamic tanh ``h = tanh(alpha x') * norm + norm_b``.  ``xidx`` / ``yidx``
+    gather the rows of ``x_in`` / ``y``; positions: sinusoids of ``pos`` with
+    ``freq`` (fp64, turns per position; even columns sine, odd cosine).  Rows are
+    zero-padded to a multiple of 4; means are over ``width``."""
     f32, bf = torch.float32, torch.bfloat16
     out = copy if copy is not None else h
-    od = out.dtype if out is not None else (y.dtype if y is not None else f32)
+    yt = next((t for t in (y, y2, ys) if t is not None), None)
+    od = out.dtype if out is not None else (yt.dtype if yt is not None else f32)
     NP = next(t.shape[1] for t in (x_out, x_in, y) if t is not None)
     _rows(x_in, 1 if xidx is not None else M, NP, "rows_update x_in", (f32,))
     _rows(x_out, M, NP, "rows_update x_out", (f32,))
+    _rows(x_add, M, NP, "rows_update x_add", (f32,))
     _rows(y, 1 if yidx is not None else M, NP, "rows_update y", (f32, bf))
+    _rows(y2, M, NP, "rows_update y2", () if yt is None else (yt.dtype,))
+    _rows(ys, 1, NP, "rows_update ys", () if yt is None else (yt.dtype,))
     _rows(copy, M, NP, "rows_update copy", (od,))
     _rows(h, M, NP, "rows_update h", (od,))
     _index(xidx, M, "rows_update xidx")
     _index(yidx, M, "rows_update yidx")
-    _weight(y_norm, NP, "rows_update y_norm")
-    _weight(norm, NP, "rows_update norm")
-    if x_in is None and y is None or (norm is None) != (h is None) or width > NP or NP % 4 or NP > WIDTH_MAX:
+    _index(ysi, M * top, "rows_update ysi")
+    _index(pos, M, "rows_update pos")
+    _weight(ysw, M * top, "rows_update ysw")
+    for t, n in ((y_norm, "y_norm"), (y2_norm, "y2_norm"), (norm, "norm"), (norm_b, "norm_b")):
+        _weight(t, NP, "rows_update " + n)
+    if x_in is None and yt is None or (norm is None) != (h is None) or width > NP or NP % 4 or NP > WIDTH_MAX \
+            or (norm_b is not None and norm is None) or (ys is not None and (ysi is None or ysw is None or top < 1)) \
+            or (y2 is not None and (y is None or y_norm is None or y2_norm is None)):
         raise ValueError(f"rows_update: unsupported call (width {width} of {NP})")
+    if freq is not None and (pos is None or freq.dtype != torch.float64 or freq.numel() < -(-width // 2)
+                             or not freq.is_contiguous()):
+        raise ValueError("rows_update: freq needs pos and fp64 entries for half the width")
     if x_in is not None and x_out is not None and x_in.stride(0) != x_out.stride(0):
         raise ValueError("rows_update: x_in and x_out must share a row stride")
-    ldx = x_in.stride(0) if x_in is not None else (x_out.stride(0) if x_out is not None else 0)
-    y32 = y is None and od == f32 or y is not None and y.dtype == f32
-    check(lib().rows_update(ptr(x_in), ptr(xidx), 0 if x_in is None else x_in.shape[0], ptr(y), ptr(yidx),
-                            0 if y is None else y.shape[0], 0 if y is None else y.stride(0), float(mult), ptr(y_norm),
-                            ptr(x_out), ldx, ptr(copy), 0 if copy is None else copy.stride(0), ptr(norm), ptr(h),
-                            0 if h is None else h.stride(0), M, width, NP, float(eps), int(y32),
-                            int(od == f32), stream_ptr()), "rows_update")
+    a = lib().RowsArgs()
+    a.M, a.N, a.NP, a.mult, a.eps = M, width, NP, float(mult), float(eps)
+    if x_in is not None:
+        a.x_in, a.xidx, a.xrows, a.ldx = ptr(x_in), ptr(xidx), x_in.shape[0], x_in.stride(0)
+    elif x_out is not None:
+        a.ldx = x_out.stride(0)
+    if y is not None:
+        a.y, a.yidx, a.yrows, a.ldy, a.y_w = ptr(y), ptr(yidx), y.shape[0], y.stride(0), ptr(y_norm)
+    if y2 is not None:
+        a.y2, a.y2_w, a.ldy2 = ptr(y2), ptr(y2_norm), y2.stride(0)
+    if ys is not None:
+        a.ys, a.ysi, a.ysw, a.top, a.ldys, a.ysrows = ptr(ys), ptr(ysi), ptr(ysw), top, ys.stride(0), ys.shape[0]
+    if x_add is not None:
+        a.x_add, a.ldadd = ptr(x_add), x_add.stride(0)
+    if freq is not None:
+        a.pos, a.freq = ptr(pos), ptr(freq)
+    a.x_out = ptr(x_out)
+    if copy is not None:
+        a.copy, a.ldcopy = ptr(copy), copy.stride(0)
+    if h is not None:
+        a.n_w, a.n_b, a.n_alpha, a.h, a.ldh = ptr(norm), ptr(norm_b), float(alpha), ptr(h), h.stride(0)
+    y32 = yt is None and od == f32 or yt is not None and yt.dtype == f32
+    check(lib().rows_update(a, int(y32), int(od == f32), stream_ptr()), "rows_update")
 
 
 def linear_f32(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
@@ -109,24 +146,25 @@ class Linear:
 
     __slots__ = ("w", "bias", "ws", "act")
 
-    def __init__(self, w: torch.Tensor, bias: Optional[torch.Tensor], dtype: torch.dtype, device, glu: bool = False,
-                 decode_copy: bool = True):
+    def __init__(self, w: torch.Tensor, bias: Optional[torch.Tensor], dtype: torch.dtype, device,
+                 act: int = G_.ACT_NONE, decode_copy: bool = True):
+        """``act``: none, or a gated activation of a packed weight (``gemm.pack_gate_up``)."""
         self.w = w.to(device=device, dtype=dtype).contiguous()
         self.bias = None if bias is None else bias.to(device=device, dtype=torch.float32).contiguous()
-        self.act = G_.ACT_GELU_TANH_MUL if glu else G_.ACT_NONE
+        self.act = act
         self.ws = G_.shuffle_weight(self.w) if dtype == torch.bfloat16 and decode_copy else None
 
     def __call__(self, x: torch.Tensor, out: torch.Tensor, gws: Optional[torch.Tensor] = None,
                  scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
         """``scratch`` (fp32 gated projections): (M, weight rows) before the activation."""
-        if self.w.dtype == torch.bfloat16:
+        if self.w.dtype == torch.bfloat16:  # ``out`` may be fp32
             return G_.linear(x, self.w, self.bias, self.act, out=out, w_shuf=self.ws, ws=gws)
         if self.act == G_.ACT_NONE:
             return linear_f32(x, self.w, self.bias, out)
         M, F = x.shape[0], self.w.shape[0] // 2
         gu = linear_f32(x, self.w, self.bias, scratch[:M])
         _rows(out, M, F, "gated linear out", (torch.float32,))
-        check(lib().glu_f32(ptr(gu), gu.stride(0), ptr(out), out.stride(0), M, F, stream_ptr()), "glu_f32")
+        check(lib().glu_f32(ptr(gu), gu.stride(0), ptr(out), out.stride(0), M, F, self.act, stream_ptr()), "glu_f32")
         return out
 
 
@@ -158,15 +196,20 @@ def token_gate(x: torch.Tensor, lin: Linear, table: torch.Tensor, off: int, ids:
 
 def paged_args(qkv: torch.Tensor, kp: torch.Tensor, vp: torch.Tensor, table: torch.Tensor, slots: torch.Tensor,
                pos: torch.Tensor, out: torch.Tensor, M: int, H: int, scale: float, window: Optional[int], keep: int,
-               gate: int = -1):
+               gate: int = -1, gate_el: bool = False, kscale: Optional[torch.Tensor] = None,
+               slopes: Optional[torch.Tensor] = None):
     """Validated arguments of the paged-attention launches.
 
     qkv rows ``[q H*DK | k G*DK | v G*DV | ...]``; ``kp`` (pages, G, 64, DK),
     ``vp`` (pages, G, 64, DV); ``table`` (slots, pages per sequence) int32;
     ``slots`` / ``pos`` per row; ``out`` rows ``[H*DV]``; ``gate``: first qkv
-    column of the per-head output gate (-1: none).  Every slot is the caller's:
-    ``0 <= slots[m] < table.shape[0]``."""
-    dt = qkv.dtype
+    column of the output gate, one per head or (``gate_el``) per head and value
+    (-1: none); ``kscale`` (pages, 64): a factor of every key's scores;
+    ``slopes`` (H,): slope * distance is taken off the scaled scores.  ``vp is
+    kp``: the values are the keys, rows have no v columns, and the rows' keys
+    are in the cache already (``mixer_ops.qk_norm``).  Every slot is the
+    caller's: ``0 <= slots[m] < table.shape[0]``."""
+    dt, shared = qkv.dtype, vp is kp
     if kp.dim() != 4 or vp.dim() != 4 or kp.shape[:3] != vp.shape[:3] or kp.shape[2] != PAGE:
         raise ValueError(f"paged attention: pages {tuple(kp.shape)} / {tuple(vp.shape)}")
     if kp.dtype != dt or vp.dtype != dt or out.dtype != dt or not (kp.is_contiguous() and vp.is_contiguous()):
@@ -175,7 +218,7 @@ def paged_args(qkv: torch.Tensor, kp: torch.Tensor, vp: torch.Tensor, table: tor
     DV = vp.shape[3]
     if DK not in HEAD_DIMS or DV not in HEAD_DIMS or H % G:
         raise ValueError(f"paged attention: {H} heads over {G}, sizes {DK} / {DV}")
-    need = max((H + G) * DK + G * DV, gate + H if gate >= 0 else 0)
+    need = max((H + G) * DK + (0 if shared else G * DV), gate + H * (DV if gate_el else 1) if gate >= 0 else 0)
     _rows(qkv, M, need, "paged attention qkv", (torch.float32, torch.bfloat16))
     _rows(out, M, H * DV, "paged attention out", (dt,))
     _index(slots, M, "paged attention slots")
@@ -184,10 +227,16 @@ def paged_args(qkv: torch.Tensor, kp: torch.Tensor, vp: torch.Tensor, table: tor
         raise ValueError("paged attention: block table must be contiguous int32 (slots, pages)")
     if not scale > 0:
         raise ValueError("paged attention: the score scale must be positive")
+    if kscale is not None and (kscale.dtype != torch.float32 or tuple(kscale.shape) != (P, PAGE)
+                               or not kscale.is_contiguous()):
+        raise ValueError("paged attention: kscale must be contiguous fp32 (pages, 64)")
+    _weight(slopes, H, "paged attention slopes")
     keep = min(int(keep), 1 << 30)
-    return lib().PagedAttnArgs(ptr(qkv), qkv.stride(0), ptr(kp), ptr(vp), ptr(table), table.shape[1], P, ptr(slots),
-                               ptr(pos), ptr(out), out.stride(0), M, H, G, DK, DV, gate,
-                               NO_WINDOW if window is None else int(window), keep, float(scale))
+    a = lib().PagedAttnArgs(ptr(qkv), qkv.stride(0), ptr(kp), ptr(vp), ptr(table), table.shape[1], P, ptr(slots),
+                            ptr(pos), ptr(out), out.stride(0), M, H, G, DK, DV, gate,
+                            NO_WINDOW if window is None else int(window), keep, float(scale))
+    a.kscale, a.slopes, a.gate_el, a.shared, a.written = ptr(kscale), ptr(slopes), int(gate_el), int(shared), int(shared)
+    return a
 
 
 def paged_write(args, f32: bool) -> None:

@@ -1,0 +1,230 @@
+"""Wrappers of the recurrent-mixer and mixture-of-experts kernels
+(``csrc/kernels/recurrence.hip``, ``moe.hip``, ``qk_norm.hip``).
+
+Operands are bf16 (serving) or fp32 (exact mode); step sizes, decays, states,
+router logits and weights are fp32 in both.  As in ``decoder_ops``, every shape
+is validated on the host before a launch.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import List, Optional
+
+import torch
+
+from . import gemm as G_
+from ._lib import check, lib, ptr, stream_ptr
+from .decoder_ops import PAGE, _index, _rows, _weight, pad64
+
+STATE_DIMS = (32, 64, 128, 256)  # state rows (key sizes) the recurrence kernels are built for
+CHUNK_TOKENS = 64                # tokens of a chunk on the MFMA (recurrence.hip SC_L)
+EXPERTS_MAX = 256
+
+
+def pad_state(n: int) -> int:
+    for p in STATE_DIMS:
+        if n <= p:
+            return p
+    raise ValueError(f"state size {n} exceeds {STATE_DIMS[-1]}")
+
+
+def _fill(a, **kw):
+    for k, v in kw.items():
+        setattr(a, k, v)
+    return a
+
+
+def _entries(ent: torch.Tensor, n: int) -> None:
+    if ent.dtype != torch.int32 or ent.dim() != 2 or ent.shape[1] != 4 or ent.shape[0] < n or not ent.is_contiguous():
+        raise ValueError("sequence entries: contiguous int32 (n, 4) expected")
+
+
+# ---------------------------------------------------------------------- attention with shared keys = values
+def qk_norm(qkv: torch.Tensor, kp: torch.Tensor, kscale: torch.Tensor, qw: torch.Tensor, table: torch.Tensor,
+            slots: torch.Tensor, pos: torch.Tensor, M: int, H: int, nq: int, nk: int, eps: float, t_every: int = 0,
+            t_coef: float = 0.0) -> None:
+    """Norm of the whole q projection of every row (in place, times ``qw`` =
+    both norm weights, times the query temperature), the keys as projected into
+    their pages and the key norms' factors into ``kscale`` (pages, 64).
+    ``nq`` / ``nk``: true widths of the (zero-padded) projections."""
+    P, G, page, DK = kp.shape
+    f32 = kp.dtype == torch.float32
+    _rows(qkv, M, (H + G) * DK, "qk_norm qkv", (kp.dtype,))
+    _weight(qw, H * DK, "qk_norm weight")
+    _index(slots, M, "qk_norm slots")
+    _index(pos, M, "qk_norm pos")
+    if page != PAGE or not kp.is_contiguous() or kscale.dtype != torch.float32 or tuple(kscale.shape) != (P, PAGE) \
+            or not kscale.is_contiguous() or table.dtype != torch.int32 or not table.is_contiguous():
+        raise ValueError("qk_norm: bad cache pool")
+    a = _fill(lib().QkNormArgs(), qkv=ptr(qkv), kp=ptr(kp), kscale=ptr(kscale), qw=ptr(qw), table=ptr(table),
+              slots=ptr(slots), pos=ptr(pos), ldq=qkv.stride(0), ldt=table.shape[1], npages=P, M=M, H=H, G=G, DK=DK,
+              nq=nq, nk=nk, t_every=t_every, t_coef=t_coef, eps=eps)
+    check(lib().qk_norm(a, int(f32), stream_ptr()), "qk_norm")
+
+
+# ---------------------------------------------------------------------- recurrences
+@dataclass
+class ConvWeights:
+    w: torch.Tensor        # (taps, C) fp32
+    b: torch.Tensor        # (C,) fp32
+    dt_bias: torch.Tensor  # (H,) fp32
+    a_log: torch.Tensor    # (H,) fp32
+
+
+def conv(rows: torch.Tensor, c: ConvWeights, ring: torch.Tensor, out: torch.Tensor, dt: torch.Tensor, la: torch.Tensor,
+         dt_col: int, start: torch.Tensor, slots: torch.Tensor, pos: torch.Tensor, ent: torch.Tensor, n_ent: int,
+         M: int) -> None:
+    """Causal convolution + silu of the first C columns of ``rows`` into
+    ``out``; dt = softplus(column dt_col + h + bias) and la = -exp(a_log) dt per
+    head; then the portions' last inputs into ``ring`` (slots, taps, C)."""
+    T, C = c.w.shape
+    H = c.dt_bias.numel()
+    f32 = rows.dtype == torch.float32
+    _rows(rows, M, max(C, dt_col + H), "conv rows", (torch.float32, torch.bfloat16))
+    _rows(out, M, C, "conv out", (rows.dtype,))
+    _entries(ent, n_ent)
+    for t, n in ((start, M), (slots, M), (pos, M)):
+        _index(t, n, "conv index")
+    for t, n in ((c.w, T * C), (c.b, C), (c.dt_bias, H), (c.a_log, H), (dt, M * H), (la, M * H)):
+        _weight(t, n, "conv weight")
+    if ring.dtype != rows.dtype or tuple(ring.shape[1:]) != (T, C) or not ring.is_contiguous():
+        raise ValueError("conv: bad ring")
+    a = _fill(lib().ConvArgs(), **{"in": ptr(rows)}, w=ptr(c.w), b=ptr(c.b), ring=ptr(ring), out=ptr(out),
+              start=ptr(start), slots=ptr(slots), pos=ptr(pos), dt_bias=ptr(c.dt_bias), a_log=ptr(c.a_log), dt=ptr(dt),
+              la=ptr(la), ldi=rows.stride(0), ldo=out.stride(0), M=M, C=C, taps=T, dt_col=dt_col, H=H,
+              nslots=ring.shape[0])
+    check(lib().conv(a, int(f32), stream_ptr()), "conv")
+    if T > 1:
+        check(lib().conv_state(a, ptr(ent), n_ent, int(f32), stream_ptr()), "conv_state")
+
+
+def scan(rows: torch.Tensor, cols, state: torch.Tensor, y: torch.Tensor, vdim: int, qdiv: int, pos: torch.Tensor,
+         ent: torch.Tensor, n_chunk: int, n_one: int, M: int, *, dt: Optional[torch.Tensor] = None,
+         la: Optional[torch.Tensor] = None, la_h: Optional[torch.Tensor] = None, dt_c: float = 1.0,
+         D: Optional[torch.Tensor] = None) -> None:
+    """The recurrence of every sequence of a step.  ``rows``: q, k, v at columns
+    ``cols``; ``state`` (slots, H, VP, NP) fp32; ``ent``: ``n_chunk`` sequences
+    of two tokens or more, then ``n_one`` of one."""
+    slots, H, VP, NP = state.shape
+    qc, kc, vc = cols
+    f32 = rows.dtype == torch.float32
+    _rows(rows, M, max(vc + H * VP, max(qc, kc) + -(-H // qdiv) * NP), "scan rows", (torch.float32, torch.bfloat16))
+    _rows(y, M, H * vdim, "scan y", (rows.dtype,))
+    _entries(ent, n_chunk + n_one)
+    _index(pos, M, "scan pos")
+    for t, n in ((dt, M * H), (la, M * H), (la_h, H), (D, H)):
+        _weight(t, n, "scan decay")
+    if state.dtype != torch.float32 or not state.is_contiguous() or NP not in STATE_DIMS:
+        raise ValueError(f"scan: bad state {tuple(state.shape)} {state.dtype}")
+    a = _fill(lib().ScanArgs(), rows=ptr(rows), dt=ptr(dt), la=ptr(la), la_h=ptr(la_h), D=ptr(D), state=ptr(state),
+              y=ptr(y), ent=ptr(ent), pos=ptr(pos), ld=rows.stride(0), ldy=y.stride(0), qcol=qc, kcol=kc, vcol=vc,
+              qdiv=qdiv, M=M, H=H, NP=NP, VP=VP, vdim=vdim, nent=n_chunk, nslots=slots, dt_c=dt_c)
+    if f32:
+        a.nent = n_chunk + n_one
+        check(lib().scan_steps(a, 1, stream_ptr()), "scan_steps")
+        return
+    if n_chunk:
+        check(lib().scan_chunks(a, stream_ptr()), "scan_chunks")
+    if n_one:
+        a.ent, a.nent = ptr(ent) + 16 * n_chunk, n_one
+        check(lib().scan_steps(a, 0, stream_ptr()), "scan_steps")
+
+
+def gated_norm(y: torch.Tensor, z: torch.Tensor, out: torch.Tensor, M: int, n: int, groups: int, eps: float,
+               w: Optional[torch.Tensor] = None, gate_first: bool = False) -> None:
+    """``gate_first``: out = norm(y * silu(z)) * w; else norm(y) * silu(z) [* w];
+    the norm runs over ``groups`` equal parts of the n columns."""
+    dt = y.dtype
+    _rows(y, M, n, "gated_norm y", (torch.float32, torch.bfloat16))
+    _rows(z, M, n, "gated_norm z", (dt,))
+    _rows(out, M, n, "gated_norm out", (dt,))
+    _weight(w, n, "gated_norm weight")
+    a = _fill(lib().GatedNormArgs(), y=ptr(y), z=ptr(z), w=ptr(w), out=ptr(out), ldy=y.stride(0), ldz=z.stride(0),
+              ldo=out.stride(0), M=M, n=n, groups=groups, gate_first=int(gate_first), eps=eps)
+    check(lib().gated_norm(a, int(dt == torch.float32), stream_ptr()), "gated_norm")
+
+
+# ---------------------------------------------------------------------- mixture of experts
+class Routing:
+    """Buffers of one step's routing: choices, weights and the rows' places
+    sorted by expert (``order`` place -> row * top + choice, ``place`` its
+    inverse, ``offs`` first place of every expert)."""
+
+    def __init__(self, rows: int, experts: int, top: int, device):
+        z = lambda n, t=torch.int32: torch.zeros((n,), dtype=t, device=device)  # noqa: E731
+        self.rows, self.experts, self.top = rows, experts, top
+        self.idx, self.rank, self.order, self.place = (z(rows * top) for _ in range(4))
+        self.w = z(rows * top, torch.float32)
+        self._sets, self._z = {}, z
+
+    def bins(self, row0: int):
+        """(counts, offs) of the rows from ``row0`` on: concurrent microbatches have their own."""
+        if row0 not in self._sets:
+            self._sets[row0] = (self._z(self.experts), self._z(self.experts + 1))
+        return self._sets[row0]
+
+
+def route(logits: torch.Tensor, r: Routing, M: int, groups: int, keep: int, row0: int = 0) -> None:
+    """Choices of M rows; the results start at entry ``row0 * top`` of the buffers."""
+    _rows(logits, M, r.experts, "route logits", (torch.float32,))
+    if row0 + M > r.rows:
+        raise ValueError(f"route: rows {row0} .. {row0 + M} of {r.rows}")
+    o = 4 * row0 * r.top
+    counts, offs = r.bins(row0)
+    a = _fill(lib().RouteArgs(), logits=ptr(logits), idx=ptr(r.idx) + o, w=ptr(r.w) + o, rank=ptr(r.rank) + o,
+              counts=ptr(counts), order=ptr(r.order) + o, place=ptr(r.place) + o, offs=ptr(offs),
+              ldl=logits.stride(0), M=M, E=r.experts, groups=groups, keep=keep, top=r.top)
+    check(lib().route(a, stream_ptr()), "route")
+
+
+class ExpertLinear:
+    """One projection of every expert: bf16 weights in fragment order only (the
+    tile kernel of many rows and the streaming kernel of few read the same
+    copy), or fp32 weights row-major.  Rows of N and K are padded to multiples
+    of 64 by the caller; gated projections come packed (``gemm.pack_gate_up``)."""
+
+    def __init__(self, ws: List[torch.Tensor], dtype: torch.dtype, device, act: int = G_.ACT_NONE):
+        self.E, (self.N, self.K) = len(ws), ws[0].shape
+        if self.N % 64 or self.K % 64 or any(w.shape != ws[0].shape for w in ws):
+            raise ValueError(f"ExpertLinear: {self.N} x {self.K}")
+        self.act, self.dtype = act, dtype
+        if dtype == torch.bfloat16:
+            self.w = torch.empty((self.E, self.N * self.K * 2), dtype=torch.uint8, device=device)
+            for e, w in enumerate(ws):
+                self.w[e].copy_(G_.shuffle_weight(w.to(device=device, dtype=dtype)))
+        else:
+            self.w = torch.stack([w.to(device=device, dtype=dtype) for w in ws]).contiguous()
+
+    @property
+    def n_out(self) -> int:
+        return self.N // 2 if self.act in G_.ACTS_GLU else self.N
+
+    def __call__(self, x: torch.Tensor, rows: int, out: torch.Tensor, r: Routing, gather: int = 0, row0: int = 0,
+                 scratch: Optional[torch.Tensor] = None, clear: bool = False) -> torch.Tensor:
+        """Products of ``rows`` places.  ``gather``: 0 = ``x`` rows are places,
+        else ``x`` row = order[place] / gather.  ``clear``: leave the counters zero."""
+        _rows(x, rows // gather if gather else rows, self.K, "expert rows", (self.dtype,))
+        _rows(out, rows, self.n_out, "expert out", (self.dtype,))
+        f32 = self.dtype == torch.float32
+        c = scratch if f32 and self.act != G_.ACT_NONE else out
+        if f32:
+            _rows(c, rows, self.N, "expert scratch", (self.dtype,))
+        counts, offs = r.bins(row0)
+        a = _fill(lib().GroupedArgs(), A=ptr(x), C=ptr(c), offs=ptr(offs),
+                  order=ptr(r.order) + 4 * row0 * r.top if gather else 0, counts=ptr(counts) if clear else 0,
+                  lda=x.stride(0), ldc=c.stride(0), rows=rows, arows=rows // gather if gather else rows,
+                  div=max(gather, 1), N=self.N, K=self.K, E=self.E, act=self.act)
+        if f32:
+            a.W = ptr(self.w)
+            check(lib().grouped_gemm_f32(a, stream_ptr()), "grouped_gemm_f32")
+            if c is not out:
+                F = self.n_out
+                check(lib().glu_f32(ptr(c), c.stride(0), ptr(out), out.stride(0), rows, F, self.act, stream_ptr()), "glu_f32")
+            return out
+        a.Wsh = ptr(self.w)
+        check(lib().grouped_gemm(a, stream_ptr()), "grouped_gemm")
+        return out
+
+
+__all__ = ["qk_norm", "ConvWeights", "conv", "scan", "gated_norm", "Routing", "route", "ExpertLinear", "pad_state",
+           "pad64", "STATE_DIMS", "CHUNK_TOKENS"]

@@ -1,8 +1,9 @@
-"""Decoder stages with an fp32 residual over a paged KV cache (Kozusun).
+"""Decoder stages with an fp32 residual over paged caches and recurrent states
+(the families of ``models.DECODERS``).
 
-A stage runs a range of layer *runs* (``models/kozusun.py``; a looped layer
-counts once per pass and has a cache per pass, its weights are shared).  One
-forward pass serves both callers:
+A stage runs a range of layer *runs* (a looped layer counts once per pass; every
+run has its own cache or state, weights are shared).  What a layer is made of is
+in ``runtime/decoder_layers.py``.  One forward pass serves both callers:
 
 * ``step_batch(StepBatch)`` — the engine's step (``runtime/engine.py``): tokens
   of any number of sequences, portions of prompts beside single tokens;
@@ -11,17 +12,11 @@ forward pass serves both callers:
   [b0, b0 + B), each with its own fixed pages, so a decode step is one HIP
   graph whose positions live on the device.
 
-Launches per layer run (bf16): q|k|v|gate projection; gate|up projection with
-the tanh-GELU product in its epilogue; attention (decode: cache write, attention
-and output gate in one launch; prefill: cache write, then flash attention) —
-both sublayers write one row ``[attention | feed-forward]``, so ONE projection
-with the two output matrices side by side gives their sum; residual update;
-token-input gate (projection, activation and product with the token's row in one
-launch) and its output projection; residual update + the next run's norm in one
-pass.  The residual, norms, scores and softmax are fp32.
-
-``dtype="float32"`` runs the same sequence with fp32 weights, activations,
-cache and matrix products (``ops/decoder_ops.py``).
+Keys live in pages (``runtime/paging.py``), recurrent states by slot; a portion
+that begins at position 0 starts from a zero state.  The residual, norms,
+scores, softmax, routers and everything of a recurrence but its projections are
+fp32.  ``dtype="float32"`` runs the same sequence with fp32 weights,
+activations, cache and matrix products (``ops/decoder_ops.py``).
 
 Stage boundary: rows ``[residual | token id | padding]`` of fp32 (the token id
 as its bits): later stages need the tokens for their per-layer inputs, and the
@@ -29,73 +24,23 @@ embedding output at a loop's entry.
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, List, Optional
 
 import torch
 
-from ..models import kozusun, model_info
+from ..models import DECODERS, model_info
 from ..ops import decoder_ops as D_
+from ..ops import mixer_ops as M_
 from ..ops import transformer_ops as T_
-from ..ops.gemm import decode_workspace, pack_gate_up
-from .paging import PAGE, StepBatch, pages_for
+from ..ops.gemm import decode_workspace
+from .decoder_layers import LAYERS, DynamicTanh, Weights, pad
+from .paging import StepBatch, pages_for
 from .stages import StageCompute, StageOutput
 
 DTYPES = {None: torch.bfloat16, "bf16": torch.bfloat16, "bfloat16": torch.bfloat16, "fp32": torch.float32,
           "float32": torch.float32}
 HOP_IDS = 4  # fp32 columns after the residual at a stage boundary: the token id's bits, padding
-
-
-def _pad(t: torch.Tensor, *shape: int) -> torch.Tensor:
-    """``t`` in the leading corner of a zero tensor of ``shape``."""
-    if tuple(t.shape) == shape:
-        return t
-    out = t.new_zeros(shape)
-    out[tuple(slice(0, n) for n in t.shape)] = t
-    return out
-
-
-def _pad_heads(w: torch.Tensor, heads: int, dim: int, to: int) -> torch.Tensor:
-    """Rows of ``heads`` groups of ``dim`` -> groups of ``to``, zeros between."""
-    w = w.view(heads, dim, *w.shape[1:])
-    return _pad(w, heads, to, *w.shape[2:]).reshape(heads * to, *w.shape[2:])
-
-
-class DecoderLayer:
-    """Packed weights of one layer."""
-
-    def __init__(self, cfg: kozusun.KozusunConfig, i: int, sd: Dict[str, torch.Tensor], dtype, device, wp: int):
-        L, m = cfg.layers[i], cfg.layers[i].mixer
-        self.mix, self.ff = m, L.ff
-        self.dk, self.dv = D_.pad_dim(m.dim), D_.pad_dim(m.vdim)
-        self.group = m.heads // m.kv_heads
-        ld = lambda n: sd[f"l{i}.{n}"].to(device=device, dtype=torch.float32)  # noqa: E731
-        lin = lambda w, b=None, glu=False: D_.Linear(w, b, dtype, device, glu)  # noqa: E731
-        self.norm1 = _pad(1 + ld("norm1"), wp)
-        self.norm1[cfg.n_embd:] = 0
-        heads = ((m.heads, m.dim, self.dk, "q"), (m.kv_heads, m.dim, self.dk, "k"), (m.kv_heads, m.vdim, self.dv, "v"))
-        w = [_pad_heads(_pad(ld(f"mix.{n}"), h * d, wp), h, d, p) for h, d, p, n in heads]
-        b = [_pad_heads(ld(f"mix.{n}.b"), h, d, p) for h, d, p, n in heads]
-        self.gate_col = sum(t.shape[0] for t in w)
-        n = self.gate_col + m.heads
-        self.n_qkv = -(-n // 16) * 16
-        self.w_qkv = lin(_pad(torch.cat(w + [_pad(ld("mix.g"), m.heads, wp)]), self.n_qkv, wp),
-                         _pad(torch.cat(b), self.n_qkv))
-        wo = ld("mix.o").view(cfg.n_embd, m.heads, m.vdim)
-        outs = [_pad(_pad(wo, cfg.n_embd, m.heads, self.dv).reshape(cfg.n_embd, -1), wp, m.heads * self.dv)]
-        self.n_att, self.n_ff = m.heads * self.dv, 0
-        self.w_up = None
-        if L.ff is not None:
-            self.n_ff = D_.pad64(L.ff)
-            self.w_up = lin(pack_gate_up(_pad(ld("mlp.gate"), self.n_ff, wp), _pad(ld("mlp.up"), self.n_ff, wp)),
-                            glu=True)
-            outs.append(_pad(ld("mlp.down"), wp, self.n_ff))
-        self.w_out = lin(torch.cat(outs, 1))
-        self.side_off = i * cfg.side_dim
-        if cfg.side_dim:
-            sp = D_.pad64(cfg.side_dim)
-            self.w_sgate = lin(_pad(ld("side.gate"), sp, wp))
-            self.w_sproj = lin(_pad(ld("side.proj"), wp, sp))
-            self.side_norm = _pad(ld("side.norm"), wp)
 
 
 class DecoderStage(StageCompute):
@@ -104,15 +49,16 @@ class DecoderStage(StageCompute):
     def __init__(self, model: str, sd: Dict[str, torch.Tensor], start: int, end: int, first: bool, last: bool,
                  device, max_batch: int = 8, max_seq: int = 1024, max_tokens: Optional[int] = None,
                  dtype: Optional[str] = None, temperature: float = 0.0, top_k: int = 0, seed: int = 0,
-                 num_pages: Optional[int] = None, cfg: Optional[kozusun.KozusunConfig] = None):
+                 num_pages: Optional[int] = None, cfg=None, num_slots: Optional[int] = None):
         """``max_batch`` x ``max_seq``: the ring's cache rows (and the default
-        ``num_pages``).  ``num_pages``: the page pool of an engine.  ``max_tokens``:
-        rows of one step.  ``cfg`` overrides the registry's configuration."""
+        ``num_pages`` / ``num_slots``).  ``num_pages``: the page pool of an
+        engine, ``num_slots``: its sequences' states.  ``max_tokens``: rows of
+        one step.  ``cfg`` overrides the registry's configuration."""
         if dtype not in DTYPES:
             raise ValueError(f"dtype {dtype!r}: this model runs in bf16 or float32")
         self.model = model
         self.cfg = c = cfg if cfg is not None else model_info(model).cfg
-        self.family = "kozusun"
+        self.family = next(f for f, mod in DECODERS.items() if type(c).__module__ == mod.__name__)
         self.start, self.end, self.first, self.last = start, end, first, last
         self.device = dev = torch.device(device)
         if dev.type != "cuda":
@@ -123,32 +69,45 @@ class DecoderStage(StageCompute):
         self.max_batch, self.max_seq = max_batch, max_seq
         self.row_pages = pages_for(max_seq)
         self.num_pages = num_pages or max_batch * self.row_pages
+        self.num_slots = max(num_slots or 0, max_batch)
         self.max_tokens = max(max_tokens or max_batch * max_seq, max_batch)
         self.width, self.wp = c.n_embd, D_.pad64(c.n_embd)
         self.V = c.vocab_size
         self.Vpad = D_.pad64(self.V)
-        self.eps, self.mult = c.norm_eps, c.residual_mult
+        self.eps, self.mult = c.norm_eps, getattr(c, "residual_mult", 1.0)
         self.runs = c.runs[start:end + 1]
         self.side = c.side_dim
         self.enters = any(r.enters for r in self.runs)
+        koz = self.family == "kozusun"
+        self.entry_projects = koz  # a loop's entry: a projection of [x | x0], or the sum x + x0
+        self.embed_mult = c.embed_scale if koz else 1.0
 
         def table(name, cols):  # gathered rows; columns padded so every row is aligned
             t = sd[name].to(device=dev, dtype=dt)
-            return _pad(t, t.shape[0], cols).contiguous()
+            return pad(t, t.shape[0], cols).contiguous()
         self.embed = table("embed", self.wp) if (first or self.enters) else None
+        self.freq: Optional[torch.Tensor] = None  # sinusoidal position vector: turns per position
+        if not koz:
+            i = torch.arange(-(-self.width // 2), dtype=torch.float64)
+            self.freq = (10000.0 ** (-2.0 * i / self.width) / (2.0 * math.pi)).to(dev)
         if self.side:
             self.side_embed = sd["side.embed"].to(device=dev, dtype=dt).contiguous()
-        if self.enters:
+        if self.enters and self.entry_projects:
             w = sd["loop.in"].to(device=dev, dtype=torch.float32)
-            w = torch.cat([_pad(w[:, :self.width], self.wp, self.wp), _pad(w[:, self.width:], self.wp, self.wp)], 1)
+            w = torch.cat([pad(w[:, :self.width], self.wp, self.wp), pad(w[:, self.width:], self.wp, self.wp)], 1)
             self.w_loop = D_.Linear(w, None, dt, dev)
-        layers = {i: DecoderLayer(c, i, sd, dt, dev, self.wp) for i in sorted({r.layer for r in self.runs})}
-        self.layers: List[DecoderLayer] = [layers[r.layer] for r in self.runs]
+        layers = {i: LAYERS[self.family](c, i, sd, dt, dev) for i in sorted({r.layer for r in self.runs})}
+        self.layers: List = [layers[r.layer] for r in self.runs]
         if last:
-            self.final_norm = _pad(1 + sd["final.norm"].to(device=dev, dtype=torch.float32), self.wp)
-            self.final_norm[self.width:] = 0
-            self.w_head = D_.Linear(_pad(sd["head"].to(device=dev, dtype=torch.float32), self.V, self.wp), None, dt, dev)
-        self.groups = sorted({L.group for L in self.layers})
+            ld = Weights(c, "", sd, dt, dev)
+            if koz:
+                w = pad(1 + ld("final.norm"), self.wp)
+                w[self.width:] = 0
+                self.final_norm = {"norm": w}
+            else:
+                self.final_norm = DynamicTanh(ld, "final.norm").prep(None)
+            self.w_head = ld.linear(ld.rows("head", self.V))
+        self.groups = sorted({g for L in self.layers for g in L.groups})
         self._alloc()
         self._ring: Dict[tuple, dict] = {}
         self._ring_table: Optional[torch.Tensor] = None
@@ -160,20 +119,25 @@ class DecoderStage(StageCompute):
         self.x = z(self.wp, torch.float32)
         self.cat = z(2 * self.wp)                     # [residual copy | embedding output]
         self.h, self.y = z(self.wp), z(self.wp)
-        self.qkv = z(max(L.n_qkv for L in self.layers))
-        self.af = z(max(L.n_att + L.n_ff for L in self.layers))
-        ff = max(L.n_ff for L in self.layers)
-        self.gu = z(2 * ff) if self.f32 and ff else None
+        # scratch rows by name, as wide as the widest layer asks for
+        cols: Dict[str, int] = {}
+        for L in self.layers:
+            for k, v in L.buffers(self.f32).items():
+                cols[k] = max(cols.get(k, 0), self.wp if v is None else v)
+        self.buf = {k: z(v, torch.float32 if k in ("dt", "la", "router") else dt) for k, v in cols.items() if v}
+        self._experts: Dict[tuple, M_.Routing] = {}
+        self._expert_rows: Dict[str, torch.Tensor] = {}
         if self.side:
             self.g = z(D_.pad64(self.side))
             self.z = z(D_.pad64(self.side)) if self.f32 else None
         if self.enters:
-            self.y32 = self.y if self.f32 else z(self.wp, torch.float32)
+            if self.entry_projects:
+                self.y32 = self.y if self.f32 else z(self.wp, torch.float32)
+            else:
+                self.x0 = z(self.wp, torch.float32)
         if not self.first:
             self.ids_in = torch.zeros((n,), dtype=torch.int32, device=dev)
-        P = self.num_pages
-        self.pages = [(torch.zeros((P, L.mix.kv_heads, PAGE, L.dk), dtype=dt, device=dev),
-                       torch.zeros((P, L.mix.kv_heads, PAGE, L.dv), dtype=dt, device=dev)) for L in self.layers]
+        self.caches = [L.new_cache(self) for L in self.layers]
         if self.last:
             self.hn = z(self.wp)
             self.logits = torch.zeros((max(self.max_batch, 1), self.Vpad), dtype=dt, device=dev)
@@ -181,6 +145,30 @@ class DecoderStage(StageCompute):
             self.amx_part = torch.empty((max(self.max_batch, 1) * 2 * T_.ARGMAX_PART_PER_ROW,), dtype=torch.int32,
                                         device=dev)
         self.ws: Optional[torch.Tensor] = None        # decode-attention partials (engine steps)
+
+    def flat(self, name: str, s: slice, cols: int) -> torch.Tensor:
+        """Rows ``s`` of a scratch buffer as dense rows of ``cols`` (buffers of
+        concurrent microbatches do not overlap: a row has at least ``cols``)."""
+        w = self.buf[name].shape[1]
+        return self.buf[name].view(-1)[s.start * w:s.start * w + (s.stop - s.start) * cols]
+
+    def experts(self, experts: int, top: int, ff: int):
+        """Routing buffers, and the rows of (token, choice) between and after the experts' projections."""
+        key, rows = (experts, top), self.max_tokens * top
+        if key not in self._experts:
+            self._experts[key] = M_.Routing(self.max_tokens, experts, top, self.device)
+        return self._experts[key], self._grown("up", rows, ff), self._grown("down", rows, self.wp)
+
+    def expert_scratch(self, cols: int, s: slice) -> torch.Tensor:
+        return self._grown("gu", s.stop, cols)[s, :cols]
+
+    def _grown(self, name: str, rows: int, cols: int) -> torch.Tensor:
+        t = self._expert_rows.get(name)
+        if t is None or t.shape[0] < rows or t.shape[1] < cols:
+            have = (0, 0) if t is None else t.shape
+            t = self._expert_rows[name] = torch.zeros((max(rows, have[0]), max(cols, have[1])), dtype=self.dtype,
+                                                      device=self.device)
+        return t
 
     # ------------------------------------------------------------------ specs
     @property
@@ -199,10 +187,25 @@ class DecoderStage(StageCompute):
         """Greedy last stage: the argmax launch writes the next input ids and advances the positions."""
         return self.last and not self.temperature > 0
 
+    def _cache_tensors(self):
+        for c in self.caches:
+            yield from ((k, t) for k, t in (c.items() if isinstance(c, dict) else zip(("kp", "vp"), c)))
+
     def reset(self):
-        for k, v in self.pages:
-            k.zero_()
-            v.zero_()
+        for _, t in self._cache_tensors():
+            t.zero_()
+
+    def save_states(self) -> List[torch.Tensor]:
+        """Copies of the recurrent states (a step that is run twice advances them twice)."""
+        return [t.clone() for k, t in self._cache_tensors() if k in ("state", "ring")]
+
+    def restore_states(self, saved: List[torch.Tensor]) -> None:
+        for t, v in zip((t for k, t in self._cache_tensors() if k in ("state", "ring")), saved):
+            t.copy_(v)
+
+    @property
+    def recurrent(self) -> bool:
+        return any(k == "state" for k, _ in self._cache_tensors())
 
     # ------------------------------------------------------------------ layers
     def _prep(self, k: int, r0: int, M: int) -> dict:
@@ -210,70 +213,42 @@ class DecoderStage(StageCompute):
         s = slice(r0, r0 + M)
         if k == len(self.runs):
             return {}
-        if self.runs[k].enters:
+        if not self.runs[k].enters:
+            return self.layers[k].prep(self.h[s])
+        if self.entry_projects:
             return {"copy": self.cat[s, :self.wp]}
-        return {"norm": self.layers[k].norm1, "h": self.h[s]}
-
-    def _splits(self, L: DecoderLayer, n: int, keys: int) -> int:
-        m = L.mix
-        return D_.paged_splits(n, m.heads, m.kv_heads, keys, m.window, m.keep_first)
+        return {"x_add": self.x0[s], **self.layers[k].prep(self.h[s])}
 
     def _ws_need(self, n: int, keys: int) -> int:
         """fp32 partials the decode launches of ``n`` sequences need."""
-        return max((n * L.mix.heads * s * (L.dv + 2) for L in self.layers
-                    for s in [self._splits(L, n, keys)] if s > 1), default=0)
-
-    def _attention(self, k: int, b: StepBatch, qkv: torch.Tensor, out: torch.Tensor, ws) -> None:
-        L, (kp, vp), m = self.layers[k], self.pages[k], self.layers[k].mix
-        args = D_.paged_args(qkv, kp, vp, b.table, b.slots, b.pos, out, b.M, m.heads, m.scale, m.window, m.keep_first,
-                             L.gate_col)
-        if self.f32:
-            D_.paged_write(args, True)
-            D_.paged_attn_f32(args)
-            return
-        if b.chunks:
-            D_.paged_write(args, False)
-            D_.paged_prefill(args, b.tiles[L.group])
-        if b.n_dec:
-            D_.paged_decode(args, b.dec_rows, b.n_dec, self._splits(L, b.n_dec, b.max_len), ws)
+        return max((L.ws_need(n, keys) for L in self.layers), default=0)
 
     def _layers(self, b: StepBatch, ids: torch.Tensor, r0: int, gws, ws) -> None:
         """Residual rows [r0, r0 + M) through this stage's runs (``self.x`` holds
         the incoming residual on a later stage)."""
         M, wp, w, s = b.M, self.wp, self.width, slice(r0, r0 + b.M)
-        x, h, y, xc = self.x[s], self.h[s], self.y[s], self.cat[s, :self.wp]
+        x = self.x[s]
         up = lambda **kw: D_.rows_update(M, w, eps=self.eps, **kw)  # noqa: E731
-        if self.enters:  # the embedding output, kept for the loop's passes
-            up(y=self.embed, yidx=ids, mult=self.cfg.embed_scale, x_out=x if self.first else None,
-               copy=self.cat[s, wp:])
+        emb = {"y": self.embed, "yidx": ids, "mult": self.embed_mult}
+        if self.freq is not None:
+            emb.update(pos=b.pos, freq=self.freq)
+        if not self.enters:
+            up(**(dict(emb, x_out=x) if self.first else {"x_in": x}), **self._prep(0, r0, M))
+        elif self.entry_projects:  # the embedding output, kept for the loop's passes
+            up(**emb, x_out=x if self.first else None, copy=self.cat[s, wp:])
             up(x_in=x, **self._prep(0, r0, M))
-        elif self.first:
-            up(y=self.embed, yidx=ids, mult=self.cfg.embed_scale, x_out=x, **self._prep(0, r0, M))
         else:
-            up(x_in=x, **self._prep(0, r0, M))
+            up(**emb, x_out=self.x0[s])
+            up(x_in=self.x0[s] if self.first else x, x_out=x, **self._prep(0, r0, M))
         for k, (run, L) in enumerate(zip(self.runs, self.layers)):
-            if run.enters:
-                up(y=self.w_loop(self.cat[s], self.y32[s], gws), x_out=x, norm=L.norm1, h=h)
-            qkv = self.qkv[s, :L.n_qkv]
-            af = self.af[s, :L.n_att + L.n_ff]
-            L.w_qkv(h, qkv, gws)
-            if L.w_up is not None:
-                L.w_up(h, af[:, L.n_att:], gws, None if self.gu is None else self.gu[:, :2 * L.n_ff])
-            self._attention(k, b, qkv, af[:, :L.n_att], ws)
-            L.w_out(af, y, gws)
-            nxt = self._prep(k + 1, r0, M)
-            if not self.side:
-                up(x_in=x, y=y, mult=self.mult, x_out=x, **nxt)
-                continue
-            up(x_in=x, y=y, mult=self.mult, x_out=x, copy=xc)
-            D_.token_gate(xc, L.w_sgate, self.side_embed, L.side_off, ids, self.g[s], self.side, self.z)
-            L.w_sproj(self.g[s], y, gws)
-            up(x_in=x, y=y, mult=self.mult, y_norm=L.side_norm, x_out=x, **nxt)
+            if run.enters and self.entry_projects:
+                up(y=self.w_loop(self.cat[s], self.y32[s], gws), x_out=x, **L.prep(self.h[s]))
+            L.run(self, self.caches[k], b, ids, s, gws, ws, self._prep(k + 1, r0, M), up)
 
     def _head(self, r0: int, M: int, rows: torch.Tensor, n: int, logits: torch.Tensor, gws=None) -> torch.Tensor:
         """Logits of ``n`` rows (``rows``: their places among the M of the step)."""
         hn = self.hn[r0:r0 + n]
-        D_.rows_update(n, self.width, x_in=self.x[r0:r0 + M], xidx=rows, norm=self.final_norm, h=hn, eps=self.eps)
+        D_.rows_update(n, self.width, x_in=self.x[r0:r0 + M], xidx=rows, eps=self.eps, **dict(self.final_norm, h=hn))
         self.w_head(hn, logits[:, :self.V], gws)
         return logits
 
@@ -339,7 +314,10 @@ class DecoderStage(StageCompute):
         c = self._ring.get((B, T, b0))
         if c is None:
             slots = torch.arange(b0, b0 + B, dtype=torch.int32, device=dev)
-            c = {"slots": slots.repeat_interleave(T).contiguous(),
+            first = torch.arange(0, B * T, T, dtype=torch.int32, device=dev)
+            ent = torch.stack([first, torch.full_like(first, T), slots, torch.zeros_like(first)], 1).contiguous()
+            c = {"slots": slots.repeat_interleave(T).contiguous(), "ent": ent,
+                 "start": first.repeat_interleave(T).contiguous(),
                  "last": torch.arange(T - 1, B * T, T, dtype=torch.int32, device=dev),
                  "rows": torch.arange(B * T, dtype=torch.int32, device=dev), "chunks": [], "tiles": None}
             if T > 1:
@@ -351,7 +329,7 @@ class DecoderStage(StageCompute):
         p = pos if T == 1 else (pos.view(B, 1) + c["steps"]).view(-1).contiguous()
         return StepBatch(M=B * T, pos=p, slots=c["slots"], table=self._ring_table,
                          dec_rows=c["rows"] if T == 1 else None, n_dec=B if T == 1 else 0, chunks=c["chunks"],
-                         max_len=self.max_seq, tiles=c["tiles"])
+                         max_len=self.max_seq, ent=c["ent"], start=c["start"], tiles=c["tiles"])
 
     def step(self, x: torch.Tensor, pos: torch.Tensor, B: int, T: int, b0: int = 0,
              out: Optional[torch.Tensor] = None, last_only: bool = True, advance=None):

@@ -1,0 +1,412 @@
+"""Layers of the paged decoder stages (``runtime/decoder.py``): packed weights,
+the caches or states of a layer run, and its launches.
+
+A *layer* holds the weights of one layer of the model; a layer that runs several
+times (a loop) has one object and a cache per run (``new_cache``).  It describes
+what it needs (``buffers``: scratch columns by name, ``groups``: query heads per
+KV head) and adds its launches in ``run``, which reads the normed input from
+``st.h`` and leaves the updated residual in ``st.x`` together with what the next
+run asks for (``nxt``, keyword arguments of ``rows_update``).
+
+* ``JointLayer`` (Kozusun): attention and feed-forward side by side behind one
+  norm, one output projection for both.
+* ``SequentialLayer`` (Funepel): a mixer, then a mixture of experts, each behind
+  a norm of its own.
+  ``Mamba2Mixer``: convolution and state-space recurrence, state by slot.
+  ``AttentionRetentionMixer``: paged attention whose values are its keys, and a
+  retention state, on the same input, by one projection.
+* ``TokenInput``: the per-layer input looked up by token, shared by both.
+
+All padding happens here, once: widths, feed-forward and side sizes to multiples
+of 64, attention heads to 64 / 128 / 256, states to 32 / 64 / 128 / 256 x
+multiples of 64, with zeros, so kernels see aligned shapes.
+"""
+from __future__ import annotations
+
+import math
+from typing import Dict, List, Optional
+
+import torch
+
+from ..models import funepel
+from ..ops import decoder_ops as D_
+from ..ops import mixer_ops as M_
+from ..ops.gemm import ACT_GELU_TANH_MUL, ACT_SILU_MUL, pack_gate_up
+from .paging import PAGE, StepBatch
+
+
+def pad(t: torch.Tensor, *shape: int) -> torch.Tensor:
+    """``t`` in the leading corner of a zero tensor of ``shape``."""
+    if tuple(t.shape) == shape:
+        return t
+    out = t.new_zeros(shape)
+    out[tuple(slice(0, n) for n in t.shape)] = t
+    return out
+
+
+def pad_heads(w: torch.Tensor, heads: int, dim: int, to: int) -> torch.Tensor:
+    """Rows of ``heads`` groups of ``dim`` -> groups of ``to``, zeros between."""
+    w = w.reshape(heads, dim, *w.shape[1:])
+    return pad(w, heads, to, *w.shape[2:]).reshape(heads * to, *w.shape[2:])
+
+
+def pad16(n: int) -> int:
+    return -(-n // 16) * 16
+
+
+class Weights:
+    """A layer's tensors as padded fp32 on the device, and packed projections."""
+
+    def __init__(self, cfg, prefix: str, sd: Dict[str, torch.Tensor], dtype, device):
+        self.cfg, self.prefix, self.sd, self.dtype, self.device = cfg, prefix, sd, dtype, device
+        self.width, self.wp = cfg.n_embd, D_.pad64(cfg.n_embd)
+
+    def sub(self, name: str) -> "Weights":
+        return Weights(self.cfg, self.prefix + name, self.sd, self.dtype, self.device)
+
+    def __call__(self, name: str) -> torch.Tensor:
+        return self.sd[self.prefix + name].to(device=self.device, dtype=torch.float32)
+
+    def has(self, name: str) -> bool:
+        return self.prefix + name in self.sd
+
+    def rows(self, name: str, n: int) -> torch.Tensor:
+        """A projection from the width: (n padded rows, padded width)."""
+        return pad(self(name), n, self.wp)
+
+    def vec(self, name: str) -> torch.Tensor:
+        return pad(self(name), self.wp)
+
+    def linear(self, w: torch.Tensor, bias=None, act: int = 0) -> D_.Linear:
+        return D_.Linear(w, bias, self.dtype, self.device, act)
+
+    def gate_up(self, n: int) -> torch.Tensor:
+        return pack_gate_up(self.rows("gate", n), self.rows("up", n))
+
+
+class TokenInput:
+    """y = W_proj (gelu_tanh(W_gate x) * the layer's part of the token's row), RMS-normed."""
+
+    def __init__(self, ld: Weights, i: int, dim: int):
+        sp = D_.pad64(dim)
+        self.off = i * dim
+        self.w_gate, self.w_proj = ld.linear(ld.rows("gate", sp)), ld.linear(pad(ld("proj"), ld.wp, sp))
+        self.norm = ld.vec("norm")
+
+    def run(self, st, s: slice, ids, gws, nxt: dict, up) -> None:
+        """The residual's copy is in ``st.cat``; the update prepares ``nxt``."""
+        x, y = st.x[s], st.y[s]
+        D_.token_gate(st.cat[s, :st.wp], self.w_gate, st.side_embed, self.off, ids, st.g[s], st.side, st.z)
+        self.w_proj(st.g[s], y, gws)
+        up(x_in=x, y=y, mult=st.mult, y_norm=self.norm, x_out=x, **nxt)
+
+
+def attention_cache(st, heads: int, dk: int, dv: Optional[int]):
+    """Key and value page pools (``dv`` None: keys only)."""
+    z = lambda d: torch.zeros((st.num_pages, heads, PAGE, d), dtype=st.dtype, device=st.device)  # noqa: E731
+    return z(dk), None if dv is None else z(dv)
+
+
+def run_attention(st, args, b: StepBatch, group: int, splits: int, ws, write: bool = True) -> None:
+    """The attention launches of one step: fp32, or bf16 portions and single tokens."""
+    if st.f32:
+        if write:
+            D_.paged_write(args, True)
+        D_.paged_attn_f32(args)
+        return
+    if b.chunks:
+        if write:
+            D_.paged_write(args, False)
+        D_.paged_prefill(args, b.tiles[group])
+    if b.n_dec:
+        D_.paged_decode(args, b.dec_rows, b.n_dec, splits, ws)
+
+
+# ---------------------------------------------------------------------- Kozusun
+class JointLayer:
+    """Attention and feed-forward on one normed input, one projection for their sum."""
+
+    def __init__(self, cfg, i: int, sd: Dict[str, torch.Tensor], dtype, device):
+        ld = Weights(cfg, f"l{i}.", sd, dtype, device)
+        L, m, wp = cfg.layers[i], cfg.layers[i].mixer, ld.wp
+        self.mix, self.ff = m, L.ff
+        self.dk, self.dv = D_.pad_dim(m.dim), D_.pad_dim(m.vdim)
+        self.group = m.heads // m.kv_heads
+        self.groups = [self.group]
+        self.norm1 = pad(1 + ld("norm1"), wp)
+        self.norm1[cfg.n_embd:] = 0
+        heads = ((m.heads, m.dim, self.dk, "q"), (m.kv_heads, m.dim, self.dk, "k"), (m.kv_heads, m.vdim, self.dv, "v"))
+        w = [pad_heads(ld.rows(f"mix.{n}", h * d), h, d, p) for h, d, p, n in heads]
+        b = [pad_heads(ld(f"mix.{n}.b"), h, d, p) for h, d, p, n in heads]
+        self.gate_col = sum(t.shape[0] for t in w)
+        self.n_qkv = pad16(self.gate_col + m.heads)
+        self.w_qkv = ld.linear(pad(torch.cat(w + [ld.rows("mix.g", m.heads)]), self.n_qkv, wp),
+                               pad(torch.cat(b), self.n_qkv))
+        wo = ld("mix.o").view(cfg.n_embd, m.heads, m.vdim)
+        outs = [pad(pad(wo, cfg.n_embd, m.heads, self.dv).reshape(cfg.n_embd, -1), wp, m.heads * self.dv)]
+        self.n_att, self.n_ff = m.heads * self.dv, 0
+        self.w_up = None
+        if L.ff is not None:
+            self.n_ff = D_.pad64(L.ff)
+            self.w_up = ld.linear(ld.sub("mlp.").gate_up(self.n_ff), act=ACT_GELU_TANH_MUL)
+            outs.append(pad(ld("mlp.down"), wp, self.n_ff))
+        self.w_out = ld.linear(torch.cat(outs, 1))
+        self.side = TokenInput(ld.sub("side."), i, cfg.side_dim) if cfg.side_dim else None
+
+    def prep(self, h: torch.Tensor) -> dict:
+        """What the residual update before a run of this layer also produces."""
+        return {"norm": self.norm1, "h": h}
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        b = {"qkv": self.n_qkv, "af": self.n_att + self.n_ff}
+        if f32 and self.n_ff:
+            b["gu"] = 2 * self.n_ff
+        return b
+
+    def new_cache(self, st):
+        return attention_cache(st, self.mix.kv_heads, self.dk, self.dv)
+
+    def splits(self, n: int, keys: int) -> int:
+        m = self.mix
+        return D_.paged_splits(n, m.heads, m.kv_heads, keys, m.window, m.keep_first)
+
+    def ws_need(self, n: int, keys: int) -> int:
+        """fp32 partials the decode launches of ``n`` sequences need."""
+        s = self.splits(n, keys)
+        return n * self.mix.heads * s * (self.dv + 2) if s > 1 else 0
+
+    def run(self, st, cache, b: StepBatch, ids, s: slice, gws, ws, nxt: dict, up) -> None:
+        m, x, h, y, (kp, vp) = self.mix, st.x[s], st.h[s], st.y[s], cache
+        qkv, af = st.buf["qkv"][s, :self.n_qkv], st.buf["af"][s, :self.n_att + self.n_ff]
+        self.w_qkv(h, qkv, gws)
+        if self.w_up is not None:
+            self.w_up(h, af[:, self.n_att:], gws, st.buf["gu"][s, :2 * self.n_ff] if st.f32 else None)
+        args = D_.paged_args(qkv, kp, vp, b.table, b.slots, b.pos, af[:, :self.n_att], b.M, m.heads, m.scale, m.window,
+                             m.keep_first, self.gate_col)
+        run_attention(st, args, b, self.group, self.splits(b.n_dec, b.max_len) if b.n_dec else 1, ws)
+        self.w_out(af, y, gws)
+        if self.side is None:
+            up(x_in=x, y=y, mult=st.mult, x_out=x, **nxt)
+            return
+        up(x_in=x, y=y, mult=st.mult, x_out=x, copy=st.cat[s, :st.wp])
+        self.side.run(st, s, ids, gws, nxt, up)
+
+
+# ---------------------------------------------------------------------- Funepel
+class DynamicTanh:
+    """tanh(alpha x) * w + b, as keyword arguments of ``rows_update``."""
+
+    def __init__(self, ld: Weights, name: str):
+        self.w, self.b, self.alpha = ld.vec(name), ld.vec(name + ".b"), float(ld(name + ".alpha"))
+
+    def prep(self, h: torch.Tensor) -> dict:
+        return {"norm": self.w, "norm_b": self.b, "alpha": self.alpha, "h": h}
+
+
+class Mamba2Mixer:
+    """Projection rows [x | B | C | z | dt]: the convolved channels first, heads
+    of x padded to multiples of 64 columns, groups of B and C to a state size."""
+
+    def __init__(self, ld: Weights, m: funepel.Mamba2Config):
+        self.m, self.groups = m, []
+        H, P, N, G = m.heads, m.vdim, m.state, m.groups
+        self.np, self.vp = M_.pad_state(N), D_.pad64(P)
+        self.C = H * self.vp + 2 * G * self.np
+        self.ip = D_.pad64(m.inner)
+        self.z_col, self.dt_col = self.C, self.C + self.ip
+        self.n_in = pad16(self.dt_col + H)
+
+        def channels(t):  # [x | B | C] rows, padded
+            x, B, C = t.split([m.inner, G * N, G * N])
+            return torch.cat([pad_heads(x, H, P, self.vp), pad_heads(B, G, N, self.np), pad_heads(C, G, N, self.np)])
+        w = pad(ld("in"), m.inner * 2 + 2 * G * N + H, ld.wp)
+        z, xbc, dt = w.split([m.inner, m.inner + 2 * G * N, H])
+        self.w_in = ld.linear(pad(torch.cat([channels(xbc), pad(z, self.ip, ld.wp), dt]), self.n_in, ld.wp))
+        self.conv = M_.ConvWeights(channels(ld("conv")).t().contiguous(), channels(ld("conv.b")).contiguous(),
+                                   ld("dt_bias").contiguous(), ld("A_log").contiguous())
+        self.D, self.norm = ld("D").contiguous(), ld("norm").contiguous()
+        self.w_o = ld.linear(pad(ld("o"), ld.wp, self.ip))
+        x1 = H * self.vp
+        self.cols = (x1 + G * self.np, x1, 0)  # q = C, k = B, v = x
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        return {"in": self.n_in, "conv": self.C, "mix": self.ip, "mixn": self.ip, "dt": self.m.heads, "la": self.m.heads}
+
+    def new_cache(self, st):
+        return {"ring": torch.zeros((st.num_slots, self.m.conv, self.C), dtype=st.dtype, device=st.device),
+                "state": torch.zeros((st.num_slots, self.m.heads, self.vp, self.np), dtype=torch.float32,
+                                     device=st.device)}
+
+    def ws_need(self, n: int, keys: int) -> int:
+        return 0
+
+    def run(self, st, cache, b: StepBatch, s: slice, gws, ws) -> dict:
+        """Returns the mixer's part of the residual update."""
+        m, M, B = self.m, b.M, st.buf
+        rows = self.w_in(st.h[s], B["in"][s, :self.n_in], gws)
+        cv, y, yn = B["conv"][s, :self.C], B["mix"][s, :self.ip], B["mixn"][s, :self.ip]
+        dt, la = st.flat("dt", s, m.heads), st.flat("la", s, m.heads)
+        M_.conv(rows, self.conv, cache["ring"], cv, dt, la, self.dt_col, b.start, b.slots, b.pos, b.ent,
+                len(b.chunks) + b.n_dec, M)
+        M_.scan(cv, self.cols, cache["state"], y, m.vdim, m.heads // m.groups, b.pos, b.ent, len(b.chunks), b.n_dec, M,
+                dt=dt, la=la, D=self.D)
+        M_.gated_norm(y, rows[:, self.z_col:], yn, M, m.inner, m.norm_groups, st.eps, self.norm, gate_first=True)
+        return {"y": self.w_o(yn, st.y[s], gws), "mult": 1.0}
+
+
+class AttentionRetentionMixer:
+    """One projection for both sides: [q | k | attention gate | retention q | k
+    | v | gate].  The key norm's weight is folded into the query's, its factor
+    per key is kept beside the pages, and the pages hold the keys as projected:
+    keys and values share one pool."""
+
+    def __init__(self, ld: Weights, m: funepel.ParallelConfig):
+        self.m = m
+        a, r = m.left, m.right
+        self.dk, self.np, self.vp = D_.pad_dim(a.dim), M_.pad_state(r.dim), D_.pad64(r.vdim)
+        self.group = a.heads // a.kv_heads
+        self.groups = [self.group]
+        self.n_att, self.n_ret = a.heads * self.dk, D_.pad64(r.heads * r.vdim)
+        wp, left, right = ld.wp, ld.sub("left."), ld.sub("right.")
+
+        def side(w, name, heads, dim, to):
+            return pad_heads(w.rows(name, heads * dim), heads, dim, to)
+        parts = [side(left, "q", a.heads, a.dim, self.dk), side(left, "k", a.kv_heads, a.dim, self.dk),
+                 side(left, "g", a.heads, a.dim, self.dk), side(right, "q", r.heads, r.dim, self.np),
+                 side(right, "k", r.heads, r.dim, self.np), side(right, "v", r.heads, r.vdim, self.vp),
+                 right.rows("g", self.n_ret)]
+        col = [0]
+        for p in parts:
+            col.append(col[-1] + p.shape[0])
+        self.gate_col, self.cols, self.rg_col = col[2], (col[3], col[4], col[5]), col[6]
+        self.n_in = pad16(col[-1])
+        self.w_in = ld.linear(pad(torch.cat(parts), self.n_in, wp))
+        qn, kn = (pad_heads(left(f"{n}.norm"), h, a.dim, self.dk) for n, h in (("q", a.heads), ("k", a.kv_heads)))
+        self.qw = (qn.view(a.kv_heads, self.group, self.dk) * kn.view(a.kv_heads, 1, self.dk)).reshape(-1).contiguous()
+        f = dict(dtype=torch.float32, device=ld.device)
+        self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / a.heads) for h in range(a.heads)], **f)
+        self.la = torch.tensor([max(math.log(d), -88.0) if d > 0 else -88.0 for d in r.decay], **f)
+        wo = pad(left("o").view(ld.width, a.heads, a.dim), ld.width, a.heads, self.dk)
+        self.w_left = ld.linear(pad(wo.reshape(ld.width, -1), wp, self.n_att))
+        self.w_right = ld.linear(pad(right("o"), wp, self.n_ret))
+        self.left_out, self.right_out = left.vec("out"), right.vec("out")
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        return {"in": self.n_in, "mix": max(self.n_att, self.n_ret), "mixn": self.n_ret, "y2": None}
+
+    def new_cache(self, st):
+        r = self.m.right
+        return {"kp": attention_cache(st, self.m.left.kv_heads, self.dk, None)[0],
+                "kscale": torch.zeros((st.num_pages, PAGE), dtype=torch.float32, device=st.device),
+                "state": torch.zeros((st.num_slots, r.heads, self.vp, self.np), dtype=torch.float32, device=st.device)}
+
+    def splits(self, n: int, keys: int) -> int:
+        a = self.m.left
+        return D_.paged_splits(n, a.heads, a.kv_heads, keys, a.window, a.keep_first)
+
+    def ws_need(self, n: int, keys: int) -> int:
+        s = self.splits(n, keys)
+        return n * self.m.left.heads * s * (self.dk + 2) if s > 1 else 0
+
+    def run(self, st, cache, b: StepBatch, s: slice, gws, ws) -> dict:
+        a, r, M, B = self.m.left, self.m.right, b.M, st.buf
+        rows = self.w_in(st.h[s], B["in"][s, :self.n_in], gws)
+        # retention
+        o, on = B["mix"][s, :self.n_ret], B["mixn"][s, :self.n_ret]
+        M_.scan(rows, self.cols, cache["state"], o, r.vdim, 1, b.pos, b.ent, len(b.chunks), b.n_dec, M, la_h=self.la,
+                dt_c=r.dim ** -0.5)
+        M_.gated_norm(o, rows[:, self.rg_col:], on, M, r.heads * r.vdim, r.heads, st.eps)
+        y2 = self.w_right(on, B["y2"][s], gws)
+        # attention
+        M_.qk_norm(rows, cache["kp"], cache["kscale"], self.qw, b.table, b.slots, b.pos, M, a.heads, a.heads * a.dim,
+                   a.kv_heads * a.dim, st.eps, a.temp_every, a.temp_coef)
+        out = B["mix"][s, :self.n_att]
+        args = D_.paged_args(rows, cache["kp"], cache["kp"], b.table, b.slots, b.pos, out, M, a.heads, a.scale, a.window,
+                             a.keep_first, self.gate_col, True, cache["kscale"], self.slopes)
+        run_attention(st, args, b, self.group, self.splits(b.n_dec, b.max_len) if b.n_dec else 1, ws, write=False)
+        y = self.w_left(out, st.y[s], gws)
+        return {"y": y, "y_norm": self.left_out, "y2": y2, "y2_norm": self.right_out, "mult": 0.5}
+
+
+class MixtureOfExperts:
+    def __init__(self, ld: Weights, m: funepel.MoEConfig):
+        self.m, self.fp, self.ep = m, D_.pad64(m.ff), pad16(m.experts)
+        self.w_router = ld.linear(ld.rows("router", self.ep))
+        experts = [ld.sub(f"e{e}.") for e in range(m.experts)]
+        self.w_up = M_.ExpertLinear([e.gate_up(self.fp) for e in experts], ld.dtype, ld.device, ACT_SILU_MUL)
+        self.w_down = M_.ExpertLinear([pad(e("down"), ld.wp, self.fp) for e in experts], ld.dtype, ld.device)
+        self.sp = D_.pad64(m.shared_ff) if m.shared_ff else 0
+        if self.sp:
+            sh = ld.sub("shared.")
+            self.w_sup = ld.linear(sh.gate_up(self.sp), act=ACT_SILU_MUL)
+            self.w_sdown = ld.linear(pad(sh("down"), ld.wp, self.sp))
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        b = {"sff": self.sp, "router": self.ep}
+        if f32:
+            b["gu"] = 2 * self.sp
+        return b
+
+    def run(self, st, s: slice, gws) -> dict:
+        """Returns the feed-forward's part of the residual update."""
+        m, h, B = self.m, st.h[s], st.buf
+        r0, M = s.start, s.stop - s.start
+        z = self.w_router(h, B["router"][s, :self.ep], gws)
+        rt, up, down = st.experts(m.experts, m.top, self.fp)
+        M_.route(z, rt, M, m.groups, m.keep, r0)
+        e = slice(r0 * m.top, (r0 + M) * m.top)
+        gu = up[e, :self.fp]
+        self.w_up(h, M * m.top, gu, rt, m.top, r0, st.expert_scratch(2 * self.fp, e) if st.f32 else None, clear=True)
+        ys = self.w_down(gu, M * m.top, down[e], rt, 0, r0)
+        part = {"ys": ys, "ysi": rt.place[e], "ysw": rt.w[e], "top": m.top, "mult": 1.0}
+        if self.sp:
+            f = self.w_sup(h, B["sff"][s, :self.sp], gws, B["gu"][s, :2 * self.sp] if st.f32 else None)
+            part["y"] = self.w_sdown(f, st.y[s], gws)
+        return part
+
+
+class SequentialLayer:
+    """Mixer, then experts, then the token input, each with its own residual update."""
+
+    def __init__(self, cfg, i: int, sd: Dict[str, torch.Tensor], dtype, device):
+        ld = Weights(cfg, f"l{i}.", sd, dtype, device)
+        L = cfg.layers[i]
+        self.norm1 = DynamicTanh(ld, "norm1")
+        mixer = Mamba2Mixer if isinstance(L.mixer, funepel.Mamba2Config) else AttentionRetentionMixer
+        self.mixer = mixer(ld.sub("mix."), L.mixer)
+        self.groups: List[int] = self.mixer.groups
+        self.ff = self.norm2 = None
+        if L.mlp is not None:
+            self.norm2, self.ff = DynamicTanh(ld, "norm2"), MixtureOfExperts(ld.sub("mlp."), L.mlp)
+        self.side = TokenInput(ld.sub("side."), i, cfg.side_dim) if cfg.side_dim else None
+
+    def prep(self, h: torch.Tensor) -> dict:
+        return self.norm1.prep(h)
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        b = dict(self.mixer.buffers(f32))
+        for k, v in (self.ff.buffers(f32) if self.ff else {}).items():
+            b[k] = max(b.get(k, 0), v)
+        return b
+
+    def new_cache(self, st):
+        return self.mixer.new_cache(st)
+
+    def ws_need(self, n: int, keys: int) -> int:
+        return self.mixer.ws_need(n, keys)
+
+    def run(self, st, cache, b: StepBatch, ids, s: slice, gws, ws, nxt: dict, up) -> None:
+        x = st.x[s]
+        last = nxt if self.side is None else {"copy": st.cat[s, :st.wp]}
+        part = self.mixer.run(st, cache, b, s, gws, ws)
+        if self.ff is None:
+            up(x_in=x, x_out=x, **part, **last)
+        else:
+            up(x_in=x, x_out=x, **part, **self.norm2.prep(st.h[s]))
+            part = self.ff.run(st, s, gws)
+            up(x_in=x, x_out=x, **part, **last)
+        if self.side is not None:
+            self.side.run(st, s, ids, gws, nxt, up)
+
+
+LAYERS = {"kozusun": JointLayer, "funepel": SequentialLayer}

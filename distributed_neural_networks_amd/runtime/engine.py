@@ -58,6 +58,9 @@ class Engine:
         pages = min(s.num_pages for s in self.stages)
         if num_pages is not None and num_pages > pages:
             raise ValueError(f"Engine: {num_pages} pages asked for, the stages hold {pages}")
+        slots = min((s.num_slots for s in self.stages if getattr(s, "recurrent", False)), default=max_slots)
+        if max_slots > slots:
+            raise ValueError(f"Engine: {max_slots} slots asked for, the stages hold the states of {slots} sequences")
         self.table = PageTable(num_pages or pages, max_slots)
         self.vocab = self.stages[0].V
         self.groups = sorted({g for s in self.stages for g in s.groups})

@@ -83,7 +83,9 @@ class PageTable:
 class StepBatch:
     """One step's rows on the device.  ``chunks``: (first row, tokens, slot) of
     the sequences that bring two tokens or more; ``dec_rows``: rows of the
-    sequences that bring one; ``max_len``: the longest sequence after the step."""
+    sequences that bring one; ``ent``: {first row, tokens, slot, 0} of all of
+    them, the chunks first; ``start``: per row, the first row of its sequence;
+    ``max_len``: the longest sequence after the step."""
     M: int
     pos: torch.Tensor
     slots: torch.Tensor
@@ -92,6 +94,8 @@ class StepBatch:
     n_dec: int
     chunks: Sequence[tuple]
     max_len: int
+    ent: torch.Tensor
+    start: torch.Tensor
     ids: Optional[torch.Tensor] = None
     want: Optional[torch.Tensor] = None
     n_want: int = 0
@@ -102,7 +106,7 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
     """``entries``: (token ids, first position, slot, wanted places) per
     sequence.  ``groups``: the query-heads-per-KV-head values of the model's
     layers.  Everything travels in one host-to-device copy."""
-    ids, pos, slots, dec, want, chunks = [], [], [], [], [], []
+    ids, pos, slots, dec, want, chunks, start = [], [], [], [], [], [], []
     for toks, p0, slot, places in entries:
         n, row = len(toks), len(ids)
         if n == 0:
@@ -111,13 +115,16 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
         ids += toks
         pos += range(p0, p0 + n)
         slots += [slot] * n
+        start += [row] * n
         if n == 1:
             dec.append(row)
         else:
             chunks.append((row, n, slot))
     parts = [("t%d" % g, np.array([t for c in chunks for t in chunk_tiles(*c, g)], dtype=np.int32).reshape(-1))
              for g in sorted(set(groups))] if chunks else []
-    parts += [("ids", np.array(ids, dtype=np.int32)), ("pos", np.array(pos, dtype=np.int32)),
+    ent = [(r, n, slot, 0) for r, n, slot in chunks] + [(r, 1, slots[r], 0) for r in dec]
+    parts += [("ent", np.array(ent, dtype=np.int32).reshape(-1)), ("start", np.array(start, dtype=np.int32)),
+              ("ids", np.array(ids, dtype=np.int32)), ("pos", np.array(pos, dtype=np.int32)),
               ("slots", np.array(slots, dtype=np.int32)), ("dec", np.array(dec, dtype=np.int32)),
               ("want", np.array(want, dtype=np.int32)), ("table", table.reshape(-1))]
     off, total = {}, 0
@@ -131,5 +138,5 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
     v = {name: dev[off[name]:off[name] + a.size] for name, a in parts}
     return StepBatch(M=len(ids), pos=v["pos"], slots=v["slots"], table=v["table"].view(table.shape),
                      dec_rows=v["dec"] if dec else None, n_dec=len(dec), chunks=chunks,
-                     max_len=max(pos) + 1, ids=v["ids"], want=v["want"] if want else None, n_want=len(want),
+                     max_len=max(pos) + 1, ent=v["ent"].view(-1, 4), start=v["start"], ids=v["ids"], want=v["want"] if want else None, n_want=len(want),
                      tiles={g: v["t%d" % g].view(-1, 4) for g in set(groups)} if chunks else None)

@@ -537,13 +537,24 @@ class DecodeRing:
         for m in range(self.M):
             snap = self.pos[m].clone()
             cur = self.cur[m].clone() if self.first else None
+            states = self._save_states()
             self._out_ready(m)
             self.graphs[m] = GraphedStep(lambda m=m: self._decode_body(m), self.dev, warmup=1)
             self.pos[m].copy_(snap)  # the warmup/capture runs advanced the position
             if cur is not None:
                 self.cur[m].copy_(cur)
+            self._restore_states(states)
         torch.cuda.synchronize(self.dev)
         self._capture_multi_step()
+
+    def _save_states(self):
+        """Recurrent states of the stages that have any: a graph's warmup advances them."""
+        return [s.save_states() if getattr(s, "recurrent", False) else None for s in self.stages]
+
+    def _restore_states(self, saved) -> None:
+        for s, v in zip(self.stages, saved):
+            if v is not None:
+                s.restore_states(v)
 
     def _capture_multi_step(self) -> None:
         K = self.multi_step
@@ -557,6 +568,7 @@ class DecodeRing:
         from .graph import GraphedStep
         snap = [p.clone() for p in self.pos]
         cur = [c.clone() for c in self.cur] if self.first else None
+        states = self._save_states()
 
         def body():
             for _ in range(K):
@@ -571,6 +583,7 @@ class DecodeRing:
         self.graph_k = GraphedStep(body, self.dev, warmup=1, reset=reset)
         self.graph_k_steps = K
         reset()  # the capture run advanced them again
+        self._restore_states(states)
         torch.cuda.synchronize(self.dev)
 
     def decode_round(self, mbs: Optional[Sequence[int]] = None) -> None:

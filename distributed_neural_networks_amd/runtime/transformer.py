@@ -32,7 +32,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from ..models import model_info
+from ..models import DECODERS, model_info
 from ..models.llama3 import rope_tables
 from ..ops import gemm as G_
 from ..ops.fp8 import mx_ok as fp8_mx_ok
@@ -580,14 +580,16 @@ def _e4m3_amax(t: torch.Tensor) -> float:
 def build_device_stage(model: str, sd, start: int, end: int, first: bool, last: bool, device, dtype=None,
                        max_batch: int = 8, max_seq: int = 1024, max_tokens: Optional[int] = None,
                        temperature: float = 0.0, top_k: int = 0, seed: int = 0, kv_dtype: str = "bf16",
-                       kv_scale: str = "calibrated", fp8_prefill: str = "e4m3", num_pages: Optional[int] = None):
-    """The GPU stage of a model family.  ``num_pages``: page pool of an engine (paged families)."""
-    if model_info(model).family == "kozusun":
+                       kv_scale: str = "calibrated", fp8_prefill: str = "e4m3", num_pages: Optional[int] = None,
+                       num_slots: Optional[int] = None):
+    """The GPU stage of a model family.  ``num_pages`` / ``num_slots``: page pool
+    and sequence states of an engine (paged families)."""
+    if model_info(model).family in DECODERS:
         from .decoder import DecoderStage
         if kv_dtype != "bf16":
             raise ValueError(f"model {model!r}: the paged cache follows the compute dtype, kv_cache_dtype {kv_dtype!r}")
         return DecoderStage(model, sd, start, end, first, last, device, max_batch, max_seq, max_tokens, dtype,
-                            temperature, top_k, seed, num_pages=num_pages)
+                            temperature, top_k, seed, num_pages=num_pages, num_slots=num_slots)
     fp8 = dtype in ("fp8", "float8_e4m3fn", "fp8_e4m3")
     info = model_info(model)
     max_seq = min(max_seq, getattr(info.cfg, "block_size", getattr(info.cfg, "max_seq", max_seq)))
@@ -596,14 +598,13 @@ def build_device_stage(model: str, sd, start: int, end: int, first: bool, last: 
 
 
 # ---------------------------------------------------------------------- smoke / golden check
-def decoder_smoke(dev) -> None:
-    """Kozusun-tiny, 2 stages: greedy tokens of the decode ring (fixed pages,
+def decoder_smoke(dev, model: str) -> None:
+    """A tiny paged decoder, 2 stages: greedy tokens of the decode ring (fixed pages,
     graphs) equal those of the engine (shared pool, prompts in portions) in the
     exact mode, and the bf16 logits stay within 3e-2 of the exact ones."""
     from .. import checkpoint as ckpt
     from .engine import Engine, Entry
     from .scheduler import DecodeRing, RingLinks
-    model = "kozusun-tiny"
     n = model_info(model).num_layers
     ranges = [(0, n // 2 - 1), (n // 2, n - 1)]
     sds = [ckpt.random_stage_state_dict(model, a, b, i == 0, i == 1, 7, nontrivial=True)
@@ -628,14 +629,15 @@ def decoder_smoke(dev) -> None:
 
 
 def smoke(dev) -> None:
-    """Kozusun-tiny: decode ring vs engine (``decoder_smoke``); GPT-2-tiny and
+    """Kozusun-tiny and Funepel-tiny: decode ring vs engine (``decoder_smoke``); GPT-2-tiny and
     Llama-tiny, 2 stages each on the decode ring, vs the fp32 torch golden: prefill logits within 2e-2 relative, the first generated
     token exact, and the greedy continuation equal to the golden's until the
     golden's top-2 logits come within bf16 resolution of each other."""
     from .. import checkpoint as ckpt
     from ..models import build_golden_stage
     from .scheduler import DecodeRing, RingLinks
-    decoder_smoke(dev)
+    decoder_smoke(dev, "kozusun-tiny")
+    decoder_smoke(dev, "funepel-tiny")
     for model in ("gpt2-tiny", "llama3-tiny"):
         n = model_info(model).num_layers
         ranges = [(0, n // 2 - 1), (n // 2, n - 1)]

@@ -50,7 +50,7 @@ def build_engine(folder: str, dtype: str, max_tokens: int):
     sd = ckpt.stage_state_dict(info.name, ckpt.load_full_state_dict(folder), 0, n - 1, True, True)
     stage = build_device_stage(info.name, sd, 0, n - 1, True, True, torch.device("cuda", 0), dtype=dtype,
                                max_batch=1, max_seq=max_tokens, max_tokens=max_tokens,
-                               num_pages=pages_for(max_tokens))
+                               num_pages=pages_for(max_tokens), num_slots=MAX_LIVE)
     return Engine([stage], max_slots=MAX_LIVE)
 
 

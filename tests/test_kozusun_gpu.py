@@ -113,11 +113,11 @@ def test_linear_f32(M, N, K):
 def test_gated_tanh_gelu(dtype, M, F, K):
     """Packed gate|up projection with the activation in the epilogue, at decode and prefill sizes."""
     from distributed_neural_networks_amd.ops import decoder_ops as D_
-    from distributed_neural_networks_amd.ops.gemm import decode_workspace, pack_gate_up
+    from distributed_neural_networks_amd.ops.gemm import ACT_GELU_TANH_MUL, decode_workspace, pack_gate_up
     g = torch.Generator().manual_seed(M)
     x = torch.randn(M, K, generator=g).to(DT[dtype])
     gate, up = (torch.randn(F, K, generator=g).bfloat16().float() / math.sqrt(K) * 2 for _ in range(2))
-    lin = D_.Linear(pack_gate_up(gate, up), None, DT[dtype], dev(), glu=True)
+    lin = D_.Linear(pack_gate_up(gate, up), None, DT[dtype], dev(), ACT_GELU_TANH_MUL)
     out = torch.zeros(M, F + 64, dtype=DT[dtype], device=dev())
     lin(x.to(dev()), out[:, 64:], decode_workspace(dev()) if M <= 64 else None,
         torch.zeros(M, 2 * F, device=dev()) if dtype == "float32" else None)
