@@ -785,9 +785,9 @@ def main():
         return rc
     if args.model != "cifar10":
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "bench"))
-        if args.model == "kozusun":
+        if args.model in ("kozusun", "funepel"):
             import decoder_bench
-            return decoder_bench.main(["--steps", str(args.steps)])
+            return decoder_bench.main(["--model", args.model, "--steps", str(args.steps)])
         import gpt_bench
         return gpt_bench.main(args)
     phases = {"startup_s": round(elapsed_s(), 2)}

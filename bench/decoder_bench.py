@@ -1,11 +1,17 @@
 #!/usr/bin/env python3
-"""Kozusun layers beside Llama layers of the same size: prefill and decode.
+"""Layers of the paged decoder families beside layers of another model of the
+same size: prefill and decode.
 
-``bench.py --model kozusun`` runs it (one GPU).  For each size, ``--layers``
-layers of random weights of either model (no loop, no head; the residual enters
-from the embedding) run on the same box in turn, timed as HIP graphs for decode
-and eagerly for prefill; medians over alternating repeats.  Kozusun's extra work
-per layer (token input, output gate, fp32 residual) is part of its time.
+``bench.py --model kozusun`` / ``--model funepel`` runs it (one GPU).  For each
+size, ``--layers`` layers of random weights of either model (no loop, no head;
+the residual enters from the embedding) run on the same box in turn, timed as
+HIP graphs for decode and eagerly for prefill; medians over alternating repeats.
+
+* kozusun: Kozusun layers beside Llama layers of the same size.
+* funepel: its two kinds of layers (a Mamba-2 mixer; attention beside
+  retention; both with experts and token input) beside Kozusun layers of the
+  same width, attention heads and token input.
+
 Prints one JSON line; ``--phase`` / ``--only`` restrict a profiler run.
 """
 from __future__ import annotations
@@ -22,13 +28,17 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 if ROOT not in sys.path:
     sys.path.insert(0, ROOT)
 
-# name -> (Kozusun preset, Llama configuration of the same layer size)
-SIZES = {"8b": ("kozusun-8b", dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=4096, ffn_dim=14336)),
-         "1b": ("kozusun-1b", dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=2048, ffn_dim=5632))}
+# name -> Llama configuration of the presets' layer size
+SIZES = {"8b": dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=4096, ffn_dim=14336),
+         "1b": dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=2048, ffn_dim=5632)}
+
+
+MODELS = {"kozusun": ("kozusun", "llama"), "funepel": ("funepel-mamba2", "funepel-parallel", "kozusun")}
 
 
 def parse(argv=None):
     ap = argparse.ArgumentParser()
+    ap.add_argument("--model", default="kozusun", choices=sorted(MODELS))
     ap.add_argument("--sizes", default="8b,1b")
     ap.add_argument("--layers", type=int, default=4)
     ap.add_argument("--batches", default="1,32,64", help="decode batch sizes")
@@ -37,28 +47,33 @@ def parse(argv=None):
     ap.add_argument("--repeats", type=int, default=7)
     ap.add_argument("--steps", type=int, default=20, help="decode steps of a repeat")
     ap.add_argument("--phase", default="both", choices=["both", "prefill", "decode"])
-    ap.add_argument("--only", default="", choices=["", "kozusun", "llama"])
+    ap.add_argument("--only", default="", choices=["", "kozusun", "llama", "funepel-mamba2", "funepel-parallel"])
     return ap.parse_args(argv)
 
 
-def build(size: str, layers: int, batch: int, seq: int, tokens: int, dev):
-    """{model: first-stage object with ``layers`` layers}"""
+def build(model: str, size: str, layers: int, batch: int, seq: int, tokens: int, dev):
+    """A first-stage object with ``layers`` layers of ``model``."""
     from dataclasses import replace
     from distributed_neural_networks_amd import checkpoint as ckpt
-    from distributed_neural_networks_amd.models import kozusun, llama3
+    from distributed_neural_networks_amd.models import funepel, kozusun, llama3
     from distributed_neural_networks_amd.runtime.decoder import DecoderStage
     from distributed_neural_networks_amd.runtime.transformer import TransformerStage
-    preset, lc = SIZES[size]
-    cfg = replace(kozusun.scaled(kozusun.KOZUSUN_CONFIGS[preset], layers), vocab_size=lc["vocab_size"])
-    sd = ckpt.random_decoder_state(kozusun, cfg, 0, layers - 1, True, False, 0, dev, True)
-    koz = DecoderStage(preset, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens,
-                       cfg=cfg)
-    del sd
-    name = "llama-layers-" + size
-    llama3.LLAMA_CONFIGS[name] = llama3.LlamaConfig(n_layer=layers, max_seq=seq, **lc)
-    sd = ckpt.random_stage_state_dict(name, 0, layers - 1, True, False, 0, device=dev)
-    lla = TransformerStage(name, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens)
-    return {"kozusun": koz, "llama": lla}
+    lc = SIZES[size]
+    if model == "llama":
+        name = "llama-layers-" + size
+        llama3.LLAMA_CONFIGS[name] = llama3.LlamaConfig(n_layer=layers, max_seq=seq, **lc)
+        sd = ckpt.random_stage_state_dict(name, 0, layers - 1, True, False, 0, device=dev)
+        return TransformerStage(name, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq,
+                                max_tokens=tokens)
+    if model == "kozusun":
+        family, cfg = kozusun, kozusun.scaled(kozusun.KOZUSUN_CONFIGS["kozusun-" + size], layers)
+    else:  # layer 0 of the presets has a Mamba-2 mixer, layer 1 attention beside retention
+        family = funepel
+        cfg = funepel.scaled(funepel.FUNEPEL_CONFIGS["funepel-" + size], (int(model == "funepel-parallel"),) * layers)
+    cfg = replace(cfg, vocab_size=lc["vocab_size"])
+    sd = ckpt.random_decoder_state(family, cfg, 0, layers - 1, True, False, 0, dev, True)
+    return DecoderStage(model, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens,
+                        cfg=cfg)
 
 
 def timed(fn, n: int) -> float:
@@ -93,11 +108,10 @@ def run(argv=None) -> dict:
         batches = [int(b) for b in a.batches.split(",")]
         maxb = max(batches + [a.prompts])
         seq, T = a.context + 64, a.context
-        stages = build(size, a.layers, maxb, seq, max(a.prompts * T, maxb), dev)
-        if a.only:
-            stages = {a.only: stages[a.only]}
+        stages = {m: build(m, size, a.layers, maxb, seq, max(a.prompts * T, maxb), dev)
+                  for m in ([a.only] if a.only else MODELS[a.model])}
         g = torch.Generator().manual_seed(1)
-        ids = torch.randint(0, SIZES[size][1]["vocab_size"], (maxb, T), generator=g).to(device=dev, dtype=torch.int32)
+        ids = torch.randint(0, SIZES[size]["vocab_size"], (maxb, T), generator=g).to(device=dev, dtype=torch.int32)
         zero = torch.zeros((maxb,), dtype=torch.int32, device=dev)
         outs = {k: torch.empty(*s.out_spec(a.prompts, T)[:1], dtype=s.out_spec(a.prompts, T)[1], device=dev)
                 for k, s in stages.items()}
@@ -126,9 +140,9 @@ def run(argv=None) -> dict:
             del graphs
         del stages, outs
         torch.cuda.empty_cache()
-    big = [r for r in rows if r["model"] == "kozusun" and r["phase"] == "decode"] or \
-        [r for r in rows if r["model"] == "kozusun"]
-    return {"metric": "layer tokens/s, Kozusun decoder layers", "value": big[-1]["tokens_per_s_layer"] if big else None,
+    mine = a.only or MODELS[a.model][0]
+    big = [r for r in rows if r["model"] == mine and r["phase"] == "decode"] or [r for r in rows if r["model"] == mine]
+    return {"metric": f"layer tokens/s, {mine} decoder layers", "value": big[-1]["tokens_per_s_layer"] if big else None,
             "unit": "tokens/s x layers", "n_gpus": 1, "higher_is_better": True, "vs_baseline": None, "dtype": "bf16",
             "data": "synthetic (random weights)", "config": {"layers": a.layers, "context": a.context}, "rows": rows}
 

@@ -17,85 +17,82 @@
 
 namespace dnn {
 
-// The choices of one row by one wave: lane l holds the logits of experts l, l + 64, ...
-struct Choice {
-  int e;
-  float s;
-};
-__device__ __forceinline__ unsigned long long wave_max_u64(unsigned long long v) {
-#pragma unroll
-  for (int o = 1; o < 64; o <<= 1) {
-    const unsigned lo = __shfl_xor((unsigned)v, o, 64), hi = __shfl_xor((unsigned)(v >> 32), o, 64);
-    const unsigned long long u = ((unsigned long long)hi << 32) | lo;
-    v = u > v ? u : v;
-  }
-  return v;
-}
-
-// f(t, expert) for every choice (every lane calls it), returning the weights through idx / w.
+// One row by half a wave: lane l of 32 holds the logits of experts l, l + 32,
+// ...; both halves call it together, a half past the rows with live = false.
+// f(t, expert) for every choice.
 template <typename F>
-__device__ __forceinline__ void route_row(const RouteArgs& a, int m, int lane, F f) {
-  float s[4];
+__device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, int l, int half, F f) {
+  constexpr int NR = EXPERTS_MAX / 32;
+  const int nr = (a.E + 31) / 32;  // registers that hold experts
+  float s[NR];
   float mx = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int e = i * 64 + lane;
-    s[i] = e < a.E ? a.logits[(size_t)m * a.ldl + e] : -INFINITY;
+  for (int i = 0; i < NR; ++i) {
+    const int e = i * 32 + l;
+    s[i] = live && i < nr && e < a.E ? a.logits[(size_t)m * a.ldl + e] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
-  mx = wave_max(mx);
+  mx = group_max<32>(mx);
+  if (!live) mx = 0.f;
   float sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < NR; ++i) {
     s[i] = expf(s[i] - mx);  // 0 past the experts
     sum += s[i];
   }
-  sum = wave_sum(sum);
-  // key of an expert: score bits, then the lower index first
-  unsigned long long key[4];
+  sum = live ? group_sum<32>(sum) : 1.f;
   const int per = a.E / a.groups;
-  int grp[4];
+  int grp[NR];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int e = i * 64 + lane;
+  for (int i = 0; i < NR; ++i) {
     s[i] /= sum;
-    grp[i] = e / per;
-    key[i] = e < a.E ? ((unsigned long long)__float_as_uint(s[i]) << 32) | (0xffffffffu - e) : 0ull;
+    grp[i] = i < nr ? (i * 32 + l) / per : 0;
   }
-  auto best = [&](const bool (&ok)[4]) __attribute__((always_inline)) {
-    unsigned long long k = 0;
+  // the best expert among ok: the largest score, the lower index first
+  auto best = [&](unsigned ok, float& v) __attribute__((always_inline)) {
+    float m1 = -1.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (ok[i] && key[i] > k) k = key[i];
-    return wave_max_u64(k);
+    for (int i = 0; i < NR; ++i)
+      if (i < nr && (ok >> i & 1) != 0 && i * 32 + l < a.E) m1 = fmaxf(m1, s[i]);
+    v = m1 = group_max<32>(m1);
+    int e = a.E - 1;
+#pragma unroll
+    for (int i = NR - 1; i >= 0; --i) {
+      if (i >= nr) continue;
+      const unsigned at = (unsigned)(__ballot((ok >> i & 1) != 0 && i * 32 + l < a.E && s[i] == m1) >> (32 * half));
+      if (at != 0) e = i * 32 + __ffs(at) - 1;
+    }
+    return e;
   };
   // the best groups: the group of the best expert outside those already taken
-  bool open[4], in[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) open[i] = true, in[i] = a.keep >= a.groups;
+  unsigned open = ~0u, in = a.keep >= a.groups ? ~0u : 0u;
   for (int k = 0; k < a.keep && a.keep < a.groups; ++k) {
-    const int e = (int)(0xffffffffu - (unsigned)best(open)), g = e / per;
+    float v;
+    const int g = best(open, v) / per;
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (grp[i] == g) open[i] = false, in[i] = true;
+    for (int i = 0; i < NR; ++i)
+      if (grp[i] == g) open &= ~(1u << i), in |= 1u << i;
   }
-  float total = 0.f, mine = 0.f;
-  int me = 0;
+  float total = 0.f;
+  float mine[2] = {0.f, 0.f};
+  int me[2] = {0, 0};
   for (int t = 0; t < a.top; ++t) {
-    const unsigned long long k = best(in);
-    const int e = min((int)(0xffffffffu - (unsigned)k), a.E - 1);
-    const float v = __uint_as_float((unsigned)(k >> 32));
+    float v;
+    const int e = best(in, v);
     total += v;
-    if (lane == t) mine = v, me = e;
+    if ((t & 31) == l) {
+      if (t < 32) mine[0] = v, me[0] = e;
+      else mine[1] = v, me[1] = e;
+    }
+    if ((e & 31) == l) in &= ~(1u << (e >> 5));
+    if (live) f(t, e);
+  }
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i * 64 + lane == e) in[i] = false;
-    f(t, e);
-  }
-  if (lane < a.top) {
-    a.idx[(size_t)m * a.top + lane] = me;
-    a.w[(size_t)m * a.top + lane] = mine / (total + 1e-20f);
-  }
+  for (int i = 0; i < 2; ++i)
+    if (live && i * 32 + l < a.top) {
+      a.idx[(size_t)m * a.top + i * 32 + l] = me[i];
+      a.w[(size_t)m * a.top + i * 32 + l] = mine[i] / (total + 1e-20f);
+    }
 }
 
 constexpr int RT_ROWS = 16;  // rows of a workgroup of 4 waves
@@ -105,10 +102,10 @@ __global__ __launch_bounds__(256) void route_kernel(RouteArgs a) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m0 = blockIdx.x * RT_ROWS;
   hist[tid] = 0;
   __syncthreads();
-  for (int r = wave; r < RT_ROWS && m0 + r < a.M; r += 4) {
-    const int m = m0 + r;
-    route_row(a, m, lane, [&](int t, int e) __attribute__((always_inline)) {
-      if (lane == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
+  for (int r = wave * 2; r < RT_ROWS; r += 8) {
+    const int half = lane >> 5, l = lane & 31, m = m0 + r + half;
+    route_row(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
+      if (l == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
     });
   }
   __syncthreads();
@@ -167,10 +164,12 @@ __global__ __launch_bounds__(1024) void route_small_kernel(RouteArgs a) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   if (tid < EXPERTS_MAX) hist[tid] = 0;
   __syncthreads();
-  for (int m = wave; m < a.M; m += 16)
-    route_row(a, m, lane, [&](int t, int e) __attribute__((always_inline)) {
-      if (lane == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
+  for (int m0 = wave * 2; m0 < a.M; m0 += 32) {
+    const int half = lane >> 5, l = lane & 31, m = m0 + half;
+    route_row(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
+      if (l == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
     });
+  }
   __syncthreads();
   expert_offsets(hist, a.E, offs, tid);
   __syncthreads();

@@ -456,23 +456,36 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
   }
 }
 
-__global__ __launch_bounds__(64) void paged_combine_kernel(PagedAttnArgs a, const int* __restrict__ rows, int ns,
-                                                           const float* __restrict__ ws) {
+// One workgroup per (sequence, head): the four waves take every fourth split.
+__global__ __launch_bounds__(256) void paged_combine_kernel(PagedAttnArgs a, const int* __restrict__ rows, int ns,
+                                                            const float* __restrict__ ws) {
+  __shared__ float acc[4][256 + 2];
   const int e = blockIdx.x / a.H, head = blockIdx.x % a.H, row = rows[e];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const float* d = ws + ((size_t)e * a.H + head) * ns * (a.DV + 2);
   float m = -INFINITY;
-  for (int s = 0; s < ns; ++s) m = fmaxf(m, d[s * (a.DV + 2)]);
-  const float gate = pa_gate(a, row, head);
-  for (int c = threadIdx.x; c < a.DV; c += 64) {
-    float l = 0.f, v = 0.f;
-    for (int s = 0; s < ns; ++s) {
-      const float* q = d + s * (a.DV + 2);
-      const float f = q[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(q[0] - m);
-      l = fmaf(q[1], f, l);
-      v = fmaf(q[2 + c], f, v);
-    }
-    reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.DV + c] = f2bf((l > 0.f ? v / l : 0.f) * gate * pa_gate_el(a, row, head * a.DV + c));
+  for (int s = lane; s < ns; s += 64) m = fmaxf(m, d[(size_t)s * (a.DV + 2)]);
+  m = wave_max(m);
+  float l = 0.f, v[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int s = wave; s < ns; s += 4) {
+    const float* q = d + (size_t)s * (a.DV + 2);
+    const float f = q[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(q[0] - m);
+    l = fmaf(q[1], f, l);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (lane + 64 * i < a.DV) v[i] = fmaf(q[2 + lane + 64 * i], f, v[i]);
   }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (lane + 64 * i < a.DV) acc[wave][lane + 64 * i] = v[i];
+  if (lane == 0) acc[wave][256] = l;
+  __syncthreads();
+  const int c = threadIdx.x;
+  if (c >= a.DV) return;
+  l = acc[0][256] + acc[1][256] + acc[2][256] + acc[3][256];
+  const float o = acc[0][c] + acc[1][c] + acc[2][c] + acc[3][c];
+  reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.DV + c] =
+      f2bf((l > 0.f ? o / l : 0.f) * pa_gate(a, row, head) * pa_gate_el(a, row, head * a.DV + c));
 }
 
 // ---------------------------------------------------------------- fp32
@@ -595,7 +608,7 @@ extern "C" int dnn_paged_decode(const PagedAttnArgs* a, const int* rows, int nro
   PA_DISPATCH(PD)
 #undef PD
   if (splits > 1)
-    hipLaunchKernelGGL(paged_combine_kernel, dim3((unsigned)(nrows * a->H)), dim3(64), 0, st, *a, rows, splits, ws);
+    hipLaunchKernelGGL(paged_combine_kernel, dim3((unsigned)(nrows * a->H)), dim3(256), 0, st, *a, rows, splits, ws);
   return (int)hipGetLastError();
 }
 

@@ -4,7 +4,8 @@
 // whose decay is data-dependent in the one and a constant per head in the other.
 //
 //   conv        short causal convolution per channel + silu, and the step sizes
-//   conv_state  the last inputs of every sequence for its next step
+//   conv_state  the last inputs of longer portions for their sequence's next
+//               step (a single token's input is stored by conv)
 //   scan_chunks bf16, sequences of 2 tokens or more: 64-token chunks on the
 //               MFMA, the state in fp32 accumulators from chunk to chunk
 //   scan_steps  token by token in fp32: single decoded tokens, and the exact mode
@@ -21,25 +22,33 @@ namespace dnn {
 typedef short s16x4 __attribute__((ext_vector_type(4)));
 constexpr float LOG2E = 1.4426950408889634f;
 
+// silu of a value that feeds a bf16 store
+__device__ __forceinline__ float silu_fast(float x) {
+  return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -LOG2E));
+}
+
 // ---------------------------------------------------------------- convolution
-// grid M * ceil((C / E + H) / 256)
+// Does row m bring the only token of its sequence in this step?
+__device__ __forceinline__ bool conv_single(const ConvArgs& a, int m) {
+  return a.start[m] == m && (m + 1 == a.M || a.start[m + 1] != m);
+}
+
 template <typename T>
-__global__ __launch_bounds__(256) void conv_kernel(ConvArgs a) {
+__device__ __forceinline__ void conv_store(const ConvArgs& a, int m, int c, float (&acc)[Vec16<T>::N]) {
+#pragma unroll
+  for (int j = 0; j < Vec16<T>::N; ++j) acc[j] = sizeof(T) == 2 ? silu_fast(acc[j]) : silu(acc[j]);
+  Vec16<T>::put(reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + c, acc);
+}
+
+// One row's channels c.., inputs from the rows of the step or the ring; a
+// single token also stores its input (its thread alone reads this channel of
+// the ring, and never the entry it overwrites).
+template <typename T>
+__device__ __forceinline__ void conv_row(const ConvArgs& a, int m, int c) {
   constexpr int E = Vec16<T>::N;
-  const int cv = a.C / E, gx = (cv + (a.dt != nullptr ? a.H : 0) + 255) / 256;
-  const int m = blockIdx.x / gx;
-  int i = (int)(blockIdx.x % gx) * 256 + threadIdx.x;
-  const T* row = reinterpret_cast<const T*>(a.in) + (size_t)m * a.ldi;
-  if (i >= cv) {
-    i -= cv;
-    if (a.dt == nullptr || i >= a.H) return;
-    const float z = to_f32(row[a.dt_col + i]) + a.dt_bias[i];
-    const float dt = z > 20.f ? z : log1pf(expf(z));
-    a.dt[(size_t)m * a.H + i] = dt;
-    a.la[(size_t)m * a.H + i] = fmaxf(-expf(a.a_log[i]) * dt, -88.f);  // exp(-88) is zero beside any state
-    return;
-  }
-  const int c = i * E, p = a.pos[m], s0 = a.start[m], slot = min(max(a.slots[m], 0), a.nslots - 1);
+  const T* row = reinterpret_cast<const T*>(a.in) + (size_t)m * a.ldi + c;
+  const int p = a.pos[m], s0 = a.start[m], slot = min(max(a.slots[m], 0), a.nslots - 1);
+  T* ring = reinterpret_cast<T*>(a.ring) + (size_t)slot * a.taps * a.C + c;
   float acc[E], v[E];
 #pragma unroll
   for (int j = 0; j < E; j += 4) {
@@ -49,9 +58,7 @@ __global__ __launch_bounds__(256) void conv_kernel(ConvArgs a) {
   }
   for (int t = 0; t < a.taps; ++t) {  // the input t positions back
     if (p - t < 0) break;
-    const T* src = m - t >= s0 ? row - (size_t)t * a.ldi + c
-                               : reinterpret_cast<const T*>(a.ring) + ((size_t)slot * a.taps + (p - t) % a.taps) * a.C + c;
-    Vec16<T>::get(src, v);
+    Vec16<T>::get(m - t >= s0 ? row - (size_t)t * a.ldi : ring + (size_t)((p - t) % a.taps) * a.C, v);
     const float* w = a.w + (size_t)(a.taps - 1 - t) * a.C + c;
 #pragma unroll
     for (int j = 0; j < E; j += 4) {
@@ -60,9 +67,70 @@ __global__ __launch_bounds__(256) void conv_kernel(ConvArgs a) {
       for (int k = 0; k < 4; ++k) acc[j + k] = fmaf(v[j + k], w4[k], acc[j + k]);
     }
   }
+  if (conv_single(a, m))
+    *reinterpret_cast<uint4*>(ring + (size_t)(p % a.taps) * a.C) = *reinterpret_cast<const uint4*>(row);
+  conv_store<T>(a, m, c, acc);
+}
+
+// grid ceil(M / R) * ceil((C / E + H) / 256); a thread takes E channels of R
+// rows.  Where the R rows and the TAPS - 1 before them are one sequence's, every
+// input is read once.
+template <typename T, int R, int TAPS>
+__global__ __launch_bounds__(256) void conv_kernel(ConvArgs a) {
+  constexpr int E = Vec16<T>::N;
+  const int cv = a.C / E, gx = (cv + (a.dt != nullptr ? a.H : 0) + 255) / 256;
+  const int m0 = (int)(blockIdx.x / gx) * R, m1 = min(m0 + R, a.M);
+  int i = (int)(blockIdx.x % gx) * 256 + threadIdx.x;
+  if (i >= cv) {
+    i -= cv;
+    if (a.dt == nullptr || i >= a.H) return;
+    const float bias = a.dt_bias[i], rate = -expf(a.a_log[i]);
+    for (int m = m0; m < m1; ++m) {
+      const float z = to_f32(reinterpret_cast<const T*>(a.in)[(size_t)m * a.ldi + a.dt_col + i]) + bias;
+      const float dt = z > 20.f ? z : log1pf(expf(z));
+      a.dt[(size_t)m * a.H + i] = dt;
+      a.la[(size_t)m * a.H + i] = fmaxf(rate * dt, -88.f);  // exp(-88) is zero beside any state
+    }
+    return;
+  }
+  const int c = i * E;
+  if constexpr (R > 1) {
+    const int s0 = a.start[m0];
+    if (m1 - m0 == R && s0 <= m0 - (TAPS - 1) && a.start[m1 - 1] == s0) {
+      const T* row = reinterpret_cast<const T*>(a.in) + (size_t)(m0 - (TAPS - 1)) * a.ldi + c;
+      float w[TAPS][E], bias[E];
 #pragma unroll
-  for (int j = 0; j < E; ++j) acc[j] = silu(acc[j]);
-  Vec16<T>::put(reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + c, acc);
+      for (int j = 0; j < E; j += 4) {
+        const f32x4 b = *reinterpret_cast<const f32x4*>(a.b + c + j);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) bias[j + k] = b[k];
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) {
+          const f32x4 v = *reinterpret_cast<const f32x4*>(a.w + (size_t)t * a.C + c + j);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) w[t][j + k] = v[k];
+        }
+      }
+      uint4 in[R + TAPS - 1];
+#pragma unroll
+      for (int r = 0; r < R + TAPS - 1; ++r) in[r] = *reinterpret_cast<const uint4*>(row + (size_t)r * a.ldi);
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        float acc[E], v[E];
+#pragma unroll
+        for (int j = 0; j < E; ++j) acc[j] = bias[j];
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) {
+          Vec16<T>::get(reinterpret_cast<const T*>(&in[r + t]), v);
+#pragma unroll
+          for (int j = 0; j < E; ++j) acc[j] = fmaf(v[j], w[t][j], acc[j]);
+        }
+        conv_store<T>(a, m0 + r, c, acc);
+      }
+      return;
+    }
+  }
+  for (int m = m0; m < m1; ++m) conv_row<T>(a, m, c);
 }
 
 // grid (ceil(C / E / 256), sequences): the raw inputs of a portion's last tokens
@@ -146,9 +214,10 @@ __global__ __launch_bounds__(256) void scan_steps_kernel(ScanArgs a) {
 // Within a chunk, A_t the running sum of la:
 //   y_t = exp(A_t) S^T q_t + sum_{s <= t} (q_t . k_s) exp(A_t - A_s) dt_s v_s + D v_t
 //   S  <- exp(A_L) S + sum_s k_s (exp(A_L - A_s) dt_s v_s)^T
-// Everything that carries a decay, and the state as an operand, goes to the
-// MFMA as two bf16 terms (value and remainder), so the recurrence keeps about
-// 16 bits of mantissa; accumulators are fp32.  Wave w: tokens (w & 1) * 32..,
+// Scores, decays and accumulators are fp32.  The state as an operand and the
+// decayed values that enter it go to the MFMA as two bf16 terms (value and
+// remainder), so the state keeps about 16 bits of mantissa through a readout
+// or an update.  Wave w: tokens (w & 1) * 32..,
 // value columns (w >> 1) * 32.. of the output; the same value columns and half
 // of the state rows in the update.
 constexpr int SC_L = 64;            // tokens of a chunk
@@ -169,14 +238,23 @@ __device__ __forceinline__ bf16x8 sc_tr(const char* tile, int stride, int s, int
   const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(p + 8 * stride));
   return bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
 }
-__device__ __forceinline__ void sc_split(float v, short& hi, short& lo) {
-  const bf16_t h = f2bf(v);
-  hi = (short)h;
-  lo = (short)f2bf(v - bf2f(h));
+// Two values as one pair of bf16 (a single conversion)
+__device__ __forceinline__ uint32_t sc_pack2(float a, float b) {
+  typedef float f32x2v __attribute__((ext_vector_type(2)));
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2v{a, b}), bf16x2v));
+}
+// ... and their remainders.
+__device__ __forceinline__ void sc_split2(float a, float b, uint32_t& hi, uint32_t& lo) {
+  hi = sc_pack2(a, b);
+  lo = sc_pack2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
+}
+__device__ __forceinline__ bf16x8 sc_frag(const uint32_t (&p)[4]) {
+  const i32x4 v = {(int)p[0], (int)p[1], (int)p[2], (int)p[3]};
+  return __builtin_bit_cast(bf16x8, v);
 }
 
 template <int NP>
-__global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
+__global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(ScanArgs a) {
   using L = ScanLds<NP>;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* ks = smem;
@@ -184,8 +262,8 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
   char* sh = vs + L::V;
   char* sl = sh + L::S;
   float* cum = reinterpret_cast<float*>(sl + L::S);
-  float* dts = cum + SC_L;
-  float* wst = dts + SC_L;
+  float* src = cum + SC_L;
+  float* wst = src + SC_L;
   constexpr int NK = NP / 16, NT = NP / 32, NTW = NT > 1 ? NT / 2 : 1;
   constexpr int CK = NP / 8, NIK = SC_L * CK / 256;  // 16-B pieces of a key row; per thread
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, hh = lane >> 5, r32 = lane & 31;
@@ -259,17 +337,12 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
       for (int i = 0; i < NTW; ++i)
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-          s16x4 hi, lo;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            short x, y;
-            sc_split(S[i][4 * q + j], x, y);
-            hi[j] = x;
-            lo[j] = y;
-          }
+          uint2 hi, lo;
+          sc_split2(S[i][4 * q], S[i][4 * q + 1], hi.x, lo.x);
+          sc_split2(S[i][4 * q + 2], S[i][4 * q + 3], hi.y, lo.y);
           const int o = (vt * 32 + r32) * L::SST + ((nt0 + i) * 32 + 8 * q + 4 * hh) * 2;
-          *reinterpret_cast<s16x4*>(sh + o) = hi;
-          *reinterpret_cast<s16x4*>(sl + o) = lo;
+          *reinterpret_cast<uint2*>(sh + o) = hi;
+          *reinterpret_cast<uint2*>(sl + o) = lo;
         }
     }
     if (wave == 0) {
@@ -279,10 +352,11 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
         const float u = __shfl_up(s, o, 64);
         if (lane >= o) s += u;
       }
+      s *= LOG2E;
+      const float w = s - __builtin_amdgcn_logf(pdt);  // dt_s exp(-A_s) as an exponent of 2 (dt 0: +inf, weight 0)
       cum[lane] = s;
-      dts[lane] = pdt;
-      const float end = __shfl(s, 63, 64);
-      wst[lane] = __expf(end - s) * pdt;
+      src[lane] = w;
+      wst[lane] = __builtin_amdgcn_exp2f(__shfl(s, 63, 64) - w);
     }
     // this wave's queries as B operand: column = token
     const int tok = tt * 32 + r32;
@@ -301,7 +375,7 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
       o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(sh + off), qf[k], o, 0, 0, 0);
       o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(sl + off), qf[k], o, 0, 0, 0);
     }
-    o *= __expf(at);
+    o *= __builtin_amdgcn_exp2f(at);
     for (int j = 0; j <= tt; ++j) {
       f32x16 g = f32x16{};
 #pragma unroll
@@ -311,24 +385,22 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const int s0 = j * 32 + 8 * q + 4 * hh;
-        const f32x4 cs = *reinterpret_cast<const f32x4*>(cum + s0), ds = *reinterpret_cast<const f32x4*>(dts + s0);
+        const f32x4 w = *reinterpret_cast<const f32x4*>(src + s0);
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          g[4 * q + i] = s0 + i <= tok ? g[4 * q + i] * (__expf(at - cs[i]) * ds[i]) : 0.f;
+        for (int i = 0; i < 4; ++i) g[4 * q + i] *= __builtin_amdgcn_exp2f(at - w[i]);
+        if (j == tt) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (s0 + i > tok) g[4 * q + i] = 0.f;
+        }
       }
 #pragma unroll
       for (int s = 0; s < 2; ++s) {
-        bf16x8 hi, lo;
+        uint32_t p[4];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          short x, y;
-          sc_split(g[8 * s + i], x, y);
-          hi[i] = x;
-          lo[i] = y;
-        }
+        for (int i = 0; i < 4; ++i) p[i] = sc_pack2(g[8 * s + 2 * i], g[8 * s + 2 * i + 1]);
         const bf16x8 vf = sc_tr(vs, SC_VST, 2 * j + s, vt * 32, lane);
-        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, hi, o, 0, 0, 0);
-        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, lo, o, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(p), o, 0, 0, 0);
       }
     }
     if (tok < len) {
@@ -351,7 +423,7 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
       }
     }
     if (mine) {
-      const float dec = __expf(cum[SC_L - 1]);
+      const float dec = __builtin_amdgcn_exp2f(cum[SC_L - 1]);
 #pragma unroll
       for (int i = 0; i < NTW; ++i) S[i] *= dec;
 #pragma unroll
@@ -359,19 +431,17 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
         const bf16x8 v = sc_tr(vs, SC_VST, s, vt * 32, lane);
         const f32x4 w0 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh);
         const f32x4 w1 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh + 8);
-        bf16x8 hi, lo;
+        uint32_t hi[4], lo[4];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          short x, y;
-          sc_split(bf2f_s(v[i]) * (i < 4 ? w0[i & 3] : w1[i & 3]), x, y);
-          hi[i] = x;
-          lo[i] = y;
+        for (int i = 0; i < 4; ++i) {
+          const f32x4& w = i < 2 ? w0 : w1;
+          sc_split2(bf2f_s(v[2 * i]) * w[2 * (i & 1)], bf2f_s(v[2 * i + 1]) * w[2 * (i & 1) + 1], hi[i], lo[i]);
         }
 #pragma unroll
         for (int i = 0; i < NTW; ++i) {
           const bf16x8 kt = sc_tr(ks, L::KST, s, (nt0 + i) * 32, lane);
-          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, hi, S[i], 0, 0, 0);
-          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, lo, S[i], 0, 0, 0);
+          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, sc_frag(hi), S[i], 0, 0, 0);
+          S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, sc_frag(lo), S[i], 0, 0, 0);
         }
       }
     }
@@ -387,14 +457,15 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(ScanArgs a) {
 }
 
 // ---------------------------------------------------------------- gate and norm
-// TPR threads per part; E values a piece (16 bytes, or one value where parts are not aligned)
-template <typename T, int TPR, int E>
+// TPR threads per part; E values a piece (16 bytes, or one value where parts
+// are not aligned), NV pieces a thread kept in registers (0: read twice)
+template <typename T, int TPR, int E, int NV>
 __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs a) {
   __shared__ float red[4];
   const int t = threadIdx.x % TPR;
   const long x = blockIdx.x * (256L / TPR) + threadIdx.x / TPR;
-  if (x >= (long)a.M * a.groups) return;  // TPR 256: uniform over the workgroup
-  const int m = (int)(x / a.groups), g = (int)(x % a.groups), n = a.n / a.groups;
+  const bool live = x < (long)a.M * a.groups;  // TPR 256: uniform over the workgroup
+  const int m = live ? (int)(x / a.groups) : 0, g = live ? (int)(x % a.groups) : 0, n = live ? a.n / a.groups : 0;
   const T* y = reinterpret_cast<const T*>(a.y) + (size_t)m * a.ldy + g * n;
   const T* z = reinterpret_cast<const T*>(a.z) + (size_t)m * a.ldz + g * n;
   T* out = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + g * n;
@@ -403,34 +474,72 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs a) {
     if constexpr (E == 1) v[0] = to_f32(*p);
     else Vec16<T>::get(p, v);
   };
-  for (int c = t * E; c < n; c += TPR * E) {
-    float u[E], v[E];
-    get(y + c, u);
-    if (a.gate_first) get(z + c, v);
+  auto act = [&](float v) __attribute__((always_inline)) { return sizeof(T) == 2 ? silu_fast(v) : silu(v); };
+  // gate: y * silu(z) or y alone, and its square
+  auto first = [&](float (&u)[E], float (&v)[E]) __attribute__((always_inline)) {
 #pragma unroll
     for (int j = 0; j < E; ++j) {
-      if (a.gate_first) u[j] *= silu(v[j]);
+      v[j] = act(v[j]);
+      if (a.gate_first) u[j] *= v[j];
       s = fmaf(u[j], u[j], s);
     }
-  }
-  s = wave_sum(s);
-  if constexpr (TPR == 256) {
-    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
-    __syncthreads();
-    s = red[0] + red[1] + red[2] + red[3];
-  }
-  const float r = 1.0f / sqrtf(s / (float)n + a.eps);
-  for (int c = t * E; c < n; c += TPR * E) {
-    float u[E], v[E];
-    get(y + c, u);
-    get(z + c, v);
+  };
+  auto last = [&](int c, float (&u)[E], const float (&v)[E], float r) __attribute__((always_inline)) {
 #pragma unroll
     for (int j = 0; j < E; ++j) {
-      u[j] *= silu(v[j]) * r;
-      if (a.w != nullptr) u[j] *= a.w[g * n + c + j];
+      u[j] *= a.gate_first ? r : r * v[j];
+      if (E == 1 && a.w != nullptr) u[j] *= a.w[g * n + c];
+    }
+    if constexpr (E > 1) {
+      if (a.w != nullptr) {
+#pragma unroll
+        for (int j = 0; j < E; j += 4) {
+          const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + g * n + c + j);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) u[j + k] *= w[k];
+        }
+      }
     }
     if constexpr (E == 1) out[c] = from_f32<T>(u[0]);
     else Vec16<T>::put(out + c, u);
+  };
+  auto sum = [&]() __attribute__((always_inline)) {
+    if constexpr (TPR <= 64) {
+      s = group_sum<TPR>(s);
+    } else {
+      s = wave_sum(s);
+      if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+      __syncthreads();
+      s = red[0] + red[1] + red[2] + red[3];
+    }
+    return 1.0f / sqrtf(s / (float)n + a.eps);
+  };
+  if constexpr (NV > 0) {
+    float u[NV][E], v[NV][E];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (t + i * TPR) * E;
+      if (c < n) get(y + c, u[i]), get(z + c, v[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if ((t + i * TPR) * E < n) first(u[i], v[i]);
+    const float r = sum();
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if ((t + i * TPR) * E < n) last((t + i * TPR) * E, u[i], v[i], r);
+  } else {
+    float u[E], v[E];
+    for (int c = t * E; c < n; c += TPR * E) {
+      get(y + c, u), get(z + c, v);
+      first(u, v);
+    }
+    const float r = sum();
+    for (int c = t * E; c < n; c += TPR * E) {
+      get(y + c, u), get(z + c, v);
+      first(u, v);
+      last(c, u, v, r);
+    }
   }
 }
 
@@ -444,11 +553,20 @@ extern "C" int dnn_conv(const ConvArgs* a, int f32, hipStream_t st) {
       a->ldo < a->C || a->nslots < 1)
     return -1;
   if (a->dt != nullptr && (a->H <= 0 || a->la == nullptr || a->dt_col < 0 || a->dt_col + a->H > a->ldi)) return -1;
-  const long n = (long)a->M * ((a->C / e + (a->dt != nullptr ? a->H : 0) + 255) / 256);
+  const int R = a->M >= 256 && a->taps >= 2 && a->taps <= 4 ? 8 : 1;
+  const long n = (long)((a->M + R - 1) / R) * ((a->C / e + (a->dt != nullptr ? a->H : 0) + 255) / 256);
   if (n > 0x7fffffff) return -1;
-  if (f32) hipLaunchKernelGGL(conv_kernel<float>, dim3((unsigned)n), dim3(256), 0, st, *a);
-  else hipLaunchKernelGGL(conv_kernel<bf16_t>, dim3((unsigned)n), dim3(256), 0, st, *a);
-  return (int)hipGetLastError();
+#define CV(R, TAPS)                                                                                             \
+  {                                                                                                             \
+    if (f32) hipLaunchKernelGGL((conv_kernel<float, R, TAPS>), dim3((unsigned)n), dim3(256), 0, st, *a);        \
+    else hipLaunchKernelGGL((conv_kernel<bf16_t, R, TAPS>), dim3((unsigned)n), dim3(256), 0, st, *a);           \
+    return (int)hipGetLastError();                                                                              \
+  }
+  if (R == 1) CV(1, 1)
+  if (a->taps == 2) CV(8, 2)
+  if (a->taps == 3) CV(8, 3)
+  CV(8, 4)
+#undef CV
 }
 
 extern "C" int dnn_conv_state(const ConvArgs* a, const int4* ent, int nent, int f32, hipStream_t st) {
@@ -502,19 +620,31 @@ extern "C" int dnn_gated_norm(const GatedNormArgs* a, int f32, hipStream_t st) {
   if (a->M <= 0 || a->n <= 0 || a->groups <= 0 || a->n % a->groups != 0 || a->ldy < a->n || a->ldz < a->n || a->ldo < a->n)
     return -1;
   const int n = a->n / a->groups, e = f32 ? 4 : 8;
-  const bool vec = n % e == 0 && (a->ldy | a->ldz | a->ldo) % e == 0 &&
+  const bool vec = n % e == 0 && ((uintptr_t)a->w & 15) == 0 && (a->ldy | a->ldz | a->ldo) % e == 0 &&
                    (((uintptr_t)a->y | (uintptr_t)a->z | (uintptr_t)a->out) & 15) == 0;
   const long parts = (long)a->M * a->groups;
-#define GN(T, E)                                                                                                         \
-  {                                                                                                                      \
-    if (n > 1024) hipLaunchKernelGGL((gated_norm_kernel<T, 256, E>), dim3((unsigned)parts), dim3(256), 0, st, *a);       \
-    else hipLaunchKernelGGL((gated_norm_kernel<T, 64, E>), dim3((unsigned)((parts + 3) / 4)), dim3(256), 0, st, *a);     \
+#define GN(T, TPR, E, NV)                                                                                              \
+  {                                                                                                                    \
+    hipLaunchKernelGGL((gated_norm_kernel<T, TPR, E, NV>), dim3((unsigned)((parts + 256 / TPR - 1) / (256 / TPR))),    \
+                       dim3(256), 0, st, *a);                                                                          \
+    return (int)hipGetLastError();                                                                                     \
+  }
+#define GN_SIZES(T, E)                         \
+  {                                            \
+    if (n <= 16 * E) GN(T, 16, E, 1)           \
+    if (n <= 32 * E) GN(T, 32, E, 1)           \
+    if (n <= 64 * E) GN(T, 64, E, 1)           \
+    if (n <= 128 * E) GN(T, 64, E, 2)          \
+    if (n <= 512 * E) GN(T, 256, E, 2)         \
+    if (n <= 1024 * E) GN(T, 256, E, 4)        \
+    GN(T, 256, E, 0)                           \
   }
   if (f32) {
-    if (vec) GN(float, 4) else GN(float, 1)
-  } else {
-    if (vec) GN(bf16_t, 8) else GN(bf16_t, 1)
+    if (vec) GN_SIZES(float, 4)
+    GN(float, 64, 1, 0)
   }
+  if (vec) GN_SIZES(bf16_t, 8)
+  GN(bf16_t, 64, 1, 0)
+#undef GN_SIZES
 #undef GN
-  return (int)hipGetLastError();
 }

@@ -12,6 +12,7 @@
 // ys are the rows of a mixture of experts, w_t their router weights.
 // Rows are NP wide (padded, zeros past N); means are over the true width N.
 // bf16 y / T in serving, fp32 in the exact mode.
+#include <algorithm>
 #include "common.h"
 #include "gemm_epilogue.h"
 #include "residual_api.h"
@@ -63,40 +64,61 @@ __device__ __forceinline__ float pos_entry(int p, const double* freq, int c) {
   return (c & 1) != 0 ? cosf(a) : sinf(a);
 }
 
-template <typename YT, typename OT, int TPR, int NC>
+// tanh for a bf16 result (straight line: one exponential, one reciprocal)
+__device__ __forceinline__ float tanh_fast(float x) {
+  return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * 2.8853900817779268f));
+}
+
+// PART: what the row needs beyond x, y and an RMS norm, so that plain rows do
+// not carry the registers of the rest.
+enum RowsPart { ROWS_PLAIN = 0, ROWS_MORE = 1, ROWS_TWO = 2, ROWS_EXPERTS = 3, ROWS_POSITIONS = 4 };
+// every part but PLAIN also has x_add and the dynamic tanh; MORE has nothing else
+
+template <typename YT, typename OT, int TPR, int NC, int PART>
 __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
   __shared__ float red[8];
   const int t = threadIdx.x % TPR;
-  const int m = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
-  if (m >= a.M) return;  // TPR 256: uniform over the workgroup
+  // few values per thread: the norm weights stay in registers over a
+  // workgroup's rows, and everything of a row is one memory round trip
+  constexpr bool PF = NC <= 4, TWO = PART == ROWS_TWO;
+  constexpr bool NB = PF && PART != ROWS_PLAIN;
+  f32x4 yw[PF ? NC : 1], nw[PF ? NC : 1], y2w[PF && TWO ? NC : 1], nb[NB ? NC : 1];
+  if constexpr (PF) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (t + TPR * i) * 4;
+      if (c >= a.NP) continue;
+      if (a.y_w != nullptr) yw[i] = ld4(a.y_w + c);
+      if (a.n_w != nullptr) nw[i] = ld4(a.n_w + c);
+      if constexpr (TWO) y2w[i] = ld4(a.y2_w + c);
+      if constexpr (NB)
+        if (a.n_b != nullptr) nb[i] = ld4(a.n_b + c);
+    }
+  }
+  // TPR 256: m is uniform over the workgroup
+  for (int m = blockIdx.x * (256 / TPR) + threadIdx.x / TPR; m < a.M; m += gridDim.x * (256 / TPR)) {
   const int xr = a.xidx != nullptr ? min(max(a.xidx[m], 0), a.xrows - 1) : m;
-  // few values per thread: the norm weights and y2 are issued with the row (one memory round trip)
-  constexpr bool PF = NC <= 4;
-  f32x4 x[NC], y[NC], yw[PF ? NC : 1], nw[PF ? NC : 1], y2[PF ? NC : 1];
+  f32x4 x[NC], y[NC], y2[PF && TWO ? NC : 1];
   const float* xp = a.x_in != nullptr ? a.x_in + (size_t)xr * a.ldx : nullptr;
   const YT* yp = nullptr;
   if (a.y != nullptr) {
     const int yr = a.yidx != nullptr ? min(max(a.yidx[m], 0), a.yrows - 1) : m;
     yp = reinterpret_cast<const YT*>(a.y) + (size_t)yr * a.ldy;
   }
-  const YT* y2p = a.y2 != nullptr ? reinterpret_cast<const YT*>(a.y2) + (size_t)m * a.ldy2 : nullptr;
+  const YT* y2p = TWO ? reinterpret_cast<const YT*>(a.y2) + (size_t)m * a.ldy2 : nullptr;
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
     const int c = (t + TPR * i) * 4;
     x[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if constexpr (PF) y2[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if constexpr (PF && TWO) y2[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c < a.NP) {
       if (xp != nullptr) x[i] = ld4(xp + c);
       if (yp != nullptr) y[i] = ld4(yp + c);
-      if constexpr (PF) {
-        if (a.y_w != nullptr) yw[i] = ld4(a.y_w + c);
-        if (a.n_w != nullptr) nw[i] = ld4(a.n_w + c);
-        if (y2p != nullptr) y2[i] = ld4(y2p + c);
-      }
+      if constexpr (PF && TWO) y2[i] = ld4(y2p + c);
     }
   }
-  if (y2p != nullptr) {  // both outputs normalised
+  if constexpr (TWO) {  // both outputs normalised
     float s1 = 0.f, s2 = 0.f;
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
@@ -116,7 +138,7 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
     for (int i = 0; i < NC; ++i) {
       const int c = (t + TPR * i) * 4;
       if (c < a.NP)
-        y[i] = y[i] * r1 * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c)) + (PF ? y2[PF ? i : 0] : ld4(y2p + c)) * r2 * ld4(a.y2_w + c);
+        y[i] = y[i] * r1 * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c)) + (PF ? y2[PF ? i : 0] * y2w[PF ? i : 0] : ld4(y2p + c) * ld4(a.y2_w + c)) * r2;
     }
   } else if (a.y_w != nullptr) {
     float s = 0.f;
@@ -131,28 +153,40 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
       if (c < a.NP) y[i] = y[i] * r * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c));
     }
   }
-  if (a.ys != nullptr) {
+  if constexpr (PART == ROWS_EXPERTS) {
     const int* si = a.ysi + (size_t)m * a.top;
     const float* sw = a.ysw + (size_t)m * a.top;
-#pragma unroll 4
-    for (int k = 0; k < a.top; ++k) {
-      const YT* p = reinterpret_cast<const YT*>(a.ys) + (size_t)min(max(si[k], 0), a.ysrows - 1) * a.ldys;
-      const float w = sw[k];
+    for (int k = 0; k < a.top; k += 4) {  // four rows in flight
+      const YT* p[4];
+      float w[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int q = min(k + u, a.top - 1);
+        p[u] = reinterpret_cast<const YT*>(a.ys) + (size_t)min(max(si[q], 0), a.ysrows - 1) * a.ldys;
+        w[u] = k + u < a.top ? sw[q] : 0.f;
+      }
 #pragma unroll
       for (int i = 0; i < NC; ++i) {
         const int c = (t + TPR * i) * 4;
-        if (c < a.NP) y[i] = y[i] + w * ld4(p + c);
+        if (c >= a.NP) continue;
+        f32x4 v[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) v[u] = ld4(p[u] + c);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) y[i][j] = fmaf(w[u], v[u][j], y[i][j]);
       }
     }
   }
-  if (a.x_add != nullptr) {
+  if (PART != ROWS_PLAIN && a.x_add != nullptr) {
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
       const int c = (t + TPR * i) * 4;
       if (c < a.NP) x[i] = x[i] + ld4(a.x_add + (size_t)m * a.ldadd + c);
     }
   }
-  if (a.freq != nullptr) {
+  if constexpr (PART == ROWS_POSITIONS) {
     const int p = a.pos[m];
 #pragma unroll
     for (int i = 0; i < NC; ++i)
@@ -176,19 +210,19 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
       if (a.copy != nullptr) st4(reinterpret_cast<OT*>(a.copy) + (size_t)m * a.ldcopy + c, x[i]);
     }
   }
-  if (a.n_w == nullptr) return;
-  if (a.n_b != nullptr) {
+  if (a.n_w == nullptr) continue;
+  if (PART != ROWS_PLAIN && a.n_b != nullptr) {
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
       const int c = (t + TPR * i) * 4;
       if (c >= a.NP) continue;
-      const f32x4 w = PF ? nw[PF ? i : 0] : ld4(a.n_w + c), b = ld4(a.n_b + c);
+      const f32x4 w = PF ? nw[PF ? i : 0] : ld4(a.n_w + c), b = NB ? nb[NB ? i : 0] : ld4(a.n_b + c);
       f32x4 v;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] = fmaf(tanhf(a.n_alpha * x[i][j]), w[j], b[j]);
+      for (int j = 0; j < 4; ++j) v[j] = fmaf(sizeof(OT) == 2 ? tanh_fast(a.n_alpha * x[i][j]) : tanhf(a.n_alpha * x[i][j]), w[j], b[j]);
       st4(reinterpret_cast<OT*>(a.h) + (size_t)m * a.ldh + c, v);
     }
-    return;
+    continue;
   }
   const float r = 1.0f / sqrtf(row_sum<TPR>(s, red) / (float)a.N + a.eps);
 #pragma unroll
@@ -196,14 +230,17 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
     const int c = (t + TPR * i) * 4;
     if (c < a.NP) st4(reinterpret_cast<OT*>(a.h) + (size_t)m * a.ldh + c, x[i] * r * (PF ? nw[PF ? i : 0] : ld4(a.n_w + c)));
   }
+  }
 }
 
-template <typename YT, typename OT>
+constexpr int ROWS_GRID = 2048;  // workgroups of a launch of many rows: they loop, eight to a CU
+
+template <typename YT, typename OT, int PART>
 static int rows_launch(const RowsArgs& a, hipStream_t st) {
 #define ROWS(TPR, NC)                                                                                             \
   {                                                                                                               \
-    hipLaunchKernelGGL((rows_update_kernel<YT, OT, TPR, NC>), dim3((a.M + 256 / TPR - 1) / (256 / TPR)), dim3(256), \
-                       0, st, a);                                                                                 \
+    hipLaunchKernelGGL((rows_update_kernel<YT, OT, TPR, NC, PART>),                                               \
+                       dim3(std::min((a.M + 256 / TPR - 1) / (256 / TPR), ROWS_GRID)), dim3(256), 0, st, a);                                                                                 \
     return (int)hipGetLastError();                                                                                \
   }
   // few rows (decode): a workgroup per row, so a row is one round trip deep
@@ -245,8 +282,21 @@ extern "C" int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStr
       (a->freq != nullptr && a->pos == nullptr))
     return -1;
   if ((a->xidx != nullptr && (a->xrows < 1 || a->x_out != nullptr)) || (a->yidx != nullptr && a->yrows < 1)) return -1;
-  if (y_f32) return out_f32 ? rows_launch<float, float>(*a, st) : rows_launch<float, bf16_t>(*a, st);
-  return out_f32 ? -1 : rows_launch<bf16_t, bf16_t>(*a, st);
+  if (a->y2 != nullptr && (a->ys != nullptr || a->freq != nullptr)) return -1;
+  if (a->ys != nullptr && a->freq != nullptr) return -1;
+  const bool more = a->x_add != nullptr || a->n_b != nullptr;
+#define ROWS_PART(YT, OT)                                                                        \
+  {                                                                                              \
+    if (a->y2 != nullptr) return rows_launch<YT, OT, ROWS_TWO>(*a, st);                          \
+    if (a->ys != nullptr) return rows_launch<YT, OT, ROWS_EXPERTS>(*a, st);                      \
+    if (a->freq != nullptr) return rows_launch<YT, OT, ROWS_POSITIONS>(*a, st);                  \
+    return more ? rows_launch<YT, OT, ROWS_MORE>(*a, st) : rows_launch<YT, OT, ROWS_PLAIN>(*a, st); \
+  }
+  if (y_f32 && out_f32) ROWS_PART(float, float)
+  if (!y_f32 && !out_f32) ROWS_PART(bf16_t, bf16_t)
+#undef ROWS_PART
+  if (!y_f32 || a->y2 != nullptr || a->ys != nullptr || a->freq != nullptr || more) return -1;
+  return rows_launch<float, bf16_t, ROWS_PLAIN>(*a, st);
 }
 
 extern "C" int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act,

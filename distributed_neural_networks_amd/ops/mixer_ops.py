@@ -72,17 +72,18 @@ class ConvWeights:
 
 
 def conv(rows: torch.Tensor, c: ConvWeights, ring: torch.Tensor, out: torch.Tensor, dt: torch.Tensor, la: torch.Tensor,
-         dt_col: int, start: torch.Tensor, slots: torch.Tensor, pos: torch.Tensor, ent: torch.Tensor, n_ent: int,
+         dt_col: int, start: torch.Tensor, slots: torch.Tensor, pos: torch.Tensor, ent: torch.Tensor, n_chunk: int,
          M: int) -> None:
     """Causal convolution + silu of the first C columns of ``rows`` into
     ``out``; dt = softplus(column dt_col + h + bias) and la = -exp(a_log) dt per
-    head; then the portions' last inputs into ``ring`` (slots, taps, C)."""
+    head; the portions' last inputs go into ``ring`` (slots, taps, C).  ``ent``:
+    ``n_chunk`` sequences that bring two tokens or more come first."""
     T, C = c.w.shape
     H = c.dt_bias.numel()
     f32 = rows.dtype == torch.float32
     _rows(rows, M, max(C, dt_col + H), "conv rows", (torch.float32, torch.bfloat16))
     _rows(out, M, C, "conv out", (rows.dtype,))
-    _entries(ent, n_ent)
+    _entries(ent, n_chunk)
     for t, n in ((start, M), (slots, M), (pos, M)):
         _index(t, n, "conv index")
     for t, n in ((c.w, T * C), (c.b, C), (c.dt_bias, H), (c.a_log, H), (dt, M * H), (la, M * H)):
@@ -94,8 +95,8 @@ def conv(rows: torch.Tensor, c: ConvWeights, ring: torch.Tensor, out: torch.Tens
               la=ptr(la), ldi=rows.stride(0), ldo=out.stride(0), M=M, C=C, taps=T, dt_col=dt_col, H=H,
               nslots=ring.shape[0])
     check(lib().conv(a, int(f32), stream_ptr()), "conv")
-    if T > 1:
-        check(lib().conv_state(a, ptr(ent), n_ent, int(f32), stream_ptr()), "conv_state")
+    if T > 1 and n_chunk:
+        check(lib().conv_state(a, ptr(ent), n_chunk, int(f32), stream_ptr()), "conv_state")
 
 
 def scan(rows: torch.Tensor, cols, state: torch.Tensor, y: torch.Tensor, vdim: int, qdiv: int, pos: torch.Tensor,

@@ -247,7 +247,7 @@ class Mamba2Mixer:
         cv, y, yn = B["conv"][s, :self.C], B["mix"][s, :self.ip], B["mixn"][s, :self.ip]
         dt, la = st.flat("dt", s, m.heads), st.flat("la", s, m.heads)
         M_.conv(rows, self.conv, cache["ring"], cv, dt, la, self.dt_col, b.start, b.slots, b.pos, b.ent,
-                len(b.chunks) + b.n_dec, M)
+                len(b.chunks), M)
         M_.scan(cv, self.cols, cache["state"], y, m.vdim, m.heads // m.groups, b.pos, b.ent, len(b.chunks), b.n_dec, M,
                 dt=dt, la=la, D=self.D)
         M_.gated_norm(y, rows[:, self.z_col:], yn, M, m.inner, m.norm_groups, st.eps, self.norm, gate_first=True)
