@@ -214,10 +214,9 @@ __global__ __launch_bounds__(256) void scan_steps_kernel(ScanArgs a) {
 // Within a chunk, A_t the running sum of la:
 //   y_t = exp(A_t) S^T q_t + sum_{s <= t} (q_t . k_s) exp(A_t - A_s) dt_s v_s + D v_t
 //   S  <- exp(A_L) S + sum_s k_s (exp(A_L - A_s) dt_s v_s)^T
-// Scores, decays and accumulators are fp32.  The state as an operand and the
-// decayed values that enter it go to the MFMA as two bf16 terms (value and
-// remainder), so the state keeps about 16 bits of mantissa through a readout
-// or an update.  Wave w: tokens (w & 1) * 32..,
+// Decays and accumulators are fp32.  Everything that carries a decay, and the
+// state as an operand, goes to the MFMA as two bf16 terms (value and
+// remainder), so the recurrence keeps about 16 bits of mantissa.  Wave w: tokens (w & 1) * 32..,
 // value columns (w >> 1) * 32.. of the output; the same value columns and half
 // of the state rows in the update.
 constexpr int SC_L = 64;            // tokens of a chunk
@@ -396,11 +395,12 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
       }
 #pragma unroll
       for (int s = 0; s < 2; ++s) {
-        uint32_t p[4];
+        uint32_t hi[4], lo[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) p[i] = sc_pack2(g[8 * s + 2 * i], g[8 * s + 2 * i + 1]);
+        for (int i = 0; i < 4; ++i) sc_split2(g[8 * s + 2 * i], g[8 * s + 2 * i + 1], hi[i], lo[i]);
         const bf16x8 vf = sc_tr(vs, SC_VST, 2 * j + s, vt * 32, lane);
-        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(p), o, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(hi), o, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(lo), o, 0, 0, 0);
       }
     }
     if (tok < len) {

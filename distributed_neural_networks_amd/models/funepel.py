@@ -68,7 +68,7 @@ class SharedKVAttentionConfig:
     kv_heads: int
     dim: int
     scale: float
-    window: int
+    window: Optional[int]   # None: every earlier key
     temp_coef: float = 0.0
     temp_every: int = 0     # 0: no query temperature
     keep_first: int = 0
@@ -141,7 +141,7 @@ def _attention(d, where) -> SharedKVAttentionConfig:
     t = d.get("q_temp")
     a = SharedKVAttentionConfig(heads=_size(d, "heads", where), kv_heads=_size(d, "kv_heads", where),
                                 dim=_size(d, "dim", where), scale=float(_get(d, "scale", where)),
-                                window=_size(d.get("mask"), "size", where + ".mask"),
+                                window=_size(d["mask"], "size", where + ".mask") if d.get("mask") else None,
                                 temp_coef=float(_get(t, "coef", where + ".q_temp")) if t else 0.0,
                                 temp_every=_size(t, "every", where + ".q_temp") if t else 0)
     _divides(a.heads, a.kv_heads, "heads over kv_heads", where)
@@ -326,7 +326,8 @@ def run_flops(cfg: FunepelConfig, layer: int, ctx: int) -> float:
     if isinstance(m, Mamba2Config):
         mix = 4.0 * m.inner * m.state + 2.0 * m.conv * (m.inner + 2 * m.groups * m.state)
     else:
-        mix = 4.0 * min(ctx, m.left.window) * m.left.heads * m.left.dim + 4.0 * m.right.heads * m.right.dim * m.right.vdim
+        keys = ctx if m.left.window is None else min(ctx, m.left.window)
+        mix = 4.0 * keys * m.left.heads * m.left.dim + 4.0 * m.right.heads * m.right.dim * m.right.vdim
     return 2.0 * mats + mix
 
 

@@ -1,0 +1,724 @@
+"""Funepel on the GPU kernels against the plain oracle (funepel_oracle.py)."""
+import copy
+import json
+import math
+import os
+import subprocess
+
+import numpy as np
+import pytest
+import torch
+
+import funepel_oracle as O
+from funepel_cases import CASES, att, config, layer, mamba2, moe, parallel, ret
+
+pytestmark = pytest.mark.gpu
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+F32_TOL = 3e-5
+DT = {"float32": torch.float32, "bf16": torch.bfloat16}
+
+
+def dev():
+    return torch.device("cuda", 0)
+
+
+def rel(got, ref):
+    got, ref = got.double().cpu(), ref.double().cpu()
+    return ((got - ref).norm() / ref.norm().clamp_min(1e-30)).item()
+
+
+def row_errors(got, ref):
+    """Relative error of every logits row (mean taken off)."""
+    d = got.double().cpu() - ref
+    d = d - d.mean(-1, keepdim=True)
+    r = ref - ref.mean(-1, keepdim=True)
+    return d.norm(dim=-1) / r.norm(dim=-1)
+
+
+def gen(seed):
+    return torch.Generator().manual_seed(seed)
+
+
+# ------------------------------------------------------------------ rows
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("M,width,NP", [(1, 60, 64), (5, 201, 256), (300, 200, 256), (3, 1100, 1152), (2600, 130, 192),
+                                        (4, 4096, 4096), (2, 9000, 9024)])
+def test_rows_update_parts(dtype, M, width, NP):
+    from distributed_neural_networks_amd.ops import decoder_ops as D_
+    g, dt, tol = gen(M + NP), DT[dtype], 1e-6 if dtype == "float32" else 4e-3
+
+    def mk(m, t, scale=1.0):
+        z = torch.zeros(m, NP)
+        z[:, :width] = scale * torch.randn(m, width, generator=g)
+        return z.to(t)
+    x, add, y, y2, tab = mk(M, torch.float32), mk(M, torch.float32), mk(M, dt), mk(M, dt, 3.0), mk(9, dt)
+    w = [mk(1, torch.float32)[0] for _ in range(4)]
+    to = lambda t: t.to(dev())  # noqa: E731
+    d = lambda t: t[..., :width].double()  # noqa: E731
+    xo, h, cp = (torch.full((M, NP), 7.0, device=dev()), torch.full((M, NP), 7.0, dtype=dt, device=dev()),
+                 torch.full((M, NP), 7.0, dtype=dt, device=dev()))
+
+    def check(ref, copy=True):
+        assert rel(xo[:, :width], ref) < 1e-6
+        if copy:
+            assert rel(cp[:, :width], ref) < tol
+        assert rel(h[:, :width], torch.tanh(0.7 * ref) * d(w[2]) + d(w[3])) < tol
+        assert (xo[:, width:] == 0).all() and (h[:, width:] == 0).all()
+    dyt = dict(norm=to(w[2]), norm_b=to(w[3]), alpha=0.7, h=h)
+    # dynamic tanh with an added row
+    D_.rows_update(M, width, x_in=to(x), y=to(y), mult=0.3, x_add=to(add), x_out=xo, copy=cp, eps=1e-2, **dyt)
+    check(d(x) + d(add) + 0.3 * d(y))
+    # two normalised outputs
+    D_.rows_update(M, width, x_in=to(x), y=to(y), y_norm=to(w[0]), y2=to(y2), y2_norm=to(w[1]), mult=0.5, x_out=xo, eps=1e-2,
+                   **dyt)
+    ref = d(x) + 0.5 * (O.rms_norm(d(y), 1e-2) * d(w[0]) + O.rms_norm(d(y2), 1e-2) * d(w[1]))
+    check(ref, False)
+    D_.rows_update(M, width, x_in=to(x), y=to(y), y_norm=to(w[0]), y2=to(y2), y2_norm=to(w[1]), mult=0.5, x_out=xo,
+                   x_add=to(add), copy=cp, eps=1e-2)
+    assert rel(xo[:, :width], ref + d(add)) < 1e-6 and rel(cp[:, :width], ref + d(add)) < tol
+    # weighted rows, with and without an output of the shared expert
+    for top in (1, 3, 6):
+        ys = mk(M * top, dt)
+        idx, sw = torch.randperm(M * top, generator=g).int(), torch.rand(M * top, generator=g)
+        mix = (sw.double().view(M, top, 1) * d(ys)[idx.long()].view(M, top, width)).sum(1)
+        kw = dict(ys=to(ys), ysi=to(idx), ysw=to(sw), top=top)
+        D_.rows_update(M, width, x_in=to(x), y=to(y), x_out=xo, copy=cp, **kw, **dyt)
+        check(d(x) + d(y) + mix)
+        D_.rows_update(M, width, x_in=to(x), x_out=xo, **kw, **dyt)
+        check(d(x) + mix, False)
+    # embedding rows with positions, near and far
+    ids, pos = torch.randint(0, 9, (M,), generator=g).int(), torch.randint(0, 5000, (M,), generator=g).int()
+    i = torch.arange(-(-width // 2), dtype=torch.float64)
+    freq = to(10000.0 ** (-2 * i / width) / (2 * math.pi))
+    D_.rows_update(M, width, y=to(tab), yidx=to(ids), pos=to(pos), freq=freq, x_out=xo, **dyt)
+    check(d(tab)[ids.long()] + O.positions(5000, width, torch.float64)[pos.long()] if width < 300 else
+          d(tab)[ids.long()] + torch.stack([torch.sin(pos.double()[:, None] * 10000.0 ** (-2 * i / width)),
+                                            torch.cos(pos.double()[:, None] * 10000.0 ** (-2 * i / width))],
+                                           -1).view(M, -1)[:, :width], False)
+
+
+# ------------------------------------------------------------------ attention with shared keys = values
+def run_shared_attention(dtype, H, G, dim, size, seqs, seed=0, standout=None, temp=(0.3, 16)):
+    """One step over sequences (cached length, new tokens), pages scattered over a
+    pool with garbage in it: norm and cache write, then attention.  ``standout``:
+    {(sequence, key): factor} makes that key a multiple of the last query."""
+    from distributed_neural_networks_amd.ops import decoder_ops as D_
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    from distributed_neural_networks_amd.runtime.paging import PAGE, PageTable, build_batch, pages_for
+    g, dt, R, dk, eps = gen(seed), DT[dtype], H // G, D_.pad_dim(dim), 1e-3
+    n_pages = sum(pages_for(a + b) for a, b in seqs) + 3
+    table = PageTable(n_pages, len(seqs))
+    table._free_pages = torch.randperm(n_pages, generator=g).tolist()
+    kp = (torch.randn(n_pages, G, PAGE, dk, generator=g) * 3).to(dt).to(dev())
+    ks = torch.rand(n_pages, PAGE, generator=g).to(dev()) * 5
+    wq, wk = 1 + 0.3 * torch.randn(H, dim, generator=g), 1 + 0.3 * torch.randn(G, dim, generator=g)
+    scale, slopes = 1.1 / math.sqrt(dim), O.slopes(H)
+    pad = lambda t: torch.nn.functional.pad(t, (0, dk - dim))  # noqa: E731
+    rows, refs, entries = [], [], []
+    for s, (old, new) in enumerate(seqs):
+        T = old + new
+        q, k, gt = (torch.randn(T, n, dim, generator=g) for n in (H, G, H))
+        for (sq, key), f in (standout or {}).items():
+            if sq == s:  # after the norms and weights, this key's score stands out
+                for c in range(G):
+                    k[key, c] = q[T - 1, c * R] * wq[c * R] / wk[c] * f
+        q, k, gt = (t.to(dt).double() for t in (q, k, gt))
+        qn = O.rms_norm(q.reshape(T, -1), eps).view(T, H, dim) * wq.double()
+        qn = qn * O.query_temperature(T, {"coef": temp[0], "every": temp[1]})[:, None, None]
+        rk = 1 / torch.sqrt((k.reshape(T, -1) ** 2).mean(-1) + eps)
+        kn, ok = k * rk[:, None, None] * wk.double(), O.visible(T, size)
+        o = [O.masked_softmax(O.biased_scores(qn[:, h], kn[:, h // R], scale, slopes[h]), ok) @ k[:, h // R]
+             * torch.sigmoid(gt[:, h]) for h in range(H)]
+        refs.append(torch.stack(o, 1)[old:])
+        slot = table.admit()
+        table.reserve(slot, T)
+        for j in range(old):
+            p = table.table[slot, j // PAGE]
+            kp[p, :, j % PAGE] = pad(k[j]).to(dt).to(dev())
+            ks[p, j % PAGE] = float(rk[j])
+        rows.append(torch.cat([pad(t[old:]).reshape(new, -1) for t in (q, k, gt)], 1))
+        entries.append(([1] * new, old, slot, []))
+    b = build_batch(entries, table.table, [R], dev())
+    raw = torch.cat(rows)
+    qkv = raw.to(dt).to(dev())
+    qw = pad(wq).view(G, R, dk) * pad(wk).view(G, 1, dk)
+    M_.qk_norm(qkv, kp, ks, qw.reshape(-1).contiguous().to(dev()), b.table, b.slots, b.pos, b.M, H, H * dim, G * dim, eps,
+               temp[1], temp[0])
+    out = torch.full((b.M, H * dk + 64), 5.0, dtype=dt, device=dev())
+    sl = torch.tensor(slopes, dtype=torch.float32, device=dev())
+    args = D_.paged_args(qkv, kp, kp, b.table, b.slots, b.pos, out[:, :H * dk], b.M, H, scale, size, 0, (H + G) * dk, True, ks,
+                         sl)
+    if dtype == "float32":
+        D_.paged_attn_f32(args)
+    else:
+        if b.chunks:
+            D_.paged_prefill(args, b.tiles[R])
+        if b.n_dec:
+            for splits in (1, 3):
+                ws = torch.empty(b.n_dec * H * splits * (dk + 2), device=dev()) if splits > 1 else None
+                D_.paged_decode(args, b.dec_rows, b.n_dec, splits, ws)
+                if splits == 1:
+                    one = out.clone()
+            assert rel(out, one) < 5e-3
+    torch.cuda.synchronize()
+    assert (out[:, H * dk:] == 5).all()
+    for (toks, old, slot, _), r in zip(entries, torch.split(raw, [len(e[0]) for e in entries])):  # keys as projected
+        for t in (0, len(toks) - 1):
+            p, o = table.table[slot, (old + t) // PAGE], (old + t) % PAGE
+            assert torch.equal(kp[p, :, o].cpu().double().view(-1), r[t, H * dk:(H + G) * dk].double())
+    return out[:, :H * dk].cpu().double().view(b.M, H, dk)[..., :dim], torch.cat(refs)
+
+
+SEQS = [(0, 1), (0, 2), (63, 1), (64, 1), (65, 2), (127, 3), (0, 130), (200, 1), (130, 77), (191, 65)]
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("H,G,dim", [(2, 2, 64), (6, 2, 40), (3, 1, 128), (40, 1, 64), (2, 1, 200), (5, 5, 16)])
+@pytest.mark.parametrize("size", [1, 50, 64, 1000])
+def test_shared_key_attention(dtype, H, G, dim, size):
+    got, ref = run_shared_attention(dtype, H, G, dim, size, SEQS, seed=H + dim)
+    err = ((got - ref).flatten(1).norm(dim=1) / ref.flatten(1).norm(dim=1)).max().item()
+    assert err < (3e-6 if dtype == "float32" else 2e-2), err
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("new", [1, 2, 40])
+@pytest.mark.parametrize("size", [32, 65, 128, 250])
+def test_window_edges_stand_out(dtype, new, size):
+    """A key that outweighs the distance bias and all others, just inside and
+    just outside the window and at page borders."""
+    T = 300
+    last = T - 1
+    for key in sorted({last - size + 1, last - size, 0, 63, 64, 127, 128, 255, 256, last}):
+        if key >= T - new and key != last:
+            continue
+        got, ref = run_shared_attention(dtype, 3, 1, 64, size, [(T - new, new)], seed=key, standout={(0, key): 40.0})
+        assert rel(got[-1], ref[-1]) < (1e-5 if dtype == "float32" else 2e-2), key  # fp32 scores of some hundreds
+
+
+# ------------------------------------------------------------------ recurrences
+def step_batch(portions, slots):
+    """A batch of (start, tokens) portions in ``slots``; pages play no role here."""
+    from distributed_neural_networks_amd.runtime.paging import build_batch
+    table = np.zeros((max(slots) + 1, 1), dtype=np.int32)
+    return build_batch([([1] * n, p0, s, []) for (p0, n), s in zip(portions, slots)], table, [], dev())
+
+
+# how three sequences of 150, 70 and 9 tokens come, step by step (0: left out)
+SCHEDULES = [[(150, 70, 9)], [(1, 2, 3), (63, 1, 1), (1, 0, 1), (2, 64, 2), (65, 1, 1), (18, 2, 1)],
+             [(64, 1, 0), (64, 66, 8), (1, 2, 0), (1, 1, 1), (20, 0, 0)], [(100, 60, 1)] + [(1, 1, 1)] * 8 + [(42, 2, 0)]]
+
+
+def portions(schedule, lengths):
+    at = [0] * len(lengths)
+    for step in schedule:
+        take = [(i, min(n, lengths[i] - at[i])) for i, n in enumerate(step)]
+        take = [(i, n) for i, n in take if n > 0]
+        yield [(i, at[i], n) for i, n in take]
+        for i, n in take:
+            at[i] += n
+    assert at == list(lengths)
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 6])
+@pytest.mark.parametrize("C,H", [(32, 3), (736, 5)])
+def test_convolution(dtype, taps, C, H):
+    """Every cut of three sequences gives the whole sequence's values; slots keep garbage of earlier sequences."""
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    g, dt = gen(taps + C), DT[dtype]
+    lengths = (300, 70, 9)
+    w, b = torch.randn(C, taps, generator=g) / math.sqrt(taps), torch.randn(C, generator=g)
+    bias, a_log = torch.randn(H, generator=g) * 3, torch.randn(H, generator=g)
+    seqs = [torch.randn(n, C + H, generator=g).to(dt) * 2 for n in lengths]
+    cw = M_.ConvWeights(*(t.contiguous().to(dev()) for t in (w.t(), b, bias, a_log)))
+    tol = 2e-6 if dtype == "float32" else 5e-3
+    ring = torch.randn(5, taps, C, generator=g).to(dt).to(dev())
+    for schedule in ([(300, 70, 9)], [(7, 1, 1), (64, 2, 2), (1, 1, 1), (1, 64, 1), (226, 1, 1), (1, 1, 3)]):
+        got, got_dt, got_la = ([torch.zeros(n, k, dtype=torch.float64) for n in lengths] for k in (C, H, H))
+        for part in portions(schedule, lengths):
+            bt = step_batch([(p0, n) for _, p0, n in part], [(4, 0, 2)[i] for i, _, _ in part])
+            rows = torch.cat([seqs[i][p0:p0 + n] for i, p0, n in part])
+            width = -(-(C + H) // 16) * 16
+            buf = torch.zeros(bt.M, width, dtype=dt)
+            buf[:, :C + H] = rows
+            buf = buf.to(dev())
+            out = torch.full((bt.M, C), 9.0, dtype=dt, device=dev())
+            d, la = torch.empty(bt.M * H, device=dev()), torch.empty(bt.M * H, device=dev())
+            M_.conv(buf, cw, ring, out, d, la, C, bt.start, bt.slots, bt.pos, bt.ent, len(bt.chunks), bt.M)
+            r = 0
+            for i, p0, n in part:
+                got[i][p0:p0 + n] = out[r:r + n].double().cpu()
+                got_dt[i][p0:p0 + n], got_la[i][p0:p0 + n] = d.view(-1, H)[r:r + n].cpu(), la.view(-1, H)[r:r + n].cpu()
+                r += n
+        for i, s in enumerate(seqs):
+            u = s.double()
+            ref = O.silu(O.causal_conv(u[:, :C], w.double(), b.double()))
+            assert ((got[i] - ref).norm(dim=1) / ref.norm(dim=1)).max() < tol
+            step = O.softplus(u[:, C:] + bias.double())
+            assert rel(got_dt[i], step) < 1e-6 and rel(got_la[i], -torch.exp(a_log.double()) * step) < 1e-6
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("schedule", range(len(SCHEDULES)))
+@pytest.mark.parametrize("H,N,P,G,fixed", [(4, 32, 64, 2, False), (3, 64, 20, 3, True), (2, 128, 130, 2, True),
+                                           (6, 128, 48, 1, False), (2, 256, 64, 1, False), (2, 200, 72, 2, True)])
+def test_recurrence(dtype, schedule, H, N, P, G, fixed):
+    """Portions and single tokens of three sequences against the token-by-token
+    recurrence, from long memories (decay 1) to none, in slots with garbage."""
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    g, dt, lengths = gen(N + P), DT[dtype], (150, 70, 9)
+    NP, VP = M_.pad_state(N), -(-P // 64) * 64
+    qdiv, decays = H // G, [1.0, 0.0, 0.97, 0.5, 0.999, 0.9][:H]
+    a_log, D = torch.linspace(-6, 3, H), None if fixed else torch.randn(H, generator=g)
+    cols = (0, G * NP, 2 * G * NP)
+    state = torch.full((4, H, VP, NP), 1e3, device=dev())
+    seqs = []
+    for n in lengths:
+        q, k, v = (torch.randn(n, m, d, generator=g).to(dt) for m, d in ((G, N), (G, N), (H, P)))
+        v[0] = (v[0].float() * 20).to(dt)  # the first token stands out in the state
+        seqs.append((q, k, v, torch.rand(n, H, generator=g) * 2))
+    refs = []
+    for q, k, v, d in seqs:
+        y = []
+        for h in range(H):
+            qh, kh, vh = q[:, h // qdiv].double(), k[:, h // qdiv].double(), v[:, h].double()
+            if fixed:
+                y.append(O.retention(qh, kh * N ** -0.5, vh, decays[h]))
+            else:
+                y.append(O.ssd(vh, kh, qh, d[:, h].double(), a_log[h].double(), D[h].double()))
+        refs.append(torch.stack(y, 1))
+    got = [torch.zeros(n, H, P, dtype=torch.float64) for n in lengths]
+    pad = torch.nn.functional.pad
+    for part in portions(SCHEDULES[schedule], lengths):
+        bt = step_batch([(p0, n) for _, p0, n in part], [(3, 0, 2)[i] for i, _, _ in part])
+        rows = torch.cat([torch.cat([pad(t[p0:p0 + n], (0, w - t.shape[2])).reshape(n, -1) for t, w in
+                                     zip(seqs[i][:3], (NP, NP, VP))], 1) for i, p0, n in part]).to(dev())
+        y = torch.full((bt.M, H * P + 8), 7.0, dtype=dt, device=dev())
+        if fixed:
+            la = torch.tensor([max(math.log(x), -88.0) if x else -88.0 for x in decays], dtype=torch.float32, device=dev())
+            kw = dict(la_h=la, dt_c=N ** -0.5)
+        else:
+            d = torch.cat([seqs[i][3][p0:p0 + n] for i, p0, n in part]).to(dev())
+            kw = dict(dt=d.reshape(-1).contiguous(), la=(-torch.exp(a_log).to(dev()) * d).clamp_min(-88).reshape(-1).contiguous(),
+                      D=D.to(dev()))
+        M_.scan(rows, cols, state, y, P, qdiv, bt.pos, bt.ent, len(bt.chunks), bt.n_dec, bt.M, **kw)
+        assert (y[:, H * P:] == 7).all()
+        r = 0
+        for i, p0, n in part:
+            got[i][p0:p0 + n] = y[r:r + n, :H * P].double().cpu().view(n, H, P)
+            r += n
+    assert (state[1] == 1e3).all()  # no sequence had this slot
+    for a, b in zip(got, refs):
+        scale = b.norm(dim=2).clamp_min(0.05 * b.norm(dim=2).mean())
+        assert ((a - b).norm(dim=2) / scale).max() < (2e-5 if dtype == "float32" else 1.5e-2)
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("M,n,groups", [(3, 24, 4), (1, 60, 5), (700, 96, 3), (5, 640, 1), (2, 1536, 2), (70, 2048, 16),
+                                        (2, 8192, 1), (2, 3000, 1), (1, 9000, 1), (3, 33, 3), (2, 24576, 2)])
+@pytest.mark.parametrize("gate_first", [False, True])
+def test_gated_norm(dtype, M, n, groups, gate_first):
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    g, dt = gen(n), DT[dtype]
+    y, z, w = torch.randn(M, n + 8, generator=g).to(dt), (2 * torch.randn(M, n + 8, generator=g)).to(dt), torch.randn(n, generator=g)
+    out = torch.full((M, n + 16), 3.0, dtype=dt, device=dev())
+    M_.gated_norm(y.to(dev()), z.to(dev()), out, M, n, groups, 1e-2, w.to(dev()) if gate_first else None, gate_first)
+    yd, zd = y[:, :n].double(), z[:, :n].double()
+    if gate_first:
+        ref = O.gated_group_norm(yd, zd, w.double(), groups, 1e-2)
+    else:
+        ref = O.rms_norm(yd.view(M, groups, -1), 1e-2).view(M, n) * O.silu(zd)
+    assert rel(out[:, :n], ref) < (1e-6 if dtype == "float32" else 5e-3) and (out[:, n:] == 3).all()
+
+
+# ------------------------------------------------------------------ experts
+@pytest.mark.parametrize("M", [1, 5, 33, 64, 65, 300])
+@pytest.mark.parametrize("E,top,groups,keep", [(1, 1, 1, 1), (8, 2, 2, 1), (12, 4, 4, 2), (70, 6, 7, 3), (256, 8, 8, 4),
+                                               (64, 40, 1, 1), (33, 33, 3, 3)])
+def test_route(M, E, top, groups, keep):
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    z = torch.randn(M, E + 3, generator=gen(M + E)) * 3
+    r = M_.Routing(M + 2, E, top, dev())
+    for row0 in (2, 0, 2):  # the counters are left as they were found
+        M_.route(z.to(dev()), r, M, groups, keep, row0)
+        counts, offs = r.bins(row0)
+        if M > 64:
+            counts.zero_()  # the grouped product does this
+        s = slice(row0 * top, (row0 + M) * top)
+        idx, w = r.idx[s].view(M, top).cpu().long(), r.w[s].view(M, top).cpu().double()
+        rd = {"top": top, "groups": {"count": groups, "keep": keep}}
+        ri, rw = O.route(z[:, :E].double(), rd)
+        assert torch.equal(idx, ri) and rel(w, rw) < 1e-6
+        order, place, o = r.order[s].cpu().long(), r.place[s].cpu().long(), offs.cpu()
+        assert torch.equal(place[order], torch.arange(M * top)) and torch.equal(order[place], torch.arange(M * top))
+        n = torch.bincount(idx.view(-1), minlength=E)
+        assert torch.equal(o[1:].long(), n.cumsum(0)) and o[0] == 0
+        assert (idx.view(-1)[order].diff() >= 0).all()  # sorted by expert
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "float32"])
+@pytest.mark.parametrize("M,E,top", [(1, 8, 2), (17, 4, 2), (40, 4, 2), (90, 4, 2), (300, 5, 2), (700, 3, 3), (66, 200, 4)])
+@pytest.mark.parametrize("F,K", [(64, 128), (192, 320)])
+def test_expert_products(dtype, M, E, top, F, K):
+    """Gated and plain products of rows grouped by expert, from a few rows an
+    expert (one of them without any) to several tiles; a heavily uneven load."""
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    from distributed_neural_networks_amd.ops.gemm import ACT_SILU_MUL, pack_gate_up
+    g, dt = gen(M + E), DT[dtype]
+    z = torch.randn(M, E, generator=g)
+    z[:, E - 1] = -50  # an expert without rows
+    z[:, 0] += 3
+    if top == E:
+        z[:, E - 1] += 50
+    r = M_.Routing(M, E, top, dev())
+    M_.route(z.to(dev()), r, M, 1, 1)
+    ws = [[(torch.randn(a, b, generator=g) * 1.5 / math.sqrt(b)).bfloat16().float() for a, b in ((F, K), (F, K), (K, F))]
+          for _ in range(E)]
+    x = torch.randn(M, K, generator=g).to(dt)
+    up = M_.ExpertLinear([pack_gate_up(a, b) for a, b, _ in ws], dt, dev(), ACT_SILU_MUL)
+    down = M_.ExpertLinear([c for _, _, c in ws], dt, dev())
+    mid = torch.full((M * top, F + 8), 5.0, dtype=dt, device=dev())
+    out = torch.full((M * top, K + 8), 5.0, dtype=dt, device=dev())
+    sc = torch.empty(M * top, 2 * F, device=dev()) if dtype == "float32" else None
+    up(x.to(dev()), M * top, mid[:, :F], r, top, scratch=sc, clear=True)
+    down(mid[:, :F], M * top, out[:, :K], r)
+    assert (r.bins(0)[0] == 0).all() and (mid[:, F:] == 5).all() and (out[:, K:] == 5).all()
+    idx, order = r.idx.cpu().long(), r.order.cpu().long()
+    tol = 3e-6 if dtype == "float32" else 1e-2
+    for p in range(M * top):
+        a, b, c = (t.double() for t in ws[idx[order[p]]])
+        xd = x[order[p] // top].double()
+        ref = O.silu(a @ xd) * (b @ xd)
+        assert rel(mid[p, :F], ref) < tol
+        assert rel(out[p, :K], c @ mid[p, :F].double().cpu()) < tol
+
+
+# ------------------------------------------------------------------ whole models
+def smooth(d):
+    """The same model with every expert chosen: no close call of a router can
+    turn rounding into another choice, so bf16 is compared sharply too."""
+    d = copy.deepcopy(d)
+    for x in d["layers"]:
+        if x["mlp"]:
+            r = x["mlp"]["router"]
+            r["experts"] = min(r["experts"], 12 if "groups" not in r else r["groups"]["count"] * 2)
+            r["top"] = r["experts"]
+            if "groups" in r:
+                r["groups"]["keep"] = r["groups"]["count"]
+    return d
+
+
+MODELS = {**CASES, **{n + "~": smooth(d) for n, d in CASES.items()}}
+SHARP = [(n, "float32") for n in sorted(CASES)] + [(n + "~", "bf16") for n in sorted(CASES)]
+_WEIGHTS = {}
+
+
+def weights(name):
+    if name not in _WEIGHTS:
+        W = O.random_weights(MODELS[name], 11, gain=1.2)
+        _WEIGHTS[name] = (W, {k: v.double() for k, v in W.items()})
+    return _WEIGHTS[name]
+
+
+def model(name, dtype, num_pages=12, stages=1, max_batch=1, max_seq=768, num_slots=4, **kw):
+    from distributed_neural_networks_amd.models import funepel
+    from distributed_neural_networks_amd.runtime.decoder import DecoderStage
+    W = weights(name)[0]
+    c = funepel.parse_config(MODELS[name])
+    n = c.n_layer
+    cuts = [round(i * n / stages) for i in range(stages + 1)]
+    st = []
+    for i in range(stages):
+        a, b, f, l = cuts[i], cuts[i + 1] - 1, i == 0, i == stages - 1
+        sd = {k: W[k] for k in funepel.stage_key_map(c, a, b, f, l)}
+        st.append(DecoderStage(name, sd, a, b, f, l, dev(), max_batch=max_batch, max_seq=max_seq, dtype=dtype,
+                               num_pages=num_pages, num_slots=num_slots, cfg=c, **kw))
+    return st
+
+
+def engine(name, dtype, **kw):
+    from distributed_neural_networks_amd.runtime.engine import Engine
+    return Engine(model(name, dtype, **kw), max_slots=4)
+
+
+def tokens(name, n, seed=0):
+    return torch.randint(0, MODELS[name]["vocab"], (n,), generator=gen(seed)).tolist()
+
+
+_REFS = {}
+
+
+def reference(name, toks, rnd=O.exact):
+    key = (name, tuple(toks), rnd.__name__)
+    if key not in _REFS:
+        _REFS[key] = O.forward(torch.tensor(toks), MODELS[name], weights(name)[1], rnd=rnd)
+    return _REFS[key]
+
+
+def tol(name, dtype):
+    """Logits tolerance: fp32 rounding, or three times the error that bf16
+    projections alone make in the oracle."""
+    if dtype == "float32":
+        return F32_TOL
+    toks = tokens(name, 210)
+    t = 3 * row_errors(reference(name, toks, O.bf16), reference(name, toks)).max().item()
+    assert t < 0.3, t
+    return t
+
+
+def feed(eng, sid, toks, sizes):
+    """All logits of one sequence brought in portions of ``sizes`` (the last repeats)."""
+    from distributed_neural_networks_amd.runtime.engine import Entry
+    out, p, i = [], 0, 0
+    while p < len(toks):
+        n = min(sizes[min(i, len(sizes) - 1)], len(toks) - p)
+        out.append(eng.step([Entry(sid, toks[p:p + n], range(n))]).float().cpu())
+        p, i = p + n, i + 1
+    return torch.cat(out)
+
+
+@pytest.mark.parametrize("name,dtype", SHARP)
+def test_portions_match_oracle(name, dtype):
+    """The same logits however the prompt is cut: whole, token by token, portions
+    of 2, 3, 7, 64, 65, and a prompt followed by long decoding.  Every cut uses
+    the pages and the slot that the one before gave back."""
+    eng = engine(name, dtype)
+    toks = tokens(name, 210)
+    ref = reference(name, toks)
+    for i, sizes in enumerate([[210], [1], [2], [3], [7, 1], [64], [65], [63, 1, 66, 2], [20, 1]]):
+        err = row_errors(feed(eng, i, toks, sizes), ref).max().item()
+        assert err < tol(name, dtype), (sizes, err)
+        eng.end(i)
+
+
+@pytest.mark.parametrize("name", ["plain", "mixed", "wide"])
+def test_bf16_with_router_choices(name):
+    """bf16 where experts are chosen: rounding may flip a close call of a router,
+    so nearly all rows, not every one, must be close."""
+    eng = engine(name, "bf16")
+    toks = tokens(name, 210)
+    ref = reference(name, toks)
+    t = 3 * row_errors(reference(name, toks, O.bf16), ref).quantile(0.5).item()
+    whole = feed(eng, 0, toks, [210])
+    for got in (whole, feed(eng, 1, toks, [50, 1])):
+        err = row_errors(got, ref)
+        assert err.quantile(0.85).item() < 2 * t and t < 0.1, (err.quantile(0.85).item(), t)
+
+
+@pytest.mark.parametrize("name,dtype", [("plain", "float32"), ("mixed", "float32"), ("plain~", "bf16"), ("mixed~", "bf16")])
+def test_mixed_batches_and_reused_pages(name, dtype):
+    """Unequal sequences together — portions beside single tokens, sequences left
+    out of steps, pages and slots given back and used again — against each alone."""
+    from distributed_neural_networks_amd.runtime.engine import Entry
+    from distributed_neural_networks_amd.runtime.paging import pages_for
+    eng = engine(name, dtype, num_pages=9)
+    g = gen(4)
+    lengths = [1, 130, 67, 5, 190, 64, 90, 2, 128, 33]
+    seqs = {i: tokens(name, n, 100 + i) for i, n in enumerate(lengths)}
+    waiting, live, got, slots_seen = list(seqs), {}, {i: [] for i in seqs}, set()
+    while waiting or live:
+        while waiting and len(live) < 4 and \
+                sum(pages_for(lengths[i]) for i in live) + pages_for(lengths[waiting[0]]) <= 9:
+            live[waiting.pop(0)] = 0
+        entries = []
+        for i, p in live.items():
+            r = int(torch.randint(0, 6, (1,), generator=g))
+            if r == 0 and len(live) > 1:
+                continue  # left out of this step
+            n = min([1, 1, 2, 9, 64][r - 1], lengths[i] - p) if r else 1
+            entries.append(Entry(i, seqs[i][p:p + n], range(n)))
+        if not entries:
+            continue
+        y = eng.step(entries).float().cpu()
+        slots_seen |= {eng.live[e.id].slot for e in entries}
+        for e, part in zip(entries, torch.split(y, [len(e.tokens) for e in entries])):
+            got[e.id].append(part)
+            live[e.id] += len(e.tokens)
+            if live[e.id] == lengths[e.id]:
+                eng.end(e.id)
+                del live[e.id]
+    assert slots_seen == {0, 1, 2, 3} and eng.table.free_pages == 9
+    for i in seqs:
+        err = row_errors(torch.cat(got[i]), reference(name, seqs[i])).max().item()
+        assert err < tol(name, dtype), (i, lengths[i], err)
+
+
+def marked_model():
+    """Attention almost one-hot on token 1 (its key along one direction, the
+    distance bias small beside it), and a retention head that never forgets."""
+    d = config([layer(parallel(att(2, 1, 64, 0.5, 80, 0.0, 64), ret(1, 32, 64, (1.0,))))] * 2, 64, 64)
+    W = O.random_weights(d, 3)
+    for i in (0, 1):
+        p = f"l{i}."
+        mark = torch.zeros(64)
+        mark[5] = 1
+        W[p + "norm1"], W[p + "norm1.b"] = torch.ones(64), torch.zeros(64)
+        W[p + "norm1.b"][9] = 2.0  # a constant entry: every query asks for the mark
+        one = torch.zeros(64)
+        one[9] = 1
+        W[p + "mix.left.q"] = torch.outer(torch.ones(128), one)
+        W[p + "mix.left.k"] = W[p + "mix.left.k"] * 0.3 + 4 * torch.outer(torch.ones(64), mark)
+    W["embed"][:, 5] = -0.3
+    W["embed"][1, 5] = 4
+    return d, {k: v.bfloat16().float() for k, v in W.items()}
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bf16"])
+def test_marked_key_through_the_model(dtype):
+    """A marked token passes the window's edge and page borders while the model
+    decodes past it; the retention state carries it on."""
+    from distributed_neural_networks_amd.models import funepel
+    from distributed_neural_networks_amd.runtime.decoder import DecoderStage
+    from distributed_neural_networks_amd.runtime.engine import Engine
+    d, W = marked_model()
+    Wd = {k: v.double() for k, v in W.items()}
+    st = DecoderStage("marked", W, 0, 1, True, True, dev(), max_batch=1, max_seq=512, dtype=dtype, num_pages=8,
+                      num_slots=2, cfg=funepel.parse_config(d))
+    eng = Engine([st], max_slots=2)
+    base = [t if t != 1 else 2 for t in torch.randint(0, 64, (230,), generator=gen(9)).tolist()]
+    plain = O.forward(torch.tensor(base), d, Wd)
+    for n, key in enumerate([0, 63, 64, 100, 127, 128]):
+        toks = list(base)
+        toks[key] = 1
+        ref = O.forward(torch.tensor(toks), d, Wd)
+        limit = F32_TOL if dtype == "float32" else 3 * row_errors(O.forward(torch.tensor(toks), d, Wd, rnd=O.bf16), ref).max().item()
+        if key == 64 and dtype == "float32":
+            d2 = copy.deepcopy(d)
+            for x in d2["layers"]:
+                x["mixer"]["left"]["mask"]["size"] += 1
+            moved = row_errors(O.forward(torch.tensor(toks), d2, Wd), ref)
+            assert moved[64 + 80] > 2 * limit  # one key more in the window shows
+            assert row_errors(plain, ref)[65:].min() > 2 * limit  # and so does the state, long after the window
+        for sizes in ([230], [70, 1], [64, 2]):
+            err = row_errors(feed(eng, n, toks, sizes), ref).max().item()
+            assert err < limit, (key, sizes, err)
+            eng.end(n)
+
+
+def greedy(name, prompt, steps):
+    """Oracle greedy continuation; also the smallest top-2 gap on the way."""
+    seq, gap = list(prompt), 1e9
+    for _ in range(steps):
+        y = O.forward(torch.tensor(seq), MODELS[name], weights(name)[1])[-1]
+        top = y.topk(2).values
+        gap = min(gap, ((top[0] - top[1]) / y.std()).item())
+        seq.append(int(y.argmax()))
+    return seq[len(prompt):], gap
+
+
+@pytest.mark.parametrize("stages", [1, 2])
+@pytest.mark.parametrize("name", ["plain", "mixed"])
+def test_greedy_generation(name, stages):
+    """Greedy tokens of the oracle from the engine (unequal prompts, queueing,
+    several budgets) and from the decode ring (graphs, microbatches, chunks)."""
+    from distributed_neural_networks_amd.runtime.engine import Engine
+    from distributed_neural_networks_amd.runtime.scheduler import DecodeRing, RingLinks
+    prompts = [tokens(name, n, 40 + n) for n in (1, 66, 5, 30)]
+    want, gaps = zip(*(greedy(name, p, 6) for p in prompts))
+    assert min(gaps) > 1e-4  # fp32 cannot flip a greedy choice
+    eng = Engine(model(name, "float32", num_pages=5, stages=stages, max_seq=96, num_slots=2), max_slots=2)
+    for budget in (0, 40, 3):
+        assert eng.generate(prompts, 6, budget) == list(want)
+    st = model(name, "float32", num_pages=None, stages=stages, max_batch=4, max_seq=96, max_tokens=160)
+    same = [tokens(name, 33, 70 + i) for i in range(4)]
+    want = [greedy(name, p, 12)[0] for p in same]
+    for M, B, chunk, multi in ((1, 4, 0, 8), (2, 2, 10, 0), (1, 4, 32, 4)):
+        ring = DecodeRing(st, RingLinks(), 1, M, B, multi_step=multi)
+        got = ring.generate([torch.tensor(same[m * B:(m + 1) * B]) for m in range(M)], 33, 12, chunk)
+        assert got.tolist() == want, (M, B, chunk)
+
+
+def test_ring_graph_replays_match_eager():
+    """Captured decode steps (a warmup runs them once more: the states must not notice) against eager ones."""
+    from distributed_neural_networks_amd.runtime.scheduler import DecodeRing, RingLinks
+    st = model("plain~", "bf16", num_pages=None, max_batch=3, max_seq=200)
+    prompt = torch.tensor([tokens("plain~", 70, i) for i in range(3)])
+    a = DecodeRing(st, RingLinks(), 1, 1, 3, use_graphs=False).generate([prompt], 70, 100)
+    for multi in (4, 0):
+        assert torch.equal(a, DecodeRing(st, RingLinks(), 1, 1, 3, multi_step=multi).generate([prompt], 70, 100))
+
+
+def test_forward_all_positions_and_sampling():
+    name = "mixed~"
+    kw = dict(num_pages=None, stages=2, max_batch=2, max_seq=128)
+    st = model(name, "bf16", temperature=0.8, top_k=20, seed=5, **kw)
+    toks = torch.tensor([tokens(name, 90, i) for i in (1, 2)])
+    h = st[0].forward(toks)
+    assert h.shape == (2, 90, st[0].d) and h.dtype == torch.float32
+    y = st[1].forward(h.cpu())
+    for i in (0, 1):
+        assert row_errors(y.probs[i].float(), reference(name, toks[i].tolist())).max().item() < tol(name, "bf16")
+    from distributed_neural_networks_amd.runtime.engine import Engine
+    eng = Engine(st, max_slots=2)
+    p = [t.tolist() for t in toks]
+    a = eng.generate(p, 10)
+    assert a == eng.generate(p, 10) and all(0 <= t < MODELS[name]["vocab"] for r in a for t in r)
+    assert a != Engine(model(name, "bf16", **kw), max_slots=2).generate(p, 10)  # not the greedy tokens
+
+
+@pytest.mark.parametrize("parts", [1, 3])
+def test_cli_generation(tmp_path, capsys, parts):
+    """node.py on a model folder: one prompt through the decode ring, several
+    unequal ones through the engine; greedy tokens equal the oracle's."""
+    from distributed_neural_networks_amd import cli
+    O.save_model(str(tmp_path), MODELS["plain"], weights("plain")[0])
+    prompts = [tokens("plain", n, 40 + n) for n in (1, 66, 30)]
+    want = [greedy("plain", p, 6)[0] for p in prompts]
+    cfg = {"nodes": [{"id": f"n{i}", "address": f"127.0.0.1:{50790 + i}", "part_index": i} for i in range(parts)],
+           "model_weights": str(tmp_path), "num_parts": parts, "transport": "colocated", "model": str(tmp_path),
+           "dtype": "float32", "decode_steps": 6, "micro_batch_size": 2, "prefill_chunk": 16}
+    (tmp_path / "node.json").write_text(json.dumps(cfg))
+    for text, ref in ((";".join(",".join(map(str, p)) for p in prompts), want), (",".join(map(str, prompts[1])), [want[1]] * 2)):
+        assert cli.main(["--node_id", "n0", "--config", str(tmp_path / "node.json"), "--prompt", text]) == 0
+        out = capsys.readouterr().out
+        assert json.loads(next(ln for ln in out.splitlines() if "generated tokens:" in ln).split("generated tokens:")[1]) == ref
+
+
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_trace_runner(tmp_path, dtype):
+    """bin/trace_run as a program: a pool of live tokens only, logits per step."""
+    name = "mixed~" if dtype == "bfloat16" else "mixed"
+    O.save_model(str(tmp_path), MODELS[name], weights(name)[0])
+    seqs = {i: tokens(name, n, 7 + i) for i, n in enumerate((70, 64, 100))}
+    steps = [([(0, 0, 69), (1, 0, 2)], []), ([(0, 69, 70), (1, 2, 40)], [0]), ([(2, 0, 100), (1, 40, 41)], []),
+             ([(1, 41, 64)], [1, 2])]
+    lines, refs = [], []
+    for n, (parts, end) in enumerate(steps):
+        lines.append(json.dumps({"step": n, "end": [f"s{i}" for i in end], "entries": [
+            {"id": f"s{i}", "tokens": seqs[i][a:b], "want": list(range(b - a))} for i, a, b in parts]}))
+        refs.append(torch.cat([reference(name, seqs[i])[a:b] for i, a, b in parts]))
+    out = tmp_path / "out"
+    r = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", dtype, "--out",
+                        str(out), "--max-tokens", "192"], input="\n".join(lines) + "\n", capture_output=True, text=True,
+                       timeout=110)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == [f"done {n}" for n in range(4)]
+    for n, ref in enumerate(refs):
+        got = torch.from_numpy(np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(-1, MODELS[name]["vocab"]))
+        assert got.shape == ref.shape
+        assert row_errors(got, ref).max().item() < tol(name, "float32" if dtype == "float32" else "bf16")
+
+
+def test_refusals():
+    from distributed_neural_networks_amd.models import funepel
+    from distributed_neural_networks_amd.ops import decoder_ops as D_
+    from distributed_neural_networks_amd.ops import mixer_ops as M_
+    from distributed_neural_networks_amd.runtime.decoder import DecoderStage
+    from distributed_neural_networks_amd.runtime.engine import Engine
+    with pytest.raises(ValueError, match="dtype"):
+        model("plain", "fp8")
+    with pytest.raises(ValueError, match="GPU"):
+        DecoderStage("plain", {}, 0, 0, True, False, "cpu", cfg=funepel.parse_config(MODELS["plain"]))
+    st = model("ones", "bf16", num_pages=4, num_slots=2)
+    with pytest.raises(ValueError, match="states"):
+        Engine(st, max_slots=3)
+    r = M_.Routing(4, 8, 2, dev())
+    with pytest.raises(ValueError):
+        M_.route(torch.zeros(4, 8, device=dev()), r, 4, 1, 1, row0=1)
+    with pytest.raises(RuntimeError):
+        M_.route(torch.zeros(4, 8, device=dev()), r, 4, 3, 1)  # 8 experts in 3 groups
+    x = torch.zeros(2, 64, device=dev())
+    with pytest.raises(ValueError):
+        D_.rows_update(2, 64, x_in=x, y2=x, y2_norm=x[0], x_out=x)
