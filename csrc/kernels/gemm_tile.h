@@ -35,18 +35,8 @@ __device__ __forceinline__ bf16x8 lds_frag(const char* tile, int row, int chunk)
 }
 
 // Tile order: the XCD remap gives each XCD a contiguous run of logical ids;
-// inside it tiles go GROUP_M rows of M-tiles at a time, M fastest, so the ~32-64
-// tiles co-resident on one XCD share a few A and W panels in its L2.
-__device__ __forceinline__ void tile_coords(int logical, int ntm, int ntn, int& tm, int& tn) {
-  constexpr int GROUP_M = 8;
-  const int per_group = GROUP_M * ntn;
-  const int grp = logical / per_group;
-  const int first = grp * GROUP_M;
-  const int gm = min(ntm - first, GROUP_M);
-  const int r = logical - grp * per_group;
-  tm = first + r % gm;
-  tn = r / gm;
-}
+// inside it tiles go in groups of row tiles (grouped_tile.h tile_coords), so the
+// ~32-64 tiles co-resident on one XCD share a few A and W panels in its L2.
 
 // ---------------------------------------------------------------------------
 // Large-tile GEMM: 256x256x64, 8 waves (2 M x 4 N), ~1 block per CU, the

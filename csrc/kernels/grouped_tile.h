@@ -22,8 +22,21 @@ struct GroupTile {
   int expert, first, rows, tm, tn;  // first place and rows of the expert; expert < 0: past the last tile
 };
 
-// Tile `bid` of tiles of `bm` rows x ntn columns (m-tile major, neighbours on
-// one XCD).  Every lane of every wave calls it.
+// Tile order of a matrix of ntm x ntn tiles: groups of 8 row tiles, row tile
+// fastest, so that tiles running at the same time share panels of both operands.
+__device__ __forceinline__ void tile_coords(int logical, int ntm, int ntn, int& tm, int& tn) {
+  constexpr int GROUP_M = 8;
+  const int per_group = GROUP_M * ntn;
+  const int grp = logical / per_group;
+  const int first = grp * GROUP_M;
+  const int gm = min(ntm - first, GROUP_M);
+  const int r = logical - grp * per_group;
+  tm = first + r % gm;
+  tn = r / gm;
+}
+
+// Tile `bid` of tiles of `bm` rows x ntn columns: expert by expert, neighbours
+// on one XCD.  Every lane of every wave calls it.
 __device__ __forceinline__ GroupTile group_tile(const GroupedRows& g, int bm, int ntn, int bid, int lane) {
   if (g.counts != nullptr && bid == 0)
     for (int e = threadIdx.x; e < g.E; e += blockDim.x) g.counts[e] = 0;
@@ -46,16 +59,17 @@ __device__ __forceinline__ GroupTile group_tile(const GroupedRows& g, int bm, in
   GroupTile t{-1, 0, 0, 0, 0};
   if (bid >= total) return t;
   const int logical = xcd_remap(bid, total), mt = logical / ntn;
-  t.tn = logical - mt * ntn;
   const int src = __ffsll((unsigned long long)__ballot(incl > mt)) - 1;  // the lane whose experts hold the tile
-  int base = incl - sum, e = lane * 4, f = first[0], r = rows[0];
+  int base = incl - sum, e = lane * 4, f = first[0], r = rows[0], n = nt[0];
 #pragma unroll
   for (int i = 0; i < 3; ++i)
-    if (mt >= base + nt[i] && e == lane * 4 + i) base += nt[i], e = lane * 4 + i + 1, f = first[i + 1], r = rows[i + 1];
+    if (mt >= base + nt[i] && e == lane * 4 + i) 
+      base += nt[i], e = lane * 4 + i + 1, f = first[i + 1], r = rows[i + 1], n = nt[i + 1];
   t.expert = __builtin_amdgcn_readfirstlane(__shfl(e, src, 64));
   t.first = __builtin_amdgcn_readfirstlane(__shfl(f, src, 64));
   t.rows = __builtin_amdgcn_readfirstlane(__shfl(r, src, 64));
-  t.tm = mt - __builtin_amdgcn_readfirstlane(__shfl(base, src, 64));
+  tile_coords(logical - __builtin_amdgcn_readfirstlane(__shfl(base, src, 64)) * ntn,
+              __builtin_amdgcn_readfirstlane(__shfl(n, src, 64)), ntn, t.tm, t.tn);
   return t;
 }
 

@@ -369,8 +369,10 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     const size_t k0 = ((size_t)page * a.G + g) * PG + (unit % (PG / DU)) * DU;
     const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kp) + (k0 + r32) * DK + 8 * h;
     const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vp) + k0 * DV;
+    if (!a.shared) {
 #pragma unroll
-    for (int s = 0; s < NKS; ++s) kf[s] = *reinterpret_cast<const bf16x8*>(kb + s * 16);
+      for (int s = 0; s < NKS; ++s) kf[s] = *reinterpret_cast<const bf16x8*>(kb + s * 16);
+    }
 #pragma unroll
     for (int it = 0; it < NIV; ++it) pv[it] = *reinterpret_cast<const i32x4*>(vb + (it * 64 + lane) * 8);
     if (terms) {
@@ -384,13 +386,23 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     const int kb0 = u.at(i) * DU;
     f32x16 s[1];
     s[0] = f32x16{};
+    auto stage_v = [&]() __attribute__((always_inline)) {
+#pragma unroll
+      for (int it = 0; it < NIV; ++it) {
+        const int c = it * 64 + lane;
+        *reinterpret_cast<i32x4*>(vs + (c / CV) * PaV<DV>::STRIDE + (c % CV) * 16) = pv[it];
+      }
+    };
+    if (a.shared) {  // the tile was read once, as values: the keys come from LDS
+      stage_v();
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+#pragma unroll
+      for (int k = 0; k < NKS; ++k)
+        kf[k] = *reinterpret_cast<const bf16x8*>(vs + r32 * PaV<DV>::STRIDE + (DK == DV ? 2 * k + h : 0) * 16);
+    }
 #pragma unroll
     for (int k = 0; k < NKS; ++k) s[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[k], qf[k], s[0], 0, 0, 0);
-#pragma unroll
-    for (int it = 0; it < NIV; ++it) {
-      const int c = it * 64 + lane;
-      *reinterpret_cast<i32x4*>(vs + (c / CV) * PaV<DV>::STRIDE + (c % CV) * 16) = pv[it];
-    }
+    if (!a.shared) stage_v();
     if (terms) {
 #pragma unroll
       for (int q = 0; q < 4; ++q)

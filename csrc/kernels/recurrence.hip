@@ -219,22 +219,30 @@ __global__ __launch_bounds__(256) void scan_steps_kernel(ScanArgs a) {
 // remainder), so the recurrence keeps about 16 bits of mantissa.  Wave w: tokens (w & 1) * 32..,
 // value columns (w >> 1) * 32.. of the output; the same value columns and half
 // of the state rows in the update.
-constexpr int SC_L = 64;            // tokens of a chunk
-constexpr int SC_VST = 64 * 2 + 64;  // bytes of a value row in LDS
+constexpr int SC_L = 64;  // tokens of a chunk
 
 template <int NP>
 struct ScanLds {
-  static constexpr int KST = NP * 2 + 64, SST = NP * 2 + 16;
-  static constexpr int K = SC_L * KST, V = SC_L * SC_VST, S = 64 * SST;
+  static constexpr int SST = NP * 2 + 16;  // bytes of a state row: 16 rows of a fragment read are 64 banks
+  static constexpr int K = SC_L * NP * 2, V = SC_L * 128, S = 64 * SST;
   static constexpr int TOTAL = K + V + 2 * S + 3 * SC_L * 4;
 };
 
-// 8 values of column (lane & 31) of a 64-row LDS tile at rows 16 s + 4 h + {0..3, 8..11}
-__device__ __forceinline__ bf16x8 sc_tr(const char* tile, int stride, int s, int col0, int lane) {
-  const char* p = tile + (16 * s + 4 * (lane >> 5) + ((lane & 15) >> 2)) * stride +
-                  (col0 + ((lane >> 4) & 1) * 16 + 4 * (lane & 3)) * 2;
-  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(p));
-  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(p + 8 * stride));
+// Byte of 16-B piece c of row r in a tile of 64 rows of W bf16 values.  The
+// piece index is swizzled by the row so that both a fragment read (one piece of
+// 16 rows) and a transposing read (4 pieces of 8 rows) spread over all banks.
+template <int W>
+__device__ __forceinline__ int sc_at(int r, int c) {
+  const int f = W == 32 ? (r >> 2) & 3 : W == 64 ? ((r << 1) & 4) | ((r >> 2) & 3) : ((r & 3) << 2) | ((r >> 2) & 3);
+  return r * W * 2 + ((c ^ f) << 4);
+}
+// 8 values of column (lane & 31) of a tile at rows 16 s + 4 h + {0..3, 8..11}
+template <int W>
+__device__ __forceinline__ bf16x8 sc_tr(const char* tile, int s, int col0, int lane) {
+  const int r = 16 * s + 4 * (lane >> 5) + ((lane & 15) >> 2);
+  const int c = (col0 >> 3) + ((lane >> 4) & 1) * 2 + ((lane >> 1) & 1), b = (lane & 1) * 8;
+  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(tile + sc_at<W>(r, c) + b));
+  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((LDS_AS s16x4*)(tile + sc_at<W>(r + 8, c) + b));
   return bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
 }
 // Two values as one pair of bf16 (a single conversion)
@@ -294,42 +302,50 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
 
   i32x4 pk[NIK], pv[2];
   float pla = 0.f, pdt = 0.f;
+  // rows past the end repeat the last one: their weights are zero
   auto fetch = [&](int c0) __attribute__((always_inline)) {
-    const int len = min(SC_L, n - c0);
+    const bf16_t* cb = base + (size_t)c0 * a.ld;
+    const int last = min(SC_L, n - c0) - 1;
 #pragma unroll
     for (int it = 0; it < NIK; ++it) {
-      const int x = it * 256 + tid, r = x / CK, c = x % CK;
-      pk[it] = i32x4{0, 0, 0, 0};
-      if (r < len) pk[it] = *reinterpret_cast<const i32x4*>(base + (size_t)(c0 + r) * a.ld + kc + c * 8);
+      const int x = it * 256 + tid;
+      pk[it] = *reinterpret_cast<const i32x4*>(cb + min(x / CK, last) * a.ld + kc + (x % CK) * 8);
     }
 #pragma unroll
     for (int it = 0; it < 2; ++it) {
-      const int x = it * 256 + tid, r = x >> 3, c = x & 7;
-      pv[it] = i32x4{0, 0, 0, 0};
-      if (r < len) pv[it] = *reinterpret_cast<const i32x4*>(base + (size_t)(c0 + r) * a.ld + vc + c * 8);
+      const int x = it * 256 + tid;
+      pv[it] = *reinterpret_cast<const i32x4*>(cb + min(x >> 3, last) * a.ld + vc + (x & 7) * 8);
     }
     if (wave == 0) {
-      pla = pdt = 0.f;
-      if (lane < len) {
-        const size_t o = (size_t)(e.x + c0 + lane) * a.H + h;
-        pdt = a.dt != nullptr ? a.dt[o] : a.dt_c;
-        pla = a.la != nullptr ? a.la[o] : a.la_h[h];
-      }
+      const size_t o = (size_t)(e.x + c0 + min(lane, last)) * a.H + h;
+      pdt = a.dt != nullptr ? a.dt[o] : a.dt_c;
+      pla = a.la != nullptr ? a.la[o] : a.la_h[h];
+      if (lane > last) pla = pdt = 0.f;
     }
   };
   fetch(0);
   for (int c0 = 0; c0 < n; c0 += SC_L) {
     const int len = min(SC_L, n - c0);
+    float ps = pla, pw = 0.f;  // wave 0: sums of the decays' logarithms (base 2) and the weights from them
+    if (wave == 0) {
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float u = __shfl_up(ps, o, 64);
+        if (lane >= o) ps += u;
+      }
+      ps *= LOG2E;
+      pw = ps - __builtin_amdgcn_logf(pdt);  // dt_s exp(-A_s) as an exponent (dt 0: +inf, weight 0)
+    }
     __syncthreads();  // the last chunk is read
 #pragma unroll
     for (int it = 0; it < NIK; ++it) {
       const int x = it * 256 + tid;
-      *reinterpret_cast<i32x4*>(ks + (x / CK) * L::KST + (x % CK) * 16) = pk[it];
+      *reinterpret_cast<i32x4*>(ks + sc_at<NP>(x / CK, x % CK)) = pk[it];
     }
 #pragma unroll
     for (int it = 0; it < 2; ++it) {
       const int x = it * 256 + tid;
-      *reinterpret_cast<i32x4*>(vs + (x >> 3) * SC_VST + (x & 7) * 16) = pv[it];
+      *reinterpret_cast<i32x4*>(vs + sc_at<64>(x >> 3, x & 7)) = pv[it];
     }
     if (mine) {  // the state as an operand: rows of value columns, two terms
 #pragma unroll
@@ -345,17 +361,9 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
         }
     }
     if (wave == 0) {
-      float s = pla;
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const float u = __shfl_up(s, o, 64);
-        if (lane >= o) s += u;
-      }
-      s *= LOG2E;
-      const float w = s - __builtin_amdgcn_logf(pdt);  // dt_s exp(-A_s) as an exponent of 2 (dt 0: +inf, weight 0)
-      cum[lane] = s;
-      src[lane] = w;
-      wst[lane] = __builtin_amdgcn_exp2f(__shfl(s, 63, 64) - w);
+      cum[lane] = ps;
+      src[lane] = pw;
+      wst[lane] = __builtin_amdgcn_exp2f(__shfl(ps, 63, 64) - pw);
     }
     // this wave's queries as B operand: column = token
     const int tok = tt * 32 + r32;
@@ -380,7 +388,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
 #pragma unroll
       for (int k = 0; k < NK; ++k)
         g = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
-            *reinterpret_cast<const bf16x8*>(ks + (j * 32 + r32) * L::KST + (k * 16 + 8 * hh) * 2), qf[k], g, 0, 0, 0);
+            *reinterpret_cast<const bf16x8*>(ks + sc_at<NP>(j * 32 + r32, 2 * k + hh)), qf[k], g, 0, 0, 0);
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const int s0 = j * 32 + 8 * q + 4 * hh;
@@ -398,7 +406,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
         uint32_t hi[4], lo[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) sc_split2(g[8 * s + 2 * i], g[8 * s + 2 * i + 1], hi[i], lo[i]);
-        const bf16x8 vf = sc_tr(vs, SC_VST, 2 * j + s, vt * 32, lane);
+        const bf16x8 vf = sc_tr<64>(vs, 2 * j + s, vt * 32, lane);
         o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(hi), o, 0, 0, 0);
         o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, sc_frag(lo), o, 0, 0, 0);
       }
@@ -409,7 +417,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const int vl = vt * 32 + 8 * q + 4 * hh, v = v0 + vl;
-        const s16x4 x = *reinterpret_cast<const s16x4*>(vs + tok * SC_VST + vl * 2);
+        const s16x4 x = *reinterpret_cast<const s16x4*>(vs + sc_at<64>(tok, vl >> 3) + (vl & 7) * 2);
         float y[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) y[i] = fmaf(d, bf2f_s(x[i]), o[4 * q + i]);
@@ -428,7 +436,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
       for (int i = 0; i < NTW; ++i) S[i] *= dec;
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
-        const bf16x8 v = sc_tr(vs, SC_VST, s, vt * 32, lane);
+        const bf16x8 v = sc_tr<64>(vs, s, vt * 32, lane);
         const f32x4 w0 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh);
         const f32x4 w1 = *reinterpret_cast<const f32x4*>(wst + 16 * s + 4 * hh + 8);
         uint32_t hi[4], lo[4];
@@ -439,7 +447,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
         }
 #pragma unroll
         for (int i = 0; i < NTW; ++i) {
-          const bf16x8 kt = sc_tr(ks, L::KST, s, (nt0 + i) * 32, lane);
+          const bf16x8 kt = sc_tr<NP>(ks, s, (nt0 + i) * 32, lane);
           S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, sc_frag(hi), S[i], 0, 0, 0);
           S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kt, sc_frag(lo), S[i], 0, 0, 0);
         }

@@ -8,6 +8,7 @@
 #include <cstdio>
 
 #include "../kernels/api.h"
+#include "../kernels/mixer_api.h"
 #include "../kernels/residual_api.h"
 
 static int g_fail = 0;
@@ -47,12 +48,71 @@ int main() {
   rb = ra, rb.xidx = ip, rb.xrows = 1;
   expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows gathered in-place");
   expect_reject(dnn_rows_update(&ra, 0, 1, st), "rows bf16 in, fp32 operand out");
+  rb = ra, rb.y2 = f;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows second output without a norm");
+  rb = ra, rb.ys = f, rb.top = 2;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows of experts without places");
+  double freq = 0;
+  rb = ra, rb.freq = &freq;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "positions without positions");
+  {
+    ConvArgs c{};
+    c.in = f, c.out = f, c.M = 4, c.C = 64, c.taps = 4, c.ldi = c.ldo = 64, c.nslots = 1;
+    ConvArgs d = c;
+    d.C = 60;
+    expect_reject(dnn_conv(&d, 0, st), "conv channels % 8");
+    d = c, d.ldi = 32;
+    expect_reject(dnn_conv(&d, 0, st), "conv row too short");
+    d = c, d.dt = f, d.la = f, d.H = 8, d.dt_col = 60;
+    expect_reject(dnn_conv(&d, 0, st), "conv step sizes past the row");
+    expect_reject(dnn_conv_state(&c, nullptr, 0, 0, st), "conv state of nothing");
+    ScanArgs a{};
+    a.M = 4, a.H = 2, a.NP = 64, a.VP = 64, a.vdim = 64, a.nent = 1, a.nslots = 1, a.qdiv = 1, a.ld = 384, a.ldy = 128;
+    a.kcol = 128, a.vcol = 256, a.la_h = f, a.state = f, a.pos = reinterpret_cast<int*>(f);
+    auto scan = [&](auto edit, const char* what) {
+      ScanArgs b = a;
+      edit(b);
+      expect_reject(dnn_scan_chunks(&b, st), what);
+      expect_reject(dnn_scan_steps(&b, 0, st), what);
+    };
+    scan([](ScanArgs& b) { b.NP = 96; }, "scan state size 96");
+    scan([](ScanArgs& b) { b.vcol = 320; }, "scan values past the row");
+    scan([](ScanArgs& b) { b.vdim = 65; }, "scan value size past its padding");
+    scan([](ScanArgs& b) { b.la_h = nullptr; }, "scan without decays");
+    scan([](ScanArgs& b) { b.nent = 0; }, "scan of nothing");
+    GatedNormArgs g{};
+    g.M = 1, g.n = 65, g.groups = 2, g.ldy = g.ldz = g.ldo = 128;
+    expect_reject(dnn_gated_norm(&g, 0, st), "gated norm in unequal parts");
+    RouteArgs r{};
+    r.M = 4, r.E = r.ldl = 8, r.groups = 2, r.keep = 1, r.top = 5;
+    expect_reject(dnn_route(&r, st), "route more experts than the groups hold");
+    r.top = 2, r.groups = 3;
+    expect_reject(dnn_route(&r, st), "route unequal groups");
+    r.groups = 2, r.E = r.ldl = 512;
+    expect_reject(dnn_route(&r, st), "route too many experts");
+    GroupedArgs e{};
+    int offs[3] = {0, 1, 2};
+    e.A = e.W = e.Wsh = e.C = nullptr, e.offs = offs, e.rows = 2, e.arows = 2, e.div = 1, e.N = e.K = 64, e.E = 2;
+    e.lda = e.ldc = 64;
+    expect_reject(dnn_grouped_gemm(&e, st), "grouped product without weights");
+    expect_reject(dnn_grouped_gemm_f32(&e, st), "fp32 grouped product without weights");
+    e.Wsh = e.W = f, e.K = 48;
+    expect_reject(dnn_grouped_gemm(&e, st), "grouped product K % 64");
+    e.K = 64, e.ldc = 32;
+    expect_reject(dnn_grouped_gemm(&e, st), "grouped product result row too short");
+    QkNormArgs q{};
+    q.M = 1, q.H = 2, q.G = 1, q.DK = 64, q.ldq = 128, q.nq = 128, q.nk = 64, q.ldt = 1, q.npages = 1;
+    expect_reject(dnn_qk_norm(&q, 0, st), "qk norm row too short");
+    q.ldq = 192, q.nk = 65;
+    expect_reject(dnn_qk_norm(&q, 0, st), "qk norm of more than the projection");
+  }
   expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 8, ip, 5, p, 64, 4, 24, 64, st), "token gate past the row");
   expect_reject(dnn_token_gate(p, 64, p, 64, nullptr, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 64, st),
                 "token gate without the fragment copy");
   expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 48, st), "token gate np%64");
   expect_reject(dnn_gemm_f32(f, 24, f, 24, f, 8, nullptr, 4, 8, 24, st), "f32 gemm K%16");
-  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 12, st), "glu F%8");
+  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 12, 3, st), "glu F%8");
+  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 8, 1, st), "glu with a plain activation");
   PagedAttnArgs pa = {};
   pa.qkv = pa.kp = pa.vp = pa.out = p, pa.table = pa.slots = pa.pos = ip;
   pa.ldq = 256, pa.ldo = 64, pa.ldt = 1, pa.npages = 1, pa.M = 1, pa.H = pa.G = 1, pa.DK = pa.DV = 64;
@@ -70,6 +130,8 @@ int main() {
   bad([](PagedAttnArgs& b) { b.gate = 256; }, "paged gate past the row");
   bad([](PagedAttnArgs& b) { b.scale = -1.f; }, "paged negative scale");
   bad([](PagedAttnArgs& b) { b.table = nullptr; }, "paged without a block table");
+  bad([](PagedAttnArgs& b) { b.gate_el = 1, b.gate = 196; }, "paged gate per element past the row");
+  bad([](PagedAttnArgs& b) { b.shared = 1, b.written = 0; }, "paged shared keys that nobody wrote");
   expect_reject(dnn_paged_decode(&pa, ip, 1, 2, f, 4, st), "paged decode workspace too small");
   expect_reject(dnn_paged_decode(&pa, ip, 0, 1, nullptr, 0, st), "paged decode of nothing");
   expect_reject(dnn_paged_prefill(&pa, ip, 0, st), "paged prefill of nothing");

@@ -21,7 +21,7 @@ def test_host_validate_asan_ubsan():
     srcs = sorted(s for s in b.sources() if s.endswith(".hip")) + [os.path.join(ROOT, "csrc", "tests",
                                                                                  "host_validate.cpp")]
     h = hashlib.sha1()
-    for s in srcs + [os.path.join(ROOT, "csrc", "kernels", n) for n in ("api.h", "residual_api.h")]:
+    for s in srcs + [os.path.join(ROOT, "csrc", "kernels", n) for n in ("api.h", "mixer_api.h", "residual_api.h")]:
         h.update(open(s, "rb").read())
     out_dir = os.path.join(ROOT, "build", "asan")
     os.makedirs(out_dir, exist_ok=True)
