@@ -249,15 +249,16 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_prefill_k
     }
     if (terms) {
       const int page = max(pa_page(a, slot, u.at(i)), 0);
+      const float off = -slope * (float)(q_abs - kb0);
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
           const int k4 = kt * 32 + 8 * q + 4 * h;
           const f32x4 f = pa_kscale4(a, page, k4) * sc0;
+          const float c = fmaf(slope, (float)k4, off);
 #pragma unroll
-          for (int j = 0; j < 4; ++j)
-            s[kt][4 * q + j] = fmaf(s[kt][4 * q + j], f[j], -slope * (float)(q_abs - (kb0 + k4 + j)));
+          for (int j = 0; j < 4; ++j) s[kt][4 * q + j] = fmaf(s[kt][4 * q + j], f[j], fmaf(slope, (float)j, c));
         }
     }
     // every key visible to every query of the wave: no mask
@@ -404,11 +405,12 @@ __global__ __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) void paged_decode_ke
     for (int k = 0; k < NKS; ++k) s[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[k], qf[k], s[0], 0, 0, 0);
     if (!a.shared) stage_v();
     if (terms) {
+      const float off = -slope * (float)(p - kb0 - 4 * h);
 #pragma unroll
       for (int q = 0; q < 4; ++q)
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          s[0][4 * q + j] = fmaf(s[0][4 * q + j], ksc[q][j], -slope * (float)(p - (kb0 + 8 * q + 4 * h + j)));
+          s[0][4 * q + j] = fmaf(s[0][4 * q + j], ksc[q][j], fmaf(slope, (float)(8 * q + j), off));
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     if (i + 4 < ue) load(i + 4);

@@ -137,15 +137,17 @@ def test_gpt2_tiny_decode_ring_four_ranks_gloo_gpu(tmp_path):
 
 
 @pytest.mark.timeout(400)
-def test_kozusun_tiny_decode_ring_three_ranks_gloo_gpu(tmp_path):
-    """Kozusun over 3 ranks on GPU 0: the looped layers' passes lie on different
-    stages, boundary rows carry the fp32 residual and the token ids, and the
-    tokens equal those of one colocated stage."""
+@pytest.mark.parametrize("model", ["kozusun-tiny", "funepel-tiny"])
+def test_paged_decoder_ring_three_ranks_gloo_gpu(tmp_path, model):
+    """A paged decoder over 3 ranks on GPU 0: the looped layers' passes lie on
+    different stages (with caches and states of their own), boundary rows carry
+    the fp32 residual and the token ids, and the tokens equal those of one
+    colocated stage."""
     common = dict(prompt_len=70, decode_steps=6, micro_batch_size=2, num_microbatches=3, prefill_chunk=32,
                   dtype="float32")
     # device-generated weights: seeded by tensor name, the same on every rank
-    dist = _run(_cfg(tmp_path, "gloo_gpu", 3, "kozusun-tiny", "synthetic:5", **common), 3)
-    one = _run(_cfg(tmp_path, "colocated", 1, "kozusun-tiny", "synthetic:5", **common), 1)
+    dist = _run(_cfg(tmp_path, "gloo_gpu", 3, model, "synthetic:5", **common), 3)
+    one = _run(_cfg(tmp_path, "colocated", 1, model, "synthetic:5", **common), 1)
     got, want = (json.loads(o.split("generated tokens:")[1].strip().splitlines()[0]) for o in (dist, one))
     assert len(got) == 6 and all(len(t) == 6 for t in got) and got == want
     assert len({tuple(t) for t in got}) > 1
