@@ -300,6 +300,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
     }
   }
 
+  const int tok = tt * 32 + r32;  // this wave's queries as B operand: column = token
   i32x4 pk[NIK], pv[2];
   float pla = 0.f, pdt = 0.f;
   // rows past the end repeat the last one: their weights are zero
@@ -326,6 +327,10 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
   fetch(0);
   for (int c0 = 0; c0 < n; c0 += SC_L) {
     const int len = min(SC_L, n - c0);
+    const bf16_t* qp = base + (size_t)c0 * a.ld + min(tok, len - 1) * a.ld + qc + 8 * hh;
+    bf16x8 qf[NK];
+#pragma unroll
+    for (int k = 0; k < NK; ++k) qf[k] = *reinterpret_cast<const bf16x8*>(qp + k * 16);
     float ps = pla, pw = 0.f;  // wave 0: sums of the decays' logarithms (base 2) and the weights from them
     if (wave == 0) {
 #pragma unroll
@@ -365,12 +370,6 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunks_kernel(Sca
       src[lane] = pw;
       wst[lane] = __builtin_amdgcn_exp2f(__shfl(ps, 63, 64) - pw);
     }
-    // this wave's queries as B operand: column = token
-    const int tok = tt * 32 + r32;
-    const bf16_t* qp = base + (size_t)min(c0 + tok, n - 1) * a.ld + qc + 8 * hh;
-    bf16x8 qf[NK];
-#pragma unroll
-    for (int k = 0; k < NK; ++k) qf[k] = *reinterpret_cast<const bf16x8*>(qp + k * 16);
     __syncthreads();
     if (c0 + SC_L < n) fetch(c0 + SC_L);
 
