@@ -38,7 +38,8 @@ Scaling is weak: each stage-0 GPU sources ``--batch`` images per step.
 
 ``--model gpt2`` runs the GPT-2 4-stage token throughput bench instead
 (bench/gpt_bench.py); ``--model kozusun`` times Kozusun layers beside Llama
-layers of the same size, prefill and decode (bench/decoder_bench.py).
+layers of the same size, ``--model funepel`` Funepel layers beside Kozusun
+layers, prefill and decode (bench/decoder_bench.py).
 """
 from __future__ import annotations
 

@@ -225,7 +225,7 @@ __device__ __forceinline__ void epi_pair_scatter(f32x4 a0, f32x4 a1, int m, int 
 // NQ = 2: 256x256 tiles (4 phases per K-tile, below).  NQ = 1: 256x128 tiles
 // for N where the 256^2 grid leaves its last round of 256 CUs half empty
 // (GPT-2's 768-wide projections at M = 32768: 384 tiles = 1.5 rounds; as
-// 256x128 768 tiles = 3 full rounds of half-size tiles, VERDICT r3 item 4).
+// 256x128 768 tiles = 3 full rounds of half-size tiles).
 // Same waves (2 M x 4 N) and LDS images; a wave owns 2 x 1 quadrants of 64x32
 // and a K-tile is two phases:
 //     ph1: read B0 (4), A0 (8)  | stage A0, B0 [t+1] -> buf^1 | vmcnt(4) | C00

@@ -4,7 +4,7 @@ Reference behaviour (``node.py:294-325``): every stage ``torch.load``s the full
 state dict on CPU, wraps a throw-away full model in its part class and calls
 ``load_state_dict(full_sd, strict=False)``; missing/unexpected keys are only
 printed.  That trick silently loads nothing for GPT stages (their attribute
-names do not match ``transformer.h.{i}.*``, SURVEY §2.2 M8).  Here:
+names do not match ``transformer.h.{i}.*``).  Here:
 
 * ``load_full_state_dict`` accepts a plain ``.pth`` state dict (reference), a
   nanoGPT ``ckpt.pt`` dict (``{"model": sd}``, ``_orig_mod.`` prefixes

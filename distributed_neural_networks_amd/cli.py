@@ -303,7 +303,7 @@ async def initiate(ctx: NodeContext, args, stage, fwd, fam) -> int:
     # a CIFAR request is micro_batch_size x num_microbatches images (1 by default:
     # the reference's single image); with --metrics, stage 0 records every
     # request's end-to-end latency (forward, hop(s), result back) — the number
-    # BASELINE.md's survey measured for the reference
+    # measured for the reference
     rows = ctx.pipeline.micro_batch_size * ctx.pipeline.num_microbatches if fam == "cifar" else 1
     met = getattr(getattr(args, "_servicer", None), "metrics", None)
     for r in range(args.num_requests):

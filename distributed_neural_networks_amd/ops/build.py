@@ -27,8 +27,8 @@ TRANSFORMER_SRCS = ("norm_embed.hip", "attention.hip", "sampler.hip", "gemm_fp8.
 # No SLP vectoriser where it packs scalar FP32 into cross-half v_pk_*_f32 (op_sel
 # reads of a pair's other half) whose low result a 32-bit VALU op reads: under two
 # workgroups per CU that read returned the pre-op value in lanes 48-63 (the
-# one-shot GEMM's row statistics, csrc/kernels/gemm_oneshot.h "The race of rounds
-# 5-6"; 100 -> 0 mismatches in 10000 calls, profiles/r6_oneshot_race_root_cause.md).
+# one-shot GEMM's row statistics, csrc/kernels/gemm_oneshot.h; 100 -> 0
+# mismatches in 10000 calls, profiles/r6_oneshot_race_root_cause.md).
 NO_SLP = ["-fno-slp-vectorize"]
 # No packed FP32 instructions anywhere (some v_pk_*_f32 forms returned wrong
 # lanes, see above): explicit float2 / ext_vector code is split per element too.

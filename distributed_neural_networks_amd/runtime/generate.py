@@ -1,4 +1,4 @@
-"""CLI generation drivers for the transformer families (GPT-2 / Llama-3 / Kozusun).
+"""CLI generation drivers for the transformer families (GPT-2 / Llama-3 / paged decoders).
 
 The reference's GPT stages exist only as modules (``partitions/
 gpt_model_parts.py:6-50``) that recompute the whole prefix per call; nothing

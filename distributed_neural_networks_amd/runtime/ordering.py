@@ -1,4 +1,4 @@
-"""Debug-mode stream-ordering checks for slot buffers (race detection).
+"""Debug-mode stream-ordering checks for slot buffers.
 
 The streaming schedules (``runtime/pipeline.py``) reuse a ring of activation
 slots: a slot may be overwritten only after every asynchronous transfer that

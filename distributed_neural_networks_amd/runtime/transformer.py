@@ -447,7 +447,7 @@ class TransformerStage(StageCompute):
         # decode row statistics produced by the residual-writing projections
         # (O, c_proj: per-16-column {mean, M2} partials of h) and merged by the
         # next folded pre-norm projection (c_fc, the next layer's QKV) instead
-        # of every column-tile workgroup re-deriving them (VERDICT r4 item 2)
+        # of every column-tile workgroup re-deriving them
         rs = self.rowstat[r0:r1] if (T == 1 and self.fuse_norm and G_.ROWSTATS) else None
         have_rs = False
         for li, L in enumerate(self.layers):

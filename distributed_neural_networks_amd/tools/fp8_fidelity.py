@@ -1,4 +1,4 @@
-"""What fp8 weights cost at the model level (VERDICT r4 item 8).
+"""What fp8 weights cost at the model level.
 
 The fp8 kernel tests pin the GPT-2 XL fp8 stage against an fp32 golden on its
 own *dequantised* e4m3 weights: kernel fidelity.  This harness instead runs
