@@ -692,11 +692,16 @@ extern "C" int dnn_gemm_bf16(const void* A, int lda, const void* W, int ldw, voi
   DISPATCH(ACT_SILU_MUL)
 #endif
 #undef DISPATCH
-  if (act == ACT_GELU_TANH_MUL && !out_f32) {
-    launch_gemm<ACT_GELU_TANH_MUL, false>(A, lda, W, ldw, C, ldc, bias, R, ldr, M, N, K, st, Wsh, rs, colsum, ws,
-                                          ws_bytes);
-    return (int)hipGetLastError();
+#define DISPATCH_GLU(a)                                                                                              \
+  if (act == a && !out_f32) {                                                                                        \
+    launch_gemm<a, false>(A, lda, W, ldw, C, ldc, bias, R, ldr, M, N, K, st, Wsh, rs, colsum, ws, ws_bytes);         \
+    return (int)hipGetLastError();                                                                                   \
   }
+  DISPATCH_GLU(ACT_GELU_TANH_MUL)
+#ifdef DNN_DECODER_ONLY
+  DISPATCH_GLU(ACT_SILU_MUL)
+#endif
+#undef DISPATCH_GLU
   return -2;
 }
 

@@ -983,6 +983,9 @@ extern "C" int dnn_gemm_skinny(const void* A, int lda, const float* sa, const vo
   if (fp8 && (sa == nullptr || sw == nullptr)) return -1;
   const int la = lda * eb, lw = ldw * eb;
 #ifdef DNN_DECODER_ONLY
+  if (act == ACT_SILU_MUL && !fp8 && !out_f32)
+    return launch_skinny<ACT_SILU_MUL, false, false>(A, la, sa, W, lw, sw, C, ldc, bias, R, ldr, M, N, kbytes, st, nullptr,
+                                                     0.f, Wsh, ws, ws_bytes);
   if (act == ACT_NONE && !fp8)
     return out_f32 ? launch_skinny<ACT_NONE, true, false>(A, la, sa, W, lw, sw, C, ldc, bias, R, ldr, M, N, kbytes, st,
                                                           nullptr, 0.f, Wsh)

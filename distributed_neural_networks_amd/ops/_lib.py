@@ -61,7 +61,9 @@ def lib():
         _lib = _load_override(os.environ["DNN_HIP_LIB"])
     if _lib is None:
         errors = []
-        for name in ("_dnn_hip", "_dnn_decoder"):  # the full library, else the decoder subset (ops/build.py)
+        # the full library, else the decoder subset (ops/build.py); DNN_KERNELS=decoder: the subset
+        names = ("_dnn_decoder",) if os.environ.get("DNN_KERNELS") == "decoder" else ("_dnn_hip", "_dnn_decoder")
+        for name in names:
             spec = importlib.util.find_spec("distributed_neural_networks_amd." + name)
             if spec is None:
                 continue

@@ -676,9 +676,22 @@ def test_cli_generation(tmp_path, capsys, parts):
         assert json.loads(next(ln for ln in out.splitlines() if "generated tokens:" in ln).split("generated tokens:")[1]) == ref
 
 
+def subset_is_built():
+    """The decoder subset library of these sources (ops/build.py) lies beside the full one."""
+    from distributed_neural_networks_amd.ops import _lib, build
+    try:
+        return bool(os.path.exists(build.lib_path("decoder")) and _lib.verify_stamp(build.lib_path("decoder")))
+    except RuntimeError:
+        return False
+
+
+@pytest.mark.parametrize("kernels", ["full", "decoder"])
 @pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
-def test_trace_runner(tmp_path, dtype):
-    """bin/trace_run as a program: a pool of live tokens only, logits per step."""
+def test_trace_runner(tmp_path, dtype, kernels):
+    """bin/trace_run as a program: a pool of live tokens only, logits per step;
+    on the full library and on the subset that a fresh checkout compiles."""
+    if kernels == "decoder" and not subset_is_built():
+        pytest.skip("the decoder subset library is not built")
     name = "mixed~" if dtype == "bfloat16" else "mixed"
     O.save_model(str(tmp_path), MODELS[name], weights(name)[0])
     seqs = {i: tokens(name, n, 7 + i) for i, n in enumerate((70, 64, 100))}
@@ -692,7 +705,7 @@ def test_trace_runner(tmp_path, dtype):
     out = tmp_path / "out"
     r = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", dtype, "--out",
                         str(out), "--max-tokens", "192"], input="\n".join(lines) + "\n", capture_output=True, text=True,
-                       timeout=110)
+                       timeout=110, env=dict(os.environ, DNN_KERNELS=kernels))
     assert r.returncode == 0, r.stderr[-2000:]
     assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == [f"done {n}" for n in range(4)]
     for n, ref in enumerate(refs):
