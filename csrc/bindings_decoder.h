@@ -52,7 +52,7 @@ inline void bind_decoder(py::module_& m) {
       PF(RowsArgs, ys) PF(RowsArgs, ysi) PF(RowsArgs, ysw) PF(RowsArgs, n_b) PF(RowsArgs, pos) PF(RowsArgs, freq)
       VF(RowsArgs, xrows) VF(RowsArgs, yrows) VF(RowsArgs, ldx) VF(RowsArgs, ldy) VF(RowsArgs, ldcopy) VF(RowsArgs, ldh)
       VF(RowsArgs, M) VF(RowsArgs, N) VF(RowsArgs, NP) VF(RowsArgs, mult) VF(RowsArgs, eps) VF(RowsArgs, ldadd)
-      VF(RowsArgs, ldy2) VF(RowsArgs, ldys) VF(RowsArgs, ysrows) VF(RowsArgs, top) VF(RowsArgs, n_alpha);
+      VF(RowsArgs, ldy2) VF(RowsArgs, ldys) VF(RowsArgs, ysrows) VF(RowsArgs, top) VF(RowsArgs, n_alpha) VF(RowsArgs, y_joined);
   m.def("rows_update", [](const RowsArgs& a, int y_f32, int out_f32, u64 st) {
     return dnn_rows_update(&a, y_f32, out_f32, ST(st));
   });
@@ -81,6 +81,64 @@ inline void bind_decoder(py::module_& m) {
       VF(ScanArgs, VP) VF(ScanArgs, vdim) VF(ScanArgs, nent) VF(ScanArgs, nslots) VF(ScanArgs, dt_c);
   m.def("scan_steps", [](const ScanArgs& a, int f32, u64 st) { return dnn_scan_steps(&a, f32, ST(st)); });
   m.def("scan_chunks", [](const ScanArgs& a, u64 st) { return dnn_scan_chunks(&a, ST(st)); });
+  py::class_<PairArgs>(m, "PairArgs")
+      .def(py::init([] { return PairArgs{}; }))
+      PF(PairArgs, ids) PF(PairArgs, start) PF(PairArgs, last) PF(PairArgs, slots) PF(PairArgs, pos) PF(PairArgs, prev)
+      PF(PairArgs, rows) VF(PairArgs, mul_prev) VF(PairArgs, mul_cur) VF(PairArgs, buckets) VF(PairArgs, M)
+      VF(PairArgs, nslots);
+  m.def("pair_rows", [](const PairArgs& a, u64 st) { return dnn_pair_rows(&a, ST(st)); });
+  py::class_<ShiftArgs>(m, "ShiftArgs")
+      .def(py::init([] { return ShiftArgs{}; }))
+      PF(ShiftArgs, x) PF(ShiftArgs, mu) PF(ShiftArgs, out) PF(ShiftArgs, state) PF(ShiftArgs, start) PF(ShiftArgs, last)
+      PF(ShiftArgs, slots) PF(ShiftArgs, pos) VF(ShiftArgs, ostride) VF(ShiftArgs, ldx) VF(ShiftArgs, ldo) VF(ShiftArgs, M)
+      VF(ShiftArgs, NP) VF(ShiftArgs, n) VF(ShiftArgs, nslots);
+  m.def("token_shift", [](const ShiftArgs& a, int f32, u64 st) { return dnn_token_shift(&a, f32, ST(st)); });
+  py::class_<DecayArgs>(m, "DecayArgs")
+      .def(py::init([] { return DecayArgs{}; }))
+      PF(DecayArgs, t) PF(DecayArgs, w2) PF(DecayArgs, w0) PF(DecayArgs, la) VF(DecayArgs, ldt) VF(DecayArgs, M)
+      VF(DecayArgs, N) VF(DecayArgs, rank);
+  m.def("decay", [](const DecayArgs& a, int f32, u64 st) { return dnn_decay(&a, f32, ST(st)); });
+  py::class_<WkvArgs>(m, "WkvArgs")
+      .def(py::init([] { return WkvArgs{}; }))
+      PF(WkvArgs, r) PF(WkvArgs, k) PF(WkvArgs, v) PF(WkvArgs, la) PF(WkvArgs, u) PF(WkvArgs, state) PF(WkvArgs, y)
+      PF(WkvArgs, ent) PF(WkvArgs, pos) VF(WkvArgs, ld) VF(WkvArgs, ldy) VF(WkvArgs, M) VF(WkvArgs, H) VF(WkvArgs, NP)
+      VF(WkvArgs, dim) VF(WkvArgs, nent) VF(WkvArgs, nslots);
+  m.def("wkv_steps", [](const WkvArgs& a, int f32, u64 st) { return dnn_wkv_steps(&a, f32, ST(st)); });
+  m.def("wkv_chunks", [](const WkvArgs& a, u64 st) { return dnn_wkv_chunks(&a, ST(st)); });
+  py::class_<PolyNormArgs>(m, "PolyNormArgs")
+      .def(py::init([] { return PolyNormArgs{}; }))
+      PF(PolyNormArgs, z) PF(PolyNormArgs, w) VF(PolyNormArgs, ld) VF(PolyNormArgs, M) VF(PolyNormArgs, n)
+      VF(PolyNormArgs, eps);
+  m.def("poly_norm", [](const PolyNormArgs& a, int f32, u64 st) { return dnn_poly_norm(&a, f32, ST(st)); });
+  py::class_<RopeTable>(m, "RopeTable")
+      .def(py::init([](u64 freq, int pairs, float mag) {
+        RopeTable r;
+        r.freq = reinterpret_cast<const double*>(CP(freq)), r.pairs = pairs, r.mag = mag;
+        return r;
+      }));
+  m.def("rope_rows", [](u64 x, int ld, int hs, int M, int H, int RP, u64 pos, const RopeTable& r, int f32, u64 st) {
+    return dnn_rope_rows(P(x), ld, hs, M, H, RP, CIP(pos), &r, f32, ST(st));
+  });
+  py::class_<LatentPrepArgs>(m, "LatentPrepArgs")
+      .def(py::init([] { return LatentPrepArgs{}; }))
+      PF(LatentPrepArgs, rows) PF(LatentPrepArgs, kp) PF(LatentPrepArgs, qw) PF(LatentPrepArgs, cw)
+      PF(LatentPrepArgs, table) PF(LatentPrepArgs, slots) PF(LatentPrepArgs, pos) VF(LatentPrepArgs, rope)
+      VF(LatentPrepArgs, ld) VF(LatentPrepArgs, ldt) VF(LatentPrepArgs, npages) VF(LatentPrepArgs, M)
+      VF(LatentPrepArgs, QN) VF(LatentPrepArgs, QP) VF(LatentPrepArgs, CN) VF(LatentPrepArgs, CP) VF(LatentPrepArgs, RP)
+      VF(LatentPrepArgs, eps);
+  m.def("latent_prep", [](const LatentPrepArgs& a, int f32, u64 st) { return dnn_latent_prep(&a, f32, ST(st)); });
+  py::class_<LatentAttnArgs>(m, "LatentAttnArgs")
+      .def(py::init([] { return LatentAttnArgs{}; }))
+      PF(LatentAttnArgs, qlat) PF(LatentAttnArgs, qrot) PF(LatentAttnArgs, kp) PF(LatentAttnArgs, table)
+      PF(LatentAttnArgs, slots) PF(LatentAttnArgs, pos) PF(LatentAttnArgs, out) PF(LatentAttnArgs, gate)
+      VF(LatentAttnArgs, ldql) VF(LatentAttnArgs, ldqr) VF(LatentAttnArgs, hs) VF(LatentAttnArgs, ldo)
+      VF(LatentAttnArgs, ldg) VF(LatentAttnArgs, ldt) VF(LatentAttnArgs, npages) VF(LatentAttnArgs, M)
+      VF(LatentAttnArgs, H) VF(LatentAttnArgs, CP) VF(LatentAttnArgs, RP) VF(LatentAttnArgs, scale);
+  m.def("latent_attn", [](const LatentAttnArgs& a, u64 tiles, int ntiles, int splits, int per_token, u64 ws,
+                          long long ws_elems, u64 st) {
+    return dnn_latent_attn(&a, CIP(tiles), ntiles, splits, per_token, FP(ws), ws_elems, ST(st));
+  });
+  m.def("latent_attn_f32", [](const LatentAttnArgs& a, u64 st) { return dnn_latent_attn_f32(&a, ST(st)); });
   py::class_<GatedNormArgs>(m, "GatedNormArgs")
       .def(py::init([] { return GatedNormArgs{}; }))
       PF(GatedNormArgs, y) PF(GatedNormArgs, z) PF(GatedNormArgs, w) PF(GatedNormArgs, out) VF(GatedNormArgs, ldy)
@@ -91,14 +149,16 @@ inline void bind_decoder(py::module_& m) {
       .def(py::init([] { return RouteArgs{}; }))
       PF(RouteArgs, logits) PF(RouteArgs, idx) PF(RouteArgs, w) PF(RouteArgs, rank) PF(RouteArgs, counts)
       PF(RouteArgs, order) PF(RouteArgs, place) PF(RouteArgs, offs) VF(RouteArgs, ldl) VF(RouteArgs, M) VF(RouteArgs, E)
-      VF(RouteArgs, groups) VF(RouteArgs, keep) VF(RouteArgs, top);
+      VF(RouteArgs, groups) VF(RouteArgs, keep) VF(RouteArgs, top) PF(RouteArgs, correction) VF(RouteArgs, sigmoid) VF(RouteArgs, group_top)
+      VF(RouteArgs, normalise);
   m.def("route", [](const RouteArgs& a, u64 st) { return dnn_route(&a, ST(st)); });
   py::class_<GroupedArgs>(m, "GroupedArgs")
       .def(py::init([] { return GroupedArgs{}; }))
       PF(GroupedArgs, A) PF(GroupedArgs, W) PF(GroupedArgs, Wsh) PF(GroupedArgs, C) PF(GroupedArgs, offs)
       PF(GroupedArgs, order) PF(GroupedArgs, counts) VF(GroupedArgs, lda) VF(GroupedArgs, ldc) VF(GroupedArgs, rows)
       VF(GroupedArgs, arows) VF(GroupedArgs, div) VF(GroupedArgs, N) VF(GroupedArgs, K) VF(GroupedArgs, E)
-      VF(GroupedArgs, act);
+      VF(GroupedArgs, act) VF(GroupedArgs, sa) VF(GroupedArgs, sc)
+      .def("set_clamp", [](GroupedArgs& a, float limit, float alpha, float shift) { a.clamp = {limit, alpha, shift}; });
   m.def("grouped_gemm", [](const GroupedArgs& a, u64 st) { return dnn_grouped_gemm(&a, ST(st)); });
   m.def("grouped_gemm_f32", [](const GroupedArgs& a, u64 st) { return dnn_grouped_gemm_f32(&a, ST(st)); });
   m.def("token_gate", [](u64 x, int ldx, u64 w, int ldw, u64 wsh, int K, u64 table, int ldt, int off, u64 tok, int V,
@@ -110,9 +170,12 @@ inline void bind_decoder(py::module_& m) {
                              int np, u64 st) {
     return dnn_token_gate_f32(CFP(z), ldz, CFP(table), ldt, off, CIP(tok), V, FP(g), ldg, M, n, np, ST(st));
   });
-  m.def("glu_f32", [](u64 gu, int ldi, u64 out, int ldo, int M, int F, int act, u64 st) {
-    return dnn_glu_f32(CFP(gu), ldi, FP(out), ldo, M, F, act, ST(st));
-  });
+  m.def("glu_f32", [](u64 gu, int ldi, u64 out, int ldo, int M, int F, int act, u64 st, float limit, float alpha,
+                      float shift) {
+    const GluClamp c{limit, alpha, shift};
+    return dnn_glu_f32(CFP(gu), ldi, FP(out), ldo, M, F, act, &c, ST(st));
+  }, py::arg("gu"), py::arg("ldi"), py::arg("out"), py::arg("ldo"), py::arg("M"), py::arg("F"), py::arg("act"),
+     py::arg("st"), py::arg("limit") = 0.f, py::arg("alpha") = 0.f, py::arg("shift") = 0.f);
   m.def("gemm_f32", [](u64 A, int lda, u64 W, int ldw, u64 C, int ldc, u64 bias, int M, int N, int K, u64 st) {
     return dnn_gemm_f32(CFP(A), lda, CFP(W), ldw, FP(C), ldc, CFP(bias), M, N, K, ST(st));
   });

@@ -4,20 +4,30 @@
 // and the 4 consecutive columns n = .. + 4*(l>>4) + r, r = 0..3.
 #pragma once
 #include "common.h"
+#include "glu_clamp.h"
 
 namespace dnn {
 
-enum Act { ACT_NONE = 0, ACT_RELU = 1, ACT_GELU = 2, ACT_SILU_MUL = 3, ACT_GELU_TANH_MUL = 4 };
+enum Act { ACT_NONE = 0, ACT_RELU = 1, ACT_GELU = 2, ACT_SILU_MUL = 3, ACT_GELU_TANH_MUL = 4, ACT_CLAMP_MUL = 5 };
 
 // Gated activations: the weight holds packed gate|up rows (ops/gemm.py
 // pack_gate_up) and the output act(gate) * up has half its columns.
-__host__ __device__ constexpr bool is_glu(int act) { return act == ACT_SILU_MUL || act == ACT_GELU_TANH_MUL; }
+__host__ __device__ constexpr bool is_glu(int act) {
+  return act == ACT_SILU_MUL || act == ACT_GELU_TANH_MUL || act == ACT_CLAMP_MUL;
+}
 
 // Activation of the gate half.
 template <int ACT>
 __device__ __forceinline__ float glu_gate(float g) {
   if constexpr (ACT == ACT_GELU_TANH_MUL) return gelu_tanh(g);
   return silu(g);
+}
+
+// Gate and up joined by the clamped activation.
+__device__ __forceinline__ float glu_clamped(float g, float u, const GluClamp& c) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * c.alpha * -1.4426950408889634f)) * (u + c.shift);
 }
 
 // Vector epilogue stores need 4-column-aligned rows and 16-B aligned bases.
@@ -339,7 +349,8 @@ __device__ __forceinline__ void epi_glu_t4(const f32x4& acc, int m, int ncol0, i
 // (ncol0 = tile j's first output column).
 template <int ACT, bool OUT_F32>
 __device__ __forceinline__ void epi_glu_pair(const f32x4& a0, const f32x4& a1, int m, int ncol0, int M, int NO,
-                                              void* __restrict__ Cv, int ldc, bool vec, int lane) {
+                                              void* __restrict__ Cv, int ldc, bool vec, int lane,
+                                              const GluClamp& clamp = {}) {
   f32x4 v;
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -347,6 +358,8 @@ __device__ __forceinline__ void epi_glu_pair(const f32x4& a0, const f32x4& a1, i
     const float g = __uint_as_float(s[0]), u = __uint_as_float(s[1]);
     if constexpr (ACT == ACT_GELU_TANH_MUL)
       v[r] = gelu_tanh(g) * u;
+    else if constexpr (ACT == ACT_CLAMP_MUL)
+      v[r] = glu_clamped(g, u, clamp);
     else
       v[r] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * -1.4426950408889634f)) * u;
   }

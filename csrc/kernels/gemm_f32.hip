@@ -27,8 +27,9 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
     if (t.expert < 0) return;
     n0 = t.tn * F32_T, m0 = t.tm * F32_T, M = t.rows;
     W += (size_t)t.expert * N * ldw;
-    C += (size_t)t.first * ldc;
-    arow = grp.row(t.first + min(m0 + row, M - 1));
+    A += grp.a_off(t.expert);
+    C += grp.c_off(t.expert, t.first, ldc);
+    arow = grp.row(t.first, min(m0 + row, M - 1));
   }
   const float* ap = A + (size_t)arow * lda + kc;
   const float* wp = W + (size_t)min(n0 + row, N - 1) * ldw + kc;
@@ -79,11 +80,12 @@ extern "C" int dnn_gemm_f32(const float* A, int lda, const float* W, int ldw, fl
 extern "C" int dnn_grouped_gemm_f32(const GroupedArgs* a, hipStream_t st) {
   using namespace dnn;
   if (a->rows <= 0 || a->E <= 0 || a->E > EXPERTS_MAX || a->N <= 0 || a->K <= 0 || a->K % F32_K != 0 || a->lda % 4 != 0 ||
-      a->lda < a->K || a->ldc < a->N || a->div < 1 || a->arows < 1 || a->W == nullptr || a->offs == nullptr)
+      a->lda < a->K || a->ldc < a->N || a->div < 1 || a->arows < 1 || a->W == nullptr ||
+      (a->offs == nullptr && (a->rows % a->E != 0 || a->sa < 0 || a->sa % 4 != 0 || a->sc < 0)))
     return -1;
   const long n = (long)group_tiles_max(a->rows, F32_T, a->E) * ((a->N + F32_T - 1) / F32_T);
   if (n > 0x7fffffff) return -1;
-  const GroupedRows g{a->offs, a->order, a->counts, a->E, a->div, a->arows};
+  const GroupedRows g{a->offs, a->order, a->counts, a->E, a->div, a->arows, a->rows / a->E, a->sa, a->sc, a->clamp};
   hipLaunchKernelGGL(gemm_f32_kernel<true>, dim3((unsigned)n), dim3(256), 0, st, (const float*)a->A, a->lda,
                      (const float*)a->W, a->K, (float*)a->C, a->ldc, (const float*)nullptr, a->rows, a->N, a->K, g);
   return (int)hipGetLastError();

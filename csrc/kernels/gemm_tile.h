@@ -253,10 +253,11 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
     if (t.expert < 0) return;
     tm = t.tm, tn = t.tn, M = t.rows;
     W += (size_t)t.expert * N * K;
-    Cv = reinterpret_cast<bf16_t*>(Cv) + (size_t)t.first * ldc;
+    A += grp.a_off(t.expert);
+    Cv = reinterpret_cast<bf16_t*>(Cv) + grp.c_off(t.expert, t.first, ldc);
 #pragma unroll
     for (int x = 0; x < 4; ++x)
-      ga[x] = grp.row(t.first + min(tm * BG_M + (x >> 1) * 128 + ((x & 1) * 8 + wave) * 8 + (lane >> 3), M - 1));
+      ga[x] = grp.row(t.first, min(tm * BG_M + (x >> 1) * 128 + ((x & 1) * 8 + wave) * 8 + (lane >> 3), M - 1));
   } else {
     const int ntm = (M + BG_M - 1) / BG_M;
     tile_coords(xcd_remap(blockIdx.x, ntm * ntn), ntm, ntn, tm, tn);
@@ -522,7 +523,8 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_256_kernel(
         const int m = m0 + mq * 128 + arow + i * 16 + (lane & 15);
         const int nb = n0 + nq * 128 + wc * 32;
         if (is_glu(ACT)) {
-          epi_glu_pair<ACT, OUT_F32>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb / 2, M, N / 2, Cv, ldc, vec, lane);
+          epi_glu_pair<ACT, OUT_F32>(acc[mq][nq][i][0], acc[mq][nq][i][1], m, nb / 2, M, N / 2, Cv, ldc, vec, lane,
+                                     grp.clamp);
         } else if (SCATTER) {
           // widened 16-B stores as in epi_pair_bf16, to the head-major / cache
           // destination of the lane's 8 columns (host: ACT_NONE, bf16 out, no

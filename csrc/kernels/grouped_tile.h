@@ -1,7 +1,9 @@
 // Tiles of rows that are sorted by expert: expert e owns the places
-// offs[e] .. offs[e + 1] - 1; a tile never crosses a border.
+// offs[e] .. offs[e + 1] - 1; a tile never crosses a border.  Without offs every
+// expert has `per` rows, at A + e * sa and C + e * sc.
 #pragma once
 #include "common.h"
+#include "glu_clamp.h"
 
 namespace dnn {
 
@@ -12,9 +14,18 @@ struct GroupedRows {
   const int* order;  // source of a place: order[place] / div (nullptr: the place itself)
   int* counts;       // zeroed by the first workgroup (nullptr: not)
   int E, div, arows;
-  __device__ __forceinline__ int row(int place) const {
-    const int r = order != nullptr ? order[place] / div : place;
-    return min(max(r, 0), arows - 1);
+  int per = 0;
+  long long sa = 0, sc = 0;
+  GluClamp clamp = {};
+  // Row r of the expert with places from `first`, among the rows from a_off on.
+  __device__ __forceinline__ int row(int first, int r) const {
+    if (offs == nullptr) return r;
+    const int x = order != nullptr ? order[first + r] / div : first + r;
+    return min(max(x, 0), arows - 1);
+  }
+  __device__ __forceinline__ size_t a_off(int expert) const { return offs == nullptr ? (size_t)(expert * sa) : 0; }
+  __device__ __forceinline__ size_t c_off(int expert, int first, int ldc) const {
+    return offs == nullptr ? (size_t)(expert * sc) : (size_t)first * ldc;
   }
 };
 
@@ -44,8 +55,13 @@ __device__ __forceinline__ GroupTile group_tile(const GroupedRows& g, int bm, in
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int e = min(lane * 4 + i, g.E);
-    first[i] = g.offs[e];
-    rows[i] = g.offs[min(e + 1, g.E)] - first[i];
+    if (g.offs != nullptr) {
+      first[i] = g.offs[e];
+      rows[i] = g.offs[min(e + 1, g.E)] - first[i];
+    } else {
+      first[i] = e * g.per;
+      rows[i] = e < g.E ? g.per : 0;
+    }
     nt[i] = (rows[i] + bm - 1) / bm;
     sum += nt[i];
   }

@@ -1,7 +1,8 @@
-// C ABI of the recurrent mixers (recurrence.hip) and the mixture of experts
-// (moe.hip).  Every function enqueues on `st`; 0 = success, negative = rejected shape.
+// C ABI of the recurrent mixers (recurrence.hip, token_shift.hip, wkv.hip) and
+// the mixture of experts (moe.hip).  Every function enqueues on `st`; 0 = success, negative = rejected shape.
 #pragma once
 #include <hip/hip_runtime.h>
+#include "glu_clamp.h"
 
 // Short causal convolution per channel over the rows of a step, with silu, and
 // the step sizes of a recurrence beside it.  `ring` keeps the last inputs of
@@ -52,9 +53,65 @@ struct GatedNormArgs {
   float eps;
 };
 
-// Router: softmax over E logits, the best `keep` of `groups` groups of
-// neighbours (by their largest score), the `top` best experts in them, weights
-// normalised over the chosen.  Sorted placement of every (row, choice):
+// Row of a table of (previous token, token) pairs for every row of a step:
+//   (prev * mul_prev + id * mul_cur) mod buckets, row `buckets` for a first token.
+// `prev` [slot] keeps the last token of every sequence.
+struct PairArgs {
+  const int* ids;
+  const int* start;    // per row: first row of its sequence's portion in this step
+  const int* last;     // per row: last row of it
+  const int* slots;
+  const int* pos;
+  int* prev;
+  int* rows;           // [M]
+  long long mul_prev, mul_cur, buckets;
+  int M, nslots;
+};
+
+// n mixes of every row of x with the row before it: out_i = x + (prev - x) * mu_i.
+struct ShiftArgs {
+  const float* x;      // rows [NP], stride ldx
+  const float* mu;     // [n][NP]
+  void* out;           // n x rows [NP], stride ldo, `ostride` elements from mix to mix
+  float* state;        // [slot][NP]: the last row of every sequence
+  const int* start;
+  const int* last;
+  const int* slots;
+  const int* pos;
+  long long ostride;
+  int ldx, ldo, M, NP, n, nslots;
+};
+
+// la = -exp(W2 tanh(t) + w0): logarithms of decays from a low-rank projection.
+struct DecayArgs {
+  const float* t;      // rows [rank], stride ldt
+  const void* w2;      // [N][rank] in bf16 (rank a multiple of 32), or fp32
+  const float* w0;     // [N]
+  float* la;           // [M][N]
+  int ldt, M, N, rank;
+};
+
+// Recurrence with a decay per key channel and a bonus u for the current token,
+// state fp32 [slot][H][NP values][NP key channels]:
+//   y = (S + diag(u) k v^T)^T r,   S <- diag(exp(la)) S + k v^T
+struct WkvArgs {
+  const void* r;       // rows [H * NP] each, stride ld
+  const void* k;
+  const void* v;
+  const float* la;     // [M][H * NP]
+  const float* u;      // [H][NP]
+  float* state;
+  void* y;             // rows [H * dim], stride ldy
+  const int4* ent;     // sequences of the step: {first row, tokens, slot, -}
+  const int* pos;
+  int ld, ldy, M, H, NP, dim, nent, nslots;
+};
+
+// Router over E logits: scores s are softmax or (sigmoid != 0) sigmoid; choice
+// scores are s + correction.  The best `keep` of `groups` groups of neighbours
+// (by the sum of their group_top largest choice scores, 1 or 2), the `top` best
+// experts in them; weights are the chosen s, normalised over the chosen if
+// asked for.  Sorted placement of every (row, choice):
 //   order[place] = row * top + choice,  place[row * top + choice],  offs[E + 1]
 struct RouteArgs {
   const float* logits;
@@ -66,10 +123,14 @@ struct RouteArgs {
   int* place;
   int* offs;
   int ldl, M, E, groups, keep, top;
+  const float* correction = nullptr;  // [E]
+  int sigmoid = 0, group_top = 1, normalise = 1;
 };
 
 // Products of rows sorted by expert with that expert's weight:
 //   C[p] = act(A[row(p)] W_e^T),  e the expert whose range holds place p.
+// Without offs, expert e has the rows / E rows A + e * sa and C + e * sc (heads
+// with projections of their own, several projections of one launch).
 struct GroupedArgs {
   const void* A;       // row(p) = order[p] / div (order == nullptr: p)
   const void* W;       // [E][N][K]
@@ -79,6 +140,8 @@ struct GroupedArgs {
   const int* order;
   int* counts;         // zeroed on the way (nullptr: not)
   int lda, ldc, rows, arows, div, N, K, E, act;
+  long long sa = 0, sc = 0;
+  GluClamp clamp = {};
 };
 
 extern "C" {
@@ -86,6 +149,11 @@ int dnn_conv(const ConvArgs* a, int f32, hipStream_t st);
 int dnn_conv_state(const ConvArgs* a, const int4* ent, int nent, int f32, hipStream_t st);
 int dnn_scan_steps(const ScanArgs* a, int f32, hipStream_t st);   // token by token
 int dnn_scan_chunks(const ScanArgs* a, hipStream_t st);           // bf16, 64-token chunks on the MFMA
+int dnn_pair_rows(const PairArgs* a, hipStream_t st);
+int dnn_token_shift(const ShiftArgs* a, int f32, hipStream_t st);
+int dnn_decay(const DecayArgs* a, int f32, hipStream_t st);
+int dnn_wkv_steps(const WkvArgs* a, int f32, hipStream_t st);     // token by token
+int dnn_wkv_chunks(const WkvArgs* a, hipStream_t st);             // bf16, on the MFMA
 int dnn_gated_norm(const GatedNormArgs* a, int f32, hipStream_t st);
 int dnn_route(const RouteArgs* a, hipStream_t st);
 int dnn_grouped_gemm(const GroupedArgs* a, hipStream_t st);       // bf16

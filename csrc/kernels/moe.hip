@@ -1,8 +1,8 @@
 // Mixture of experts (gfx950): router selection, placement of rows by expert,
 // and products of the placed rows with their experts' weights.
 //
-//   route        softmax over the router logits, the best experts within the
-//                best groups, normalised weights, and a place for every
+//   route        softmax or sigmoid of the router logits, the best experts
+//                within the best groups, their weights, and a place for every
 //                (row, choice) so that an expert's rows are neighbours; one
 //                workgroup for up to 64 rows, two launches beyond
 //   grouped GEMM many rows per expert: the 256x256 tile kernel (gemm_tile.h)
@@ -24,7 +24,7 @@ template <typename F>
 __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, int l, int half, F f) {
   constexpr int NR = EXPERTS_MAX / 32;
   const int nr = (a.E + 31) / 32;  // registers that hold experts
-  float s[NR];
+  float s[NR], w[NR];  // choice scores, scores
   float mx = -INFINITY;
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
@@ -32,25 +32,32 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, 
     s[i] = live && i < nr && e < a.E ? a.logits[(size_t)m * a.ldl + e] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
-  mx = group_max<32>(mx);
-  if (!live) mx = 0.f;
-  float sum = 0.f;
+  if (a.sigmoid) {
 #pragma unroll
-  for (int i = 0; i < NR; ++i) {
-    s[i] = expf(s[i] - mx);  // 0 past the experts
-    sum += s[i];
+    for (int i = 0; i < NR; ++i) w[i] = 1.0f / (1.0f + expf(-s[i]));
+  } else {
+    mx = group_max<32>(mx);
+    if (!live) mx = 0.f;
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      s[i] = expf(s[i] - mx);  // 0 past the experts
+      sum += s[i];
+    }
+    sum = live ? group_sum<32>(sum) : 1.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) w[i] = s[i] / sum;
   }
-  sum = live ? group_sum<32>(sum) : 1.f;
   const int per = a.E / a.groups;
   int grp[NR];
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
-    s[i] /= sum;
+    s[i] = a.correction != nullptr && i < nr && i * 32 + l < a.E ? w[i] + a.correction[i * 32 + l] : w[i];
     grp[i] = i < nr ? (i * 32 + l) / per : 0;
   }
   // the best expert among ok: the largest score, the lower index first
   auto best = [&](unsigned ok, float& v) __attribute__((always_inline)) {
-    float m1 = -1.f;
+    float m1 = -INFINITY;
 #pragma unroll
     for (int i = 0; i < NR; ++i)
       if (i < nr && (ok >> i & 1) != 0 && i * 32 + l < a.E) m1 = fmaxf(m1, s[i]);
@@ -64,14 +71,48 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, 
     }
     return e;
   };
-  // the best groups: the group of the best expert outside those already taken
   unsigned open = ~0u, in = a.keep >= a.groups ? ~0u : 0u;
-  for (int k = 0; k < a.keep && a.keep < a.groups; ++k) {
-    float v;
-    const int g = best(open, v) / per;
+  if (a.keep < a.groups && a.group_top > 1 && per > 1) {
+    // every expert takes its group's score, the sum of its two best, and groups
+    // are chosen by it: the lower group first where two are equal
+    float gs[NR];
+    for (int g = 0; g < a.groups; ++g) {
+      unsigned ok = 0u;
 #pragma unroll
-    for (int i = 0; i < NR; ++i)
-      if (grp[i] == g) open &= ~(1u << i), in |= 1u << i;
+      for (int i = 0; i < NR; ++i)
+        if (i < nr && grp[i] == g) ok |= 1u << i;
+      float v1, v2;
+      const int e = best(ok, v1);
+      if ((e & 31) == l) ok &= ~(1u << (e >> 5));
+      best(ok, v2);
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (grp[i] == g) gs[i] = v1 + v2;
+    }
+    for (int k = 0; k < a.keep; ++k) {
+      float m1 = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (i < nr && (open >> i & 1) != 0 && i * 32 + l < a.E) m1 = fmaxf(m1, gs[i]);
+      m1 = group_max<32>(m1);
+      int g = a.groups;
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (i < nr && (open >> i & 1) != 0 && i * 32 + l < a.E && gs[i] == m1) g = min(g, grp[i]);
+      g = (int)-group_max<32>(-(float)g);
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (grp[i] == g) open &= ~(1u << i), in |= 1u << i;
+    }
+  } else {
+    // the best groups: the group of the best expert outside those already taken
+    for (int k = 0; k < a.keep && a.keep < a.groups; ++k) {
+      float v;
+      const int g = best(open, v) / per;
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (grp[i] == g) open &= ~(1u << i), in |= 1u << i;
+    }
   }
   float total = 0.f;
   float mine[2] = {0.f, 0.f};
@@ -79,6 +120,13 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, 
   for (int t = 0; t < a.top; ++t) {
     float v;
     const int e = best(in, v);
+    if (a.correction != nullptr) {
+      v = 0.f;
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (i == e >> 5) v = w[i];
+      v = __shfl(v, half * 32 + (e & 31), 64);
+    }
     total += v;
     if ((t & 31) == l) {
       if (t < 32) mine[0] = v, me[0] = e;
@@ -91,7 +139,7 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, 
   for (int i = 0; i < 2; ++i)
     if (live && i * 32 + l < a.top) {
       a.idx[(size_t)m * a.top + i * 32 + l] = me[i];
-      a.w[(size_t)m * a.top + i * 32 + l] = mine[i] / (total + 1e-20f);
+      a.w[(size_t)m * a.top + i * 32 + l] = a.normalise ? mine[i] / (total + 1e-20f) : mine[i];
     }
 }
 
@@ -197,7 +245,7 @@ __global__ __launch_bounds__(256) void grouped_skinny_kernel(const bf16_t* __res
   const bf16_t* ap[MT];
 #pragma unroll
   for (int i = 0; i < MT; ++i)
-    ap[i] = A + (size_t)g.row(t.first + min(r0 + i * 16 + (lane & 15), t.rows - 1)) * lda + (lane >> 4) * 8;
+    ap[i] = A + g.a_off(t.expert) + (size_t)g.row(t.first, min(r0 + i * 16 + (lane & 15), t.rows - 1)) * lda + (lane >> 4) * 8;
   const uint8_t* wp = wsh + ((size_t)t.expert * (N / 16) + (size_t)t.tn * NT) * nch * 1024 + lane * 16;
   f32x4 acc[MT][NT];
 #pragma unroll
@@ -237,15 +285,18 @@ __global__ __launch_bounds__(256) void grouped_skinny_kernel(const bf16_t* __res
 #pragma unroll
     for (int w = 1; w < 4; ++w) z += red[w][x][lane];
     const int i = x / NT, j = x % NT, r = r0 + i * 16 + (lane & 15), nb = (t.tn * NT + j) * 16;
-    bf16_t* crow = C + (size_t)(t.first + min(r, t.rows - 1)) * ldc;
+    bf16_t* crow = C + g.c_off(t.expert, t.first, ldc) + (size_t)min(r, t.rows - 1) * ldc;
     if constexpr (is_glu(ACT)) {  // columns 0..7 of the tile are gates, 8..15 their partners
       f32x4 u;
 #pragma unroll
       for (int q = 0; q < 4; ++q) u[q] = __shfl_xor(z[q], 32, 64);
+      auto join = [&](float gate, float up) __attribute__((always_inline)) {
+        if constexpr (ACT == ACT_CLAMP_MUL) return glu_clamped(gate, up, g.clamp);
+        else return glu_gate<ACT>(gate) * up;
+      };
       if (lane < 32 && r < t.rows)
         *reinterpret_cast<uint2*>(crow + nb / 2 + (lane >> 4) * 4) =
-            make_uint2(pack2bf(glu_gate<ACT>(z[0]) * u[0], glu_gate<ACT>(z[1]) * u[1]),
-                       pack2bf(glu_gate<ACT>(z[2]) * u[2], glu_gate<ACT>(z[3]) * u[3]));
+            make_uint2(pack2bf(join(z[0], u[0]), join(z[1], u[1])), pack2bf(join(z[2], u[2]), join(z[3], u[3])));
     } else {
       if (r < t.rows)
         *reinterpret_cast<uint2*>(crow + nb + (lane >> 4) * 4) = make_uint2(pack2bf(z[0], z[1]), pack2bf(z[2], z[3]));
@@ -259,7 +310,7 @@ using namespace dnn;
 
 extern "C" int dnn_route(const RouteArgs* a, hipStream_t st) {
   if (a->M <= 0 || a->E <= 0 || a->E > EXPERTS_MAX || a->ldl < a->E || a->groups <= 0 || a->E % a->groups != 0 ||
-      a->keep < 1 || a->keep > a->groups || a->top < 1 || a->top > 64 || a->top > a->E / a->groups * a->keep ||
+      a->keep < 1 || a->keep > a->groups || a->top < 1 || a->top > 64 || a->top > a->E / a->groups * a->keep || a->group_top < 1 || a->group_top > 2 ||
       a->M > (1 << 30) / a->top)
     return -1;
   if (a->M <= RT_SMALL) {
@@ -300,11 +351,12 @@ extern "C" int dnn_grouped_gemm(const GroupedArgs* a, hipStream_t st) {
   const int nc = is_glu(a->act) ? a->N / 2 : a->N;
   if (a->rows <= 0 || a->E <= 0 || a->E > EXPERTS_MAX || a->N <= 0 || a->N % 32 != 0 || a->K <= 0 || a->K % 64 != 0 ||
       a->lda % 8 != 0 || a->lda < a->K || a->ldc % 8 != 0 || a->ldc < nc || a->div < 1 || a->arows < 1 || a->Wsh == nullptr ||
-      a->offs == nullptr)
+      (a->offs == nullptr && (a->rows % a->E != 0 || a->sa < 0 || a->sa % 8 != 0 || a->sc < 0 || a->sc % 8 != 0)))
     return -1;
   if ((((uintptr_t)a->A | (uintptr_t)a->Wsh | (uintptr_t)a->C) & 15) != 0) return -1;
-  const GroupedRows g{a->offs, a->order, a->counts, a->E, a->div, a->arows};
+  const GroupedRows g{a->offs, a->order, a->counts, a->E, a->div, a->arows, a->rows / a->E, a->sa, a->sc, a->clamp};
   if (a->act == ACT_SILU_MUL) return grouped_launch<ACT_SILU_MUL>(*a, g, st);
+  if (a->act == ACT_CLAMP_MUL) return grouped_launch<ACT_CLAMP_MUL>(*a, g, st);
   if (a->act == ACT_NONE) return grouped_launch<ACT_NONE>(*a, g, st);
   return -1;
 }

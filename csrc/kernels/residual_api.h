@@ -1,9 +1,10 @@
 // C ABI of the decoder kernels with an fp32 residual and a paged KV cache
 // (residual_rows.hip, token_gate.hip, gemm_f32.hip,
-// paged_attention.hip).  As in api.h: every
+// paged_attention.hip, latent_attention.hip, poly_norm.hip).  As in api.h: every
 // function enqueues on `st`; 0 = success, negative = rejected shape.
 #pragma once
 #include <hip/hip_runtime.h>
+#include "glu_clamp.h"
 
 struct RowsArgs {
   const float* x_in;   // residual rows (nullptr: 0)
@@ -29,6 +30,7 @@ struct RowsArgs {
   const double* freq = nullptr;     //   sin, 2i + 1 cos of 2 pi * pos * freq[i] (freq in turns)
   int ldadd = 0, ldy2 = 0, ldys = 0, ysrows = 0, top = 0;
   float n_alpha = 0.f;
+  int y_joined = 0;                 // with ys: y_w norms the joined row instead of y alone
 };
 
 // One sequence's key range, masks and scales of a paged attention launch.
@@ -70,7 +72,60 @@ struct QkNormArgs {
   float t_coef, eps;
 };
 
+// out = a N(z) + b N(z^2) + c N(z^3) + e in place, N(y) = y / sqrt(mean(y^2) + eps);
+// rows of n values, zero up to the next 16 bytes.
+struct PolyNormArgs {
+  void* z;
+  const float* w;  // {a, b, c, e}
+  int ld, M, n;
+  float eps;
+};
+
+// Rotation of neighbouring pairs: freq[i] turns per position, cos and sin times mag.
+struct RopeTable {
+  const double* freq = nullptr;
+  int pairs = 0;
+  float mag = 1.f;
+};
+
+// Rows [query latent QP | latent CP | shared key part RP]: RMS norms of the two
+// latents (true widths QN, CN) with weights qw, cw and rotation of the key part,
+// in place; [latent | key part] goes into the cache [page][64][CP + RP].
+struct LatentPrepArgs {
+  void* rows;
+  void* kp;
+  const float* qw;
+  const float* cw;
+  const int* table;
+  const int* slots;
+  const int* pos;
+  RopeTable rope;
+  int ld, ldt, npages, M, QN, QP, CN, CP, RP;
+  float eps;
+};
+
+// Causal attention of every head over latent cache rows; out = sum of latents.
+struct LatentAttnArgs {
+  const void* qlat;    // rows [H][CP], stride ldql
+  const void* qrot;    // rows: head h at h * hs, RP columns, stride ldqr
+  const void* kp;      // [page][64][CP + RP]
+  const int* table;
+  const int* slots;
+  const int* pos;
+  void* out;           // rows [H][CP], stride ldo
+  const void* gate;    // rows [H] of gate logits, stride ldg (nullptr: none)
+  int ldql, ldqr, hs, ldo, ldg, ldt, npages, M, H, CP, RP;
+  float scale;
+};
+
 extern "C" {
+int dnn_poly_norm(const PolyNormArgs* a, int f32, hipStream_t st);
+int dnn_rope_rows(void* x, int ld, int hs, int M, int H, int RP, const int* pos, const RopeTable* r, int f32,
+                  hipStream_t st);
+int dnn_latent_prep(const LatentPrepArgs* a, int f32, hipStream_t st);
+int dnn_latent_attn(const LatentAttnArgs* a, const int* tiles, int ntiles, int splits, int per_token, float* ws,
+                    long long ws_elems, hipStream_t st);
+int dnn_latent_attn_f32(const LatentAttnArgs* a, hipStream_t st);
 int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStream_t st);
 // g = gelu_tanh(x W^T) * table[tok]: bf16, wsh = W in fragment order; _f32: from z = x W^T
 int dnn_token_gate(const void* x, int ldx, const void* w, int ldw, const void* wsh, int K, const void* table, int ldt,
@@ -78,7 +133,8 @@ int dnn_token_gate(const void* x, int ldx, const void* w, int ldw, const void* w
 int dnn_token_gate_f32(const float* z, int ldz, const float* table, int ldt, int off, const int* tok, int V, float* g,
                        int ldg, int M, int n, int np, hipStream_t st);
 int dnn_qk_norm(const QkNormArgs* a, int f32, hipStream_t st);
-int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act, hipStream_t st);
+int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act, const GluClamp* clamp,
+                hipStream_t st);
 int dnn_gemm_f32(const float* A, int lda, const float* W, int ldw, float* C, int ldc, const float* bias, int M, int N,
                  int K, hipStream_t st);
 int dnn_paged_write(const PagedAttnArgs* a, int f32, hipStream_t st);

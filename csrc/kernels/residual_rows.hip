@@ -2,7 +2,8 @@
 //
 // rows_update: one pass over a row that joins sublayer outputs into the
 // residual and prepares the next projection's input,
-//   z  = y * [rsqrt(mean(y^2) + eps) * yw] [+ the same of y2] [+ sum_t w_t ys_t]
+//   z  = y * [rsqrt(mean(y^2) + eps) * yw] [+ the same of y2] [+ sum_t w_t ys_t],
+//        or the norm of y + sum_t w_t ys_t
 //   x' = [x] [+ x_add] [+ position vector] + mult * z        (fp32)
 //   copy = T(x')              the residual as a GEMM operand
 //   h    = T(x' * rsqrt(mean(x'^2) + eps) * nw)               RMS norm, or
@@ -140,7 +141,7 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
       if (c < a.NP)
         y[i] = y[i] * r1 * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c)) + (PF ? y2[PF ? i : 0] * y2w[PF ? i : 0] : ld4(y2p + c) * ld4(a.y2_w + c)) * r2;
     }
-  } else if (a.y_w != nullptr) {
+  } else if (a.y_w != nullptr && !(PART == ROWS_EXPERTS && a.y_joined)) {
     float s = 0.f;
 #pragma unroll
     for (int i = 0; i < NC; ++i)
@@ -176,6 +177,19 @@ __global__ __launch_bounds__(256) void rows_update_kernel(RowsArgs a) {
         for (int u = 0; u < 4; ++u)
 #pragma unroll
           for (int j = 0; j < 4; ++j) y[i][j] = fmaf(w[u], v[u][j], y[i][j]);
+      }
+    }
+    if (a.y_joined) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < NC; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s = fmaf(y[i][j], y[i][j], s);
+      const float r = 1.0f / sqrtf(row_sum<TPR>(s, red) / (float)a.N + a.eps);
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const int c = (t + TPR * i) * 4;
+        if (c < a.NP) y[i] = y[i] * r * (PF ? yw[PF ? i : 0] : ld4(a.y_w + c));
       }
     }
   }
@@ -259,12 +273,17 @@ static int rows_launch(const RowsArgs& a, hipStream_t st) {
 
 // fp32 gated activation of packed gate|up columns (8 gate, 8 up, ...): out = act(gate) * up.
 __global__ __launch_bounds__(256) void glu_f32_kernel(const float* __restrict__ gu, int ldi, float* __restrict__ out,
-                                                      int ldo, int M, int F, int act) {
+                                                      int ldo, int M, int F, int act, GluClamp clamp) {
   const long i = blockIdx.x * 256L + threadIdx.x;
   if (i >= (long)M * F) return;
   const int m = (int)(i / F), c = (int)(i % F);
   const float* p = gu + (size_t)m * ldi + (c >> 3) * 16 + (c & 7);
   const float x = p[0];
+  if (act == ACT_CLAMP_MUL) {
+    const float g = fminf(x, clamp.limit), u = fminf(fmaxf(p[8], -clamp.limit), clamp.limit);
+    out[(size_t)m * ldo + c] = g / (1.0f + expf(-clamp.alpha * g)) * (u + clamp.shift);
+    return;
+  }
   const float g = act == ACT_SILU_MUL ? x / (1.0f + expf(-x))
                                       : 0.5f * x * (1.0f + tanhf(0.797884560802865f * (x + 0.044715f * x * x * x)));
   out[(size_t)m * ldo + c] = g * p[8];
@@ -279,6 +298,7 @@ extern "C" int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStr
     return -1;
   if ((a->ldadd | a->ldy2 | a->ldys) % 4 != 0 || (a->y2 != nullptr && (a->y2_w == nullptr || a->y_w == nullptr)) ||
       (a->ys != nullptr && (a->ysi == nullptr || a->ysw == nullptr || a->top < 1 || a->ysrows < 1)) ||
+      (a->y_joined && (a->ys == nullptr || a->y_w == nullptr)) ||
       (a->freq != nullptr && a->pos == nullptr))
     return -1;
   if ((a->xidx != nullptr && (a->xrows < 1 || a->x_out != nullptr)) || (a->yidx != nullptr && a->yrows < 1)) return -1;
@@ -300,9 +320,9 @@ extern "C" int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStr
 }
 
 extern "C" int dnn_glu_f32(const float* gu, int ldi, float* out, int ldo, int M, int F, int act,
-                           hipStream_t st) {
-  if (M <= 0 || F <= 0 || F % 8 != 0 || ldi < 2 * F || ldo < F || !is_glu(act)) return -1;
+                           const GluClamp* clamp, hipStream_t st) {
+  if (M <= 0 || F <= 0 || F % 8 != 0 || ldi < 2 * F || ldo < F || !is_glu(act) || (act == ACT_CLAMP_MUL && clamp == nullptr)) return -1;
   hipLaunchKernelGGL(glu_f32_kernel, dim3((unsigned)(((long)M * F + 255) / 256)), dim3(256), 0, st, gu, ldi, out, ldo,
-                     M, F, act);
+                     M, F, act, clamp != nullptr ? *clamp : GluClamp{});
   return (int)hipGetLastError();
 }

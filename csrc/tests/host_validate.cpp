@@ -111,8 +111,8 @@ int main() {
                 "token gate without the fragment copy");
   expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 48, st), "token gate np%64");
   expect_reject(dnn_gemm_f32(f, 24, f, 24, f, 8, nullptr, 4, 8, 24, st), "f32 gemm K%16");
-  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 12, 3, st), "glu F%8");
-  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 8, 1, st), "glu with a plain activation");
+  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 12, 3, nullptr, st), "glu F%8");
+  expect_reject(dnn_glu_f32(f, 16, f, 16, 4, 8, 1, nullptr, st), "glu with a plain activation");
   PagedAttnArgs pa = {};
   pa.qkv = pa.kp = pa.vp = pa.out = p, pa.table = pa.slots = pa.pos = ip;
   pa.ldq = 256, pa.ldo = 64, pa.ldt = 1, pa.npages = 1, pa.M = 1, pa.H = pa.G = 1, pa.DK = pa.DV = 64;

@@ -29,6 +29,9 @@ import torch
 from .models import DECODERS, cifar, gpt2, llama3, model_info
 
 
+FREE_SIZE = 16  # random weights: a size that no configuration fixes
+
+
 class CheckpointError(Exception):
     pass
 
@@ -138,10 +141,15 @@ def stage_state_dict(model: str, full_sd, start: int, end: int, first: bool,
     sd = {local: full_sd[full] for local, full in want.items()}
     if info.family in DECODERS:  # every size comes from the config: the tensors must agree with it
         shapes = DECODERS[info.family].stage_shapes(info.cfg, start, end, first, last)
-        bad = [f"{k} {tuple(v.shape)} (config: {shapes[k]})" for k, v in sd.items() if tuple(v.shape) != shapes[k]]
+        bad = [f"{k} {tuple(v.shape)} (config: {shapes[k]})" for k, v in sd.items() if not shape_fits(v.shape, shapes[k])]
         if bad:
             raise CheckpointError(f"tensors that do not fit the config: {bad[:8]}")
     return sd
+
+
+def shape_fits(shape, want) -> bool:
+    """``want``: a size may be None where the checkpoint alone fixes it."""
+    return len(shape) == len(want) and all(w is None or s == w for s, w in zip(shape, want))
 
 
 def unexpected_keys(model: str, full_sd, start: int, end: int, first: bool, last: bool) -> List[str]:
@@ -201,6 +209,7 @@ def random_decoder_state(family, cfg, start, end, first, last, seed, dev, nontri
     sd = {}
     for k, shape in family.stage_shapes(cfg, start, end, first, last).items():
         g = torch.Generator(device=dev).manual_seed(_key_seed(seed, k))
+        shape = tuple(FREE_SIZE if n is None else n for n in shape)
         sd[k] = family.random_tensor(cfg, k, torch.randn(shape, generator=g, device=dev), nontrivial)
     return sd
 

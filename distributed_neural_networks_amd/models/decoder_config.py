@@ -1,5 +1,5 @@
-"""What the paged decoder families (``kozusun.py``, ``funepel.py``) share in
-their configurations: the folder's file name, checked reads of config.json, the
+"""What the paged decoder families (``kozusun.py``, ``funepel.py``,
+``tizalorn.py``) share in their configurations: the folder's file name, checked reads of config.json, the
 loop over a layer range, and the sequence of layer runs that pipeline stages
 split.
 """
@@ -22,6 +22,28 @@ class LayerRun:
     """One execution of a layer; ``enters``: the loop's entry step comes before it."""
     layer: int
     enters: bool
+
+
+@dataclass(frozen=True)
+class MoEConfig:
+    """Mixture of experts: the router's scores (softmax, or sigmoid), a
+    correction that enters the choice only, groups of neighbours scored by their
+    ``group_top`` best experts, weights normalised over the chosen or as scored;
+    ``limit``: experts with the clamped gated activation (g = min(gate, limit),
+    u = clamp(up, +-limit), g sigmoid(alpha g) (u + shift)) instead of silu."""
+    experts: int
+    top: int
+    ff: int
+    groups: int = 1
+    keep: int = 1
+    shared_ff: int = 0      # 0: no shared expert
+    sigmoid: bool = False
+    correction: bool = False
+    group_top: int = 1
+    normalise: bool = True
+    limit: Optional[float] = None
+    alpha: float = 1.0
+    shift: float = 0.0
 
 
 def layer_runs(n: int, loop: Optional[Tuple[int, int, int]], first_pass_enters: bool) -> List[LayerRun]:

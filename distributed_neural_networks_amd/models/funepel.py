@@ -39,7 +39,7 @@ from __future__ import annotations
 from dataclasses import dataclass, replace
 from typing import Dict, List, Optional, Tuple, Union
 
-from .decoder_config import (ModelConfigError, LayerRun, get_loop, get_number as _get, get_size as _size, layer_runs,
+from .decoder_config import (MoEConfig, ModelConfigError, LayerRun, get_loop, get_number as _get, get_size as _size, layer_runs,
                              load_json)
 
 ARCHITECTURE = "Funepel"
@@ -86,16 +86,6 @@ class RetentionConfig:
 class ParallelConfig:
     left: SharedKVAttentionConfig
     right: RetentionConfig
-
-
-@dataclass(frozen=True)
-class MoEConfig:
-    experts: int
-    top: int
-    ff: int
-    groups: int = 1
-    keep: int = 1
-    shared_ff: int = 0      # 0: no shared expert
 
 
 @dataclass(frozen=True)

@@ -1,0 +1,337 @@
+"""Tizalorn: a decoder of WKV layers (a recurrence with a decay per key channel)
+and latent-attention layers, each followed by a dense feed-forward or a mixture
+of experts, with the norms on the sublayers' outputs.
+
+The residual ``x`` is fp32; ``N(y) = y / sqrt(mean(y^2) + eps)``, and a norm's
+weight is one number:
+
+    x  = N(embed[token] + bigram[pair of (previous token, token)]) * g
+    x += N(mixer(x)) * g1;  x += N(feed-forward(x)) * g2
+
+* mixer ``wkv``: r, k, v, a gate and a decay read their own mixes of the token
+  and the one before it; per head S <- diag(w_t) S + k v^T with w = exp(-exp(W2
+  tanh(W1 m) + w0)), o = (S + diag(u) k v^T)^T r before the update; heads
+  RMS-normed, gated by silu.
+* mixer ``latent_attention``: queries through a latent, keys and values from a
+  cached latent per token and one rotated key part for all heads (rotary
+  positions with YaRN scaling), a sigmoid gate per head.
+* feed-forward ``dense``: W_down act(W_up x) with a polynomial of normed powers;
+  ``moe``: sigmoid router with a correction for the choice, groups scored by
+  their two best experts, weights not renormalised, a clamped gated activation.
+
+A model is a folder with ``config.json`` ("architecture": "Tizalorn") and
+safetensors weights named ``embed``, ``bigram``, ``embed.norm``,
+``l<i>.norm{1,2}``, ``l<i>.mix.*``, ``l<i>.mlp.*``, ``final.norm``, ``head``;
+linear weights ``[out, in]``; every size and constant comes from the config, but
+the rank of the decay's projection, which is its tensors' shape.
+
+This module holds the description only; ``runtime/decoder.py`` runs it.
+"""
+from __future__ import annotations
+
+import math
+from dataclasses import dataclass, replace
+from typing import Dict, List, Optional, Tuple, Union
+
+from .decoder_config import (MoEConfig, ModelConfigError, LayerRun, get_number as _get, get_size as _size, layer_runs, load_json)
+
+ARCHITECTURE = "Tizalorn"
+STATE_MAX = 256          # head sizes the recurrence kernels are built for
+LATENT_MAX, ROT_MAX = 512, 128
+EXPERTS_MAX = 256
+BUCKETS_MAX = (1 << 30) - 1  # rows of the pair table
+GATE_ALPHA, UP_SHIFT = 1.702, 1.0  # clamped gated activation: g sigmoid(alpha g) (u + shift)
+
+
+@dataclass(frozen=True)
+class BigramConfig:
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass(frozen=True)
+class WkvConfig:
+    heads: int
+    dim: int
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.dim
+
+
+@dataclass(frozen=True)
+class YarnConfig:
+    """Frequencies of slow pairs divided by ``factor``, with a ramp between the
+    pairs that turn ``fast`` and ``slow`` times over ``original`` positions."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotaryConfig:
+    base: float
+    dims: int
+    scaling: Optional[YarnConfig] = None
+
+    def frequencies(self) -> Tuple[List[float], float]:
+        """(radians per position of every pair, factor of cos and sin)."""
+        d, s = self.dims, self.scaling
+        f = [self.base ** (-2.0 * i / d) for i in range(d // 2)]
+        if s is None:
+            return f, 1.0
+        at = [d * math.log(s.original / (2 * math.pi * turns)) / (2 * math.log(self.base)) for turns in (s.fast, s.slow)]
+        lo, hi = max(math.floor(at[0]), 0), min(math.ceil(at[1]), d - 1)
+        ramp = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(d // 2)]
+        return [x / s.factor * r + x * (1 - r) for x, r in zip(f, ramp)], 0.1 * math.log(s.factor) + 1
+
+
+@dataclass(frozen=True)
+class LatentAttentionConfig:
+    heads: int
+    dim: int        # unrotated query / key dimensions of a head
+    rot_dim: int    # rotated ones, shared by all heads in the key
+    vdim: int
+    kv_rank: int
+    q_rank: int
+    scale: float
+    rot: RotaryConfig
+
+
+@dataclass(frozen=True)
+class DenseConfig:
+    ff: int
+
+
+def _experts(experts: int, top: int, ff: int, limit: float, groups: int = 1, keep: int = 1) -> MoEConfig:
+    """This family's router and expert activation."""
+    return MoEConfig(experts, top, ff, groups, keep, sigmoid=True, correction=True, group_top=2, normalise=False,
+                     limit=limit, alpha=GATE_ALPHA, shift=UP_SHIFT)
+
+
+@dataclass(frozen=True)
+class LayerConfig:
+    mixer: Union[WkvConfig, LatentAttentionConfig]
+    mlp: Optional[Union[DenseConfig, MoEConfig]]
+
+
+@dataclass(frozen=True)
+class TizalornConfig:
+    vocab_size: int
+    n_embd: int
+    layers: Tuple[LayerConfig, ...]
+    norm_eps: float
+    bigram: BigramConfig
+    decay_rank: Optional[int] = None   # None: whatever the checkpoint holds
+    max_seq: int = 1 << 20             # bounded by the cache only
+    side_dim: int = 0                  # no per-layer token input
+
+    @property
+    def n_layer(self) -> int:
+        return len(self.layers)
+
+    @property
+    def runs(self) -> List[LayerRun]:
+        return layer_runs(len(self.layers), None, False)
+
+
+def _wkv(d, where) -> WkvConfig:
+    m = WkvConfig(_size(d, "heads", where), _size(d, "dim", where))
+    if m.dim > STATE_MAX:
+        raise ModelConfigError(f"{where}: 'dim' {m.dim} exceeds {STATE_MAX}")
+    return m
+
+
+def _rotary(d, rot_dim, where) -> RotaryConfig:
+    r = RotaryConfig(float(_get(d, "base", where)), _size(d, "dims", where, 2))
+    if r.dims % 2 or r.dims > rot_dim:
+        raise ModelConfigError(f"{where}: 'dims' {r.dims} must be even and at most 'rot_dim' {rot_dim}")
+    if not r.base > 1:
+        raise ModelConfigError(f"{where}: 'base' must exceed 1")
+    s = d.get("scaling")
+    if s is None:
+        return r
+    y = YarnConfig(**{k: float(_get(s, k, where + ".scaling")) for k in ("factor", "original", "fast", "slow")})
+    if not all(v > 0 for v in (y.factor, y.original, y.fast, y.slow)):
+        raise ModelConfigError(f"{where}.scaling: every number must be positive")
+    return replace(r, scaling=y)
+
+
+def _latent(d, where) -> LatentAttentionConfig:
+    n = {k: _size(d, k, where) for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank")}
+    a = LatentAttentionConfig(scale=float(_get(d, "scale", where)), rot=_rotary(d.get("rot"), n["rot_dim"], where + ".rot"), **n)
+    if not a.scale > 0:
+        raise ModelConfigError(f"{where}: 'scale' must be positive")
+    if a.kv_rank > LATENT_MAX or a.rot_dim > ROT_MAX or a.heads > EXPERTS_MAX:
+        raise ModelConfigError(f"{where}: 'kv_rank' up to {LATENT_MAX}, 'rot_dim' up to {ROT_MAX}, 'heads' up to "
+                               f"{EXPERTS_MAX}; got {a.kv_rank}, {a.rot_dim}, {a.heads}")
+    return a
+
+
+def _mlp(d, where) -> Union[DenseConfig, MoEConfig]:
+    kind = d.get("kind")
+    if kind == "dense":
+        return DenseConfig(_size(d, "ff", where))
+    if kind != "moe":
+        raise ModelConfigError(f"{where}: unknown feed-forward kind {kind!r}")
+    r, g, e = d.get("router") or {}, (d.get("router") or {}).get("groups"), d.get("expert")
+    m = _experts(_size(r, "experts", where + ".router"), _size(r, "top", where + ".router"),
+                 _size(e, "ff", where + ".expert"), float(_get(e, "limit", where + ".expert")),
+                 _size(g, "count", where + ".router.groups") if g else 1,
+                 _size(g, "keep", where + ".router.groups") if g else 1)
+    if m.experts % m.groups:
+        raise ModelConfigError(f"{where}: {m.experts} experts do not divide over {m.groups} groups")
+    if m.keep > m.groups or m.top > m.experts // m.groups * m.keep or m.experts > EXPERTS_MAX or m.top > 64:
+        raise ModelConfigError(f"{where}: {m.top} of {m.experts} experts from {m.keep} of {m.groups} groups")
+    if not m.limit > 0:
+        raise ModelConfigError(f"{where}: 'limit' must be positive")
+    return m
+
+
+def _layer(d, i) -> LayerConfig:
+    where = f"layers[{i}]"
+    kind, m = (d.get("type"), d.get("mixer") or {}) if isinstance(d, dict) else (d, {})
+    if kind == "wkv":
+        mixer = _wkv(m, where + ".mixer")
+    elif kind == "latent_attention":
+        mixer = _latent(m, where + ".mixer")
+    else:
+        raise ModelConfigError(f"{where}: unknown mixer type {kind!r}")
+    return LayerConfig(mixer, None if d.get("mlp") is None else _mlp(d["mlp"], where + ".mlp"))
+
+
+def parse_config(d: Dict) -> TizalornConfig:
+    if d.get("architecture") != ARCHITECTURE:
+        raise ModelConfigError(f"architecture {d.get('architecture')!r} is not {ARCHITECTURE!r}")
+    raw = d.get("layers")
+    if not isinstance(raw, list) or not raw:
+        raise ModelConfigError("'layers' must be a list with at least one layer")
+    b = (d.get("embedding") or {}).get("bigram")
+    buckets = _size(b, "buckets", "embedding.bigram")
+    if buckets > BUCKETS_MAX:
+        raise ModelConfigError(f"embedding.bigram: 'buckets' {buckets} exceeds {BUCKETS_MAX}")
+    # only the multipliers' residues matter
+    bigram = BigramConfig(buckets, *(_get(b, k, "embedding.bigram", (int,)) % buckets for k in ("mul_prev", "mul_cur")))
+    return TizalornConfig(vocab_size=_size(d, "vocab", "config"), n_embd=_size(d, "width", "config"),
+                          layers=tuple(_layer(x, i) for i, x in enumerate(raw)),
+                          norm_eps=float(_get(d.get("norm"), "eps", "norm")), bigram=bigram)
+
+
+def load_config(folder: str) -> TizalornConfig:
+    return load_json(folder, parse_config)
+
+
+TIZALORN_CONFIGS: Dict[str, TizalornConfig] = {}
+
+
+def _preset(name: str, vocab: int, width: int, pattern: str, wkv: WkvConfig, att: LatentAttentionConfig, dense: DenseConfig,
+            moe: MoEConfig, bigram: BigramConfig, rank: int) -> None:
+    """``pattern``: a layer's mixer (w: WKV, a: attention), upper case with the dense feed-forward."""
+    layers = tuple(LayerConfig(wkv if c.lower() == "w" else att, dense if c.isupper() else moe) for c in pattern)
+    TIZALORN_CONFIGS[name] = TizalornConfig(vocab, width, layers, 1e-6, bigram, rank)
+
+
+_ROT = RotaryConfig(10000.0, 64, YarnConfig(8.0, 4096, 32.0, 1.0))
+_preset("tizalorn-tiny", 512, 192, "WaWw", WkvConfig(3, 64),
+        LatentAttentionConfig(4, 48, 24, 40, 80, 96, 0.12, RotaryConfig(5000.0, 24, YarnConfig(4.0, 256, 16.0, 1.0))),
+        DenseConfig(448), _experts(12, 3, 96, 4.0, 3, 2), BigramConfig(1021, 31, 7), 24)
+# layers of a 1B model's and of Llama-3 8B's width; active feed-forward columns near theirs
+_preset("tizalorn-1b", 32768, 2048, "WwwawwwaWwwa", WkvConfig(32, 64),
+        LatentAttentionConfig(16, 128, 64, 128, 512, 768, 192 ** -0.5, _ROT), DenseConfig(8448),
+        _experts(32, 4, 1408, 7.0, 4, 2), BigramConfig(65521, 8191, 127), 64)
+_preset("tizalorn-8b", 128256, 4096, "Wwwa" * 6, WkvConfig(64, 64),
+        LatentAttentionConfig(32, 128, 64, 128, 512, 1536, 192 ** -0.5, _ROT), DenseConfig(21504),
+        _experts(32, 4, 3584, 7.0, 4, 2), BigramConfig(262139, 8191, 127), 64)
+
+
+def _layer_shapes(cfg: TizalornConfig, i: int) -> Dict[str, Tuple[Optional[int], ...]]:
+    L, w, p = cfg.layers[i], cfg.n_embd, f"l{i}."
+    s: Dict[str, Tuple[Optional[int], ...]] = {p + "norm1": ()}
+    m, q = L.mixer, p + "mix."
+    if isinstance(m, WkvConfig):
+        s.update({q + "mu." + n: (w,) for n in "rkvgw"})
+        s.update({q + n: (m.inner, w) for n in "rkvg"})
+        s[q + "w1"], s[q + "w2"], s[q + "w0"] = (cfg.decay_rank, w), (m.inner, cfg.decay_rank), (m.inner,)
+        s[q + "u"], s[q + "norm"], s[q + "o"] = (m.heads, m.dim), (m.inner,), (w, m.inner)
+    else:
+        s[q + "dq"], s[q + "dq.norm"], s[q + "uq"] = (m.q_rank, w), (m.q_rank,), (m.heads * (m.dim + m.rot_dim), m.q_rank)
+        s[q + "dkv"], s[q + "dkv.norm"] = (m.kv_rank + m.rot_dim, w), (m.kv_rank,)
+        s[q + "uk"], s[q + "uv"] = (m.heads * m.dim, m.kv_rank), (m.heads * m.vdim, m.kv_rank)
+        s[q + "g"], s[q + "o"] = (m.heads, w), (w, m.heads * m.vdim)
+    f, q = L.mlp, p + "mlp."
+    if f is not None:
+        s[p + "norm2"] = ()
+    if isinstance(f, DenseConfig):
+        s[q + "up"], s[q + "down"], s[q + "act"] = (f.ff, w), (w, f.ff), (4,)
+    elif f is not None:
+        s[q + "router"], s[q + "correction"] = (f.experts, w), (f.experts,)
+        for e in range(f.experts):
+            s[f"{q}e{e}.gate"], s[f"{q}e{e}.up"], s[f"{q}e{e}.down"] = (f.ff, w), (f.ff, w), (w, f.ff)
+    return s
+
+
+def stage_shapes(cfg: TizalornConfig, start: int, end: int, first: bool, last: bool) -> Dict[str, Tuple[Optional[int], ...]]:
+    """name -> shape of the tensors that layers ``start .. end`` need (checkpoint names; None: any size)."""
+    s: Dict[str, Tuple[Optional[int], ...]] = {}
+    if first:
+        s["embed"], s["bigram"], s["embed.norm"] = (cfg.vocab_size, cfg.n_embd), (cfg.bigram.buckets + 1, cfg.n_embd), ()
+    for i in range(start, end + 1):
+        s.update(_layer_shapes(cfg, i))
+    if last:
+        s["final.norm"], s["head"] = (), (cfg.vocab_size, cfg.n_embd)
+    return s
+
+
+def stage_key_map(cfg: TizalornConfig, start: int, end: int, first: bool, last: bool) -> Dict[str, str]:
+    return {k: k for k in stage_shapes(cfg, start, end, first, last)}
+
+
+def random_tensor(cfg: TizalornConfig, name: str, noise, nontrivial: bool):
+    """A random weight from unit ``noise`` of its shape: projections of unit
+    gain, norm weights one, or noise around those with ``nontrivial``; decays of
+    a few to a few hundred tokens."""
+    shape, extra = tuple(noise.shape), 0.1 * noise if nontrivial else 0 * noise
+    if name.endswith("mix.w0"):
+        return 1.5 * noise - 3.5
+    if ".mu." in name:
+        return 0.5 + 0.2 * noise
+    if name.endswith("mix.u"):
+        return 0.5 * noise
+    if name.endswith("mlp.act"):
+        return noise.new_tensor([0.6, 0.4, 0.2, 0.0]) + extra
+    if name.endswith("mlp.correction"):
+        return extra
+    if len(shape) < 2:
+        return 1 + extra
+    if name in ("embed", "bigram"):
+        return noise
+    return noise * shape[1] ** -0.5
+
+
+def run_flops(cfg: TizalornConfig, layer: int, ctx: int) -> float:
+    """Forward FLOPs of one token through ``layer`` with ``ctx`` tokens before it
+    (attention with the keys and values of the heads, as at prefill)."""
+    L, w, m = cfg.layers[layer], cfg.n_embd, cfg.layers[layer].mixer
+    if isinstance(m, WkvConfig):
+        mats, mix = m.inner * w * 5 + (cfg.decay_rank or 16) * (w + m.inner), 4.0 * m.inner * m.dim
+    else:
+        mats = (m.q_rank + m.kv_rank + m.rot_dim + m.heads) * w + m.heads * (m.dim + m.rot_dim) * m.q_rank
+        mats += m.heads * (m.dim + m.vdim) * m.kv_rank + w * m.heads * m.vdim
+        mix = 2.0 * ctx * m.heads * (m.dim + m.rot_dim + m.vdim)
+    if isinstance(L.mlp, DenseConfig):
+        mats += 2 * L.mlp.ff * w
+    elif L.mlp is not None:
+        mats += (L.mlp.experts + 3 * L.mlp.top * L.mlp.ff) * w
+    return 2.0 * mats + mix
+
+
+def flops_per_token(cfg: TizalornConfig, runs: List[LayerRun], ctx: int, lm_head: bool = True) -> float:
+    f = sum(run_flops(cfg, r.layer, ctx) for r in runs)
+    return f + (2.0 * cfg.n_embd * cfg.vocab_size if lm_head else 0.0)
+
+
+def scaled(cfg: TizalornConfig, pattern: Tuple[int, ...]) -> TizalornConfig:
+    """The layers ``pattern`` of ``cfg`` (benches)."""
+    return replace(cfg, layers=tuple(cfg.layers[i] for i in pattern))

@@ -1,6 +1,6 @@
 """Wrappers of the decoder kernels with an fp32 residual and a paged KV cache
 (``csrc/kernels/residual_rows.hip``, ``token_gate.hip``, ``gemm_f32.hip``,
-``paged_attention.hip``).
+``paged_attention.hip``, ``latent_attention.hip``, ``poly_norm.hip``).
 
 Operands are bf16 (serving) or fp32 (exact mode: fp32 weights, activations,
 cache and MFMA); the residual stream is fp32 in both.  As in
@@ -56,7 +56,7 @@ def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx
                 y: Optional[torch.Tensor] = None, yidx: Optional[torch.Tensor] = None, mult: float = 1.0,
                 y_norm: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None,
                 y2_norm: Optional[torch.Tensor] = None, ys: Optional[torch.Tensor] = None,
-                ysi: Optional[torch.Tensor] = None, ysw: Optional[torch.Tensor] = None, top: int = 0,
+                ysi: Optional[torch.Tensor] = None, ysw: Optional[torch.Tensor] = None, top: int = 0, y_joined: bool = False,
                 x_add: Optional[torch.Tensor] = None, pos: Optional[torch.Tensor] = None,
                 freq: Optional[torch.Tensor] = None, x_out: Optional[torch.Tensor] = None,
                 copy: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
@@ -64,7 +64,8 @@ def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx
                 eps: float = 1e-5) -> None:
     """``x' = [x_in] [+ x_add] [+ positions] + mult * z`` with ``z = y`` (RMS-
     normalised with weight ``y_norm`` first, if given) ``[+ y2`` normalised with
-    ``y2_norm] [+ sum_t ysw[m, t] ys[ysi[m, t]]]``, then any of ``x_out = x'``
+    ``y2_norm] [+ sum_t ysw[m, t] ys[ysi[m, t]]]`` (``y_joined``: ``y_norm`` norms
+    ``y`` with that sum instead), then any of ``x_out = x'``
     (fp32), ``copy = x'`` and ``h = RMSnorm(x') * norm``, or with ``norm_b`` the
     dynamic tanh ``h = tanh(alpha x') * norm + norm_b``.  ``xidx`` / ``yidx``
     gather the rows of ``x_in`` / ``y``; positions: sinusoids of ``pos`` with
@@ -90,6 +91,8 @@ def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx
     _weight(ysw, M * top, "rows_update ysw")
     for t, n in ((y_norm, "y_norm"), (y2_norm, "y2_norm"), (norm, "norm"), (norm_b, "norm_b")):
         _weight(t, NP, "rows_update " + n)
+    if y_joined and (ys is None or y_norm is None):
+        raise ValueError("rows_update: y_joined norms the sum with ys")
     if x_in is None and yt is None or (norm is None) != (h is None) or width > NP or NP % 4 or NP > WIDTH_MAX \
             or (norm_b is not None and norm is None) or (ys is not None and (ysi is None or ysw is None or top < 1)) \
             or (y2 is not None and (y is None or y_norm is None or y2_norm is None)):
@@ -106,7 +109,8 @@ def rows_update(M: int, width: int, *, x_in: Optional[torch.Tensor] = None, xidx
     elif x_out is not None:
         a.ldx = x_out.stride(0)
     if y is not None:
-        a.y, a.yidx, a.yrows, a.ldy, a.y_w = ptr(y), ptr(yidx), y.shape[0], y.stride(0), ptr(y_norm)
+        a.y, a.yidx, a.yrows, a.ldy = ptr(y), ptr(yidx), y.shape[0], y.stride(0)
+    a.y_w, a.y_joined = ptr(y_norm), int(y_joined)
     if y2 is not None:
         a.y2, a.y2_w, a.ldy2 = ptr(y2), ptr(y2_norm), y2.stride(0)
     if ys is not None:
@@ -255,10 +259,10 @@ def paged_prefill(args, tiles: torch.Tensor) -> None:
         check(lib().paged_prefill(args, ptr(part), part.shape[0], stream_ptr()), "paged_prefill")
 
 
-def chunk_tiles(row0: int, tokens: int, slot: int, group: int) -> list:
+def chunk_tiles(row0: int, tokens: int, slot: int, group: int, rows: int = TILE_ROWS) -> list:
     """Prefill workgroups of one chunk: ``tokens * group`` packed rows (group =
-    query heads per KV head), the last (longest) ones first."""
-    return [(row0, tokens, slot, r) for r in range(0, tokens * group, TILE_ROWS)][::-1]
+    query heads per KV head) in groups of ``rows``, the last (longest) ones first."""
+    return [(row0, tokens, slot, r) for r in range(0, tokens * group, rows)][::-1]
 
 
 def paged_splits(n_seq: int, H: int, G: int, keys: int, window: Optional[int], keep: int) -> int:
@@ -284,3 +288,127 @@ def paged_decode(args, rows: torch.Tensor, n: int, splits: int, ws: Optional[tor
 def paged_attn_f32(args) -> None:
     """fp32 attention of every row (cache already written)."""
     check(lib().paged_attn_f32(args, stream_ptr()), "paged_attn_f32")
+
+
+def poly_norm(z: torch.Tensor, w: torch.Tensor, M: int, n: int, eps: float) -> None:
+    """``z <- a N(z) + b N(z^2) + c N(z^3) + e`` in place over the first n columns,
+    ``w`` = (a, b, c, e), ``N(y) = y / sqrt(mean(y^2) + eps)``."""
+    f32 = z.dtype == torch.float32
+    _rows(z, M, -(-n // 8) * 8, "poly_norm z", (torch.float32, torch.bfloat16))
+    _weight(w, 4, "poly_norm weight")
+    a = lib().PolyNormArgs()
+    a.z, a.w, a.ld, a.M, a.n, a.eps = ptr(z), ptr(w), z.stride(0), M, n, eps
+    check(lib().poly_norm(a, int(f32), stream_ptr()), "poly_norm")
+
+
+# ---------------------------------------------------------------------- attention over a latent cache
+LATENT_DIMS, LATENT_ROT = (128, 256, 512), (64, 128)  # latent columns and key-part columns the kernels are built for
+LATENT_ROWS = 64                                      # packed (token, head) rows of one workgroup
+
+
+def pad_to(n: int, sizes, what: str) -> int:
+    for p in sizes:
+        if n <= p:
+            return p
+    raise ValueError(f"{what} {n} exceeds {sizes[-1]}")
+
+
+class Rope:
+    """Rotation of neighbouring pairs: radians per position of every pair, and
+    the factor of cos and sin."""
+
+    def __init__(self, freqs, mag: float, device):
+        import math
+        self.freq = torch.tensor(freqs, dtype=torch.float64, device=device) / (2.0 * math.pi)
+        self.pairs, self.mag = len(freqs), float(mag)
+
+    def table(self):
+        return lib().RopeTable(ptr(self.freq), self.pairs, self.mag)
+
+
+def rope_rows(x: torch.Tensor, M: int, H: int, hs: int, col: int, RP: int, pos: torch.Tensor, rope: Rope) -> None:
+    """Rotate columns ``h * hs + col ..`` of every row and head in place."""
+    _rows(x, M, (H - 1) * hs + col + RP, "rope rows", (torch.float32, torch.bfloat16))
+    _index(pos, M, "rope pos")
+    es = x.element_size()
+    if col * es % 16 or 2 * rope.pairs > RP or hs < RP:
+        raise ValueError(f"rope_rows: {rope.pairs} pairs in {RP} columns at {col}")
+    check(lib().rope_rows(ptr(x) + col * es, x.stride(0), hs, M, H, RP, ptr(pos), rope.table(),
+                          int(x.dtype == torch.float32), stream_ptr()), "rope_rows")
+
+
+def _latent_pool(kp: torch.Tensor, dtype) -> None:
+    if kp.dim() != 3 or kp.shape[1] != PAGE or kp.dtype != dtype or not kp.is_contiguous():
+        raise ValueError(f"latent cache: contiguous (pages, {PAGE}, columns) of {dtype} expected, got {tuple(kp.shape)}")
+
+
+def latent_prep(rows: torch.Tensor, kp: torch.Tensor, qw: torch.Tensor, cw: torch.Tensor, rope: Rope, table: torch.Tensor,
+                slots: torch.Tensor, pos: torch.Tensor, M: int, QN: int, CN: int, CP: int, eps: float) -> None:
+    """Rows ``[query latent | latent CP | key part]`` in place: RMS norms of the
+    latents (true widths QN, CN; weights ``qw``, ``cw`` padded with zeros),
+    rotation of the key part; latent and key part into the cache ``kp``."""
+    _latent_pool(kp, rows.dtype)
+    QP, RP = qw.numel(), kp.shape[2] - CP
+    _rows(rows, M, QP + kp.shape[2], "latent rows", (rows.dtype,))
+    _weight(qw, QP, "latent query norm")
+    _weight(cw, CP, "latent norm")
+    _index(slots, M, "latent slots")
+    _index(pos, M, "latent pos")
+    if table.dtype != torch.int32 or table.dim() != 2 or not table.is_contiguous() or RP < 2 * rope.pairs:
+        raise ValueError("latent_prep: bad block table or key part")
+    a = lib().LatentPrepArgs()
+    a.rows, a.kp, a.qw, a.cw, a.table, a.slots, a.pos = (ptr(t) for t in (rows, kp, qw, cw, table, slots, pos))
+    a.rope, a.ld, a.ldt, a.npages, a.M = rope.table(), rows.stride(0), table.shape[1], kp.shape[0], M
+    a.QN, a.QP, a.CN, a.CP, a.RP, a.eps = QN, QP, CN, CP, RP, eps
+    check(lib().latent_prep(a, int(rows.dtype == torch.float32), stream_ptr()), "latent_prep")
+
+
+def latent_args(qlat: torch.Tensor, q: torch.Tensor, rot_col: int, hs: int, kp: torch.Tensor, table: torch.Tensor,
+                slots: torch.Tensor, pos: torch.Tensor, out: torch.Tensor, M: int, H: int, CP: int, scale: float,
+                gate: Optional[torch.Tensor] = None):
+    """Validated arguments of the latent-attention launches: ``qlat`` rows
+    [H][CP], the rotated query parts at columns ``h * hs + rot_col`` of ``q``,
+    ``out`` rows [H][CP], ``gate`` rows of one logit per head."""
+    dt = qlat.dtype
+    _latent_pool(kp, dt)
+    RP = kp.shape[2] - CP
+    if CP not in LATENT_DIMS or RP not in LATENT_ROT:
+        raise ValueError(f"latent attention: {CP} + {RP} columns")
+    _rows(qlat, M, H * CP, "latent qlat", (torch.float32, torch.bfloat16))
+    _rows(q, M, (H - 1) * hs + rot_col + RP, "latent q", (dt,))
+    _rows(out, M, H * CP, "latent out", (dt,))
+    if gate is not None:
+        _rows(gate, M, H, "latent gate", (dt,))
+    _index(slots, M, "latent slots")
+    _index(pos, M, "latent pos")
+    if table.dtype != torch.int32 or table.dim() != 2 or not table.is_contiguous() or not scale > 0:
+        raise ValueError("latent attention: bad block table or score scale")
+    a = lib().LatentAttnArgs()
+    a.qlat, a.qrot, a.kp, a.table = ptr(qlat), ptr(q) + rot_col * q.element_size(), ptr(kp), ptr(table)
+    a.slots, a.pos, a.out, a.gate = ptr(slots), ptr(pos), ptr(out), ptr(gate)
+    a.ldql, a.ldqr, a.hs, a.ldo, a.ldg = qlat.stride(0), q.stride(0), hs, out.stride(0), gate.stride(0) if gate is not None else 0
+    a.ldt, a.npages, a.M, a.H, a.CP, a.RP, a.scale = table.shape[1], kp.shape[0], M, H, CP, RP, scale
+    return a
+
+
+def latent_splits(n_seq: int, H: int, keys: int) -> int:
+    """Workgroups per 64 heads of a decoded token: one per CU, two pages each."""
+    pages = -(-max(keys, 1) // PAGE)
+    return max(1, min(-(-256 // (n_seq * -(-H // LATENT_ROWS))), pages // 2, 64))
+
+
+def latent_attn(args, tiles: torch.Tensor, splits: int = 1, per_token: int = 1, ws: Optional[torch.Tensor] = None) -> None:
+    """``tiles`` (n, 4) int32: {first row, tokens, slot, first packed row of 64}
+    (``chunk_tiles`` with ``rows=LATENT_ROWS``).  ``splits`` > 1: single tokens,
+    ``per_token`` tiles each; ``ws``: fp32, tokens * H * splits * (CP + 2)."""
+    if tiles.dtype != torch.int32 or tiles.dim() != 2 or tiles.shape[1] != 4 or not tiles.is_contiguous():
+        raise ValueError("latent_attn: tiles must be contiguous int32 (n, 4)")
+    if splits > 1 and (ws is None or ws.dtype != torch.float32 or not ws.is_contiguous()):
+        raise ValueError("latent_attn: splits > 1 needs an fp32 workspace")
+    check(lib().latent_attn(args, ptr(tiles), tiles.shape[0], splits, per_token, ptr(ws), 0 if ws is None else ws.numel(),
+                            stream_ptr()), "latent_attn")
+
+
+def latent_attn_f32(args) -> None:
+    """fp32 attention of every row (cache already written)."""
+    check(lib().latent_attn_f32(args, stream_ptr()), "latent_attn_f32")

@@ -12,8 +12,8 @@ import torch
 
 from ._lib import check, lib, ptr, stream_ptr
 
-ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU_MUL, ACT_GELU_TANH_MUL = 0, 1, 2, 3, 4
-ACTS_GLU = (ACT_SILU_MUL, ACT_GELU_TANH_MUL)  # packed gate|up weight (pack_gate_up), half-width output
+ACT_NONE, ACT_RELU, ACT_GELU, ACT_SILU_MUL, ACT_GELU_TANH_MUL, ACT_CLAMP_MUL = 0, 1, 2, 3, 4, 5
+ACTS_GLU = (ACT_SILU_MUL, ACT_GELU_TANH_MUL, ACT_CLAMP_MUL)  # packed gate|up weight (pack_gate_up), half-width output
 SKINNY_MAX_M = 256
 
 

@@ -1,5 +1,6 @@
 """Wrappers of the recurrent-mixer and mixture-of-experts kernels
-(``csrc/kernels/recurrence.hip``, ``moe.hip``, ``qk_norm.hip``).
+(``csrc/kernels/recurrence.hip``, ``wkv.hip``, ``token_shift.hip``, ``moe.hip``,
+``qk_norm.hip``).
 
 Operands are bf16 (serving) or fp32 (exact mode); step sizes, decays, states,
 router logits and weights are fp32 in both.  As in ``decoder_ops``, every shape
@@ -131,6 +132,87 @@ def scan(rows: torch.Tensor, cols, state: torch.Tensor, y: torch.Tensor, vdim: i
         check(lib().scan_steps(a, 0, stream_ptr()), "scan_steps")
 
 
+# ---------------------------------------------------------------------- the token before
+def pair_rows(ids: torch.Tensor, prev: torch.Tensor, rows: torch.Tensor, start: torch.Tensor, last: torch.Tensor,
+              slots: torch.Tensor, pos: torch.Tensor, M: int, mul_prev: int, mul_cur: int, buckets: int) -> None:
+    """``rows[m] = (previous token * mul_prev + ids[m] * mul_cur) % buckets``, or
+    ``buckets`` for a sequence's first token; ``prev`` (slots,) keeps every
+    sequence's last token."""
+    for t, n in ((ids, M), (rows, M), (start, M), (last, M), (slots, M), (pos, M), (prev, 1)):
+        _index(t, n, "pair_rows index")
+    a = _fill(lib().PairArgs(), ids=ptr(ids), prev=ptr(prev), rows=ptr(rows), start=ptr(start), last=ptr(last),
+              slots=ptr(slots), pos=ptr(pos), mul_prev=mul_prev, mul_cur=mul_cur, buckets=buckets, M=M,
+              nslots=prev.numel())
+    check(lib().pair_rows(a, stream_ptr()), "pair_rows")
+
+
+def token_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, out: torch.Tensor, start: torch.Tensor,
+                last: torch.Tensor, slots: torch.Tensor, pos: torch.Tensor, M: int) -> None:
+    """``out[i] = x + (x of the token before - x) * mu[i]`` for every row of ``mu``
+    (n, NP); ``out`` (n, M, NP); ``state`` (slots, NP) keeps every sequence's last row."""
+    n, NP = mu.shape
+    _rows(x, M, NP, "token_shift x", (torch.float32,))
+    _weight(mu, n * NP, "token_shift mu")
+    if tuple(out.shape) != (n, M, NP) or out.stride(2) != 1 or out.dtype not in (torch.float32, torch.bfloat16) \
+            or state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] != NP or not state.is_contiguous():
+        raise ValueError(f"token_shift: out {tuple(out.shape)}, state {tuple(state.shape)}")
+    for t in (start, last, slots, pos):
+        _index(t, M, "token_shift index")
+    a = _fill(lib().ShiftArgs(), x=ptr(x), mu=ptr(mu), out=ptr(out), state=ptr(state), start=ptr(start), last=ptr(last),
+              slots=ptr(slots), pos=ptr(pos), ostride=out.stride(0), ldx=x.stride(0), ldo=out.stride(1), M=M, NP=NP, n=n,
+              nslots=state.shape[0])
+    check(lib().token_shift(a, int(out.dtype == torch.float32), stream_ptr()), "token_shift")
+
+
+# ---------------------------------------------------------------------- recurrence with a decay per key channel
+WKV_DIMS = (64, 128, 256)  # padded head sizes the kernels are built for
+
+
+def decay(t: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor, la: torch.Tensor, M: int) -> None:
+    """``la = -exp(tanh(t) w2^T + w0)`` (M, N) fp32; ``t`` fp32 rows, ``w2``
+    (N, rank) in bf16 (two-term products on the MFMA) or fp32 (exact)."""
+    N, rank = w2.shape
+    _rows(t, M, rank, "decay t", (torch.float32,))
+    _weight(w0, N, "decay w0")
+    _weight(la, M * N, "decay la")
+    if not w2.is_contiguous() or w2.dtype not in (torch.float32, torch.bfloat16):
+        raise ValueError("decay: w2 must be contiguous bf16 or fp32")
+    a = _fill(lib().DecayArgs(), t=ptr(t), w2=ptr(w2), w0=ptr(w0), la=ptr(la), ldt=t.stride(0), M=M, N=N, rank=rank)
+    check(lib().decay(a, int(w2.dtype == torch.float32), stream_ptr()), "decay")
+
+
+def wkv(rkv: torch.Tensor, la: torch.Tensor, u: torch.Tensor, state: torch.Tensor, y: torch.Tensor, dim: int,
+        pos: torch.Tensor, ent: torch.Tensor, n_chunk: int, n_one: int, M: int) -> None:
+    """The recurrence of every sequence of a step.  ``rkv`` (3 or more, M, H * NP):
+    r, k, v rows with heads padded to NP; ``la`` (M, H * NP) logarithms of the
+    decays; ``u`` (H, NP); ``state`` (slots, H, NP values, NP channels) fp32;
+    ``ent``: ``n_chunk`` sequences of two tokens or more, then ``n_one`` of one."""
+    slots, H, VP, NP = state.shape
+    f32 = rkv.dtype == torch.float32
+    if rkv.dim() != 3 or rkv.shape[0] < 3 or rkv.shape[1] < M or rkv.shape[2] < H * NP or rkv.stride(2) != 1 \
+            or rkv.dtype not in (torch.float32, torch.bfloat16):
+        raise ValueError(f"wkv: r, k, v {tuple(rkv.shape)} {rkv.dtype}")
+    _rows(y, M, H * dim, "wkv y", (rkv.dtype,))
+    _entries(ent, n_chunk + n_one)
+    _index(pos, M, "wkv pos")
+    _weight(la, M * H * NP, "wkv la")
+    _weight(u, H * NP, "wkv u")
+    if state.dtype != torch.float32 or not state.is_contiguous() or NP not in WKV_DIMS or VP != NP or dim > NP:
+        raise ValueError(f"wkv: bad state {tuple(state.shape)} {state.dtype}")
+    a = _fill(lib().WkvArgs(), r=ptr(rkv[0]), k=ptr(rkv[1]), v=ptr(rkv[2]), la=ptr(la), u=ptr(u), state=ptr(state), y=ptr(y),
+              ent=ptr(ent), pos=ptr(pos), ld=rkv.stride(1), ldy=y.stride(0), M=M, H=H, NP=NP, dim=dim, nent=n_chunk,
+              nslots=slots)
+    if f32:
+        a.nent = n_chunk + n_one
+        check(lib().wkv_steps(a, 1, stream_ptr()), "wkv_steps")
+        return
+    if n_chunk:
+        check(lib().wkv_chunks(a, stream_ptr()), "wkv_chunks")
+    if n_one:
+        a.ent, a.nent = ptr(ent) + 16 * n_chunk, n_one
+        check(lib().wkv_steps(a, 0, stream_ptr()), "wkv_steps")
+
+
 def gated_norm(y: torch.Tensor, z: torch.Tensor, out: torch.Tensor, M: int, n: int, groups: int, eps: float,
                w: Optional[torch.Tensor] = None, gate_first: bool = False) -> None:
     """``gate_first``: out = norm(y * silu(z)) * w; else norm(y) * silu(z) [* w];
@@ -165,8 +247,12 @@ class Routing:
         return self._sets[row0]
 
 
-def route(logits: torch.Tensor, r: Routing, M: int, groups: int, keep: int, row0: int = 0) -> None:
-    """Choices of M rows; the results start at entry ``row0 * top`` of the buffers."""
+def route(logits: torch.Tensor, r: Routing, M: int, groups: int, keep: int, row0: int = 0, *, sigmoid: bool = False,
+          correction: Optional[torch.Tensor] = None, group_top: int = 1, normalise: bool = True) -> None:
+    """Choices of M rows; the results start at entry ``row0 * top`` of the buffers.
+    ``correction`` (experts,) joins the scores for the choice only."""
+    if correction is not None:
+        _weight(correction, r.experts, "route correction")
     _rows(logits, M, r.experts, "route logits", (torch.float32,))
     if row0 + M > r.rows:
         raise ValueError(f"route: rows {row0} .. {row0 + M} of {r.rows}")
@@ -174,7 +260,8 @@ def route(logits: torch.Tensor, r: Routing, M: int, groups: int, keep: int, row0
     counts, offs = r.bins(row0)
     a = _fill(lib().RouteArgs(), logits=ptr(logits), idx=ptr(r.idx) + o, w=ptr(r.w) + o, rank=ptr(r.rank) + o,
               counts=ptr(counts), order=ptr(r.order) + o, place=ptr(r.place) + o, offs=ptr(offs),
-              ldl=logits.stride(0), M=M, E=r.experts, groups=groups, keep=keep, top=r.top)
+              ldl=logits.stride(0), M=M, E=r.experts, groups=groups, keep=keep, top=r.top,
+              correction=ptr(correction), sigmoid=int(sigmoid), group_top=group_top, normalise=int(normalise))
     check(lib().route(a, stream_ptr()), "route")
 
 
@@ -184,7 +271,11 @@ class ExpertLinear:
     copy), or fp32 weights row-major.  Rows of N and K are padded to multiples
     of 64 by the caller; gated projections come packed (``gemm.pack_gate_up``)."""
 
-    def __init__(self, ws: List[torch.Tensor], dtype: torch.dtype, device, act: int = G_.ACT_NONE):
+    def __init__(self, ws: List[torch.Tensor], dtype: torch.dtype, device, act: int = G_.ACT_NONE, clamp=None):
+        """``clamp``: (limit, alpha, shift) of the clamped gated activation."""
+        self.clamp = clamp
+        if (clamp is not None) != (act == G_.ACT_CLAMP_MUL):
+            raise ValueError("ExpertLinear: the clamped activation and its constants go together")
         self.E, (self.N, self.K) = len(ws), ws[0].shape
         if self.N % 64 or self.K % 64 or any(w.shape != ws[0].shape for w in ws):
             raise ValueError(f"ExpertLinear: {self.N} x {self.K}")
@@ -215,17 +306,40 @@ class ExpertLinear:
                   order=ptr(r.order) + 4 * row0 * r.top if gather else 0, counts=ptr(counts) if clear else 0,
                   lda=x.stride(0), ldc=c.stride(0), rows=rows, arows=rows // gather if gather else rows,
                   div=max(gather, 1), N=self.N, K=self.K, E=self.E, act=self.act)
+        if self.clamp is not None:
+            a.set_clamp(*self.clamp)
         if f32:
             a.W = ptr(self.w)
             check(lib().grouped_gemm_f32(a, stream_ptr()), "grouped_gemm_f32")
             if c is not out:
                 F = self.n_out
-                check(lib().glu_f32(ptr(c), c.stride(0), ptr(out), out.stride(0), rows, F, self.act, stream_ptr()), "glu_f32")
+                check(lib().glu_f32(ptr(c), c.stride(0), ptr(out), out.stride(0), rows, F, self.act, stream_ptr(),
+                                    *(self.clamp or ())), "glu_f32")
             return out
         a.Wsh = ptr(self.w)
         check(lib().grouped_gemm(a, stream_ptr()), "grouped_gemm")
         return out
 
 
-__all__ = ["qk_norm", "ConvWeights", "conv", "scan", "gated_norm", "Routing", "route", "ExpertLinear", "pad_state",
+    def each(self, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+        """``out[e] = x[e] W_e^T`` for every projection: ``x`` (E, M, K) and ``out``
+        (E, M, N), of any row and projection strides (heads side by side in a
+        row, or one operand after the other).  No activation."""
+        E, M, K = x.shape
+        if (E, K) != (self.E, self.K) or tuple(out.shape) != (E, M, self.N) or self.act != G_.ACT_NONE \
+                or x.dtype != self.dtype or out.dtype != self.dtype or x.stride(2) != 1 or out.stride(2) != 1:
+            raise ValueError(f"ExpertLinear.each: {tuple(x.shape)} {x.dtype} to {tuple(out.shape)}, weights "
+                             f"{self.E} x {self.N} x {self.K}")
+        a = _fill(lib().GroupedArgs(), A=ptr(x), C=ptr(out), lda=x.stride(1), ldc=out.stride(1), rows=E * M, arows=E * M,
+                  div=1, N=self.N, K=K, E=E, act=self.act, sa=x.stride(0), sc=out.stride(0))
+        if self.dtype == torch.float32:
+            a.W = ptr(self.w)
+            check(lib().grouped_gemm_f32(a, stream_ptr()), "grouped_gemm_f32")
+        else:
+            a.Wsh = ptr(self.w)
+            check(lib().grouped_gemm(a, stream_ptr()), "grouped_gemm")
+        return out
+
+
+__all__ = ["pair_rows", "token_shift", "decay", "wkv", "qk_norm", "ConvWeights", "conv", "scan", "gated_norm", "Routing", "route", "ExpertLinear", "pad_state",
            "pad64", "STATE_DIMS", "CHUNK_TOKENS"]

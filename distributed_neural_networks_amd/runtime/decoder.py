@@ -34,12 +34,14 @@ from ..ops import decoder_ops as D_
 from ..ops import mixer_ops as M_
 from ..ops import transformer_ops as T_
 from ..ops.gemm import decode_workspace
-from .decoder_layers import LAYERS, DynamicTanh, Weights, pad
-from .paging import StepBatch, pages_for
+from .decoder_layers import LAYERS, DynamicTanh, ScalarNorm, Weights, pad
+from .paging import StepBatch, pages_for, tile_lists
 from .stages import StageCompute, StageOutput
 
 DTYPES = {None: torch.bfloat16, "bf16": torch.bfloat16, "bfloat16": torch.bfloat16, "fp32": torch.float32,
           "float32": torch.float32}
+STATES = ("state", "ring", "shift", "prev")  # tensors by slot that a step advances
+F32_BUFFERS = ("dt", "la", "router", "lowrank")
 HOP_IDS = 4  # fp32 columns after the residual at a stage boundary: the token id's bits, padding
 
 
@@ -78,7 +80,7 @@ class DecoderStage(StageCompute):
         self.runs = c.runs[start:end + 1]
         self.side = c.side_dim
         self.enters = any(r.enters for r in self.runs)
-        koz = self.family == "kozusun"
+        koz, tiz = self.family == "kozusun", self.family == "tizalorn"
         self.entry_projects = koz  # a loop's entry: a projection of [x | x0], or the sum x + x0
         self.embed_mult = c.embed_scale if koz else 1.0
 
@@ -87,9 +89,13 @@ class DecoderStage(StageCompute):
             return pad(t, t.shape[0], cols).contiguous()
         self.embed = table("embed", self.wp) if (first or self.enters) else None
         self.freq: Optional[torch.Tensor] = None  # sinusoidal position vector: turns per position
-        if not koz:
+        if self.family == "funepel":
             i = torch.arange(-(-self.width // 2), dtype=torch.float64)
             self.freq = (10000.0 ** (-2.0 * i / self.width) / (2.0 * math.pi)).to(dev)
+        self.pairs = c.bigram if tiz and first else None  # a table of token pairs joins the embedding, normed
+        if self.pairs is not None:
+            self.pair_embed = table("bigram", self.wp)
+            self.embed_norm = ScalarNorm(Weights(c, "", sd, dt, dev), "embed.norm")
         if self.side:
             self.side_embed = sd["side.embed"].to(device=dev, dtype=dt).contiguous()
         if self.enters and self.entry_projects:
@@ -104,10 +110,12 @@ class DecoderStage(StageCompute):
                 w = pad(1 + ld("final.norm"), self.wp)
                 w[self.width:] = 0
                 self.final_norm = {"norm": w}
+            elif tiz:
+                self.final_norm = {"norm": ScalarNorm(ld, "final.norm").w}
             else:
                 self.final_norm = DynamicTanh(ld, "final.norm").prep(None)
             self.w_head = ld.linear(ld.rows("head", self.V))
-        self.groups = sorted({g for L in self.layers for g in L.groups})
+        self.groups = sorted({g for L in self.layers for g in L.groups}, key=str)
         self._alloc()
         self._ring: Dict[tuple, dict] = {}
         self._ring_table: Optional[torch.Tensor] = None
@@ -124,7 +132,7 @@ class DecoderStage(StageCompute):
         for L in self.layers:
             for k, v in L.buffers(self.f32).items():
                 cols[k] = max(cols.get(k, 0), self.wp if v is None else v)
-        self.buf = {k: z(v, torch.float32 if k in ("dt", "la", "router") else dt) for k, v in cols.items() if v}
+        self.buf = {k: z(v, torch.float32 if k in F32_BUFFERS else dt) for k, v in cols.items() if v}
         self._experts: Dict[tuple, M_.Routing] = {}
         self._expert_rows: Dict[str, torch.Tensor] = {}
         if self.side:
@@ -135,6 +143,10 @@ class DecoderStage(StageCompute):
                 self.y32 = self.y if self.f32 else z(self.wp, torch.float32)
             else:
                 self.x0 = z(self.wp, torch.float32)
+        if self.pairs is not None:
+            self.pair_row = torch.zeros((n,), dtype=torch.int32, device=dev)
+            self.ones = torch.ones((n,), dtype=torch.float32, device=dev)
+            self.prev = torch.zeros((self.num_slots,), dtype=torch.int32, device=dev)
         if not self.first:
             self.ids_in = torch.zeros((n,), dtype=torch.int32, device=dev)
         self.caches = [L.new_cache(self) for L in self.layers]
@@ -188,6 +200,8 @@ class DecoderStage(StageCompute):
         return self.last and not self.temperature > 0
 
     def _cache_tensors(self):
+        if self.pairs is not None:
+            yield "prev", self.prev
         for c in self.caches:
             yield from ((k, t) for k, t in (c.items() if isinstance(c, dict) else zip(("kp", "vp"), c)))
 
@@ -197,15 +211,15 @@ class DecoderStage(StageCompute):
 
     def save_states(self) -> List[torch.Tensor]:
         """Copies of the recurrent states (a step that is run twice advances them twice)."""
-        return [t.clone() for k, t in self._cache_tensors() if k in ("state", "ring")]
+        return [t.clone() for k, t in self._cache_tensors() if k in STATES]
 
     def restore_states(self, saved: List[torch.Tensor]) -> None:
-        for t, v in zip((t for k, t in self._cache_tensors() if k in ("state", "ring")), saved):
+        for t, v in zip((t for k, t in self._cache_tensors() if k in STATES), saved):
             t.copy_(v)
 
     @property
     def recurrent(self) -> bool:
-        return any(k == "state" for k, _ in self._cache_tensors())
+        return any(k in STATES for k, _ in self._cache_tensors())
 
     # ------------------------------------------------------------------ layers
     def _prep(self, k: int, r0: int, M: int) -> dict:
@@ -232,6 +246,10 @@ class DecoderStage(StageCompute):
         emb = {"y": self.embed, "yidx": ids, "mult": self.embed_mult}
         if self.freq is not None:
             emb.update(pos=b.pos, freq=self.freq)
+        if self.pairs is not None:
+            p, rows = self.pairs, self.pair_row[s]
+            M_.pair_rows(ids, self.prev, rows, b.start, b.last, b.slots, b.pos, M, p.mul_prev, p.mul_cur, p.buckets)
+            emb.update(ys=self.pair_embed, ysi=rows, ysw=self.ones[s], top=1, **self.embed_norm.joined)
         if not self.enters:
             up(**(dict(emb, x_out=x) if self.first else {"x_in": x}), **self._prep(0, r0, M))
         elif self.entry_projects:  # the embedding output, kept for the loop's passes
@@ -319,17 +337,19 @@ class DecoderStage(StageCompute):
             c = {"slots": slots.repeat_interleave(T).contiguous(), "ent": ent,
                  "start": first.repeat_interleave(T).contiguous(),
                  "last": torch.arange(T - 1, B * T, T, dtype=torch.int32, device=dev),
-                 "rows": torch.arange(B * T, dtype=torch.int32, device=dev), "chunks": [], "tiles": None}
+                 "ends": (first + (T - 1)).repeat_interleave(T).contiguous(),
+                 "rows": torch.arange(B * T, dtype=torch.int32, device=dev), "chunks": []}
+            seqs = [(i * T, T, b0 + i) for i in range(B)]
+            lists = tile_lists(self.groups, seqs, []) if T > 1 else tile_lists(self.groups, [], seqs)
+            c["tiles"] = {k: torch.tensor(v, dtype=torch.int32, device=dev) for k, v in lists.items()}
             if T > 1:
-                c["chunks"] = [(i * T, T, b0 + i) for i in range(B)]
-                c["tiles"] = {g: torch.tensor([t for ch in c["chunks"] for t in D_.chunk_tiles(*ch, g)],
-                                              dtype=torch.int32, device=dev) for g in self.groups}
+                c["chunks"] = seqs
                 c["steps"] = torch.arange(T, dtype=torch.int32, device=dev)
             self._ring[(B, T, b0)] = c
         p = pos if T == 1 else (pos.view(B, 1) + c["steps"]).view(-1).contiguous()
         return StepBatch(M=B * T, pos=p, slots=c["slots"], table=self._ring_table,
                          dec_rows=c["rows"] if T == 1 else None, n_dec=B if T == 1 else 0, chunks=c["chunks"],
-                         max_len=self.max_seq, ent=c["ent"], start=c["start"], tiles=c["tiles"])
+                         max_len=self.max_seq, ent=c["ent"], start=c["start"], last=c["ends"], tiles=c["tiles"])
 
     def step(self, x: torch.Tensor, pos: torch.Tensor, B: int, T: int, b0: int = 0,
              out: Optional[torch.Tensor] = None, last_only: bool = True, advance=None):

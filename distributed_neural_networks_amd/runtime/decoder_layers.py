@@ -15,6 +15,12 @@ run asks for (``nxt``, keyword arguments of ``rows_update``).
   ``Mamba2Mixer``: convolution and state-space recurrence, state by slot.
   ``AttentionRetentionMixer``: paged attention whose values are its keys, and a
   retention state, on the same input, by one projection.
+* ``PostNormLayer`` (Tizalorn): a mixer, then a feed-forward, each with a norm on
+  its output; the sublayers read the residual itself.
+  ``WkvMixer``: mixes with the token before, recurrence with a decay per key
+  channel, states by slot.  ``LatentAttentionMixer``: every head over one cached
+  latent per token.  ``PolyNormFeedForward``: powers normed over the row.
+* ``MixtureOfExperts``: both routers and expert activations of ``MoEConfig``.
 * ``TokenInput``: the per-layer input looked up by token, shared by both.
 
 All padding happens here, once: widths, feed-forward and side sizes to multiples
@@ -28,11 +34,12 @@ from typing import Dict, List, Optional
 
 import torch
 
-from ..models import funepel
+from ..models import funepel, tizalorn
 from ..ops import decoder_ops as D_
+from ..models.decoder_config import MoEConfig
 from ..ops import mixer_ops as M_
-from ..ops.gemm import ACT_GELU_TANH_MUL, ACT_SILU_MUL, pack_gate_up
-from .paging import PAGE, StepBatch
+from ..ops.gemm import ACT_CLAMP_MUL, ACT_GELU_TANH_MUL, ACT_SILU_MUL, pack_gate_up
+from .paging import PAGE, LatentHeads, StepBatch
 
 
 def pad(t: torch.Tensor, *shape: int) -> torch.Tensor:
@@ -329,11 +336,14 @@ class AttentionRetentionMixer:
 
 
 class MixtureOfExperts:
-    def __init__(self, ld: Weights, m: funepel.MoEConfig):
+    def __init__(self, ld: Weights, m: MoEConfig):
         self.m, self.fp, self.ep = m, D_.pad64(m.ff), pad16(m.experts)
         self.w_router = ld.linear(ld.rows("router", self.ep))
         experts = [ld.sub(f"e{e}.") for e in range(m.experts)]
-        self.w_up = M_.ExpertLinear([e.gate_up(self.fp) for e in experts], ld.dtype, ld.device, ACT_SILU_MUL)
+        act = (ACT_SILU_MUL, None) if m.limit is None else (ACT_CLAMP_MUL, (m.limit, m.alpha, m.shift))
+        self.w_up = M_.ExpertLinear([e.gate_up(self.fp) for e in experts], ld.dtype, ld.device, *act)
+        self.routing = {"sigmoid": m.sigmoid, "group_top": m.group_top, "normalise": m.normalise,
+                        "correction": ld("correction").contiguous() if m.correction else None}
         self.w_down = M_.ExpertLinear([pad(e("down"), ld.wp, self.fp) for e in experts], ld.dtype, ld.device)
         self.sp = D_.pad64(m.shared_ff) if m.shared_ff else 0
         if self.sp:
@@ -353,7 +363,7 @@ class MixtureOfExperts:
         r0, M = s.start, s.stop - s.start
         z = self.w_router(h, B["router"][s, :self.ep], gws)
         rt, up, down = st.experts(m.experts, m.top, self.fp)
-        M_.route(z, rt, M, m.groups, m.keep, r0)
+        M_.route(z, rt, M, m.groups, m.keep, r0, **self.routing)
         e = slice(r0 * m.top, (r0 + M) * m.top)
         gu = up[e, :self.fp]
         self.w_up(h, M * m.top, gu, rt, m.top, r0, st.expert_scratch(2 * self.fp, e) if st.f32 else None, clear=True)
@@ -409,4 +419,193 @@ class SequentialLayer:
             self.side.run(st, s, ids, gws, nxt, up)
 
 
-LAYERS = {"kozusun": JointLayer, "funepel": SequentialLayer}
+# ---------------------------------------------------------------------- Tizalorn
+class ScalarNorm:
+    """RMS norm of a sublayer's output times one number, as keyword arguments of ``rows_update``."""
+
+    def __init__(self, ld: Weights, name: str):
+        self.w = torch.zeros(ld.wp, dtype=torch.float32, device=ld.device)
+        self.w[:ld.width] = ld(name)
+
+    @property
+    def joined(self) -> dict:
+        """... of the whole sum, where weighted rows join the output."""
+        return {"y_norm": self.w, "y_joined": True}
+
+    def of(self, part: dict) -> dict:
+        return dict(part, **(self.joined if "ys" in part else {"y_norm": self.w}))
+
+
+class WkvMixer:
+    """r, k, v and the gate in one launch (four projections of operands of their
+    own), heads of r, k and v padded to a state size; the decay by way of its
+    low-rank projection in fp32."""
+    groups: List = []
+    reads_copy = False  # it reads the fp32 residual
+
+    def __init__(self, ld: Weights, m: tizalorn.WkvConfig):
+        self.m = m
+        self.np = max(64, M_.pad_state(m.dim))
+        self.n, self.inner, self.ip = m.heads * self.np, m.inner, D_.pad64(m.inner)
+        self.mu = torch.stack([ld.vec("mu." + n) for n in "rkvgw"]).contiguous()
+        heads = [pad_heads(ld.rows(n, m.inner), m.heads, m.dim, self.np) for n in "rkv"]
+        self.w_in = M_.ExpertLinear(heads + [ld.rows("g", self.n)], ld.dtype, ld.device)
+        w1, w2 = ld("w1"), ld("w2")
+        if w1.shape[0] != w2.shape[1]:
+            raise ValueError(f"{ld.prefix}: w1 {tuple(w1.shape)} does not fit w2 {tuple(w2.shape)}")
+        self.rank = D_.pad64(w1.shape[0])
+        self.w1 = ld.linear(pad(w1, self.rank, ld.wp))
+        self.w2 = pad(pad_heads(w2, m.heads, m.dim, self.np), self.n, self.rank).to(ld.dtype).contiguous()
+        self.w0 = pad_heads(ld("w0"), m.heads, m.dim, self.np).contiguous()
+        self.u = pad(ld("u"), m.heads, self.np).contiguous()
+        self.norm = ld("norm").contiguous()
+        self.w_o = ld.linear(pad(ld("o"), ld.wp, self.ip))
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        return {"mixes": 5 * self.mu.shape[1], "rkvg": 4 * self.n, "lowrank": self.rank, "la": self.n, "mix": self.ip,
+                "mixn": self.ip}
+
+    def new_cache(self, st):
+        f = dict(dtype=torch.float32, device=st.device)
+        return {"shift": torch.zeros((st.num_slots, st.wp), **f),
+                "state": torch.zeros((st.num_slots, self.m.heads, self.np, self.np), **f)}
+
+    def ws_need(self, n: int, keys: int) -> int:
+        return 0
+
+    def run(self, st, cache, b: StepBatch, s: slice, gws, ws) -> dict:
+        m, M, B, wp = self.m, b.M, st.buf, st.wp
+        mixes = st.flat("mixes", s, 5 * wp).view(5, M, wp)
+        M_.token_shift(st.x[s], self.mu, cache["shift"], mixes, b.start, b.last, b.slots, b.pos, M)
+        rkvg = self.w_in.each(mixes[:4], st.flat("rkvg", s, 4 * self.n).view(4, M, self.n))
+        la = st.flat("la", s, self.n)
+        M_.decay(self.w1(mixes[4], B["lowrank"][s, :self.rank], gws), self.w2, self.w0, la, M)
+        o, on = B["mix"][s, :self.ip], B["mixn"][s, :self.ip]
+        M_.wkv(rkvg, la, self.u, cache["state"], o, m.dim, b.pos, b.ent, len(b.chunks), b.n_dec, M)
+        M_.gated_norm(o, rkvg[3], on, M, self.inner, m.heads, st.eps, self.norm)
+        return {"y": self.w_o(on, st.y[s], gws), "mult": 1.0}
+
+
+class LatentAttentionMixer:
+    """One projection to [query latent | latent | key part | gate]; the heads'
+    query projection to [unrotated | rotated] parts; the key projection applied
+    to the query and the value projection to the summed latents, both head by head."""
+    reads_copy = True
+
+    def __init__(self, ld: Weights, m: tizalorn.LatentAttentionConfig):
+        self.m, self.tiles = m, LatentHeads(m.heads)
+        self.groups: List = [self.tiles]
+        H, D, R, V = m.heads, m.dim, m.rot_dim, m.vdim
+        self.cp, self.rp = D_.pad_to(m.kv_rank, D_.LATENT_DIMS, "latent size"), D_.pad_to(R, D_.LATENT_ROT, "rotated size")
+        self.dp, self.vp, self.qp = D_.pad64(D), D_.pad64(V), D_.pad64(m.q_rank)
+        self.hs = self.dp + self.rp
+        kv = ld("dkv")
+        parts = [ld.rows("dq", self.qp), pad(kv[:m.kv_rank], self.cp, ld.wp), pad(kv[m.kv_rank:], self.rp, ld.wp),
+                 ld.rows("g", H)]
+        self.gate_col = self.qp + self.cp + self.rp
+        self.n_in = pad16(self.gate_col + H)
+        self.w_in = ld.linear(pad(torch.cat(parts), self.n_in, ld.wp))
+        self.qw, self.cw = pad(ld("dq.norm"), self.qp).contiguous(), pad(ld("dkv.norm"), self.cp).contiguous()
+        uq = ld("uq").view(H, D + R, m.q_rank)
+        uq = torch.cat([pad(uq[:, :D], H, self.dp, self.qp), pad(uq[:, D:], H, self.rp, self.qp)], 1)
+        self.w_uq = ld.linear(uq.reshape(H * self.hs, self.qp))
+        uk, uv = ld("uk").view(H, D, m.kv_rank), ld("uv").view(H, V, m.kv_rank)
+        self.w_uk = M_.ExpertLinear([pad(w.t().contiguous(), self.cp, self.dp) for w in uk], ld.dtype, ld.device)
+        self.w_uv = M_.ExpertLinear([pad(w, self.vp, self.cp) for w in uv], ld.dtype, ld.device)
+        self.w_o = ld.linear(pad(pad(ld("o").view(ld.width, H, V), ld.width, H, self.vp).reshape(ld.width, -1), ld.wp,
+                                 H * self.vp))
+        self.rope = D_.Rope(*m.rot.frequencies(), ld.device)
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        H = self.m.heads
+        return {"in": self.n_in, "q": H * self.hs, "qlat": H * self.cp, "olat": H * self.cp, "mix": H * self.vp}
+
+    def new_cache(self, st):
+        return {"kp": torch.zeros((st.num_pages, PAGE, self.cp + self.rp), dtype=st.dtype, device=st.device)}
+
+    def splits(self, n: int, keys: int) -> int:
+        return D_.latent_splits(n, self.m.heads, keys)
+
+    def ws_need(self, n: int, keys: int) -> int:
+        s = self.splits(n, keys)
+        return n * self.m.heads * s * (self.cp + 2) if s > 1 else 0
+
+    def run(self, st, cache, b: StepBatch, s: slice, gws, ws) -> dict:
+        m, H, M, B, kp = self.m, self.m.heads, b.M, st.buf, cache["kp"]
+        rows = self.w_in(st.h[s], B["in"][s, :self.n_in], gws)
+        D_.latent_prep(rows, kp, self.qw, self.cw, self.rope, b.table, b.slots, b.pos, M, m.q_rank, m.kv_rank, self.cp,
+                       st.eps)
+        q = self.w_uq(rows[:, :self.qp], B["q"][s, :H * self.hs], gws)
+        D_.rope_rows(q, M, H, self.hs, self.dp, self.rp, b.pos, self.rope)
+        heads = lambda t, n: t.unflatten(1, (H, n)).transpose(0, 1)  # noqa: E731  (M, H n) -> (H, M, n)
+        qlat, olat, out = (B[k][s, :H * n] for k, n in (("qlat", self.cp), ("olat", self.cp), ("mix", self.vp)))
+        self.w_uk.each(heads(q, self.hs)[..., :self.dp], heads(qlat, self.cp))
+        args = D_.latent_args(qlat, q, self.dp, self.hs, kp, b.table, b.slots, b.pos, olat, M, H, self.cp, m.scale,
+                              rows[:, self.gate_col:])
+        if st.f32:
+            D_.latent_attn_f32(args)
+        else:
+            if b.chunks:
+                D_.latent_attn(args, b.tiles[self.tiles, "chunks"])
+            if b.n_dec:
+                D_.latent_attn(args, b.tiles[self.tiles, "ones"], self.splits(b.n_dec, b.max_len), self.tiles.per_token, ws)
+        self.w_uv.each(heads(olat, self.cp), heads(out, self.vp))
+        return {"y": self.w_o(out, st.y[s], gws), "mult": 1.0}
+
+
+class PolyNormFeedForward:
+    def __init__(self, ld: Weights, m: tizalorn.DenseConfig):
+        self.m, self.fp = m, D_.pad64(m.ff)
+        self.w_up, self.w_down = ld.linear(ld.rows("up", self.fp)), ld.linear(pad(ld("down"), ld.wp, self.fp))
+        self.act = ld("act").contiguous()
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        return {"ff": self.fp}
+
+    def run(self, st, s: slice, gws) -> dict:
+        z = self.w_up(st.h[s], st.buf["ff"][s, :self.fp], gws)
+        D_.poly_norm(z, self.act, s.stop - s.start, self.m.ff, st.eps)
+        return {"y": self.w_down(z, st.y[s], gws), "mult": 1.0}
+
+
+class PostNormLayer:
+    """x += N(mixer(x)) g1, x += N(feed-forward(x)) g2."""
+    side = None
+
+    def __init__(self, cfg, i: int, sd: Dict[str, torch.Tensor], dtype, device):
+        ld = Weights(cfg, f"l{i}.", sd, dtype, device)
+        L = cfg.layers[i]
+        mixer = WkvMixer if isinstance(L.mixer, tizalorn.WkvConfig) else LatentAttentionMixer
+        self.mixer, self.norm1 = mixer(ld.sub("mix."), L.mixer), ScalarNorm(ld, "norm1")
+        self.groups: List = self.mixer.groups
+        self.ff = self.norm2 = None
+        if L.mlp is not None:
+            ff = PolyNormFeedForward if isinstance(L.mlp, tizalorn.DenseConfig) else MixtureOfExperts
+            self.ff, self.norm2 = ff(ld.sub("mlp."), L.mlp), ScalarNorm(ld, "norm2")
+
+    def prep(self, h: torch.Tensor) -> dict:
+        return {"copy": h} if self.mixer.reads_copy else {}
+
+    def buffers(self, f32: bool) -> Dict[str, int]:
+        b = dict(self.mixer.buffers(f32))
+        for k, v in (self.ff.buffers(f32) if self.ff else {}).items():
+            b[k] = max(b.get(k, 0), v)
+        return b
+
+    def new_cache(self, st):
+        return self.mixer.new_cache(st)
+
+    def ws_need(self, n: int, keys: int) -> int:
+        return self.mixer.ws_need(n, keys)
+
+    def run(self, st, cache, b: StepBatch, ids, s: slice, gws, ws, nxt: dict, up) -> None:
+        x = st.x[s]
+        part = self.norm1.of(self.mixer.run(st, cache, b, s, gws, ws))
+        if self.ff is None:
+            up(x_in=x, x_out=x, **part, **nxt)
+            return
+        up(x_in=x, x_out=x, **part, copy=st.h[s])
+        up(x_in=x, x_out=x, **self.norm2.of(self.ff.run(st, s, gws)), **nxt)
+
+
+LAYERS = {"kozusun": JointLayer, "funepel": SequentialLayer, "tizalorn": PostNormLayer}

@@ -63,7 +63,7 @@ class Engine:
             raise ValueError(f"Engine: {max_slots} slots asked for, the stages hold the states of {slots} sequences")
         self.table = PageTable(num_pages or pages, max_slots)
         self.vocab = self.stages[0].V
-        self.groups = sorted({g for s in self.stages for g in s.groups})
+        self.groups = sorted({g for s in self.stages for g in s.groups}, key=str)
         self.max_tokens = min(s.max_tokens for s in self.stages)
         self.live: Dict[Hashable, _Live] = {}
         self._pos: Optional[torch.Tensor] = None

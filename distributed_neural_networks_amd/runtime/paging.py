@@ -19,7 +19,7 @@ from typing import Dict, List, Optional, Sequence
 import numpy as np
 import torch
 
-from ..ops.decoder_ops import PAGE, chunk_tiles
+from ..ops.decoder_ops import LATENT_ROWS, PAGE, chunk_tiles
 
 
 class OutOfPages(RuntimeError):
@@ -84,8 +84,9 @@ class StepBatch:
     """One step's rows on the device.  ``chunks``: (first row, tokens, slot) of
     the sequences that bring two tokens or more; ``dec_rows``: rows of the
     sequences that bring one; ``ent``: {first row, tokens, slot, 0} of all of
-    them, the chunks first; ``start``: per row, the first row of its sequence;
-    ``max_len``: the longest sequence after the step."""
+    them, the chunks first; ``start`` / ``last``: per row, the first and last row
+    of its sequence; ``max_len``: the longest sequence after the step.
+    ``tiles``: attention workgroups by key (``tile_lists``)."""
     M: int
     pos: torch.Tensor
     slots: torch.Tensor
@@ -96,17 +97,44 @@ class StepBatch:
     max_len: int
     ent: torch.Tensor
     start: torch.Tensor
+    last: torch.Tensor
     ids: Optional[torch.Tensor] = None
     want: Optional[torch.Tensor] = None
     n_want: int = 0
-    tiles: Optional[Dict[int, torch.Tensor]] = None  # query heads per KV head -> prefill tiles
+    tiles: Optional[Dict[object, torch.Tensor]] = None
+
+
+@dataclass(frozen=True)
+class LatentHeads:
+    """Attention of ``heads`` heads over one latent cache, as an entry of a
+    stage's ``groups`` (an int there: query heads per KV head)."""
+    heads: int
+
+    @property
+    def per_token(self) -> int:
+        return -(-self.heads // LATENT_ROWS)
+
+
+def tile_lists(groups: Sequence, chunks: Sequence[tuple], ones: Sequence[tuple]) -> Dict[object, list]:
+    """Workgroups of the attention launches of a step.  ``chunks`` / ``ones``:
+    (first row, tokens, slot) of the sequences that bring several tokens / one.
+    Key ``g`` (query heads per KV head): prefill tiles; ``(LatentHeads, "chunks")``
+    and ``(LatentHeads, "ones")``: tiles of either kind of sequence."""
+    out: Dict[object, list] = {}
+    for g in groups:
+        if isinstance(g, LatentHeads):
+            out[g, "chunks"] = [t for c in chunks for t in chunk_tiles(*c, g.heads, LATENT_ROWS)]
+            out[g, "ones"] = [t for c in ones for t in chunk_tiles(*c, g.heads, LATENT_ROWS)]
+        else:
+            out[g] = [t for c in chunks for t in chunk_tiles(*c, g)]
+    return {k: v for k, v in out.items() if v}
 
 
 def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[int], device) -> StepBatch:
     """``entries``: (token ids, first position, slot, wanted places) per
-    sequence.  ``groups``: the query-heads-per-KV-head values of the model's
-    layers.  Everything travels in one host-to-device copy."""
-    ids, pos, slots, dec, want, chunks, start = [], [], [], [], [], [], []
+    sequence.  ``groups``: the kinds of attention of the model's layers
+    (``tile_lists``).  Everything travels in one host-to-device copy."""
+    ids, pos, slots, dec, want, chunks, start, last = [], [], [], [], [], [], [], []
     for toks, p0, slot, places in entries:
         n, row = len(toks), len(ids)
         if n == 0:
@@ -116,14 +144,16 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
         pos += range(p0, p0 + n)
         slots += [slot] * n
         start += [row] * n
+        last += [row + n - 1] * n
         if n == 1:
             dec.append(row)
         else:
             chunks.append((row, n, slot))
-    parts = [("t%d" % g, np.array([t for c in chunks for t in chunk_tiles(*c, g)], dtype=np.int32).reshape(-1))
-             for g in sorted(set(groups))] if chunks else []
+    tiles = tile_lists(groups, chunks, [(r, 1, slots[r]) for r in dec])
+    parts = [(k, np.array(t, dtype=np.int32).reshape(-1)) for k, t in tiles.items()]
     ent = [(r, n, slot, 0) for r, n, slot in chunks] + [(r, 1, slots[r], 0) for r in dec]
     parts += [("ent", np.array(ent, dtype=np.int32).reshape(-1)), ("start", np.array(start, dtype=np.int32)),
+              ("last", np.array(last, dtype=np.int32)),
               ("ids", np.array(ids, dtype=np.int32)), ("pos", np.array(pos, dtype=np.int32)),
               ("slots", np.array(slots, dtype=np.int32)), ("dec", np.array(dec, dtype=np.int32)),
               ("want", np.array(want, dtype=np.int32)), ("table", table.reshape(-1))]
@@ -138,5 +168,5 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
     v = {name: dev[off[name]:off[name] + a.size] for name, a in parts}
     return StepBatch(M=len(ids), pos=v["pos"], slots=v["slots"], table=v["table"].view(table.shape),
                      dec_rows=v["dec"] if dec else None, n_dec=len(dec), chunks=chunks,
-                     max_len=max(pos) + 1, ent=v["ent"].view(-1, 4), start=v["start"], ids=v["ids"], want=v["want"] if want else None, n_want=len(want),
-                     tiles={g: v["t%d" % g].view(-1, 4) for g in set(groups)} if chunks else None)
+                     max_len=max(pos) + 1, ent=v["ent"].view(-1, 4), start=v["start"], last=v["last"], ids=v["ids"],
+                     want=v["want"] if want else None, n_want=len(want), tiles={k: v[k].view(-1, 4) for k in tiles})
