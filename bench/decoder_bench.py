@@ -2,7 +2,7 @@
 """Layers of the paged decoder families beside layers of another model of the
 same size: prefill and decode.
 
-``bench.py --model kozusun`` / ``--model funepel`` runs it (one GPU).  For each
+``bench.py --model kozusun`` / ``funepel`` / ``tizalorn`` runs it (one GPU).  For each
 size, ``--layers`` layers of random weights of either model (no loop, no head;
 the residual enters from the embedding) run on the same box in turn, timed as
 HIP graphs for decode and eagerly for prefill; medians over alternating repeats.
@@ -11,6 +11,9 @@ HIP graphs for decode and eagerly for prefill; medians over alternating repeats.
 * funepel: its two kinds of layers (a Mamba-2 mixer; attention beside
   retention; both with experts and token input) beside Kozusun layers of the
   same width, attention heads and token input.
+* tizalorn: WKV and latent-attention layers with experts, and a WKV layer with
+  the dense feed-forward, beside both kinds of Funepel layers of the same width
+  and as many active feed-forward columns.
 
 Prints one JSON line; ``--phase`` / ``--only`` restrict a profiler run.
 """
@@ -33,7 +36,10 @@ SIZES = {"8b": dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=4096, ffn_d
          "1b": dict(vocab_size=32768, n_head=32, n_kv_head=8, n_embd=2048, ffn_dim=5632)}
 
 
-MODELS = {"kozusun": ("kozusun", "llama"), "funepel": ("funepel-mamba2", "funepel-parallel", "kozusun")}
+MODELS = {"kozusun": ("kozusun", "llama"), "funepel": ("funepel-mamba2", "funepel-parallel", "kozusun"),
+          "tizalorn": ("tizalorn-wkv", "tizalorn-latent", "tizalorn-dense", "funepel-mamba2", "funepel-parallel")}
+# kind of layer -> layer of the family's presets that is of this kind
+KINDS = {"funepel-mamba2": 0, "funepel-parallel": 1, "tizalorn-dense": 0, "tizalorn-wkv": 1, "tizalorn-latent": 3}
 
 
 def parse(argv=None):
@@ -47,7 +53,7 @@ def parse(argv=None):
     ap.add_argument("--repeats", type=int, default=7)
     ap.add_argument("--steps", type=int, default=20, help="decode steps of a repeat")
     ap.add_argument("--phase", default="both", choices=["both", "prefill", "decode"])
-    ap.add_argument("--only", default="", choices=["", "kozusun", "llama", "funepel-mamba2", "funepel-parallel"])
+    ap.add_argument("--only", default="", choices=["", "kozusun", "llama"] + sorted(KINDS))
     return ap.parse_args(argv)
 
 
@@ -55,7 +61,7 @@ def build(model: str, size: str, layers: int, batch: int, seq: int, tokens: int,
     """A first-stage object with ``layers`` layers of ``model``."""
     from dataclasses import replace
     from distributed_neural_networks_amd import checkpoint as ckpt
-    from distributed_neural_networks_amd.models import funepel, kozusun, llama3
+    from distributed_neural_networks_amd.models import DECODERS, kozusun, llama3, model_info
     from distributed_neural_networks_amd.runtime.decoder import DecoderStage
     from distributed_neural_networks_amd.runtime.transformer import TransformerStage
     lc = SIZES[size]
@@ -67,9 +73,10 @@ def build(model: str, size: str, layers: int, batch: int, seq: int, tokens: int,
                                 max_tokens=tokens)
     if model == "kozusun":
         family, cfg = kozusun, kozusun.scaled(kozusun.KOZUSUN_CONFIGS["kozusun-" + size], layers)
-    else:  # layer 0 of the presets has a Mamba-2 mixer, layer 1 attention beside retention
-        family = funepel
-        cfg = funepel.scaled(funepel.FUNEPEL_CONFIGS["funepel-" + size], (int(model == "funepel-parallel"),) * layers)
+    else:
+        name = model.split("-")[0]
+        family = DECODERS[name]
+        cfg = family.scaled(model_info(f"{name}-{size}").cfg, (KINDS[model],) * layers)
     cfg = replace(cfg, vocab_size=lc["vocab_size"])
     sd = ckpt.random_decoder_state(family, cfg, 0, layers - 1, True, False, 0, dev, True)
     return DecoderStage(model, sd, 0, layers - 1, True, False, dev, max_batch=batch, max_seq=seq, max_tokens=tokens,
