@@ -270,7 +270,7 @@ def random_weights(cfg, seed=0, gain=1.0, w1_rank=16):
         elif n.endswith("mix.w2"):
             t = t / math.sqrt(s[1])
         elif n.endswith("mix.u"):
-            t = 0.8 * t
+            t = 0.5 + 0.5 * t.abs()
         elif len(s) == 1:
             t = 1 + 0.2 * t
         elif n.endswith("mlp.router"):
@@ -278,6 +278,13 @@ def random_weights(cfg, seed=0, gain=1.0, w1_rank=16):
         elif n not in ("embed", "bigram"):
             t = t * gain / math.sqrt(s[1])
         W[n] = t.bfloat16().float()
+    # A head's output is normed, so a first token whose r . (u k) is near zero
+    # would turn rounding into another sign: r and k point the same way.
+    for i, L in enumerate(cfg["layers"]):
+        if L["type"] == "wkv":
+            p = f"l{i}.mix."
+            for a, b in ((p + "mu.k", p + "mu.r"), (p + "k", p + "r")):
+                W[a] = (0.6 * W[a] + 0.6 * W[b]).bfloat16().float()
     return W
 
 
