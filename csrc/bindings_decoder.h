@@ -134,9 +134,21 @@ inline void bind_decoder(py::module_& m) {
       VF(LatentAttnArgs, ldql) VF(LatentAttnArgs, ldqr) VF(LatentAttnArgs, hs) VF(LatentAttnArgs, ldo)
       VF(LatentAttnArgs, ldg) VF(LatentAttnArgs, ldt) VF(LatentAttnArgs, npages) VF(LatentAttnArgs, M)
       VF(LatentAttnArgs, H) VF(LatentAttnArgs, CP) VF(LatentAttnArgs, RP) VF(LatentAttnArgs, scale);
-  m.def("latent_attn", [](const LatentAttnArgs& a, u64 tiles, int ntiles, int splits, int per_token, u64 ws,
+  m.def("latent_attn", [](const LatentAttnArgs& a, u64 tiles, int ntiles, int rows, int splits, int per_token, u64 ws,
                           long long ws_elems, u64 st) {
-    return dnn_latent_attn(&a, CIP(tiles), ntiles, splits, per_token, FP(ws), ws_elems, ST(st));
+    return dnn_latent_attn(&a, CIP(tiles), ntiles, rows, splits, per_token, FP(ws), ws_elems, ST(st));
+  });
+  m.def("latent_gather", [](u64 kp, int cols, u64 table, int ldt, int npages, u64 ent, int nent, u64 out, int rows, u64 st) {
+    return dnn_latent_gather(P(kp), cols, CIP(table), ldt, npages, CIP(ent), nent, P(out), rows, ST(st));
+  });
+  py::class_<LatentKeysArgs>(m, "LatentKeysArgs")
+      .def(py::init([] { return LatentKeysArgs{}; }))
+      PF(LatentKeysArgs, q) PF(LatentKeysArgs, kv) PF(LatentKeysArgs, krot) PF(LatentKeysArgs, pos) PF(LatentKeysArgs, out)
+      PF(LatentKeysArgs, gate) VF(LatentKeysArgs, ldq) VF(LatentKeysArgs, ldkv) VF(LatentKeysArgs, ldr)
+      VF(LatentKeysArgs, ldo) VF(LatentKeysArgs, ldg) VF(LatentKeysArgs, M) VF(LatentKeysArgs, H) VF(LatentKeysArgs, DP)
+      VF(LatentKeysArgs, RP) VF(LatentKeysArgs, VP) VF(LatentKeysArgs, keys) VF(LatentKeysArgs, scale);
+  m.def("latent_prefill", [](const LatentKeysArgs& a, u64 tiles, int ntiles, u64 st) {
+    return dnn_latent_prefill(&a, CIP(tiles), ntiles, ST(st));
   });
   m.def("latent_attn_f32", [](const LatentAttnArgs& a, u64 st) { return dnn_latent_attn_f32(&a, ST(st)); });
   py::class_<GatedNormArgs>(m, "GatedNormArgs")

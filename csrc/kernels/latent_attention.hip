@@ -2,30 +2,33 @@
 //
 // The cache holds one row per token for all heads, [page][64][CP + RP]: a normed
 // latent of CP columns and a rotated key part of RP.  A head's unrotated key and
-// its value are linear in the latent, so the key projection is moved to the
-// query (q . W_uk c = (W_uk^T q) . c) and the value projection behind the
-// softmax: every head scores whole cache rows and sums their latents.
+// its value are linear in the latent.  Two ways to score:
+//   over latents   the key projection is moved to the query (q . W_uk c =
+//                  (W_uk^T q) . c) and the value projection behind the softmax:
+//                  every head reads whole cache rows and sums their latents.
+//                  Single tokens, short portions
+//   over keys      the sequence's cache rows are gathered and projected to the
+//                  heads' keys and values first: fewer operations per score
+//                  where many queries share them.  Long portions
 //
 //   latent_prep      norms of the query's and the cache's latent, rotation of the
 //                    shared key part, cache write
 //   rope_rows        rotation of every head's rotated part, in place
-//   latent_attn      bf16; a workgroup takes 64 packed (token, head) rows and
-//                    walks the pages: its 4 waves take a quarter each of the
-//                    64 x 64 scores, then a quarter each of the latent columns.
-//                    Portions of prompts, and single tokens (over `splits`
-//                    workgroups, then a combine)
+//   latent_attn      bf16, over latents; a workgroup takes 32 or 64 packed (token,
+//                    head) rows and walks the pages.  Its 8 waves take a part each
+//                    of keys, rows and columns of the scores, then a part of the
+//                    latent columns.  Single tokens may be split over workgroups
+//                    (then a combine)
+//   latent_gather    cache pages -> rows
+//   latent_prefill   bf16, over keys; a workgroup takes 128 tokens of a head
 //   latent_attn_f32  fp32, one wave per (row, head): the exact mode
 //
 // Scores, softmax and accumulation are fp32.
-#include "common.h"
+#include "attention_tile.h"
 #include "residual_api.h"
 #include "vec16.h"
 
 namespace dnn {
-
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-constexpr int PG = 64;  // keys per page
-constexpr float LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ int la_page(const int* table, int ldt, int npages, int slot, int blk) {
   if (blk < 0 || blk >= ldt) return -1;
@@ -121,12 +124,20 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
   }
 }
 
-// ---------------------------------------------------------------- MFMA attention
-template <int CP, int RP>
-struct LaLds {
-  static constexpr int DK = CP + RP;
+// ---------------------------------------------------------------- over latents
+// ROWS packed rows and 64 keys of a page, 8 waves.  Scores: wave (kh, rh, kq) of
+// 2 key halves x RH row halves x KQ parts of the columns; the parts are summed
+// through LDS, where each wave of a group ends with EN of the 16 keys of a lane.
+template <int CP, int RP, int ROWS>
+struct LaTile {
+  static constexpr int DK = CP + RP, RH = ROWS / 32, KQ = 4 / RH, EN = 16 / KQ;
   static constexpr int RS = (DK * 2 + 255) / 256 * 256;  // bytes of a key row: whole groups of 16 pieces
-  static constexpr int K = PG * RS, P = 8 * 1024, TOTAL = K + P + 2 * 2 * 32 * 4;
+  static constexpr int NK = DK / 16 / KQ;                // MFMA steps of a wave's part
+  static constexpr int NI = PG * (DK / 8) / 512;         // 16-byte pieces of a page per thread
+  static constexpr int NC = CP >= 256 ? CP / 256 : 1;    // 32-column groups of the latent per wave
+  static constexpr int O_X = PG * RS, O_P = O_X + 8 * 4 * 1024, O_R = O_P + RH * 4 * 1024;
+  static constexpr int TOTAL = O_R + 8 * 32 * 4;
+  static_assert(DK % (16 * KQ) == 0 && PG * (DK / 8) % 512 == 0, "tile");
 };
 // Byte of 16-B piece c of key r; swizzled within groups of 16 pieces so that a
 // fragment read (one piece of 16 rows) and a transposing read (4 pieces of 4
@@ -150,114 +161,149 @@ __device__ __forceinline__ float la_gate(const LatentAttnArgs& a, int row, int h
   return 1.0f / (1.0f + __expf(-bf2f(reinterpret_cast<const bf16_t*>(a.gate)[(size_t)row * a.ldg + head])));
 }
 
+constexpr int LA_WS = 4;  // floats of a partial before its columns: {max, sum, -, -}
+
 // grid (tiles, splits); tiles: {first batch row, tokens, slot, first packed row}.
 // With splits the tiles are single tokens, per_token tiles each, and
-// ws = [token][H][splits][CP + 2] takes {max, sum, O} partials.
-template <int CP, int RP>
-__global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a, const int4* __restrict__ tiles,
+// ws = [token][H][splits][LA_WS + CP] takes the partials.
+template <int CP, int RP, int ROWS>
+__global__ __launch_bounds__(512, 1) void latent_attn_kernel(LatentAttnArgs a, const int4* __restrict__ tiles,
                                                              int per_token, float* __restrict__ ws) {
-  using L = LaLds<CP, RP>;
-  constexpr int DK = L::DK, RS = L::RS, NKS = DK / 16, CK = DK / 8, NI = PG * CK / 256, NC = CP / 128;
+  using L = LaTile<CP, RP, ROWS>;
+  constexpr int DK = L::DK, RS = L::RS, CK = DK / 8, RH = L::RH, KQ = L::KQ, EN = L::EN, NK = L::NK, NI = L::NI, NC = L::NC;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* ks = smem;
-  char* ps = smem + L::K;
-  float* red = reinterpret_cast<float*>(ps + L::P);  // [row half][key half][32]
+  char* xs = smem + L::O_X;
+  char* ps = smem + L::O_P;
+  float* red = reinterpret_cast<float*>(smem + L::O_R);  // [wave][32]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = lane >> 5, r32 = lane & 31;
-  const int rh = wave >> 1, kh = wave & 1, ns = gridDim.y;
+  const int kh = wave & 1, rh = (wave >> 1) & (RH - 1), kq = wave / (2 * RH), ns = gridDim.y;
   const int4 t = tiles[blockIdx.x];
   const int tok0 = t.x, n = t.y, slot = t.z, row0 = t.w, last = n - 1;
   const int p0 = a.pos[tok0];
   const int row = row0 + rh * 32 + r32, tk = min(row / a.H, last), head = row % a.H, q_abs = p0 + tk;
   const int q_min = p0 + min((row0 + rh * 32) / a.H, last);
-  const int total = (p0 + min((row0 + 63) / a.H, last)) / PG + 1;
+  const int total = (p0 + min((row0 + ROWS - 1) / a.H, last)) / PG + 1;
   const int ub = (int)((long)total * blockIdx.y / ns), ue = (int)((long)total * (blockIdx.y + 1) / ns);
-
-  bf16x8 qf[NKS];
-  {
-    const bf16_t* ql = reinterpret_cast<const bf16_t*>(a.qlat) + (size_t)(tok0 + tk) * a.ldql + head * CP + 8 * h;
-    const bf16_t* qr = reinterpret_cast<const bf16_t*>(a.qrot) + (size_t)(tok0 + tk) * a.ldqr + head * a.hs + 8 * h;
-#pragma unroll
-    for (int s = 0; s < CP / 16; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(ql + s * 16);
-#pragma unroll
-    for (int s = 0; s < RP / 16; ++s) qf[CP / 16 + s] = *reinterpret_cast<const bf16x8*>(qr + s * 16);
-  }
-  f32x16 o[2][NC];
-#pragma unroll
-  for (int i = 0; i < 2; ++i)
-#pragma unroll
-    for (int j = 0; j < NC; ++j) o[i][j] = f32x16{};
-  float m0 = -INFINITY, m1 = -INFINITY, l_i = 0.f;
-  const float sc = a.scale * LOG2E;
 
   i32x4 pk[NI];
   auto fetch = [&](int i) __attribute__((always_inline)) {
     const int page = max(la_page(a.table, a.ldt, a.npages, slot, i), 0);  // a missing page is never visible; stay in the pool
     const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kp) + (size_t)page * PG * DK;
 #pragma unroll
-    for (int it = 0; it < NI; ++it) pk[it] = *reinterpret_cast<const i32x4*>(kb + (it * 256 + tid) * 8);
+    for (int it = 0; it < NI; ++it) pk[it] = *reinterpret_cast<const i32x4*>(kb + (it * 512 + tid) * 8);
   };
   if (ub < ue) fetch(ub);
+  bf16x8 qf[NK];
+  {
+    const bf16_t* ql = reinterpret_cast<const bf16_t*>(a.qlat) + (size_t)(tok0 + tk) * a.ldql + head * CP + 8 * h;
+    const bf16_t* qr = reinterpret_cast<const bf16_t*>(a.qrot) + (size_t)(tok0 + tk) * a.ldqr + head * a.hs + 8 * h;
+#pragma unroll
+    for (int s = 0; s < NK; ++s) {
+      const int k = kq * NK + s;
+      qf[s] = *reinterpret_cast<const bf16x8*>(k < CP / 16 ? ql + k * 16 : qr + (k - CP / 16) * 16);
+    }
+  }
+  f32x16 o[RH][NC];
+  float m[RH], l_i = 0.f;
+#pragma unroll
+  for (int i = 0; i < RH; ++i) {
+    m[i] = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < NC; ++j) o[i][j] = f32x16{};
+  }
+  const float sc = a.scale * LOG2E;
+  const bool has_cols = wave * NC * 32 < CP;
+
   for (int i = ub; i < ue; ++i) {
-    const int kb0 = i * PG + kh * 32;
     __syncthreads();  // the last page is read
 #pragma unroll
     for (int it = 0; it < NI; ++it) {
-      const int x = it * 256 + tid;
+      const int x = it * 512 + tid;
       *reinterpret_cast<i32x4*>(ks + la_at<RS>(x / CK, x % CK)) = pk[it];
     }
     __syncthreads();
     if (i + 1 < ue) fetch(i + 1);
-    f32x16 s = f32x16{};
+    {
+      f32x16 s = f32x16{};
 #pragma unroll
-    for (int k = 0; k < NKS; ++k)
-      s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(ks + la_at<RS>(kh * 32 + r32, 2 * k + h)),
-                                                 qf[k], s, 0, 0, 0);
-    if (kb0 + 31 > q_min) {
+      for (int k = 0; k < NK; ++k)
+        s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
+            *reinterpret_cast<const bf16x8*>(ks + la_at<RS>(kh * 32 + r32, 2 * (kq * NK + k) + h)), qf[k], s, 0, 0, 0);
 #pragma unroll
-      for (int e = 0; e < 16; ++e)
-        if (kb0 + (e & 3) + 8 * (e >> 2) + 4 * h > q_abs) s[e] = -INFINITY;
+      for (int q = 0; q < 4; ++q)
+        *reinterpret_cast<f32x4*>(xs + (wave * 4 + q) * 1024 + lane * 16) = f32x4{s[4 * q], s[4 * q + 1], s[4 * q + 2], s[4 * q + 3]};
+    }
+    __syncthreads();
+    float s[EN];
+#pragma unroll
+    for (int q = 0; q < EN / 4; ++q) {
+      f32x4 z = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int w = 0; w < KQ; ++w)
+        z += *reinterpret_cast<const f32x4*>(xs + ((w * 2 * RH + rh * 2 + kh) * 4 + kq * (EN / 4) + q) * 1024 + lane * 16);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) s[4 * q + j] = z[j];
+    }
+    const int kb0 = i * PG + kh * 32 + kq * (EN / 4) * 8 + 4 * h;  // key of s[0]; s[4 q + j]: + 8 q + j
+    if (i * PG + kh * 32 + 31 > q_min) {
+#pragma unroll
+      for (int e = 0; e < EN; ++e)
+        if (kb0 + 8 * (e >> 2) + (e & 3) > q_abs) s[e] = -INFINITY;
     }
     float mx = -INFINITY;
 #pragma unroll
-    for (int e = 0; e < 16; ++e) mx = fmaxf(mx, s[e]);
+    for (int e = 0; e < EN; ++e) mx = fmaxf(mx, s[e]);
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     if (h == 0) red[wave * 32 + r32] = mx;
     __syncthreads();
-    const float n0 = fmaxf(m0, fmaxf(red[r32], red[32 + r32]) * sc), n1 = fmaxf(m1, fmaxf(red[64 + r32], red[96 + r32]) * sc);
-    const float u0 = n0 == -INFINITY ? 0.f : n0, u1 = n1 == -INFINITY ? 0.f : n1;
-    const float a0 = __builtin_amdgcn_exp2f(m0 - u0), a1 = __builtin_amdgcn_exp2f(m1 - u1);
-    m0 = n0, m1 = n1;
-    const float mu = rh == 0 ? u0 : u1;
+    float al[RH], mu = 0.f, mine = 1.f;
+    bool same = true;
+#pragma unroll
+    for (int x = 0; x < RH; ++x) {
+      float v = -INFINITY;
+#pragma unroll
+      for (int w = 0; w < KQ; ++w)
+        v = fmaxf(v, fmaxf(red[((w * RH + x) * 2) * 32 + r32], red[((w * RH + x) * 2 + 1) * 32 + r32]));
+      const float nx = fmaxf(m[x], v * sc), u = nx == -INFINITY ? 0.f : nx;
+      al[x] = __builtin_amdgcn_exp2f(m[x] - u);
+      m[x] = nx;
+      same = same && al[x] == 1.f;
+      if (x == rh) mu = u, mine = al[x];
+    }
     float rs = 0.f;
 #pragma unroll
-    for (int e = 0; e < 16; ++e) {
+    for (int e = 0; e < EN; ++e) {
       s[e] = __builtin_amdgcn_exp2f(fmaf(s[e], sc, -mu));
       rs += s[e];
     }
     rs += __shfl_xor(rs, 32, 64);
-    l_i = fmaf(l_i, rh == 0 ? a0 : a1, rs);
-#pragma unroll
-    for (int x = 0; x < 2; ++x)
-      *reinterpret_cast<uint4*>(ps + (wave * 2 + x) * 1024 + lane * 16) =
-          make_uint4(pack2bf(s[8 * x], s[8 * x + 1]), pack2bf(s[8 * x + 2], s[8 * x + 3]), pack2bf(s[8 * x + 4], s[8 * x + 5]),
-                     pack2bf(s[8 * x + 6], s[8 * x + 7]));
+    l_i = fmaf(l_i, mine, rs);
+    {  // fragment of 16 keys: this lane's 8, of which a wave has EN
+      char* d = ps + ((rh * 4 + kh * 2 + kq * EN / 8) * 64 + lane) * 16;
+      if constexpr (EN == 8)
+        *reinterpret_cast<uint4*>(d) = make_uint4(pack2bf(s[0], s[1]), pack2bf(s[2], s[3]), pack2bf(s[4], s[5]), pack2bf(s[6], s[7]));
+      else
+        *reinterpret_cast<uint2*>(d + (kq & 1) * 8) = make_uint2(pack2bf(s[0], s[1]), pack2bf(s[2], s[3]));
+    }
     __syncthreads();
-    if (!__all(a0 == 1.f && a1 == 1.f)) {
+    if (!has_cols) continue;
+    if (!__all(same)) {
 #pragma unroll
-      for (int j = 0; j < NC; ++j) {
-        o[0][j] *= a0;
-        o[1][j] *= a1;
-      }
+      for (int x = 0; x < RH; ++x)
+#pragma unroll
+        for (int j = 0; j < NC; ++j) o[x][j] *= al[x];
     }
 #pragma unroll
     for (int x = 0; x < 4; ++x) {  // 16 keys each
-      const bf16x8 f0 = *reinterpret_cast<const bf16x8*>(ps + x * 1024 + lane * 16);
-      const bf16x8 f1 = *reinterpret_cast<const bf16x8*>(ps + (4 + x) * 1024 + lane * 16);
+      bf16x8 f[RH];
+#pragma unroll
+      for (int r = 0; r < RH; ++r) f[r] = *reinterpret_cast<const bf16x8*>(ps + ((r * 4 + x) * 64 + lane) * 16);
 #pragma unroll
       for (int j = 0; j < NC; ++j) {
         const bf16x8 vf = la_tr<RS>(ks, x, (wave * NC + j) * 32, lane);
-        o[0][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, f0, o[0][j], 0, 0, 0);
-        o[1][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, f1, o[1][j], 0, 0, 0);
+#pragma unroll
+        for (int r = 0; r < RH; ++r) o[r][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, f[r], o[r][j], 0, 0, 0);
       }
     }
   }
@@ -265,25 +311,29 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentAttnArgs a, c
   if (h == 0) red[wave * 32 + r32] = l_i;
   __syncthreads();
 #pragma unroll
-  for (int x = 0; x < 2; ++x) {
+  for (int x = 0; x < RH; ++x) {
     const int rw = row0 + x * 32 + r32;
-    if (rw >= n * a.H) continue;
-    const int tok = tok0 + rw / a.H, hd = rw % a.H;
-    const float l = red[x * 64 + r32] + red[x * 64 + 32 + r32];
+    if (!has_cols || rw >= n * a.H) continue;
+    const int tok = tok0 + rw / a.H, hd = rw % a.H, c0 = wave * NC * 32 + 4 * h;
+    float l = 0.f;
+#pragma unroll
+    for (int w = 0; w < KQ; ++w) l += red[((w * RH + x) * 2) * 32 + r32] + red[((w * RH + x) * 2 + 1) * 32 + r32];
     if (ns > 1) {
-      float* d = ws + (((size_t)(blockIdx.x / per_token) * a.H + hd) * ns + blockIdx.y) * (CP + 2);
+      float* d = ws + (((size_t)(blockIdx.x / per_token) * a.H + hd) * ns + blockIdx.y) * (LA_WS + CP);
       if (wave == 0 && h == 0) {
-        d[0] = x == 0 ? m0 : m1;
+        d[0] = m[x];
         d[1] = l;
       }
 #pragma unroll
       for (int j = 0; j < NC; ++j)
 #pragma unroll
-        for (int e = 0; e < 16; ++e) d[2 + (wave * NC + j) * 32 + (e & 3) + 8 * (e >> 2) + 4 * h] = o[x][j][e];
+        for (int q = 0; q < 4; ++q)
+          *reinterpret_cast<f32x4*>(d + LA_WS + c0 + j * 32 + 8 * q) =
+              f32x4{o[x][j][4 * q], o[x][j][4 * q + 1], o[x][j][4 * q + 2], o[x][j][4 * q + 3]};
       continue;
     }
     const float f = (l > 0.f ? 1.f / l : 0.f) * la_gate(a, tok, hd);
-    bf16_t* op = reinterpret_cast<bf16_t*>(a.out) + (size_t)tok * a.ldo + hd * CP + wave * NC * 32 + 4 * h;
+    bf16_t* op = reinterpret_cast<bf16_t*>(a.out) + (size_t)tok * a.ldo + hd * CP + c0;
 #pragma unroll
     for (int j = 0; j < NC; ++j)
 #pragma unroll
@@ -298,18 +348,18 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a, c
                                                              int ns, const float* __restrict__ ws) {
   __shared__ float acc[4][130];
   const int e = blockIdx.x / a.H, head = blockIdx.x % a.H, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int row = tiles[(size_t)e * per_token].x, c0 = blockIdx.y * 128;
-  const float* d = ws + ((size_t)e * a.H + head) * ns * (a.CP + 2);
+  const int row = tiles[(size_t)e * per_token].x, c0 = blockIdx.y * 128, st = LA_WS + a.CP;
+  const float* d = ws + ((size_t)e * a.H + head) * ns * st;
   float m = -INFINITY;
-  for (int s = lane; s < ns; s += 64) m = fmaxf(m, d[(size_t)s * (a.CP + 2)]);
+  for (int s = lane; s < ns; s += 64) m = fmaxf(m, d[(size_t)s * st]);
   m = wave_max(m);
   float l = 0.f, v[2] = {0.f, 0.f};
   for (int s = wave; s < ns; s += 4) {
-    const float* q = d + (size_t)s * (a.CP + 2);
+    const float* q = d + (size_t)s * st;
     const float f = q[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(q[0] - m);
     l = fmaf(q[1], f, l);
-    v[0] = fmaf(q[2 + c0 + lane], f, v[0]);
-    v[1] = fmaf(q[2 + c0 + 64 + lane], f, v[1]);
+    v[0] = fmaf(q[LA_WS + c0 + lane], f, v[0]);
+    v[1] = fmaf(q[LA_WS + c0 + 64 + lane], f, v[1]);
   }
   acc[wave][lane] = v[0];
   acc[wave][64 + lane] = v[1];
@@ -321,6 +371,130 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a, c
   const float o = acc[0][c] + acc[1][c] + acc[2][c] + acc[3][c];
   reinterpret_cast<bf16_t*>(a.out)[(size_t)row * a.ldo + head * a.CP + c0 + c] =
       f2bf((l > 0.f ? o / l : 0.f) * la_gate(a, row, head));
+}
+
+// ---------------------------------------------------------------- over keys
+// grid (pages, 4): 16 rows each; ent: {first row of the 64, slot, block, -}
+__global__ __launch_bounds__(256) void latent_gather_kernel(const uint4* __restrict__ kp, const int* __restrict__ table, int ldt,
+                                                            int npages, const int4* __restrict__ ent, int rows, int pieces,
+                                                            uint4* __restrict__ out) {
+  const int4 e = ent[blockIdx.x];
+  const int page = la_page(table, ldt, npages, e.y, e.z);
+  const int n = min(PG, rows - e.x) * pieces, part = PG / 4 * pieces;
+  const uint4* src = kp + (size_t)max(page, 0) * PG * pieces;
+  uint4* dst = out + (size_t)e.x * pieces;
+  for (int i = blockIdx.y * part + threadIdx.x; i < min(n, (int)(blockIdx.y + 1) * part); i += 256) dst[i] = page >= 0 ? src[i] : make_uint4(0, 0, 0, 0);
+}
+
+template <int DP, int RP, int VP>
+struct LpTile {
+  static constexpr int D = DP + RP, RS = (D * 2 + 255) / 256 * 256, O_V = PG * RS, TOTAL = O_V + PG * PaV<VP>::STRIDE;
+};
+
+// grid (H, tiles); tiles: {first batch row, tokens, first key row, first token}
+template <int DP, int RP, int VP>
+__global__ __launch_bounds__(256, DP + RP + VP > 320 ? 1 : 2) void latent_prefill_kernel(LatentKeysArgs a, const int4* __restrict__ tiles) {
+  using L = LpTile<DP, RP, VP>;
+  constexpr int D = L::D, RS = L::RS, NKS = D / 16, NDT = VP / 32;
+  constexpr int CU = DP / 8, CR = RP / 8, CV = VP / 8, NU = PG * CU / 256, NR = PG * CR / 256, NV = PG * CV / 256;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  char* ks = smem;
+  char* vs = smem + L::O_V;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = lane >> 5, r32 = lane & 31, head = blockIdx.x;
+  const int4 t = tiles[blockIdx.y];
+  const int tok0 = t.x, n = t.y, key0 = t.z, last = n - 1;
+  const int p0 = a.pos[tok0], w0 = t.w + wave * 32, tk = min(w0 + r32, last), q_abs = p0 + tk;
+  const int q_min = p0 + min(w0, last), q_max = p0 + min(w0 + 31, last);
+  const int total = (p0 + min(t.w + 127, last)) / PG + 1;
+  bf16x8 qf[NKS];
+  {
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.q) + (size_t)(tok0 + tk) * a.ldq + head * D + 8 * h;
+#pragma unroll
+    for (int s = 0; s < NKS; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(qp + s * 16);
+  }
+  f32x16 o[NDT];
+#pragma unroll
+  for (int i = 0; i < NDT; ++i) o[i] = f32x16{};
+  float m_i = -INFINITY, l_i = 0.f;
+  const float sc = a.scale * LOG2E;
+  const bf16_t* kv = reinterpret_cast<const bf16_t*>(a.kv) + head * (DP + VP);
+  const bf16_t* kr = reinterpret_cast<const bf16_t*>(a.krot);
+  i32x4 pu[NU], pr[NR], pv[NV];
+  auto fetch = [&](int i) __attribute__((always_inline)) {
+    const int k0 = key0 + i * PG;
+#pragma unroll
+    for (int it = 0; it < NU; ++it) {
+      const int x = it * 256 + tid;
+      pu[it] = *reinterpret_cast<const i32x4*>(kv + (size_t)min(k0 + x / CU, a.keys - 1) * a.ldkv + x % CU * 8);
+    }
+#pragma unroll
+    for (int it = 0; it < NR; ++it) {
+      const int x = it * 256 + tid;
+      pr[it] = *reinterpret_cast<const i32x4*>(kr + (size_t)min(k0 + x / CR, a.keys - 1) * a.ldr + x % CR * 8);
+    }
+#pragma unroll
+    for (int it = 0; it < NV; ++it) {
+      const int x = it * 256 + tid;
+      pv[it] = *reinterpret_cast<const i32x4*>(kv + (size_t)min(k0 + x / CV, a.keys - 1) * a.ldkv + DP + x % CV * 8);
+    }
+  };
+  fetch(0);
+  for (int i = 0; i < total; ++i) {
+    const int kb0 = i * PG;
+    __syncthreads();
+#pragma unroll
+    for (int it = 0; it < NU; ++it) {
+      const int x = it * 256 + tid;
+      *reinterpret_cast<i32x4*>(ks + la_at<RS>(x / CU, x % CU)) = pu[it];
+    }
+#pragma unroll
+    for (int it = 0; it < NR; ++it) {
+      const int x = it * 256 + tid;
+      *reinterpret_cast<i32x4*>(ks + la_at<RS>(x / CR, CU + x % CR)) = pr[it];
+    }
+#pragma unroll
+    for (int it = 0; it < NV; ++it) {
+      const int x = it * 256 + tid;
+      *reinterpret_cast<i32x4*>(vs + x / CV * PaV<VP>::STRIDE + x % CV * 16) = pv[it];
+    }
+    __syncthreads();
+    if (i + 1 < total) fetch(i + 1);
+    if (kb0 > q_max) continue;
+    f32x16 s[2];
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) {
+      s[kt] = f32x16{};
+#pragma unroll
+      for (int k = 0; k < NKS; ++k)
+        s[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
+            *reinterpret_cast<const bf16x8*>(ks + la_at<RS>(kt * 32 + r32, 2 * k + h)), qf[k], s[kt], 0, 0, 0);
+    }
+    if (kb0 + PG - 1 > q_min) {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+          if (kb0 + kt * 32 + (e & 3) + 8 * (e >> 2) + 4 * h > q_abs) s[kt][e] = -INFINITY;
+    }
+    const float alpha = pa_softmax<2>(s, sc, m_i, l_i);
+    if (!__all(alpha == 1.f)) {
+#pragma unroll
+      for (int d = 0; d < NDT; ++d) o[d] *= alpha;
+    }
+    pa_pv<VP>(vs, s[0], o, lane);
+    pa_pv<VP>(vs + 32 * PaV<VP>::STRIDE, s[1], o, lane);
+  }
+  if (w0 + r32 >= n) return;
+  float f = l_i > 0.f ? 1.f / l_i : 0.f;
+  if (a.gate != nullptr)
+    f /= 1.0f + __expf(-bf2f(reinterpret_cast<const bf16_t*>(a.gate)[(size_t)(tok0 + tk) * a.ldg + head]));
+  bf16_t* op = reinterpret_cast<bf16_t*>(a.out) + (size_t)(tok0 + tk) * a.ldo + head * VP + 4 * h;
+#pragma unroll
+  for (int d = 0; d < NDT; ++d)
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      *reinterpret_cast<uint2*>(op + d * 32 + 8 * q) =
+          make_uint2(pack2bf(o[d][4 * q] * f, o[d][4 * q + 1] * f), pack2bf(o[d][4 * q + 2] * f, o[d][4 * q + 3] * f));
 }
 
 // ---------------------------------------------------------------- fp32
@@ -413,30 +587,72 @@ static bool la_ok(const LatentAttnArgs& a, int e) {
          a.table != nullptr && a.slots != nullptr && a.pos != nullptr;
 }
 
-extern "C" int dnn_latent_attn(const LatentAttnArgs* a, const int* tiles, int ntiles, int splits, int per_token, float* ws,
-                               long long ws_elems, hipStream_t st) {
-  if (!la_ok(*a, 8) || ntiles <= 0 || splits < 1 || splits > 256 || per_token < 1 || ntiles % per_token != 0 ||
-      ((uintptr_t)tiles & 15) != 0)
+extern "C" int dnn_latent_attn(const LatentAttnArgs* a, const int* tiles, int ntiles, int rows, int splits, int per_token,
+                               float* ws, long long ws_elems, hipStream_t st) {
+  if (!la_ok(*a, 8) || ntiles <= 0 || (rows != 32 && rows != 64) || splits < 1 || splits > 256 || per_token < 1 ||
+      ntiles % per_token != 0 || ((uintptr_t)tiles & 15) != 0)
     return -1;
   const int tokens = ntiles / per_token;
-  if (splits > 1 && (ws == nullptr || per_token != (a->H + 63) / 64 || (long)tokens * a->H > 0x7fffffff ||
-                     ws_elems < (long long)tokens * a->H * splits * (a->CP + 2)))
+  if (splits > 1 && (ws == nullptr || ((uintptr_t)ws & 15) != 0 || per_token != (a->H + rows - 1) / rows ||
+                     (long)tokens * a->H > 0x7fffffff || ws_elems < (long long)tokens * a->H * splits * (LA_WS + a->CP)))
     return -1;
   const dim3 grid(ntiles, splits);
-#define LA(C, R) hipLaunchKernelGGL((latent_attn_kernel<C, R>), grid, dim3(256), (LaLds<C, R>::TOTAL), st, *a, (const int4*)tiles, per_token, ws)
-  if (a->RP == 64) {
-    if (a->CP == 128) LA(128, 64);
-    else if (a->CP == 256) LA(256, 64);
-    else LA(512, 64);
-  } else {
-    if (a->CP == 128) LA(128, 128);
-    else if (a->CP == 256) LA(256, 128);
-    else LA(512, 128);
+#define LA(C, R, N)                                                                                                           \
+  hipLaunchKernelGGL((latent_attn_kernel<C, R, N>), grid, dim3(512), (LaTile<C, R, N>::TOTAL), st, *a, (const int4*)tiles, \
+                     per_token, ws)
+#define LAR(C, R)             \
+  {                           \
+    if (rows == 32) LA(C, R, 32); \
+    else LA(C, R, 64);        \
   }
+  if (a->RP == 64) {
+    if (a->CP == 128) LAR(128, 64)
+    else if (a->CP == 256) LAR(256, 64)
+    else LAR(512, 64)
+  } else {
+    if (a->CP == 128) LAR(128, 128)
+    else if (a->CP == 256) LAR(256, 128)
+    else LAR(512, 128)
+  }
+#undef LAR
 #undef LA
   if (splits > 1)
     hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)(tokens * a->H), a->CP / 128), dim3(256), 0, st, *a,
                        (const int4*)tiles, per_token, splits, ws);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_latent_gather(const void* kp, int cols, const int* table, int ldt, int npages, const int* ent, int nent,
+                                 void* out, int rows, hipStream_t st) {
+  if (cols <= 0 || cols % 8 != 0 || ldt <= 0 || npages <= 0 || nent <= 0 || rows <= 0 ||
+      (((uintptr_t)kp | (uintptr_t)out | (uintptr_t)ent) & 15) != 0)
+    return -1;
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(nent, 4), dim3(256), 0, st, (const uint4*)kp, table, ldt, npages, (const int4*)ent,
+                     rows, cols / 8, (uint4*)out);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dnn_latent_prefill(const LatentKeysArgs* a, const int* tiles, int ntiles, hipStream_t st) {
+  const int D = a->DP + a->RP;
+  if (a->M <= 0 || a->H <= 0 || a->keys <= 0 || ntiles <= 0 || ntiles > 65535 || (a->DP != 64 && a->DP != 128) ||
+      (a->RP != 64 && a->RP != 128) || (a->VP != 64 && a->VP != 128) || (a->ldq | a->ldkv | a->ldr) % 8 != 0 ||
+      a->ldq < a->H * D || a->ldkv < a->H * (a->DP + a->VP) || a->ldr < a->RP || a->ldo % 4 != 0 || a->ldo < a->H * a->VP ||
+      (a->gate != nullptr && a->ldg < a->H) || !(a->scale > 0.f) || a->pos == nullptr ||
+      (((uintptr_t)a->q | (uintptr_t)a->kv | (uintptr_t)a->krot | (uintptr_t)a->out | (uintptr_t)tiles) & 15) != 0)
+    return -1;
+#define LP(X, R, V)                                                                                                       \
+  if (a->DP == X && a->RP == R && a->VP == V)                                                                             \
+  hipLaunchKernelGGL((latent_prefill_kernel<X, R, V>), dim3(a->H, ntiles), dim3(256), (LpTile<X, R, V>::TOTAL), st, *a, \
+                     (const int4*)tiles)
+  LP(64, 64, 64);
+  LP(64, 64, 128);
+  LP(64, 128, 64);
+  LP(64, 128, 128);
+  LP(128, 64, 64);
+  LP(128, 64, 128);
+  LP(128, 128, 64);
+  LP(128, 128, 128);
+#undef LP
   return (int)hipGetLastError();
 }
 

@@ -19,10 +19,9 @@ namespace dnn {
 
 // One row by half a wave: lane l of 32 holds the logits of experts l, l + 32,
 // ...; both halves call it together, a half past the rows with live = false.
-// f(t, expert) for every choice.
-template <typename F>
+// f(t, expert) for every choice.  NR: experts a lane holds at most.
+template <int NR, typename F>
 __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, int l, int half, F f) {
-  constexpr int NR = EXPERTS_MAX / 32;
   const int nr = (a.E + 31) / 32;  // registers that hold experts
   float s[NR], w[NR];  // choice scores, scores
   float mx = -INFINITY;
@@ -145,6 +144,7 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int m, bool live, 
 
 constexpr int RT_ROWS = 16;  // rows of a workgroup of 4 waves
 
+template <int NR>
 __global__ __launch_bounds__(256) void route_kernel(RouteArgs a) {
   __shared__ int hist[EXPERTS_MAX], base[EXPERTS_MAX];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m0 = blockIdx.x * RT_ROWS;
@@ -152,7 +152,7 @@ __global__ __launch_bounds__(256) void route_kernel(RouteArgs a) {
   __syncthreads();
   for (int r = wave * 2; r < RT_ROWS; r += 8) {
     const int half = lane >> 5, l = lane & 31, m = m0 + r + half;
-    route_row(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
+    route_row<NR>(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
       if (l == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
     });
   }
@@ -207,6 +207,7 @@ __global__ __launch_bounds__(256) void place_kernel(RouteArgs a) {
 
 constexpr int RT_SMALL = 64;  // rows of the one-workgroup launch
 
+template <int NR>
 __global__ __launch_bounds__(1024) void route_small_kernel(RouteArgs a) {
   __shared__ int hist[EXPERTS_MAX], offs[EXPERTS_MAX + 1];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -214,7 +215,7 @@ __global__ __launch_bounds__(1024) void route_small_kernel(RouteArgs a) {
   __syncthreads();
   for (int m0 = wave * 2; m0 < a.M; m0 += 32) {
     const int half = lane >> 5, l = lane & 31, m = m0 + half;
-    route_row(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
+    route_row<NR>(a, m, m < a.M, l, half, [&](int t, int e) __attribute__((always_inline)) {
       if (l == 0) a.rank[(size_t)m * a.top + t] = atomicAdd(&hist[e], 1);
     });
   }
@@ -313,10 +314,16 @@ extern "C" int dnn_route(const RouteArgs* a, hipStream_t st) {
       a->keep < 1 || a->keep > a->groups || a->top < 1 || a->top > 64 || a->top > a->E / a->groups * a->keep || a->group_top < 1 || a->group_top > 2 ||
       a->M > (1 << 30) / a->top)
     return -1;
-  if (a->M <= RT_SMALL) {
-    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, st, *a);
-  } else {
-    hipLaunchKernelGGL(route_kernel, dim3((a->M + RT_ROWS - 1) / RT_ROWS), dim3(256), 0, st, *a);
+#define ROUTE(N)                                                                                                       \
+  {                                                                                                                    \
+    if (a->M <= RT_SMALL) hipLaunchKernelGGL(route_small_kernel<N>, dim3(1), dim3(1024), 0, st, *a);                   \
+    else hipLaunchKernelGGL(route_kernel<N>, dim3((a->M + RT_ROWS - 1) / RT_ROWS), dim3(256), 0, st, *a);              \
+  }
+  if (a->E <= 32) ROUTE(1)
+  else if (a->E <= 64) ROUTE(2)
+  else ROUTE(EXPERTS_MAX / 32)
+#undef ROUTE
+  if (a->M > RT_SMALL) {
     hipLaunchKernelGGL(place_kernel, dim3((a->M * a->top + 255) / 256), dim3(256), 0, st, *a);
   }
   return (int)hipGetLastError();
@@ -335,8 +342,9 @@ static int grouped_launch(const GroupedArgs& a, const GroupedRows& g, hipStream_
                        (const uint8_t*)a.Wsh, C, a.ldc, a.N, a.K, g);                                               \
     return (int)hipGetLastError();                                                                                  \
   }
-  if (avg <= 12) SKINNY(1, 1)
-  if (avg <= 28) SKINNY(2, 2)
+  const bool even = a.offs == nullptr;  // every expert has avg rows
+  if (avg <= (even ? 16 : 12)) SKINNY(1, 1)
+  if (avg <= (even ? 32 : 28)) SKINNY(2, 2)
   if (avg <= 64) SKINNY(4, 2)
 #undef SKINNY
   const long n = (long)group_tiles_max(a.rows, BG_M, a.E) * ((a.N + BG_N - 1) / BG_N);

@@ -82,6 +82,7 @@ extern "C" int dnn_poly_norm(const PolyNormArgs* a, int f32, hipStream_t st) {
     if (np <= 256) hipLaunchKernelGGL((poly_norm_kernel<T, 1>), dim3(a->M), dim3(256), 0, st, *a);  \
     else if (np <= 512) hipLaunchKernelGGL((poly_norm_kernel<T, 2>), dim3(a->M), dim3(256), 0, st, *a); \
     else if (np <= 2048) hipLaunchKernelGGL((poly_norm_kernel<T, 8>), dim3(a->M), dim3(256), 0, st, *a); \
+    else if (np <= 3072) hipLaunchKernelGGL((poly_norm_kernel<T, 12>), dim3(a->M), dim3(256), 0, st, *a); \
     else hipLaunchKernelGGL((poly_norm_kernel<T, 0>), dim3(a->M), dim3(256), 0, st, *a);            \
   }
   if (f32) PN(float)

@@ -118,13 +118,29 @@ struct LatentAttnArgs {
   float scale;
 };
 
+// The same attention over keys and values of every head, for portions whose
+// sequences' cache rows were gathered and projected.
+struct LatentKeysArgs {
+  const void* q;       // rows [H][DP + RP], stride ldq
+  const void* kv;      // key rows [H][DP | VP], stride ldkv
+  const void* krot;    // key rows [RP], stride ldr
+  const int* pos;
+  void* out;           // rows [H][VP], stride ldo
+  const void* gate;    // rows [H] of gate logits, stride ldg (nullptr: none)
+  int ldq, ldkv, ldr, ldo, ldg, M, H, DP, RP, VP, keys;
+  float scale;
+};
+
 extern "C" {
 int dnn_poly_norm(const PolyNormArgs* a, int f32, hipStream_t st);
 int dnn_rope_rows(void* x, int ld, int hs, int M, int H, int RP, const int* pos, const RopeTable* r, int f32,
                   hipStream_t st);
 int dnn_latent_prep(const LatentPrepArgs* a, int f32, hipStream_t st);
-int dnn_latent_attn(const LatentAttnArgs* a, const int* tiles, int ntiles, int splits, int per_token, float* ws,
-                    long long ws_elems, hipStream_t st);
+int dnn_latent_attn(const LatentAttnArgs* a, const int* tiles, int ntiles, int rows, int splits, int per_token, float* ws,
+                    long long ws_elems, hipStream_t st);  // rows: packed rows of a tile, 32 or 64
+int dnn_latent_gather(const void* kp, int cols, const int* table, int ldt, int npages, const int* ent, int nent, void* out,
+                      int rows, hipStream_t st);
+int dnn_latent_prefill(const LatentKeysArgs* a, const int* tiles, int ntiles, hipStream_t st);
 int dnn_latent_attn_f32(const LatentAttnArgs* a, hipStream_t st);
 int dnn_rows_update(const RowsArgs* a, int y_f32, int out_f32, hipStream_t st);
 // g = gelu_tanh(x W^T) * table[tok]: bf16, wsh = W in fragment order; _f32: from z = x W^T

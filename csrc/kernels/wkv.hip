@@ -37,37 +37,58 @@ __device__ __forceinline__ bf16x8 wk_frag(const uint2& a, const uint2& b) {
 }
 
 // ---------------------------------------------------------------- decay
-// grid (ceil(N / 256), ceil(M / 64)); a wave takes 16 rows x 256 columns, tanh
-// in two bf16 terms, W2 rows [N][rank] in bf16.
-__global__ __launch_bounds__(256) void decay_kernel(DecayArgs a) {
+// A wave takes 16 rows x `cols` columns, grid (ceil(N / (4 cols)), ceil(M / 16));
+// tanh in two bf16 terms, W2 rows [N][rank] in bf16.  KS: 32-column steps of the
+// rank whose terms stay in registers (0: formed again for every 64 columns).
+__device__ __forceinline__ void decay_terms(const float* tp, bf16x8& hi, bf16x8& lo) {
+  float v[8];
+#pragma unroll
+  for (int j = 0; j < 8; j += 4) {
+    const f32x4 x = *reinterpret_cast<const f32x4*>(tp + j);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      v[j + i] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x[i] * (2.0f * LOG2E)));
+  }
+  uint2 h0, h1, l0, l1;
+  wk_split4(v, h0, l0);
+  wk_split4(v + 4, h1, l1);
+  hi = wk_frag(h0, h1), lo = wk_frag(l0, l1);
+}
+
+template <int KS>
+__global__ __launch_bounds__(256) void decay_kernel(DecayArgs a, int cols) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4;
-  const int m = blockIdx.y * 64 + wave * 16 + (lane & 15);
+  const int m = blockIdx.y * 16 + (lane & 15), first = (blockIdx.x * 4 + wave) * cols;
   const float* tp = a.t + (size_t)min(m, a.M - 1) * a.ldt + 8 * g;
-  const bf16_t* w2 = reinterpret_cast<const bf16_t*>(a.w2);
-  for (int nb = 0; nb < 256; nb += 64) {
-    const int n0 = blockIdx.x * 256 + nb;
-    if (n0 >= a.N) return;
+  const bf16_t* w2 = reinterpret_cast<const bf16_t*>(a.w2) + 8 * g;
+  bf16x8 hi[KS > 0 ? KS : 1], lo[KS > 0 ? KS : 1];
+  if constexpr (KS > 0) {
+#pragma unroll
+    for (int k = 0; k < KS; ++k) decay_terms(tp + k * 32, hi[k], lo[k]);
+  }
+  for (int n0 = first; n0 < min(first + cols, a.N); n0 += 64) {
     f32x4 acc[4];
+    const bf16_t* wr[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < a.rank; k += 32) {
-      float v[8];
-#pragma unroll
-      for (int j = 0; j < 8; j += 4) {
-        const f32x4 x = *reinterpret_cast<const f32x4*>(tp + k + j);
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          v[j + i] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x[i] * (2.0f * LOG2E)));
-      }
-      uint2 h0, h1, l0, l1;
-      wk_split4(v, h0, l0);
-      wk_split4(v + 4, h1, l1);
-      const bf16x8 hi = wk_frag(h0, h1), lo = wk_frag(l0, l1);
+    for (int j = 0; j < 4; ++j) {
+      acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+      wr[j] = w2 + (size_t)min(n0 + j * 16 + (lane & 15), a.N - 1) * a.rank;
+    }
+    auto step = [&](int k, const bf16x8& h, const bf16x8& l) __attribute__((always_inline)) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const bf16x8 w = *reinterpret_cast<const bf16x8*>(w2 + (size_t)min(n0 + j * 16 + (lane & 15), a.N - 1) * a.rank + k + 8 * g);
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, hi, acc[j], 0, 0, 0);
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, lo, acc[j], 0, 0, 0);
+        const bf16x8 w = *reinterpret_cast<const bf16x8*>(wr[j] + k);
+        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, h, acc[j], 0, 0, 0);
+        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, l, acc[j], 0, 0, 0);
+      }
+    };
+    if constexpr (KS > 0) {
+#pragma unroll
+      for (int k = 0; k < KS; ++k) step(k * 32, hi[k], lo[k]);
+    } else {
+      for (int k = 0; k < a.rank; k += 32) {
+        decay_terms(tp + k, hi[0], lo[0]);
+        step(k, hi[0], lo[0]);
       }
     }
     if (m >= a.M) continue;
@@ -177,8 +198,11 @@ __global__ __launch_bounds__(256) void wkv_steps_kernel(WkvArgs a) {
 // accumulators, which are the next product's operand as they lie.
 //
 // A factorises around the middle of the part: exp(E_t - M) exp(M - L_s) where
-// neither half decays by more than 2^-40; else it is summed pair by pair.
+// neither half decays by more than 2^-60; else it is summed pair by pair.
 // Whatever carries a decay, and the state, enters the MFMA as two bf16 terms.
+//
+// PIPE: 8 waves, four prepare 64 tokens while the other four walk the 64 before
+// (two sets of parts in LDS); else 4 waves do both in turn.
 //
 // A lane of a preparing wave has token lane & 15 and, of every 32 channels, the
 // 8 that a fragment of the products holds: 4 g + {0..3} and 16 + 4 g + {0..3},
@@ -192,7 +216,7 @@ struct WkvLds {
   static constexpr int O_A = R, O_K = R + A, O_D = O_K + 2 * K, O_V = O_D + NP * 4;
   static constexpr int PART = O_V + V, TOTAL = 4 * PART;
 };
-constexpr float WK_HALF = 40.f;
+constexpr float WK_HALF = 60.f;
 
 // 4 rows of one column: rows 4 g.., column (lane & 15) of the 16 from `col`
 __device__ __forceinline__ s16x4 wk_tr(const char* rows, int stride, int col, int lane) {
@@ -205,12 +229,13 @@ __device__ __forceinline__ float wk_left(float x) {
   return __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(x), 0x110 | N, 0xf, 0xf, true));
 }
 
-template <int NP>
-__global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void wkv_chunks_kernel(WkvArgs a) {
+template <int NP, bool PIPE>
+__global__ __launch_bounds__(PIPE ? 512 : 256, 1) void wkv_chunks_kernel(WkvArgs a) {
   using L = WkvLds<NP>;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   constexpr int PAIRS = L::PAIRS;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t16 = lane & 15, g = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3, t16 = lane & 15, g = lane >> 4;
+  const bool prepares = !PIPE || tid >= 256, walks = !PIPE || tid < 256;
   const int h = blockIdx.x, v0 = blockIdx.y * 64;
   const int4 e = a.ent[blockIdx.z];
   const int n = e.y, slot = min(max(e.z, 0), a.nslots - 1);
@@ -220,7 +245,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void wkv_chunks_kernel(WkvA
 #pragma unroll
   for (int i = 0; i < 2 * PAIRS; ++i) {
     S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (!fresh) S[i] = *reinterpret_cast<const f32x4*>(state + 16 * i);
+    if (walks && !fresh) S[i] = *reinterpret_cast<const f32x4*>(state + 16 * i);
   }
   const bf16_t* rb = reinterpret_cast<const bf16_t*>(a.r) + h * NP + 4 * g;
   const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.k) + h * NP + 4 * g;
@@ -245,112 +270,116 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void wkv_chunks_kernel(WkvA
 #pragma unroll
     for (int q = 0; q < 2; ++q) pv[q] = *reinterpret_cast<const i32x4*>(vb + mv * a.ld + q * 8);
   };
-  fetch(0);
-  for (int c0 = 0; c0 < n; c0 += 64) {
-    __syncthreads();  // the last 64 tokens are read
-    {                 // ------------------------------------------------ this wave's part
-      char* part = smem + wave * L::PART;
-      const bool live = c0 + wave * 16 + t16 < n;  // past the end: no decay, no key
-      f32x4 A = f32x4{0.f, 0.f, 0.f, 0.f};
-      float own = 0.f;
+  auto prepare = [&](int c0, char* buf) __attribute__((always_inline)) {  // this wave's part
+    char* part = buf + wave * L::PART;
+    s16x4 cr[PAIRS][2], ck[PAIRS][2];
+    f32x4 cl[PAIRS][2];
+    i32x4 cv[2] = {pv[0], pv[1]};
 #pragma unroll
-      for (int p = 0; p < PAIRS; ++p) {
-        float r[8], k[8], Lc[8], E[8], tot[8], mid[8], x[8], y[8];
-        float span = 0.f;
+    for (int p = 0; p < PAIRS; ++p)
+#pragma unroll
+      for (int q = 0; q < 2; ++q) cr[p][q] = pr[p][q], ck[p][q] = pk[p][q], cl[p][q] = pl[p][q];
+    if (PIPE && c0 + 64 < n) fetch(c0 + 64);
+    const bool live = c0 + wave * 16 + t16 < n;  // past the end: no decay, no key
+    f32x4 A = f32x4{0.f, 0.f, 0.f, 0.f};
+    float own = 0.f;
+#pragma unroll
+    for (int p = 0; p < PAIRS; ++p) {
+      float r[8], k[8], Lc[8], E[8], tot[8], mid[8], x[8], y[8];
+      float span = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int q = j >> 2, i = j & 3;
+        r[j] = bf2f_s(cr[p][q][i]);
+        k[j] = live ? bf2f_s(ck[p][q][i]) : 0.f;
+        const float la = live ? cl[p][q][i] * LOG2E : 0.f;
+        float s = la;
+        s += wk_left<1>(s);
+        s += wk_left<2>(s);
+        s += wk_left<4>(s);
+        s += wk_left<8>(s);
+        Lc[j] = s;
+        E[j] = s - la;
+        tot[j] = __shfl(s, (lane & 48) | 15, 64);
+        mid[j] = __shfl(s, (lane & 48) | 7, 64);
+        span = fmaxf(span, fmaxf(-mid[j], mid[j] - tot[j]));
+      }
+#pragma unroll
+      for (int q = 0; q < 2; ++q) {
+        const f32x4 u = *reinterpret_cast<const f32x4*>(ub + p * 32 + q * 16);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) own = fmaf(r[q * 4 + i] * u[i], k[q * 4 + i], own);
+      }
+      uint2 h0, h1, l0, l1;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        x[j] = r[j] * __builtin_amdgcn_exp2f(E[j]);
+        y[j] = k[j] * __builtin_amdgcn_exp2f(tot[j] - Lc[j]);
+      }
+      wk_split4(x, h0, l0);
+      wk_split4(x + 4, h1, l1);
+      *reinterpret_cast<bf16x8*>(part + (p * 2) * 1024 + lane * 16) = wk_frag(h0, h1);
+      *reinterpret_cast<bf16x8*>(part + (p * 2 + 1) * 1024 + lane * 16) = wk_frag(l0, l1);
+      wk_split4(y, h0, l0);
+      wk_split4(y + 4, h1, l1);
+      char* kr = part + L::O_K + t16 * L::KST + (p * 32 + 4 * g) * 2;
+      *reinterpret_cast<uint2*>(kr) = h0;
+      *reinterpret_cast<uint2*>(kr + 32) = h1;
+      *reinterpret_cast<uint2*>(kr + L::K) = l0;
+      *reinterpret_cast<uint2*>(kr + L::K + 32) = l1;
+      if (t16 == 0) {
+        float* d = reinterpret_cast<float*>(part + L::O_D) + p * 32 + 4 * g;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) d[(j >> 2) * 16 + (j & 3)] = __builtin_amdgcn_exp2f(tot[j]);
+      }
+      if (__all(span <= WK_HALF)) {
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          const int q = j >> 2, i = j & 3;
-          r[j] = bf2f_s(pr[p][q][i]);
-          k[j] = live ? bf2f_s(pk[p][q][i]) : 0.f;
-          const float la = live ? pl[p][q][i] * LOG2E : 0.f;
-          float s = la;
-          s += wk_left<1>(s);
-          s += wk_left<2>(s);
-          s += wk_left<4>(s);
-          s += wk_left<8>(s);
-          Lc[j] = s;
-          E[j] = s - la;
-          tot[j] = __shfl(s, (lane & 48) | 15, 64);
-          mid[j] = __shfl(s, (lane & 48) | 7, 64);
-          span = fmaxf(span, fmaxf(-mid[j], mid[j] - tot[j]));
-        }
-#pragma unroll
-        for (int q = 0; q < 2; ++q) {
-          const f32x4 u = *reinterpret_cast<const f32x4*>(ub + p * 32 + q * 16);
-#pragma unroll
-          for (int i = 0; i < 4; ++i) own = fmaf(r[q * 4 + i] * u[i], k[q * 4 + i], own);
-        }
-        uint2 h0, h1, l0, l1;
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          x[j] = r[j] * __builtin_amdgcn_exp2f(E[j]);
-          y[j] = k[j] * __builtin_amdgcn_exp2f(tot[j] - Lc[j]);
+          x[j] = r[j] * __builtin_amdgcn_exp2f(E[j] - mid[j]);
+          y[j] = k[j] * __builtin_amdgcn_exp2f(mid[j] - Lc[j]);
         }
         wk_split4(x, h0, l0);
         wk_split4(x + 4, h1, l1);
-        *reinterpret_cast<bf16x8*>(part + (p * 2) * 1024 + lane * 16) = wk_frag(h0, h1);
-        *reinterpret_cast<bf16x8*>(part + (p * 2 + 1) * 1024 + lane * 16) = wk_frag(l0, l1);
+        const bf16x8 xh = wk_frag(h0, h1), xl = wk_frag(l0, l1);
         wk_split4(y, h0, l0);
         wk_split4(y + 4, h1, l1);
-        char* kr = part + L::O_K + t16 * L::KST + (p * 32 + 4 * g) * 2;
-        *reinterpret_cast<uint2*>(kr) = h0;
-        *reinterpret_cast<uint2*>(kr + 32) = h1;
-        *reinterpret_cast<uint2*>(kr + L::K) = l0;
-        *reinterpret_cast<uint2*>(kr + L::K + 32) = l1;
-        if (t16 == 0) {
-          float* d = reinterpret_cast<float*>(part + L::O_D) + p * 32 + 4 * g;
+        const bf16x8 yh = wk_frag(h0, h1), yl = wk_frag(l0, l1);
+        f32x4 d = f32x4{0.f, 0.f, 0.f, 0.f};
+        d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yh, xh, d, 0, 0, 0);
+        d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yh, xl, d, 0, 0, 0);
+        d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yl, xh, d, 0, 0, 0);
+        A += d;
+      } else {
+        for (int sq = 0; sq < 4; ++sq)
 #pragma unroll
-          for (int j = 0; j < 8; ++j) d[(j >> 2) * 16 + (j & 3)] = __builtin_amdgcn_exp2f(tot[j]);
-        }
-        if (__all(span <= WK_HALF)) {
+          for (int i = 0; i < 4; ++i) {
+            const int src = (lane & 48) | (sq * 4 + i);
+            float v = 0.f;
 #pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            x[j] = r[j] * __builtin_amdgcn_exp2f(E[j] - mid[j]);
-            y[j] = k[j] * __builtin_amdgcn_exp2f(mid[j] - Lc[j]);
+            for (int j = 0; j < 8; ++j)
+              v = fmaf(r[j] * __shfl(k[j], src, 64), __builtin_amdgcn_exp2f(fminf(E[j] - __shfl(Lc[j], src, 64), 0.f)), v);
+            v += __shfl_xor(v, 16, 64);
+            v += __shfl_xor(v, 32, 64);
+            if (g == sq) A[i] += v;
           }
-          wk_split4(x, h0, l0);
-          wk_split4(x + 4, h1, l1);
-          const bf16x8 xh = wk_frag(h0, h1), xl = wk_frag(l0, l1);
-          wk_split4(y, h0, l0);
-          wk_split4(y + 4, h1, l1);
-          const bf16x8 yh = wk_frag(h0, h1), yl = wk_frag(l0, l1);
-          f32x4 d = f32x4{0.f, 0.f, 0.f, 0.f};
-          d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yh, xh, d, 0, 0, 0);
-          d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yh, xl, d, 0, 0, 0);
-          d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(yl, xh, d, 0, 0, 0);
-          A += d;
-        } else {
-          for (int sq = 0; sq < 4; ++sq)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              const int src = (lane & 48) | (sq * 4 + i);
-              float v = 0.f;
-#pragma unroll
-              for (int j = 0; j < 8; ++j)
-                v = fmaf(r[j] * __shfl(k[j], src, 64), __builtin_amdgcn_exp2f(fminf(E[j] - __shfl(Lc[j], src, 64), 0.f)), v);
-              v += __shfl_xor(v, 16, 64);
-              v += __shfl_xor(v, 32, 64);
-              if (g == sq) A[i] += v;
-            }
-        }
       }
-      own += __shfl_xor(own, 16, 64);
-      own += __shfl_xor(own, 32, 64);
-      float m[4];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) m[i] = 4 * g + i < t16 ? A[i] : 4 * g + i == t16 ? own : 0.f;
-      uint2 hi, lo;
-      wk_split4(m, hi, lo);
-      *reinterpret_cast<bf16x8*>(part + L::O_A + lane * 16) = wk_frag(hi, lo);
-#pragma unroll
-      for (int q = 0; q < 2; ++q)
-        *reinterpret_cast<i32x4*>(part + L::O_V + (lane >> 2) * L::VST + (lane & 3) * 32 + q * 16) = pv[q];
     }
-    __syncthreads();
-    if (c0 + 64 < n) fetch(c0 + 64);
+    own += __shfl_xor(own, 16, 64);
+    own += __shfl_xor(own, 32, 64);
+    float m[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) m[i] = 4 * g + i < t16 ? A[i] : 4 * g + i == t16 ? own : 0.f;
+    uint2 hi, lo;
+    wk_split4(m, hi, lo);
+    *reinterpret_cast<bf16x8*>(part + L::O_A + lane * 16) = wk_frag(hi, lo);
+#pragma unroll
+    for (int q = 0; q < 2; ++q)
+      *reinterpret_cast<i32x4*>(part + L::O_V + (lane >> 2) * L::VST + (lane & 3) * 32 + q * 16) = cv[q];
+  };
+  auto walk = [&](int c0, const char* buf) __attribute__((always_inline)) {  // the parts in order
     const int parts = min(4, (n - c0 + 15) >> 4);
-    for (int s = 0; s < parts; ++s) {  // -------------------------- the parts in order
-      const char* part = smem + s * L::PART;
+    for (int s = 0; s < parts; ++s) {
+      const char* part = buf + s * L::PART;
       const s16x4 v4 = wk_tr(part + L::O_V, L::VST, wave * 16, lane);
       const bf16x8 vv = {v4[0], v4[1], v4[2], v4[3], v4[0], v4[1], v4[2], v4[3]};
       f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -384,7 +413,25 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void wkv_chunks_kernel(WkvA
         if (t < n && v < a.dim) reinterpret_cast<bf16_t*>(a.y)[(size_t)(e.x + t) * a.ldy + h * a.dim + v] = f2bf(o[i]);
       }
     }
+  };
+  if (prepares) fetch(0);
+  if constexpr (PIPE) {
+    const int chunks = (n + 63) / 64;
+    for (int i = 0; i <= chunks; ++i) {
+      if (prepares && i < chunks) prepare(i * 64, smem + (i & 1) * L::TOTAL);
+      if (walks && i > 0) walk((i - 1) * 64, smem + ((i - 1) & 1) * L::TOTAL);
+      __syncthreads();
+    }
+  } else {
+    for (int c0 = 0; c0 < n; c0 += 64) {
+      __syncthreads();  // the last 64 tokens are read
+      prepare(c0, smem);
+      __syncthreads();
+      if (c0 + 64 < n) fetch(c0 + 64);
+      walk(c0, smem);
+    }
   }
+  if (!walks) return;
 #pragma unroll
   for (int i = 0; i < 2 * PAIRS; ++i) *reinterpret_cast<f32x4*>(state + 16 * i) = S[i];
 }
@@ -399,8 +446,14 @@ extern "C" int dnn_decay(const DecayArgs* a, int f32, hipStream_t st) {
     if (a->M > 65535) return -1;
     hipLaunchKernelGGL(decay_f32_kernel, dim3((a->N + 255) / 256, a->M), dim3(256), 0, st, *a);
   } else {
-    if (a->N % 64 != 0 || a->rank % 32 != 0 || (a->M + 63) / 64 > 65535) return -1;
-    hipLaunchKernelGGL(decay_kernel, dim3((a->N + 255) / 256, (a->M + 63) / 64), dim3(256), 0, st, *a);
+    const int rows = (a->M + 15) / 16;
+    if (a->N % 64 != 0 || a->rank % 32 != 0 || rows > 65535) return -1;
+    int cols = 64;  // per wave: wide where the rows alone fill the chip
+    while (cols < 256 && (long)rows * (a->N / (8 * cols)) >= 512) cols *= 2;
+    const dim3 grid((a->N + 4 * cols - 1) / (4 * cols), rows);
+    if (a->rank == 64) hipLaunchKernelGGL(decay_kernel<2>, grid, dim3(256), 0, st, *a, cols);
+    else if (a->rank == 128) hipLaunchKernelGGL(decay_kernel<4>, grid, dim3(256), 0, st, *a, cols);
+    else hipLaunchKernelGGL(decay_kernel<0>, grid, dim3(256), 0, st, *a, cols);
   }
   return (int)hipGetLastError();
 }
@@ -428,10 +481,10 @@ extern "C" int dnn_wkv_steps(const WkvArgs* a, int f32, hipStream_t st) {
 extern "C" int dnn_wkv_chunks(const WkvArgs* a, hipStream_t st) {
   if (!wkv_ok(*a)) return -1;
   const dim3 grid(a->H, a->NP / 64, a->nent);
-#define WC(N) hipLaunchKernelGGL((wkv_chunks_kernel<N>), grid, dim3(256), WkvLds<N>::TOTAL, st, *a)
-  if (a->NP == 64) WC(64);
-  else if (a->NP == 128) WC(128);
-  else WC(256);
+#define WC(N, P) hipLaunchKernelGGL((wkv_chunks_kernel<N, P>), grid, dim3(P ? 512 : 256), (P ? 2 : 1) * WkvLds<N>::TOTAL, st, *a)
+  if (a->NP == 64) WC(64, true);
+  else if (a->NP == 128) WC(128, false);
+  else WC(256, false);
 #undef WC
   return (int)hipGetLastError();
 }

@@ -303,7 +303,8 @@ def poly_norm(z: torch.Tensor, w: torch.Tensor, M: int, n: int, eps: float) -> N
 
 # ---------------------------------------------------------------------- attention over a latent cache
 LATENT_DIMS, LATENT_ROT = (128, 256, 512), (64, 128)  # latent columns and key-part columns the kernels are built for
-LATENT_ROWS = 64                                      # packed (token, head) rows of one workgroup
+LATENT_ROWS = (32, 64)                                # packed (token, head) rows of one workgroup
+LATENT_KEYS = (64, 128)                               # head sizes of keys and values for scores over keys
 
 
 def pad_to(n: int, sizes, what: str) -> int:
@@ -391,22 +392,68 @@ def latent_args(qlat: torch.Tensor, q: torch.Tensor, rot_col: int, hs: int, kp: 
     return a
 
 
-def latent_splits(n_seq: int, H: int, keys: int) -> int:
-    """Workgroups per 64 heads of a decoded token: one per CU, two pages each."""
+def latent_splits(n_seq: int, tiles: int, keys: int) -> int:
+    """Workgroups per tile of a decoded token (``tiles`` a token): one per CU, two pages each."""
     pages = -(-max(keys, 1) // PAGE)
-    return max(1, min(-(-256 // (n_seq * -(-H // LATENT_ROWS))), pages // 2, 64))
+    return max(1, min(-(-256 // (n_seq * tiles)), pages // 2, 64))
 
 
-def latent_attn(args, tiles: torch.Tensor, splits: int = 1, per_token: int = 1, ws: Optional[torch.Tensor] = None) -> None:
-    """``tiles`` (n, 4) int32: {first row, tokens, slot, first packed row of 64}
-    (``chunk_tiles`` with ``rows=LATENT_ROWS``).  ``splits`` > 1: single tokens,
-    ``per_token`` tiles each; ``ws``: fp32, tokens * H * splits * (CP + 2)."""
-    if tiles.dtype != torch.int32 or tiles.dim() != 2 or tiles.shape[1] != 4 or not tiles.is_contiguous():
-        raise ValueError("latent_attn: tiles must be contiguous int32 (n, 4)")
+def latent_ws(n_seq: int, H: int, splits: int, CP: int) -> int:
+    """fp32 partials of ``n_seq`` decoded tokens."""
+    return n_seq * H * splits * (CP + 4) if splits > 1 else 0
+
+
+def latent_attn(args, tiles: torch.Tensor, rows: int, splits: int = 1, per_token: int = 1,
+                ws: Optional[torch.Tensor] = None) -> None:
+    """``tiles`` (n, 4) int32: {first row, tokens, slot, first packed row of ``rows``}
+    (``chunk_tiles``).  ``splits`` > 1: single tokens, ``per_token`` tiles each;
+    ``ws``: fp32, ``latent_ws``."""
+    _tiles(tiles, "latent_attn")
     if splits > 1 and (ws is None or ws.dtype != torch.float32 or not ws.is_contiguous()):
         raise ValueError("latent_attn: splits > 1 needs an fp32 workspace")
-    check(lib().latent_attn(args, ptr(tiles), tiles.shape[0], splits, per_token, ptr(ws), 0 if ws is None else ws.numel(),
+    check(lib().latent_attn(args, ptr(tiles), tiles.shape[0], rows, splits, per_token, ptr(ws), 0 if ws is None else ws.numel(),
                             stream_ptr()), "latent_attn")
+
+
+def _tiles(t: torch.Tensor, what: str) -> None:
+    if t.dtype != torch.int32 or t.dim() != 2 or t.shape[1] != 4 or not t.is_contiguous():
+        raise ValueError(f"{what}: tiles must be contiguous int32 (n, 4)")
+
+
+def latent_gather(kp: torch.Tensor, table: torch.Tensor, ent: torch.Tensor, out: torch.Tensor) -> None:
+    """Cache pages to rows: ``ent`` (n, 4) int32 {first row of the page's 64, slot,
+    block, 0}; ``out`` (rows, CP + RP)."""
+    _latent_pool(kp, torch.bfloat16)
+    _tiles(ent, "latent_gather")
+    if out.dtype != kp.dtype or out.dim() != 2 or out.shape[1] != kp.shape[2] or not out.is_contiguous() \
+            or table.dtype != torch.int32 or table.dim() != 2 or not table.is_contiguous():
+        raise ValueError(f"latent_gather: rows {tuple(out.shape)} {out.dtype} of pages {tuple(kp.shape)}")
+    check(lib().latent_gather(ptr(kp), kp.shape[2], ptr(table), table.shape[1], kp.shape[0], ptr(ent), ent.shape[0], ptr(out),
+                              out.shape[0], stream_ptr()), "latent_gather")
+
+
+def latent_prefill(q: torch.Tensor, kv: torch.Tensor, krot: torch.Tensor, pos: torch.Tensor, out: torch.Tensor, M: int, H: int,
+                   DP: int, VP: int, scale: float, tiles: torch.Tensor, gate: Optional[torch.Tensor] = None) -> None:
+    """Causal attention over gathered keys: ``q`` rows [H][DP + RP], ``kv`` key rows
+    [H][DP | VP], ``krot`` key rows [RP], ``out`` rows [H][VP]; ``tiles`` (n, 4)
+    int32 {first row, tokens, first key row, first token of 128}."""
+    keys, RP = krot.shape
+    dt = torch.bfloat16
+    if DP not in LATENT_KEYS or VP not in LATENT_KEYS or RP not in LATENT_ROT or not scale > 0:
+        raise ValueError(f"latent_prefill: {DP} + {RP} key and {VP} value columns")
+    _rows(q, M, H * (DP + RP), "latent q", (dt,))
+    _rows(kv, keys, H * (DP + VP), "latent keys", (dt,))
+    _rows(krot, keys, RP, "latent key part", (dt,))
+    _rows(out, M, H * VP, "latent out", (dt,))
+    if gate is not None:
+        _rows(gate, M, H, "latent gate", (dt,))
+    _index(pos, M, "latent pos")
+    _tiles(tiles, "latent_prefill")
+    a = lib().LatentKeysArgs()
+    a.q, a.kv, a.krot, a.pos, a.out, a.gate = ptr(q), ptr(kv), ptr(krot), ptr(pos), ptr(out), ptr(gate)
+    a.ldq, a.ldkv, a.ldr, a.ldo, a.ldg = (t.stride(0) if t is not None else 0 for t in (q, kv, krot, out, gate))
+    a.M, a.H, a.DP, a.RP, a.VP, a.keys, a.scale = M, H, DP, RP, VP, keys, scale
+    check(lib().latent_prefill(a, ptr(tiles), tiles.shape[0], stream_ptr()), "latent_prefill")
 
 
 def latent_attn_f32(args) -> None:

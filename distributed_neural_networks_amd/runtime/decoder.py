@@ -35,7 +35,7 @@ from ..ops import mixer_ops as M_
 from ..ops import transformer_ops as T_
 from ..ops.gemm import decode_workspace
 from .decoder_layers import LAYERS, DynamicTanh, ScalarNorm, Weights, pad
-from .paging import StepBatch, pages_for, tile_lists
+from .paging import LatentHeads, StepBatch, pages_for, tile_lists
 from .stages import StageCompute, StageOutput
 
 DTYPES = {None: torch.bfloat16, "bf16": torch.bfloat16, "bfloat16": torch.bfloat16, "fp32": torch.float32,
@@ -135,6 +135,7 @@ class DecoderStage(StageCompute):
         self.buf = {k: z(v, torch.float32 if k in F32_BUFFERS else dt) for k, v in cols.items() if v}
         self._experts: Dict[tuple, M_.Routing] = {}
         self._expert_rows: Dict[str, torch.Tensor] = {}
+        self._flat: Dict[str, torch.Tensor] = {}
         if self.side:
             self.g = z(D_.pad64(self.side))
             self.z = z(D_.pad64(self.side)) if self.f32 else None
@@ -173,6 +174,13 @@ class DecoderStage(StageCompute):
 
     def expert_scratch(self, cols: int, s: slice) -> torch.Tensor:
         return self._grown("gu", s.stop, cols)[s, :cols]
+
+    def scratch(self, name: str, rows: int, cols: int) -> torch.Tensor:
+        """Dense rows that no graph and no concurrent microbatch uses (prefill)."""
+        t = self._flat.get(name)
+        if t is None or t.numel() < rows * cols:
+            t = self._flat[name] = torch.empty((rows * cols,), dtype=self.dtype, device=self.device)
+        return t[:rows * cols].view(rows, cols)
 
     def _grown(self, name: str, rows: int, cols: int) -> torch.Tensor:
         t = self._expert_rows.get(name)
@@ -322,6 +330,10 @@ class DecoderStage(StageCompute):
         return out
 
     # ------------------------------------------------------------------ ring step
+    def _tiles(self, chunks, ones, starts=None) -> Dict[object, torch.Tensor]:
+        return {k: torch.tensor(v, dtype=torch.int32, device=self.device)
+                for k, v in tile_lists(self.groups, chunks, ones, starts).items()}
+
     def _ring_batch(self, pos: torch.Tensor, B: int, T: int, b0: int) -> StepBatch:
         """B sequences of T tokens on cache rows [b0, b0 + B), each with fixed pages."""
         dev, W = self.device, self.row_pages
@@ -340,13 +352,18 @@ class DecoderStage(StageCompute):
                  "ends": (first + (T - 1)).repeat_interleave(T).contiguous(),
                  "rows": torch.arange(B * T, dtype=torch.int32, device=dev), "chunks": []}
             seqs = [(i * T, T, b0 + i) for i in range(B)]
-            lists = tile_lists(self.groups, seqs, []) if T > 1 else tile_lists(self.groups, [], seqs)
-            c["tiles"] = {k: torch.tensor(v, dtype=torch.int32, device=dev) for k, v in lists.items()}
             if T > 1:
                 c["chunks"] = seqs
                 c["steps"] = torch.arange(T, dtype=torch.int32, device=dev)
+            else:
+                c["tiles"] = self._tiles([], seqs)
             self._ring[(B, T, b0)] = c
-        p = pos if T == 1 else (pos.view(B, 1) + c["steps"]).view(-1).contiguous()
+        p = pos
+        if T > 1:
+            p = (pos.view(B, 1) + c["steps"]).view(-1).contiguous()
+            starts = pos.tolist() if any(isinstance(g, LatentHeads) for g in self.groups) else None
+            if c.get("starts", ()) != starts:  # tiles over a latent cache depend on the portions' places
+                c["tiles"], c["starts"] = self._tiles(c["chunks"], [], starts), starts
         return StepBatch(M=B * T, pos=p, slots=c["slots"], table=self._ring_table,
                          dec_rows=c["rows"] if T == 1 else None, n_dec=B if T == 1 else 0, chunks=c["chunks"],
                          max_len=self.max_seq, ent=c["ent"], start=c["start"], last=c["ends"], tiles=c["tiles"])

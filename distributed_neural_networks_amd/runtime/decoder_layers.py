@@ -488,17 +488,21 @@ class WkvMixer:
 
 class LatentAttentionMixer:
     """One projection to [query latent | latent | key part | gate]; the heads'
-    query projection to [unrotated | rotated] parts; the key projection applied
-    to the query and the value projection to the summed latents, both head by head."""
+    query projection to [unrotated | rotated] parts.  Over latents: the key
+    projection applied to the query and the value projection to the summed
+    latents, both head by head.  Over keys (long portions): both applied to the
+    sequence's gathered latents, one projection."""
     reads_copy = True
 
     def __init__(self, ld: Weights, m: tizalorn.LatentAttentionConfig):
-        self.m, self.tiles = m, LatentHeads(m.heads)
-        self.groups: List = [self.tiles]
+        self.m = m
         H, D, R, V = m.heads, m.dim, m.rot_dim, m.vdim
         self.cp, self.rp = D_.pad_to(m.kv_rank, D_.LATENT_DIMS, "latent size"), D_.pad_to(R, D_.LATENT_ROT, "rotated size")
         self.dp, self.vp, self.qp = D_.pad64(D), D_.pad64(V), D_.pad64(m.q_rank)
         self.hs = self.dp + self.rp
+        by_keys = ld.dtype == torch.bfloat16 and self.dp in D_.LATENT_KEYS and self.vp in D_.LATENT_KEYS
+        self.tiles = LatentHeads(H, self.cp, self.dp, self.vp, by_keys)
+        self.groups: List = [self.tiles]
         kv = ld("dkv")
         parts = [ld.rows("dq", self.qp), pad(kv[:m.kv_rank], self.cp, ld.wp), pad(kv[m.kv_rank:], self.rp, ld.wp),
                  ld.rows("g", H)]
@@ -512,6 +516,9 @@ class LatentAttentionMixer:
         uk, uv = ld("uk").view(H, D, m.kv_rank), ld("uv").view(H, V, m.kv_rank)
         self.w_uk = M_.ExpertLinear([pad(w.t().contiguous(), self.cp, self.dp) for w in uk], ld.dtype, ld.device)
         self.w_uv = M_.ExpertLinear([pad(w, self.vp, self.cp) for w in uv], ld.dtype, ld.device)
+        if by_keys:
+            ukv = torch.cat([pad(uk, H, self.dp, self.cp), pad(uv, H, self.vp, self.cp)], 1)
+            self.w_ukv = ld.linear(ukv.reshape(-1, self.cp))
         self.w_o = ld.linear(pad(pad(ld("o").view(ld.width, H, V), ld.width, H, self.vp).reshape(ld.width, -1), ld.wp,
                                  H * self.vp))
         self.rope = D_.Rope(*m.rot.frequencies(), ld.device)
@@ -524,32 +531,39 @@ class LatentAttentionMixer:
         return {"kp": torch.zeros((st.num_pages, PAGE, self.cp + self.rp), dtype=st.dtype, device=st.device)}
 
     def splits(self, n: int, keys: int) -> int:
-        return D_.latent_splits(n, self.m.heads, keys)
+        return D_.latent_splits(n, self.tiles.per_token, keys)
 
     def ws_need(self, n: int, keys: int) -> int:
-        s = self.splits(n, keys)
-        return n * self.m.heads * s * (self.cp + 2) if s > 1 else 0
+        return D_.latent_ws(n, self.m.heads, self.splits(n, keys), self.cp)
 
     def run(self, st, cache, b: StepBatch, s: slice, gws, ws) -> dict:
-        m, H, M, B, kp = self.m, self.m.heads, b.M, st.buf, cache["kp"]
+        m, H, M, B, kp, g = self.m, self.m.heads, b.M, st.buf, cache["kp"], self.tiles
         rows = self.w_in(st.h[s], B["in"][s, :self.n_in], gws)
         D_.latent_prep(rows, kp, self.qw, self.cw, self.rope, b.table, b.slots, b.pos, M, m.q_rank, m.kv_rank, self.cp,
                        st.eps)
         q = self.w_uq(rows[:, :self.qp], B["q"][s, :H * self.hs], gws)
         D_.rope_rows(q, M, H, self.hs, self.dp, self.rp, b.pos, self.rope)
-        heads = lambda t, n: t.unflatten(1, (H, n)).transpose(0, 1)  # noqa: E731  (M, H n) -> (H, M, n)
-        qlat, olat, out = (B[k][s, :H * n] for k, n in (("qlat", self.cp), ("olat", self.cp), ("mix", self.vp)))
-        self.w_uk.each(heads(q, self.hs)[..., :self.dp], heads(qlat, self.cp))
-        args = D_.latent_args(qlat, q, self.dp, self.hs, kp, b.table, b.slots, b.pos, olat, M, H, self.cp, m.scale,
-                              rows[:, self.gate_col:])
-        if st.f32:
-            D_.latent_attn_f32(args)
-        else:
-            if b.chunks:
-                D_.latent_attn(args, b.tiles[self.tiles, "chunks"])
-            if b.n_dec:
-                D_.latent_attn(args, b.tiles[self.tiles, "ones"], self.splits(b.n_dec, b.max_len), self.tiles.per_token, ws)
-        self.w_uv.each(heads(olat, self.cp), heads(out, self.vp))
+        out, gate = B["mix"][s, :H * self.vp], rows[:, self.gate_col:]
+        over, ones, keys = (b.tiles.get((g, k)) for k in ("chunks", "ones", "keys"))
+        if st.f32 or over is not None or ones is not None:
+            heads = lambda t, n: t.unflatten(1, (H, n)).transpose(0, 1)  # noqa: E731  (M, H n) -> (H, M, n)
+            qlat, olat = (B[k][s, :H * self.cp] for k in ("qlat", "olat"))
+            self.w_uk.each(heads(q, self.hs)[..., :self.dp], heads(qlat, self.cp))
+            args = D_.latent_args(qlat, q, self.dp, self.hs, kp, b.table, b.slots, b.pos, olat, M, H, self.cp, m.scale, gate)
+            if st.f32:
+                D_.latent_attn_f32(args)
+            if not st.f32 and over is not None:
+                D_.latent_attn(args, over, D_.LATENT_ROWS[1])
+            if not st.f32 and ones is not None:
+                D_.latent_attn(args, ones, g.rows, self.splits(b.n_dec, b.max_len), g.per_token, ws)
+            self.w_uv.each(heads(olat, self.cp), heads(out, self.vp))
+        if keys is not None:  # after the others: every row of `out` is written above
+            pages = b.tiles[g, "pages"]
+            n = pages.shape[0] * PAGE
+            lat = st.scratch("latents", n, self.cp + self.rp)
+            D_.latent_gather(kp, b.table, pages, lat)
+            kv = self.w_ukv(lat[:, :self.cp], st.scratch("keys", n, H * (self.dp + self.vp)))
+            D_.latent_prefill(q, kv, lat[:, self.cp:], b.pos, out, M, H, self.dp, self.vp, m.scale, keys, gate)
         return {"y": self.w_o(out, st.y[s], gws), "mult": 1.0}
 
 

@@ -104,29 +104,62 @@ class StepBatch:
     tiles: Optional[Dict[object, torch.Tensor]] = None
 
 
+KEY_ROWS = 1 << 15    # most keys of a step that are projected to heads
+KEY_TOKENS = 32       # fewest tokens of a portion that does so
+
+
 @dataclass(frozen=True)
 class LatentHeads:
     """Attention of ``heads`` heads over one latent cache, as an entry of a
-    stage's ``groups`` (an int there: query heads per KV head)."""
+    stage's ``groups`` (an int there: query heads per KV head).  ``latent``,
+    ``dim``, ``vdim``: padded columns of a latent, of a head's unrotated key and
+    of its value; ``by_keys``: portions may be scored over keys."""
     heads: int
+    latent: int = 128
+    dim: int = 64
+    vdim: int = 64
+    by_keys: bool = False
+
+    @property
+    def rows(self) -> int:
+        """Packed rows of a single token's tile."""
+        return LATENT_ROWS[0] if self.heads <= LATENT_ROWS[0] else LATENT_ROWS[1]
 
     @property
     def per_token(self) -> int:
-        return -(-self.heads // LATENT_ROWS)
+        return -(-self.heads // self.rows)
+
+    def over_keys(self, n: int, p0: int) -> bool:
+        """Is a portion of ``n`` tokens from position ``p0`` on cheaper over keys?
+        What its scores save, against the projection of the keys before it."""
+        per_key = self.latent * (self.dim + self.vdim)
+        return self.by_keys and n >= KEY_TOKENS and n * (p0 + n / 2) * (2 * self.latent - self.dim - self.vdim) > p0 * per_key
 
 
-def tile_lists(groups: Sequence, chunks: Sequence[tuple], ones: Sequence[tuple]) -> Dict[object, list]:
+def tile_lists(groups: Sequence, chunks: Sequence[tuple], ones: Sequence[tuple],
+               starts: Optional[Sequence[int]] = None) -> Dict[object, list]:
     """Workgroups of the attention launches of a step.  ``chunks`` / ``ones``:
-    (first row, tokens, slot) of the sequences that bring several tokens / one.
-    Key ``g`` (query heads per KV head): prefill tiles; ``(LatentHeads, "chunks")``
-    and ``(LatentHeads, "ones")``: tiles of either kind of sequence."""
+    (first row, tokens, slot) of the sequences that bring several tokens / one;
+    ``starts``: first positions of the chunks, where known.  Key ``g`` (query
+    heads per KV head): prefill tiles; for a ``LatentHeads``: ``(g, "chunks")`` and
+    ``(g, "ones")``, tiles of either kind of sequence over latents; ``(g, "keys")``,
+    tiles over keys, with the pages to gather in ``(g, "pages")``."""
     out: Dict[object, list] = {}
     for g in groups:
-        if isinstance(g, LatentHeads):
-            out[g, "chunks"] = [t for c in chunks for t in chunk_tiles(*c, g.heads, LATENT_ROWS)]
-            out[g, "ones"] = [t for c in ones for t in chunk_tiles(*c, g.heads, LATENT_ROWS)]
-        else:
+        if not isinstance(g, LatentHeads):
             out[g] = [t for c in chunks for t in chunk_tiles(*c, g)]
+            continue
+        over, keys, pages, rows = [], [], [], 0
+        for i, (row, n, slot) in enumerate(chunks):
+            blocks = 0 if starts is None else pages_for(starts[i] + n)
+            if blocks and g.over_keys(n, starts[i]) and rows + blocks * PAGE <= KEY_ROWS:
+                keys += chunk_tiles(row, n, rows, 1)
+                pages += [(rows + b * PAGE, slot, b, 0) for b in range(blocks)]
+                rows += blocks * PAGE
+            else:
+                over += chunk_tiles(row, n, slot, g.heads, LATENT_ROWS[1])
+        out[g, "chunks"], out[g, "keys"], out[g, "pages"] = over, keys, pages
+        out[g, "ones"] = [t for c in ones for t in chunk_tiles(*c, g.heads, g.rows)]
     return {k: v for k, v in out.items() if v}
 
 
@@ -134,7 +167,7 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
     """``entries``: (token ids, first position, slot, wanted places) per
     sequence.  ``groups``: the kinds of attention of the model's layers
     (``tile_lists``).  Everything travels in one host-to-device copy."""
-    ids, pos, slots, dec, want, chunks, start, last = [], [], [], [], [], [], [], []
+    ids, pos, slots, dec, want, chunks, starts, start, last = [], [], [], [], [], [], [], [], []
     for toks, p0, slot, places in entries:
         n, row = len(toks), len(ids)
         if n == 0:
@@ -149,7 +182,8 @@ def build_batch(entries: Sequence[tuple], table: np.ndarray, groups: Sequence[in
             dec.append(row)
         else:
             chunks.append((row, n, slot))
-    tiles = tile_lists(groups, chunks, [(r, 1, slots[r]) for r in dec])
+            starts.append(p0)
+    tiles = tile_lists(groups, chunks, [(r, 1, slots[r]) for r in dec], starts)
     parts = [(k, np.array(t, dtype=np.int32).reshape(-1)) for k, t in tiles.items()]
     ent = [(r, n, slot, 0) for r, n, slot in chunks] + [(r, 1, slots[r], 0) for r in dec]
     parts += [("ent", np.array(ent, dtype=np.int32).reshape(-1)), ("start", np.array(start, dtype=np.int32)),

@@ -13,7 +13,7 @@ from distributed_neural_networks_amd import checkpoint as ckpt
 from distributed_neural_networks_amd.config import parse_pipeline
 from distributed_neural_networks_amd.models import build_golden_stage, default_ranges, model_info, tizalorn
 from distributed_neural_networks_amd.ops import decoder_ops as D_
-from distributed_neural_networks_amd.runtime.paging import LatentHeads, PageTable, build_batch
+from distributed_neural_networks_amd.runtime.paging import KEY_ROWS, LatentHeads, PageTable, build_batch, tile_lists
 
 
 # ------------------------------------------------------------------ configuration
@@ -104,18 +104,35 @@ def test_step_rows_and_latent_tiles():
     assert b.start.tolist() == [0, 1, 1, 1, 4, 5, 5] and b.last.tolist() == [0, 3, 3, 3, 4, 6, 6]
     assert b.tiles[g, "chunks"].tolist() == [[1, 3, s[1], 64], [1, 3, s[1], 0], [5, 2, s[3], 64], [5, 2, s[3], 0]]
     assert b.tiles[g, "ones"].tolist() == [[0, 1, s[0], 0], [4, 1, s[2], 0]]
-    assert LatentHeads(64).per_token == 1 and LatentHeads(65).per_token == 2
+    assert [(LatentHeads(n).rows, LatentHeads(n).per_token) for n in (1, 32, 33, 64, 65)] == [(32, 1), (32, 1), (64, 1),
+                                                                                           (64, 1), (64, 2)]
     assert all(v.data_ptr() % 16 == b.ids.data_ptr() % 16 for v in b.tiles.values())
     only = build_batch([([7], 64, s[0], [])], t.table, [g], "cpu")
     assert (g, "chunks") not in only.tiles
+
+
+def test_portions_over_keys():
+    """Long portions are scored over keys: their pages in rows of 64, as many as
+    fit, the others over latents; unknown places stay over latents."""
+    g = LatentHeads(2, 512, 128, 128, True)
+    chunks, starts = [(0, 200, 3), (200, 31, 1), (231, 40, 0), (271, 40, 2)], [70, 0, 0, 5000]
+    t = tile_lists([g], chunks, [(311, 1, 5)], starts)
+    assert t[g, "keys"] == [(0, 200, 0, 128), (0, 200, 0, 0), (231, 40, 320, 0)]
+    assert t[g, "pages"] == [(64 * i, 3, i, 0) for i in range(5)] + [(320, 0, 0, 0)]
+    assert t[g, "chunks"] == [(200, 31, 1, 0), (271, 40, 2, 64), (271, 40, 2, 0)] and t[g, "ones"] == [(311, 1, 5, 0)]
+    for other in (tile_lists([g], chunks, []), tile_lists([LatentHeads(2, 512, 128, 128)], chunks, [], starts)):
+        assert [k for _, k in other] == ["chunks"]
+    n = KEY_ROWS // 2
+    two = tile_lists([g], [(0, n, 0), (n, n, 1), (2 * n, n, 2)], [], [0, 0, 0])  # the third does not fit
+    assert len(two[g, "pages"]) == KEY_ROWS // 64 and {x[2] for x in two[g, "chunks"]} == {2}
 
 
 def test_padding_rules():
     assert [D_.pad_to(n, D_.LATENT_DIMS, "x") for n in (1, 128, 129, 300, 512)] == [128, 128, 256, 512, 512]
     with pytest.raises(ValueError):
         D_.pad_to(513, D_.LATENT_DIMS, "x")
-    assert D_.latent_splits(1, 16, 64) == 1 and D_.latent_splits(1, 16, 10000) > 8
-    assert D_.latent_splits(300, 16, 10000) == 1
+    assert D_.latent_splits(1, 1, 64) == 1 and D_.latent_splits(1, 1, 10000) > 8
+    assert D_.latent_splits(300, 1, 10000) == 1 and D_.latent_ws(3, 2, 1, 128) == 0
 
 
 # ------------------------------------------------------------------ what the inputs reveal

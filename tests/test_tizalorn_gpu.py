@@ -355,11 +355,11 @@ def run_latent_attention(dtype, H, CN, R, seqs, seed=0, standout=None):
         D_.latent_attn_f32(args)
     else:
         if b.chunks:
-            D_.latent_attn(args, b.tiles[gr, "chunks"])
+            D_.latent_attn(args, b.tiles[gr, "chunks"], 64)
         if b.n_dec:
             for splits in (1, 3, 7):
-                ws = torch.empty(b.n_dec * H * splits * (CP + 2), device=dev()) if splits > 1 else None
-                D_.latent_attn(args, b.tiles[gr, "ones"], splits, gr.per_token, ws)
+                ws = torch.empty(D_.latent_ws(b.n_dec, H, splits, CP), device=dev()) if splits > 1 else None
+                D_.latent_attn(args, b.tiles[gr, "ones"], gr.rows, splits, gr.per_token, ws)
                 if splits == 1:
                     one = out.clone()
                 assert rel(out, one) < 5e-3
@@ -393,6 +393,68 @@ def test_one_key_among_many_stands_out(dtype, new):
         got, ref = run_latent_attention(dtype, 3, 72, 20, [(T - new, new)], seed=key, standout={(0, key): 3.0})
         assert rel(got[-1], ref[-1]) < (1e-5 if dtype == "float32" else 1e-2), key
         assert rel(got, ref) < (1e-5 if dtype == "float32" else 1e-2), key
+
+
+@pytest.mark.parametrize("H,D,R,V,standout", [(1, 64, 64, 64, None), (5, 40, 20, 72, None), (3, 128, 64, 128, 3.0),
+                                              (2, 100, 128, 30, 3.0), (2, 64, 70, 128, None), (2, 128, 128, 128, None)])
+def test_attention_over_keys(H, D, R, V, standout):
+    """Portions over gathered pages: rows of the gathered pages, and attention
+    with a key part shared by the heads; in the second portion keys at page
+    borders outweigh all others."""
+    from distributed_neural_networks_amd.ops import decoder_ops as D_
+    from distributed_neural_networks_amd.runtime.paging import PAGE, LatentHeads, PageTable, build_batch, pages_for
+    g, dt = gen(H + D), torch.bfloat16
+    dp, vp, RP, scale = D_.pad64(D), D_.pad64(V), D_.pad_to(R, D_.LATENT_ROT, ""), 1.1 / math.sqrt(D + R)
+    gr = LatentHeads(H, 512, dp, vp, True)
+    seqs = [(0, 40), (70, 200), (0, 1), (2, 33), (0, 129), (300, 2), (63, 150)]
+    n_pages = sum(pages_for(a + n) for a, n in seqs) + 2
+    table = PageTable(n_pages, len(seqs))
+    table._free_pages = torch.randperm(n_pages, generator=g).tolist()
+    entries = []
+    for old, new in seqs:
+        s = table.admit()
+        table.reserve(s, old + new)
+        entries.append(([1] * new, old, s, []))
+    b = build_batch(entries, table.table, [gr], dev())
+    pages, tiles = b.tiles[gr, "pages"], b.tiles[gr, "keys"]
+    chosen = [i for i, (old, new) in enumerate(seqs) if gr.over_keys(new, old)]
+    assert chosen == [0, 1, 3, 4, 6] and pages.shape[0] == sum(pages_for(sum(seqs[i])) for i in chosen)
+    kp = torch.randn(n_pages, PAGE, 128 + RP, generator=g).to(dt).to(dev())
+    lat = torch.full((pages.shape[0] * PAGE, 128 + RP), 9.0, dtype=dt, device=dev())
+    D_.latent_gather(kp, b.table, pages, lat)
+    for row, slot, blk, _ in pages.tolist():
+        assert torch.equal(lat[row:row + PAGE], kp[table.table[slot, blk]])
+    pad = lambda t, n: torch.nn.functional.pad(t, (0, n - t.shape[-1]))  # noqa: E731
+    q, gate = torch.randn(b.M, H, D + R, generator=g).to(dt), torch.randn(b.M, H, generator=g).to(dt)
+    k, v, kr = (torch.randn(len(lat), n, generator=g).to(dt) for n in (H * D, H * V, R))
+    k, v = k.view(-1, H, D), v.view(-1, H, V)
+    base = {i: min(p[0] for p in pages.tolist() if p[1] == entries[i][2]) for i in chosen}
+    rows = {i: sum(n for _, n in seqs[:i]) for i in range(len(seqs))}
+    if standout:
+        last = q[rows[1] + 199]
+        for key in (0, 63, 64, 128, 269):
+            k[base[1] + key] = last[:, :D] * standout
+            kr[base[1] + key] = last[0, D:]
+    qp = torch.cat([pad(q[..., :D], dp), pad(q[..., D:], RP)], -1).reshape(b.M, -1).to(dev())
+    kv = torch.cat([pad(k, dp), pad(v, vp)], -1).reshape(len(lat), -1).to(dev())
+    lat[:, 128:] = pad(kr, RP).to(dev())
+    out = torch.full((b.M, H * vp + 8), 5.0, dtype=dt, device=dev())
+    D_.latent_prefill(qp, kv, lat[:, 128:], b.pos, out[:, :H * vp], b.M, H, dp, vp, scale, tiles, gate.to(dev()))
+    assert (out[:, H * vp:] == 5).all()
+    got = out[:, :H * vp].double().cpu().view(b.M, H, vp)
+    for i, (old, new) in enumerate(seqs):
+        o = got[rows[i]:rows[i] + new]
+        if i not in chosen:
+            assert (o == 5).all()
+            continue
+        ks = slice(base[i], base[i] + old + new)
+        sc = torch.stack([q[rows[i]:rows[i] + new, h].double() @ torch.cat([k[ks, h], kr[ks]], -1).double().t()
+                          for h in range(H)]) * scale
+        sc = sc.masked_fill(torch.arange(old + new) > (old + torch.arange(new))[:, None], -math.inf)
+        ref = torch.stack([torch.softmax(sc[h], -1) @ v[ks, h].double() for h in range(H)], 1)
+        ref = ref * torch.sigmoid(gate[rows[i]:rows[i] + new].double())[..., None]
+        err = (o[..., :V] - ref).flatten(1).norm(dim=1) / ref.flatten(1).norm(dim=1)
+        assert err.max() < 1.5e-2 and (o[..., V:] == 0).all(), (i, err.max())
 
 
 # ------------------------------------------------------------------ experts
