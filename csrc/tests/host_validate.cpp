@@ -105,6 +105,86 @@ int main() {
     expect_reject(dnn_qk_norm(&q, 0, st), "qk norm row too short");
     q.ldq = 192, q.nk = 65;
     expect_reject(dnn_qk_norm(&q, 0, st), "qk norm of more than the projection");
+    r.E = r.ldl = 8, r.group_top = 3;
+    expect_reject(dnn_route(&r, st), "route groups by three experts");
+    e.ldc = 64, e.offs = nullptr, e.rows = 3;
+    expect_reject(dnn_grouped_gemm(&e, st), "even product of rows that do not divide");
+    e.rows = 4, e.sa = 4;
+    expect_reject(dnn_grouped_gemm(&e, st), "even product at unaligned operands");
+  }
+  rb = ra, rb.y_joined = 1, rb.y_w = f, rb.y = f;
+  expect_reject(dnn_rows_update(&rb, 0, 0, st), "rows norm of a sum without rows");
+  {
+    PolyNormArgs a{p, f, 64, 1, 65, 1e-5f};
+    expect_reject(dnn_poly_norm(&a, 0, st), "poly norm past the row");
+    a.n = 64, a.w = nullptr;
+    expect_reject(dnn_poly_norm(&a, 0, st), "poly norm without weights");
+    PairArgs b{};
+    b.M = 1, b.nslots = 1, b.buckets = 0;
+    expect_reject(dnn_pair_rows(&b, st), "pair rows of no buckets");
+    b.buckets = 5, b.mul_prev = -1;
+    expect_reject(dnn_pair_rows(&b, st), "pair rows with a negative factor");
+    ShiftArgs s{};
+    s.M = 1, s.NP = s.ldx = s.ldo = 64, s.nslots = 1, s.n = 9;
+    expect_reject(dnn_token_shift(&s, 0, st), "token shift of nine mixes");
+    s.n = 1, s.ldx = 32;
+    expect_reject(dnn_token_shift(&s, 0, st), "token shift row too short");
+    DecayArgs d{};
+    d.M = 1, d.N = 64, d.rank = 48, d.ldt = 64;
+    expect_reject(dnn_decay(&d, 0, st), "decay rank % 32");
+    d.rank = 64, d.ldt = 32;
+    expect_reject(dnn_decay(&d, 1, st), "decay row too short");
+    WkvArgs w{};
+    w.M = 2, w.H = 2, w.NP = 64, w.dim = 64, w.nent = w.nslots = 1, w.ld = 128, w.ldy = 128;
+    w.state = f, w.pos = ip, w.la = f, w.u = f;
+    auto wkv = [&](auto edit, const char* what) {
+      WkvArgs x = w;
+      edit(x);
+      expect_reject(dnn_wkv_steps(&x, 0, st), what);
+      expect_reject(dnn_wkv_chunks(&x, st), what);
+    };
+    wkv([](WkvArgs& x) { x.NP = 96; }, "wkv head size 96");
+    wkv([](WkvArgs& x) { x.dim = 65; }, "wkv head past its padding");
+    wkv([](WkvArgs& x) { x.ld = 64; }, "wkv row too short");
+    wkv([](WkvArgs& x) { x.u = nullptr; }, "wkv without a bonus");
+    wkv([](WkvArgs& x) { x.nent = 0; }, "wkv of nothing");
+  }
+  {
+    RopeTable rt{nullptr, 4, 1.f};
+    expect_reject(dnn_rope_rows(p, 64, 64, 1, 2, 64, ip, &rt, 0, st), "rope past the row");
+    rt.pairs = 33;
+    expect_reject(dnn_rope_rows(p, 64, 64, 1, 1, 64, ip, &rt, 0, st), "rope more pairs than columns");
+    LatentPrepArgs a{};
+    a.M = 1, a.QP = a.RP = 64, a.CP = 128, a.ld = 256, a.QN = 64, a.CN = 129, a.rope.pairs = 4, a.ldt = a.npages = 1;
+    expect_reject(dnn_latent_prep(&a, 0, st), "latent norm past its padding");
+    a.CN = 128, a.ld = 192;
+    expect_reject(dnn_latent_prep(&a, 0, st), "latent row too short");
+    LatentAttnArgs b{};
+    b.M = b.H = 1, b.CP = 128, b.RP = b.hs = 64, b.ldql = b.ldo = 128, b.ldqr = 64, b.ldt = b.npages = 1, b.scale = 1.f;
+    b.table = b.slots = b.pos = ip;
+    auto latent = [&](auto edit, const char* what) {
+      LatentAttnArgs x = b;
+      edit(x);
+      expect_reject(dnn_latent_attn(&x, ip, 1, 32, 1, 1, nullptr, 0, st), what);
+      expect_reject(dnn_latent_attn_f32(&x, st), what);
+    };
+    latent([](LatentAttnArgs& x) { x.CP = 192; }, "latent size 192");
+    latent([](LatentAttnArgs& x) { x.ldo = 64; }, "latent result row too short");
+    latent([](LatentAttnArgs& x) { x.hs = 32; }, "latent rotated part past its head");
+    latent([](LatentAttnArgs& x) { x.table = nullptr; }, "latent without a block table");
+    expect_reject(dnn_latent_attn(&b, ip, 1, 48, 1, 1, nullptr, 0, st), "latent tiles of 48 rows");
+    expect_reject(dnn_latent_attn(&b, ip, 1, 32, 2, 1, nullptr, 0, st), "latent splits without a workspace");
+    expect_reject(dnn_latent_gather(p, 192, ip, 1, 1, ip, 0, p, 64, st), "latent gather of nothing");
+    LatentKeysArgs k{};
+    k.M = k.H = 1, k.keys = 64, k.DP = k.RP = k.VP = 64, k.ldq = k.ldkv = 128, k.ldr = k.ldo = 64, k.scale = 1.f, k.pos = ip;
+    auto keys = [&](auto edit, const char* what) {
+      LatentKeysArgs x = k;
+      edit(x);
+      expect_reject(dnn_latent_prefill(&x, ip, 1, st), what);
+    };
+    keys([](LatentKeysArgs& x) { x.DP = 96; }, "attention over keys of 96");
+    keys([](LatentKeysArgs& x) { x.ldkv = 64; }, "attention over keys, key row too short");
+    keys([](LatentKeysArgs& x) { x.keys = 0; }, "attention over no keys");
   }
   expect_reject(dnn_token_gate(p, 64, p, 64, p, 64, p, 24, 8, ip, 5, p, 64, 4, 24, 64, st), "token gate past the row");
   expect_reject(dnn_token_gate(p, 64, p, 64, nullptr, 64, p, 24, 0, ip, 5, p, 64, 4, 24, 64, st),
