@@ -37,7 +37,7 @@ __device__ __forceinline__ bf16x8 wk_frag(const uint2& a, const uint2& b) {
 }
 
 // ---------------------------------------------------------------- decay
-// A wave takes 16 rows x `cols` columns, grid (ceil(N / (4 cols)), ceil(M / 16));
+// A wave takes 16 R rows x `cols` columns, grid (ceil(N / (4 cols)), ceil(M / 16 R));
 // tanh in two bf16 terms, W2 rows [N][rank] in bf16.  KS: 32-column steps of the
 // rank whose terms stay in registers (0: formed again for every 64 columns).
 __device__ __forceinline__ void decay_terms(const float* tp, bf16x8& hi, bf16x8& lo) {
@@ -55,52 +55,64 @@ __device__ __forceinline__ void decay_terms(const float* tp, bf16x8& hi, bf16x8&
   hi = wk_frag(h0, h1), lo = wk_frag(l0, l1);
 }
 
-template <int KS>
+template <int KS, int R>
 __global__ __launch_bounds__(256) void decay_kernel(DecayArgs a, int cols) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4;
-  const int m = blockIdx.y * 16 + (lane & 15), first = (blockIdx.x * 4 + wave) * cols;
-  const float* tp = a.t + (size_t)min(m, a.M - 1) * a.ldt + 8 * g;
+  const int m0 = blockIdx.y * 16 * R + (lane & 15), first = (blockIdx.x * 4 + wave) * cols;
   const bf16_t* w2 = reinterpret_cast<const bf16_t*>(a.w2) + 8 * g;
-  bf16x8 hi[KS > 0 ? KS : 1], lo[KS > 0 ? KS : 1];
-  if constexpr (KS > 0) {
+  const float* tp[R];
+  bf16x8 hi[R][KS > 0 ? KS : 1], lo[R][KS > 0 ? KS : 1];
 #pragma unroll
-    for (int k = 0; k < KS; ++k) decay_terms(tp + k * 32, hi[k], lo[k]);
+  for (int r = 0; r < R; ++r) {
+    tp[r] = a.t + (size_t)min(m0 + 16 * r, a.M - 1) * a.ldt + 8 * g;
+    if constexpr (KS > 0) {
+#pragma unroll
+      for (int k = 0; k < KS; ++k) decay_terms(tp[r] + k * 32, hi[r][k], lo[r][k]);
+    }
   }
   for (int n0 = first; n0 < min(first + cols, a.N); n0 += 64) {
-    f32x4 acc[4];
+    f32x4 acc[R][4], w0[4];
     const bf16_t* wr[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int r = 0; r < R; ++r) acc[r][j] = f32x4{0.f, 0.f, 0.f, 0.f};
       wr[j] = w2 + (size_t)min(n0 + j * 16 + (lane & 15), a.N - 1) * a.rank;
+      w0[j] = *reinterpret_cast<const f32x4*>(a.w0 + min(n0 + j * 16 + 4 * g, a.N - 4));
     }
-    auto step = [&](int k, const bf16x8& h, const bf16x8& l) __attribute__((always_inline)) {
+    auto step = [&](int col, int k) __attribute__((always_inline)) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const bf16x8 w = *reinterpret_cast<const bf16x8*>(wr[j] + k);
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, h, acc[j], 0, 0, 0);
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, l, acc[j], 0, 0, 0);
+        const bf16x8 w = *reinterpret_cast<const bf16x8*>(wr[j] + col);
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          acc[r][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, hi[r][k], acc[r][j], 0, 0, 0);
+          acc[r][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, lo[r][k], acc[r][j], 0, 0, 0);
+        }
       }
     };
     if constexpr (KS > 0) {
 #pragma unroll
-      for (int k = 0; k < KS; ++k) step(k * 32, hi[k], lo[k]);
+      for (int k = 0; k < KS; ++k) step(k * 32, k);
     } else {
       for (int k = 0; k < a.rank; k += 32) {
-        decay_terms(tp + k, hi[0], lo[0]);
-        step(k, hi[0], lo[0]);
+#pragma unroll
+        for (int r = 0; r < R; ++r) decay_terms(tp[r] + k, hi[r][0], lo[r][0]);
+        step(k, 0);
       }
     }
-    if (m >= a.M) continue;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int n = n0 + j * 16 + 4 * g;
-      if (n >= a.N) continue;
-      const f32x4 w0 = *reinterpret_cast<const f32x4*>(a.w0 + n);
-      f32x4 o;
+    for (int r = 0; r < R; ++r) {
+      if (m0 + 16 * r >= a.M) continue;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] = fmaxf(-__builtin_amdgcn_exp2f((acc[j][i] + w0[i]) * LOG2E), LA_MIN);
-      *reinterpret_cast<f32x4*>(a.la + (size_t)m * a.N + n) = o;
+      for (int j = 0; j < 4; ++j) {
+        const int n = n0 + j * 16 + 4 * g;
+        if (n >= a.N) continue;
+        f32x4 o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = fmaxf(-__builtin_amdgcn_exp2f((acc[r][j][i] + w0[j][i]) * LOG2E), LA_MIN);
+        *reinterpret_cast<f32x4*>(a.la + (size_t)(m0 + 16 * r) * a.N + n) = o;
+      }
     }
   }
 }
@@ -446,14 +458,20 @@ extern "C" int dnn_decay(const DecayArgs* a, int f32, hipStream_t st) {
     if (a->M > 65535) return -1;
     hipLaunchKernelGGL(decay_f32_kernel, dim3((a->N + 255) / 256, a->M), dim3(256), 0, st, *a);
   } else {
-    const int rows = (a->M + 15) / 16;
+    const int R = a->M >= 1024 ? 4 : 1, rows = (a->M + 16 * R - 1) / (16 * R);
     if (a->N % 64 != 0 || a->rank % 32 != 0 || rows > 65535) return -1;
     int cols = 64;  // per wave: wide where the rows alone fill the chip
     while (cols < 256 && (long)rows * (a->N / (8 * cols)) >= 512) cols *= 2;
     const dim3 grid((a->N + 4 * cols - 1) / (4 * cols), rows);
-    if (a->rank == 64) hipLaunchKernelGGL(decay_kernel<2>, grid, dim3(256), 0, st, *a, cols);
-    else if (a->rank == 128) hipLaunchKernelGGL(decay_kernel<4>, grid, dim3(256), 0, st, *a, cols);
-    else hipLaunchKernelGGL(decay_kernel<0>, grid, dim3(256), 0, st, *a, cols);
+#define DECAY(K)                                                                                   \
+  {                                                                                                \
+    if (R == 1) hipLaunchKernelGGL((decay_kernel<K, 1>), grid, dim3(256), 0, st, *a, cols);        \
+    else hipLaunchKernelGGL((decay_kernel<K, 4>), grid, dim3(256), 0, st, *a, cols);               \
+  }
+    if (a->rank == 64) DECAY(2)
+    else if (a->rank == 128) DECAY(4)
+    else DECAY(0)
+#undef DECAY
   }
   return (int)hipGetLastError();
 }

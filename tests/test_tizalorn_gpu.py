@@ -167,7 +167,8 @@ def test_token_shift(dtype, schedule, lengths, NP, n):
 
 # ------------------------------------------------------------------ recurrence
 @pytest.mark.parametrize("dtype", ["bf16", "float32"])
-@pytest.mark.parametrize("M,N,rank", [(1, 64, 64), (5, 192, 64), (70, 4096, 64), (300, 320, 320), (64, 256, 576)])
+@pytest.mark.parametrize("M,N,rank", [(1, 64, 64), (5, 192, 64), (70, 4096, 64), (300, 320, 320), (64, 256, 576), (1025, 192, 64),
+                                      (1100, 64, 128), (1030, 128, 192)])
 def test_decay(dtype, M, N, rank):
     from distributed_neural_networks_amd.ops import mixer_ops as M_
     g = gen(M + N)
